@@ -20,15 +20,12 @@
 // tile's global loads in flight under the current tile's MFMAs (T14); online
 // softmax lane-local (query on the lane), max/row-sum in exp2 units with the
 // scale folded into one FMA, deferred rescale (T13, threshold 8).
-#include "common.h"
+#include "attn_tile.h"
 
 #include <type_traits>
 
 namespace {
 
-constexpr float kLog2e = 1.4426950408889634f;
-constexpr float kLn2 = 0.6931471805599453f;
-constexpr float kRescaleThr = 8.0f;
 
 // Diagnostic build only (-DKCA_ATTN_STAMPS, bench/attn_stamps.py): per-wave s_memtime segment
 // sums of the main loops, added into g_attn_stamps once per wave at the end (fwd slots 0..7,
@@ -78,32 +75,6 @@ struct FastFwdParams {
   int B, Sq, Sk, H, Hkv;
   float scale;
 };
-
-typedef __attribute__((address_space(3))) bf16x4 lds_bf16x4_t;
-typedef unsigned int u32x4 __attribute__((ext_vector_type(4)));
-
-__device__ __forceinline__ bf16x4 lds_tr4(const char* base, int byte_off) {
-  return __builtin_amdgcn_ds_read_tr16_b64_v4bf16(
-      (lds_bf16x4_t*)(reinterpret_cast<uintptr_t>(base + byte_off)));
-}
-
-__device__ __forceinline__ bf16x8 lds_b128(const char* base, int byte_off) {
-  return *reinterpret_cast<const bf16x8*>(base + byte_off);
-}
-
-// byte offset of 16-B chunk `ch` of row `row` in a [32][D] image (see header)
-template <int D>
-__device__ __forceinline__ int img_off(int row, int ch) {
-  return (row >> 3) * 16 * D + 512 * (ch >> 2) + 64 * (row & 7) + 16 * ((ch & 3) ^ ((row >> 2) & 3));
-}
-
-__device__ __forceinline__ bf16x8 cat8(bf16x4 a, bf16x4 b) {
-  return __builtin_shufflevector(a, b, 0, 1, 2, 3, 4, 5, 6, 7);
-}
-
-__device__ __forceinline__ uint32_t pk_bf16(float lo, float hi) {
-  return pack_bf16x2(lo, hi);
-}
 
 // buffer resource over one (batch, head) slice; the base is workgroup-uniform (readfirstlane'd so
 // the descriptor is provably scalar: no waterfall loop, T20)

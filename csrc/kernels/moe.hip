@@ -1,0 +1,482 @@
+// Mixture of gated experts: sigmoid router, grouping, expert products.
+//
+//   s = sigmoid(W_router h); the `top` experts with the largest scores take the token, with weight s
+//   expert(x) = W_down (silu(W_gate x) * (W_up x))
+// A weight scales the expert's input -- both first products are linear, so it multiplies their fp32 sums
+// before the activation -- or its output (`scale_in` 0). The router (and the shared expert's gate, one
+// more row) accumulates in fp32 and is never rounded.
+//
+//   route   scores, top-k, weights of each token (bf16: matrix cores, 16 tokens per workgroup)
+//   group   assignments sorted by expert and cut in row tiles that hold one expert each
+//   gemv    expert products of tiles of up to 8 rows: streams the weight rows on the vector units
+//           (decode; any dims, fp32 too)
+//   gemm    expert products of tiles of up to 128 rows on the matrix cores (prompts)
+// Expert weights are stacked: gate-and-up [E][2F][d] (gate rows first), down [E][d][F]. The sorted rows'
+// activations are [n][F], their outputs [n][d]; the residual pass (rms_shift.hip) sums a token's outputs
+// through `inv`.
+#include "common.h"
+
+namespace {
+
+typedef unsigned int u32x4 __attribute__((ext_vector_type(4)));
+
+template <typename E> __device__ __forceinline__ float lde(const E* p);
+template <> __device__ __forceinline__ float lde<float>(const float* p) { return *p; }
+template <> __device__ __forceinline__ float lde<bf16_t>(const bf16_t* p) { return bf2f(*p); }
+template <typename E> __device__ __forceinline__ void ste(E* p, float v);
+template <> __device__ __forceinline__ void ste<float>(float* p, float v) { *p = v; }
+template <> __device__ __forceinline__ void ste<bf16_t>(bf16_t* p, float v) { *p = f2bf(v); }
+
+__device__ __forceinline__ float sigmoid(float x) { return 1.f / (1.f + expf(-x)); }
+
+struct RouteArgs {
+  const void* h;       // [T][d]
+  const void* wr;      // [E][d]
+  const void* wsg;     // [d] shared expert's gate (nullable)
+  int* ids;            // [T][top]
+  float* wts;          // [T][top]
+  float* sg;           // [T]
+  int T, d, E, top;
+};
+
+// One wave: the top experts of one token from its logits z[E] (LDS); ties go to the lower index.
+__device__ __forceinline__ void pick(const RouteArgs& p, float* z, int t, int lane) {
+  for (int k = 0; k < p.top; ++k) {
+    float best = -INFINITY;
+    int bi = 0x7fffffff;
+    for (int e = lane; e < p.E; e += 64)
+      if (z[e] > best) best = z[e], bi = e;
+#pragma unroll
+    for (int o = 32; o > 0; o >>= 1) {
+      const float ob = __shfl_xor(best, o, 64);
+      const int oi = __shfl_xor(bi, o, 64);
+      if (ob > best || (ob == best && oi < bi)) best = ob, bi = oi;
+    }
+    if (bi >= p.E) bi = 0;  // (no finite score left)
+    if (lane == 0) {
+      p.ids[(long long)t * p.top + k] = bi;
+      p.wts[(long long)t * p.top + k] = sigmoid(best);
+      z[bi] = -INFINITY;
+    }
+    __builtin_amdgcn_fence(__ATOMIC_RELEASE, "wavefront");
+    __builtin_amdgcn_wave_barrier();
+    __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "wavefront");
+  }
+}
+
+// any dims and type: one token per workgroup, a wave per expert row
+template <typename E>
+__global__ void __launch_bounds__(256) route_rows_kernel(RouteArgs p) {
+  extern __shared__ float z[];  // [E + 1]
+  const int lane = threadIdx.x & 63, wv = threadIdx.x >> 6, t = blockIdx.x;
+  const E* h = reinterpret_cast<const E*>(p.h) + (long long)t * p.d;
+  const int n = p.E + (p.wsg ? 1 : 0);
+  for (int e = wv; e < n; e += 4) {
+    const E* w = e < p.E ? reinterpret_cast<const E*>(p.wr) + (long long)e * p.d : reinterpret_cast<const E*>(p.wsg);
+    float s = 0.f;
+    for (int i = lane; i < p.d; i += 64) s = fmaf(lde<E>(h + i), lde<E>(w + i), s);
+    s = wave_sum(s);
+    if (lane == 0) z[e] = s;
+  }
+  __syncthreads();
+  if (wv == 0) pick(p, z, t, lane);
+  if (threadIdx.x == 64 && p.wsg) p.sg[t] = sigmoid(z[p.E]);
+}
+
+// bf16: 16 tokens per workgroup, the K range cut over 8 waves, 64 experts at a time
+__global__ void __launch_bounds__(512) route_mfma_kernel(RouteArgs p) {
+  extern __shared__ __attribute__((aligned(16))) float lds[];  // z[16][zs], part[8][16][64]
+  const int n = p.E + (p.wsg ? 1 : 0), zs = (n + 63) / 64 * 64;
+  float *z = lds, *part = lds + 16 * zs;
+  const int tid = threadIdx.x, lane = tid & 63, wv = tid >> 6, r16 = lane & 15, g = lane >> 4;
+  const int t0 = blockIdx.x * 16, d = p.d;
+  const bf16_t* h = reinterpret_cast<const bf16_t*>(p.h) + (long long)min(t0 + r16, p.T - 1) * d;
+  const int nk = (d + 31) / 32;
+  for (int e0 = 0; e0 < n; e0 += 64) {
+    const bf16_t* w[4];
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      const int e = min(e0 + 16 * i + r16, n - 1);
+      w[i] = e < p.E ? reinterpret_cast<const bf16_t*>(p.wr) + (long long)e * d : reinterpret_cast<const bf16_t*>(p.wsg);
+    }
+    const int nt = min(4, (n - e0 + 15) / 16);
+    f32x4 acc[4];
+#pragma unroll
+    for (int i = 0; i < 4; ++i) acc[i] = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll 2
+    for (int k = wv; k < nk; k += 8) {
+      const int c = k * 32 + g * 8;
+      const u32x4 zero = {0u, 0u, 0u, 0u};
+      const u32x4 b = c < d ? *reinterpret_cast<const u32x4*>(h + c) : zero;
+#pragma unroll
+      for (int i = 0; i < 4; ++i)
+        if (i < nt) {
+          const u32x4 a = c < d ? *reinterpret_cast<const u32x4*>(w[i] + c) : zero;
+          acc[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8, a), __builtin_bit_cast(bf16x8, b),
+                                                           acc[i], 0, 0, 0);
+        }
+    }
+    __syncthreads();
+#pragma unroll
+    for (int i = 0; i < 4; ++i)
+#pragma unroll
+      for (int r = 0; r < 4; ++r) part[(wv * 16 + r16) * 64 + i * 16 + g * 4 + r] = acc[i][r];
+    __syncthreads();
+    for (int i = tid; i < 1024; i += 512) {
+      float s = 0.f;
+#pragma unroll
+      for (int w8 = 0; w8 < 8; ++w8) s += part[w8 * 1024 + i];
+      z[(i >> 6) * zs + e0 + (i & 63)] = s;
+    }
+  }
+  __syncthreads();
+  for (int r = wv; r < 16; r += 8) {
+    if (t0 + r >= p.T) break;
+    if (p.wsg && lane == 0) p.sg[t0 + r] = sigmoid(z[r * zs + p.E]);
+    pick(p, z + r * zs, t0 + r, lane);
+  }
+}
+
+// n assignments -> perm (sorted position -> assignment), inv (assignment -> sorted position), tiles
+// [ntiles][3] (expert, first sorted position, rows <= mt) and their count. One workgroup.
+__global__ void __launch_bounds__(1024) group_kernel(const int* ids, int n, int E, int mt, int* perm, int* inv,
+                                                     int* tiles, int* ntiles) {
+  extern __shared__ int sh[];  // cnt[E], off[E + 1], toff[E + 1]
+  int *cnt = sh, *off = sh + E, *toff = off + E + 1;
+  const int tid = threadIdx.x;
+  for (int e = tid; e < E; e += 1024) cnt[e] = 0;
+  __syncthreads();
+  for (int i = tid; i < n; i += 1024) atomicAdd(&cnt[ids[i]], 1);
+  __syncthreads();
+  if (tid < 64) {  // exclusive sums over the experts, 64 at a time
+    int co = 0, to = 0;
+    for (int e0 = 0; e0 < E; e0 += 64) {
+      const int e = e0 + tid, c = e < E ? cnt[e] : 0, t = (c + mt - 1) / mt;
+      int cs = c, ts = t;
+#pragma unroll
+      for (int o = 1; o < 64; o <<= 1) {
+        const int a = __shfl_up(cs, o, 64), b = __shfl_up(ts, o, 64);
+        if (tid >= o) cs += a, ts += b;
+      }
+      if (e < E) off[e] = co + cs - c, toff[e] = to + ts - t;
+      co += __shfl(cs, 63, 64);
+      to += __shfl(ts, 63, 64);
+    }
+    if (tid == 0) off[E] = co, toff[E] = to, *ntiles = to;
+  }
+  __syncthreads();
+  for (int e = tid; e < E; e += 1024) {
+    const int c = cnt[e];
+    for (int j = 0; j * mt < c; ++j) {
+      int* t = tiles + (toff[e] + j) * 3;
+      t[0] = e;
+      t[1] = off[e] + j * mt;
+      t[2] = min(mt, c - j * mt);
+    }
+  }
+  __syncthreads();
+  for (int e = tid; e < E; e += 1024) cnt[e] = off[e];
+  __syncthreads();
+  for (int i = tid; i < n; i += 1024) {  // (the order within an expert does not matter: rows are independent)
+    const int pos = atomicAdd(&cnt[ids[i]], 1);
+    perm[pos] = i;
+    inv[i] = pos;
+  }
+}
+
+struct ExpertArgs {
+  const void* x;        // gate-up: [T][K] token rows; down: [n][K] sorted rows
+  const void* w;        // [E][2N or N][K]
+  void* y;              // [n][N] sorted rows
+  const int* perm;
+  const float* wts;     // [n] by assignment
+  const int* tiles;
+  const int* ntiles;
+  int top, N, K, up, scale;  // up: gate-and-up (x gathered by token, silu product); scale: the weight applies here
+};
+
+// ------------------------------------------------------------------------------------------------ gemv
+// Workgroup: one tile (<= MT rows of one expert) x 4 waves, a wave streams two weight rows (gate and up
+// of one output, or two outputs); the activation rows of a K chunk are staged in LDS for the four.
+template <typename E, int MT, bool VEC>
+__global__ void __launch_bounds__(256) expert_gemv_kernel(ExpertArgs p) {
+  constexpr int KC = 2048, EPL = 16 / (int)sizeof(E), NL = KC / (64 * EPL);  // elements per lane and load
+  extern __shared__ __attribute__((aligned(16))) char raw[];
+  E* xs = reinterpret_cast<E*>(raw);  // [MT][KC]
+  if ((int)blockIdx.y >= *p.ntiles) return;
+  const int tid = threadIdx.x, lane = tid & 63, wv = tid >> 6;
+  const int* tl = p.tiles + blockIdx.y * 3;
+  const int ex = tl[0], lo = tl[1], nr = tl[2], K = p.K;
+  const int n0 = p.up ? blockIdx.x * 4 + wv : (blockIdx.x * 4 + wv) * 2;
+  const int rows = p.up ? 2 * p.N : p.N;
+  const int ra = min(n0, p.N - 1), rb = p.up ? p.N + ra : min(n0 + 1, p.N - 1);
+  const E* wa = reinterpret_cast<const E*>(p.w) + ((long long)ex * rows + ra) * K;
+  const E* wb = reinterpret_cast<const E*>(p.w) + ((long long)ex * rows + rb) * K;
+  float acc[2][MT];
+#pragma unroll
+  for (int r = 0; r < MT; ++r) acc[0][r] = acc[1][r] = 0.f;
+  for (int k0 = 0; k0 < K; k0 += KC) {
+    const int kn = min(KC, K - k0);
+    u32x4 va[NL], vb[NL];
+    if constexpr (VEC) {
+#pragma unroll
+      for (int i = 0; i < NL; ++i) {
+        const int k = (i * 64 + lane) * EPL;
+        if (k < kn) {
+          va[i] = __builtin_nontemporal_load(reinterpret_cast<const u32x4*>(wa + k0 + k));
+          vb[i] = __builtin_nontemporal_load(reinterpret_cast<const u32x4*>(wb + k0 + k));
+        }
+      }
+    }
+    __syncthreads();
+    for (int r = 0; r < nr; ++r) {
+      const long long src = p.up ? p.perm[lo + r] / p.top : lo + r;
+      const E* x = reinterpret_cast<const E*>(p.x) + src * K + k0;
+      if constexpr (VEC) {
+        for (int i = tid * EPL; i < kn; i += 256 * EPL)
+          *reinterpret_cast<u32x4*>(xs + r * KC + i) = *reinterpret_cast<const u32x4*>(x + i);
+      } else {
+        for (int i = tid; i < kn; i += 256) xs[r * KC + i] = x[i];
+      }
+    }
+    __syncthreads();
+    if constexpr (VEC) {
+#pragma unroll
+      for (int i = 0; i < NL; ++i) {
+        const int k = (i * 64 + lane) * EPL;
+        if (k < kn) {
+#pragma unroll
+          for (int r = 0; r < MT; ++r)
+            if (r < nr) {
+              const u32x4 x = *reinterpret_cast<const u32x4*>(xs + r * KC + k);
+#pragma unroll
+              for (int e = 0; e < 4; ++e) {
+                if constexpr (sizeof(E) == 2) {
+                  acc[0][r] = dot2_acc<0>(va[i][e], x[e], acc[0][r]);
+                  acc[1][r] = dot2_acc<0>(vb[i][e], x[e], acc[1][r]);
+                } else {
+                  acc[0][r] = fmaf(__uint_as_float(va[i][e]), __uint_as_float(x[e]), acc[0][r]);
+                  acc[1][r] = fmaf(__uint_as_float(vb[i][e]), __uint_as_float(x[e]), acc[1][r]);
+                }
+              }
+            }
+        }
+      }
+    } else {
+      for (int k = lane; k < kn; k += 64) {
+        const float a = lde<E>(wa + k0 + k), b = lde<E>(wb + k0 + k);
+#pragma unroll
+        for (int r = 0; r < MT; ++r)
+          if (r < nr) {
+            const float x = lde<E>(xs + r * KC + k);
+            acc[0][r] = fmaf(a, x, acc[0][r]);
+            acc[1][r] = fmaf(b, x, acc[1][r]);
+          }
+      }
+    }
+  }
+#pragma unroll
+  for (int r = 0; r < MT; ++r) {
+    if (r >= nr) break;
+    float a = wave_sum(acc[0][r]), b = wave_sum(acc[1][r]);
+    if (lane) continue;
+    if (p.scale) {
+      const float s = p.wts[p.perm[lo + r]];
+      a *= s;
+      b *= s;
+    }
+    E* y = reinterpret_cast<E*>(p.y) + (long long)(lo + r) * p.N;
+    if (p.up) {
+      if (n0 < p.N) ste<E>(y + n0, a * sigmoid(a) * b);
+    } else {
+      if (n0 < p.N) ste<E>(y + n0, a);
+      if (n0 + 1 < p.N) ste<E>(y + n0 + 1, b);
+    }
+  }
+}
+
+// ------------------------------------------------------------------------------------------------ gemm
+// bf16, 128 rows x 128 weight rows x 64 per step, 4 waves of 64 x 64 (32x32x16 tiles); weights are the A
+// operand, so a lane holds one activation row and runs of four outputs. up: a workgroup covers 64 gate
+// and the matching 64 up rows, each wave 32 of both.
+template <bool UP>
+__global__ void __launch_bounds__(256, 2) expert_gemm_kernel(ExpertArgs p) {
+  constexpr int BK = 64;
+  __shared__ __attribute__((aligned(16))) bf16_t sw[2][128 * BK], sx[2][128 * BK];
+  if ((int)blockIdx.y >= *p.ntiles) return;
+  const int tid = threadIdx.x, lane = tid & 63, wv = tid >> 6, l32 = lane & 31, hh = lane >> 5;
+  const int wn = wv >> 1, wm = wv & 1;
+  const int* tl = p.tiles + blockIdx.y * 3;
+  const int ex = tl[0], lo = tl[1], nr = tl[2], K = p.K, N = p.N;
+  const int n0 = blockIdx.x * (UP ? 64 : 128);
+  // staging: thread tid owns 16-B chunk tid % 8 of rows tid / 8 + 32 i
+  const int ch = tid & 7, sr = tid >> 3;
+  const bf16_t *wp[4], *xp[4];
+#pragma unroll
+  for (int i = 0; i < 4; ++i) {
+    const int r = sr + 32 * i;
+    long long wr;
+    if constexpr (UP) wr = (r < 64 ? 0 : N) + min(n0 + (r & 63), N - 1);
+    else wr = min(n0 + r, N - 1);
+    wp[i] = reinterpret_cast<const bf16_t*>(p.w) + ((long long)ex * (UP ? 2 * N : N) + wr) * K;
+    const int xr = lo + min(r, nr - 1);
+    const long long src = UP ? p.perm[xr] / p.top : xr;
+    xp[i] = reinterpret_cast<const bf16_t*>(p.x) + src * K;
+  }
+  u32x4 rw[4], rx[4];
+  auto load = [&](int k0) {
+    const int k = k0 + ch * 8;
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      rw[i] = k < K ? *reinterpret_cast<const u32x4*>(wp[i] + k) : u32x4{0u, 0u, 0u, 0u};
+      rx[i] = k < K ? *reinterpret_cast<const u32x4*>(xp[i] + k) : u32x4{0u, 0u, 0u, 0u};
+    }
+  };
+  auto store = [&](int b) {
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      const int r = sr + 32 * i, o = r * BK + ((ch ^ (r & 7)) << 3);
+      *reinterpret_cast<u32x4*>(&sw[b][o]) = rw[i];
+      *reinterpret_cast<u32x4*>(&sx[b][o]) = rx[i];
+    }
+  };
+  f32x16 acc[2][2];
+#pragma unroll
+  for (int i = 0; i < 2; ++i)
+#pragma unroll
+    for (int j = 0; j < 2; ++j)
+#pragma unroll
+      for (int r = 0; r < 16; ++r) acc[i][j][r] = 0.f;
+  int ar[2], br[2];
+#pragma unroll
+  for (int i = 0; i < 2; ++i) {
+    ar[i] = (UP ? i * 64 + wn * 32 : wn * 64 + i * 32) + l32;
+    br[i] = wm * 64 + i * 32 + l32;
+  }
+  const int nk = (K + BK - 1) / BK;
+  const bool live = wm * 64 < nr;
+  load(0);
+  store(0);
+  __syncthreads();
+  for (int t = 0; t < nk; ++t) {
+    const int b = t & 1;
+    if (t + 1 < nk) load((t + 1) * BK);
+    if (live) {
+#pragma unroll
+      for (int s = 0; s < BK / 16; ++s) {
+        bf16x8 a[2], x[2];
+#pragma unroll
+        for (int i = 0; i < 2; ++i) {
+          a[i] = *reinterpret_cast<const bf16x8*>(&sw[b][ar[i] * BK + (((2 * s + hh) ^ (ar[i] & 7)) << 3)]);
+          x[i] = *reinterpret_cast<const bf16x8*>(&sx[b][br[i] * BK + (((2 * s + hh) ^ (br[i] & 7)) << 3)]);
+        }
+#pragma unroll
+        for (int i = 0; i < 2; ++i)
+#pragma unroll
+          for (int j = 0; j < 2; ++j) acc[i][j] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(a[i], x[j], acc[i][j], 0, 0, 0);
+      }
+    }
+    if (t + 1 < nk) store(b ^ 1);
+    __syncthreads();
+  }
+#pragma unroll
+  for (int j = 0; j < 2; ++j) {
+    const int r = br[j];
+    if (r >= nr) continue;
+    const float s = p.scale ? p.wts[p.perm[lo + r]] : 1.f;
+    bf16_t* y = reinterpret_cast<bf16_t*>(p.y) + (long long)(lo + r) * N;
+#pragma unroll
+    for (int i = 0; i < (UP ? 1 : 2); ++i)
+#pragma unroll
+      for (int q = 0; q < 4; ++q) {
+        const int n = n0 + (UP ? wn * 32 : wn * 64 + i * 32) + 8 * q + 4 * hh;
+        if (n >= N) continue;  // (N % 4 == 0)
+        float o[4];
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+          if constexpr (UP) {
+            const float gt = acc[0][j][4 * q + e] * s, up = acc[1][j][4 * q + e] * s;
+            o[e] = gt * __builtin_amdgcn_rcpf(1.f + __expf(-gt)) * up;
+          } else {
+            o[e] = acc[i][j][4 * q + e] * s;
+          }
+        }
+        *reinterpret_cast<uint2*>(y + n) = make_uint2(pack_bf16x2(o[0], o[1]), pack_bf16x2(o[2], o[3]));
+      }
+  }
+}
+
+template <typename E, bool VEC>
+int gemv_go(const ExpertArgs& a, int mt, int max_tiles, hipStream_t s) {
+  const dim3 g((a.N + (a.up ? 4 : 8) - 1) / (a.up ? 4 : 8), max_tiles);
+#define GO(M)                                                                                                  \
+  do {                                                                                                         \
+    constexpr int lds = M * 2048 * (int)sizeof(E);                                                             \
+    auto kern = expert_gemv_kernel<E, M, VEC>;                                                                 \
+    if (lds > 48 * 1024 &&                                                                                     \
+        hipFuncSetAttribute((const void*)kern, hipFuncAttributeMaxDynamicSharedMemorySize, lds) != hipSuccess) \
+      return 5;                                                                                                \
+    hipLaunchKernelGGL(kern, g, dim3(256), lds, s, a);                                                         \
+  } while (0)
+  if (mt == 1) GO(1);
+  else if (mt == 2) GO(2);
+  else if (mt == 4) GO(4);
+  else if (mt == 8) GO(8);
+  else return 6;
+#undef GO
+  return hipGetLastError() == hipSuccess ? 0 : 4;
+}
+
+bool al16(const void* p) { return (uintptr_t)p % 16 == 0; }
+
+}  // namespace
+
+// dtype: 0 fp32, 1 bf16
+KCA_API int kca_moe_route(int dtype, const void* h, const void* wr, const void* wsg, void* ids, void* wts, void* sg,
+                          int T, int d, int E, int top, hipStream_t s) {
+  if (T < 1 || d < 1 || E < 1 || E > 1024 || top < 1 || top > E || !h || !wr || !ids || !wts || (wsg && !sg)) return 1;
+  const RouteArgs a{h, wr, wsg, (int*)ids, (float*)wts, (float*)sg, T, d, E, top};
+  if (dtype == 1 && d % 8 == 0 && al16(h) && al16(wr) && al16(wsg)) {
+    const int zs = (E + (wsg ? 1 : 0) + 63) / 64 * 64, lds = (16 * zs + 8 * 1024) * 4;
+    if (lds > 48 * 1024 && hipFuncSetAttribute((const void*)route_mfma_kernel, hipFuncAttributeMaxDynamicSharedMemorySize,
+                                               lds) != hipSuccess)
+      return 5;
+    hipLaunchKernelGGL(route_mfma_kernel, dim3((T + 15) / 16), dim3(512), lds, s, a);
+  } else if (dtype == 1) {
+    hipLaunchKernelGGL(route_rows_kernel<bf16_t>, dim3(T), dim3(256), (E + 1) * 4, s, a);
+  } else if (dtype == 0) {
+    hipLaunchKernelGGL(route_rows_kernel<float>, dim3(T), dim3(256), (E + 1) * 4, s, a);
+  } else {
+    return 3;
+  }
+  return hipGetLastError() == hipSuccess ? 0 : 4;
+}
+
+// tiles: [max_tiles][3] with max_tiles >= min(E, n) + n / mt
+KCA_API int kca_moe_group(const void* ids, int n, int E, int mt, void* perm, void* inv, void* tiles, int max_tiles,
+                          void* ntiles, hipStream_t s) {
+  if (n < 1 || E < 1 || E > 1024 || mt < 1 || !ids || !perm || !inv || !tiles || !ntiles) return 1;
+  if (max_tiles < (E < n ? E : n) + n / mt) return 2;
+  hipLaunchKernelGGL(group_kernel, dim3(1), dim3(1024), (3 * E + 2) * 4, s, (const int*)ids, n, E, mt, (int*)perm,
+                     (int*)inv, (int*)tiles, (int*)ntiles);
+  return hipGetLastError() == hipSuccess ? 0 : 4;
+}
+
+// One expert product of every tile. mt: the tiles' row limit (1, 2, 4, 8: gemv; 128: gemm, bf16 with
+// K % 8 == 0 and N % 4 == 0).
+KCA_API int kca_moe_expert(int dtype, const void* x, const void* w, void* y, const void* perm, const void* wts,
+                           const void* tiles, const void* ntiles, int max_tiles, int mt, int top, int N, int K, int up,
+                           int scale, hipStream_t s) {
+  if (max_tiles < 1 || max_tiles > 65535 || N < 1 || K < 1 || top < 1 || !x || !w || !y || !perm || !wts || !tiles || !ntiles) return 1;
+  const ExpertArgs a{x, w, y, (const int*)perm, (const float*)wts, (const int*)tiles, (const int*)ntiles, top, N, K, up, scale};
+  if (mt == 128) {
+    if (dtype != 1 || K % 8 || N % 4 || !al16(x) || !al16(w) || (uintptr_t)y % 8) return 10;
+    if (up) hipLaunchKernelGGL(expert_gemm_kernel<true>, dim3((N + 63) / 64, max_tiles), dim3(256), 0, s, a);
+    else hipLaunchKernelGGL(expert_gemm_kernel<false>, dim3((N + 127) / 128, max_tiles), dim3(256), 0, s, a);
+    return hipGetLastError() == hipSuccess ? 0 : 4;
+  }
+  const bool vec = K % (dtype == 1 ? 8 : 4) == 0 && al16(x) && al16(w);
+  if (dtype == 0) return vec ? gemv_go<float, true>(a, mt, max_tiles, s) : gemv_go<float, false>(a, mt, max_tiles, s);
+  if (dtype == 1) return vec ? gemv_go<bf16_t, true>(a, mt, max_tiles, s) : gemv_go<bf16_t, false>(a, mt, max_tiles, s);
+  return 3;
+}

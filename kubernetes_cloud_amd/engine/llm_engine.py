@@ -43,7 +43,8 @@ from concurrent.futures import Future
 
 import torch
 
-from .runner import ModelRunner, mix_seed
+from ..models.registry import family_of
+from .runner import mix_seed
 
 
 @dataclasses.dataclass
@@ -93,8 +94,9 @@ class LLMEngine:
                  max_prefill_tokens: int = 16384, runner=None, page_size: int | None = None,
                  kv_pages: int | None = None, prefill_chunk: int | None = None, pipeline: bool | None = None):
         # ``runner``: e.g. a tp_driver.CollectiveRunner that mirrors every call to TP follower ranks
-        self.runner = runner or ModelRunner(model, max_slots=max_slots, max_len=max_len, use_graphs=use_graphs,
-                                            page_size=page_size, kv_pages=kv_pages)
+        self.runner = runner or family_of(model.cfg).runner()(model, max_slots=max_slots, max_len=max_len,
+                                                              use_graphs=use_graphs, page_size=page_size,
+                                                              kv_pages=kv_pages)
         max_slots = self.runner.max_slots
         self.max_len = self.runner.max_len
         self.free = list(range(max_slots))[::-1]

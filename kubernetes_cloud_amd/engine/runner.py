@@ -74,7 +74,11 @@ class KVCache:
 
     def __init__(self, n_layers: int, slots: int, kv_heads: int, max_len: int, head_dim: int,
                  device, dtype=torch.bfloat16, page_size: int = 0, n_pages: int | None = None,
-                 layer_devices: list | None = None):
+                 layer_devices: list | None = None, layer_shapes: list | None = None):
+        """``layer_shapes``: per layer (key heads, key size, value heads, value size) where they differ from
+        ``kv_heads`` x ``head_dim`` for both."""
+        if layer_shapes is None:
+            layer_shapes = [(kv_heads, head_dim, kv_heads, head_dim)] * n_layers
         self.slots, self.max_len, self.scratch = slots, max_len, slots
         self.page_size = page_size
         self.device = torch.device(device)
@@ -89,7 +93,7 @@ class KVCache:
             # for beam forks (a fork copies a partial tail page before the old one is dropped)
             self.n_pages = int(n_pages or slots * (self.blocks + 1))
             self.scratch_page = self.n_pages
-            shape = (self.n_pages + 1, kv_heads, page_size, head_dim)
+            rows, per = self.n_pages + 1, page_size
             self.table_h = torch.full((slots + 1, self.blocks), self.n_pages, dtype=torch.int32)
             self.tables = {d: self.table_h.to(d) for d in self.devices}
             self.table = self.tables[self.device]
@@ -100,10 +104,12 @@ class KVCache:
         else:
             self.table = None
             self.n_pages = 0
-            shape = (slots + 1, kv_heads, max_len, head_dim)
+            rows, per = slots + 1, max_len
             self.tables = {}
-        self.k = [torch.zeros(shape, device=d, dtype=dtype) for d in self.layer_devices]
-        self.v = [torch.zeros(shape, device=d, dtype=dtype) for d in self.layer_devices]
+        self.k = [torch.zeros((rows, kh, per, kd), device=d, dtype=dtype)
+                  for d, (kh, kd, _, _) in zip(self.layer_devices, layer_shapes)]
+        self.v = [torch.zeros((rows, vh, per, vd), device=d, dtype=dtype)
+                  for d, (_, _, vh, vd) in zip(self.layer_devices, layer_shapes)]
 
     def nbytes(self) -> int:
         return sum(t.numel() * t.element_size() for t in self.k + self.v)
@@ -309,29 +315,339 @@ class DecodeHandle:
         return self._res
 
 
-class ModelRunner:
-    def __init__(self, model, max_slots: int = 32, max_len: int | None = None, use_graphs: bool | None = None,
-                 max_bans: int = 16, page_size: int | None = None, kv_pages: int | None = None):
+class SlotState:
+    """Recurrent state of the serving slots: named fp32 tensors [n, slots + 1, width], row ``slot`` of each
+    belonging to the slot's sequence (the last row is scratch, as in ``KVCache``). A sequence's state counts
+    as zero at position 0 -- the kernels test the position -- so a reused slot needs no clearing."""
+
+    def __init__(self, slots: int, widths: dict, device):
+        self.t = {k: torch.zeros(n, slots + 1, w, device=device, dtype=torch.float32) for k, (n, w) in widths.items()}
+
+    def __getitem__(self, k):
+        return self.t[k]
+
+    def nbytes(self) -> int:
+        return sum(t.numel() * 4 for t in self.t.values())
+
+    def fork(self, dst: list[int], src: list[int]):
+        """State of slots ``src`` -> ``dst`` (a permutation is safe: the right side is gathered first)."""
+        for t in self.t.values():
+            t[:, dst] = t[:, src]
+
+
+class StepRunner:
+    """What every model family's runner shares: slots, sampling inputs, HIP-graph decode steps, lookahead
+    chaining. A family provides ``self.cache``, ``prefill``, ``_step_buffers`` (its part of a bucket's static
+    buffers), ``_step_logits`` (the step of a bucket) and ``_eager_logits`` (one eager decode step)."""
+
+    pipelined = True       # supports decode_async (the engine's one-step lookahead)
+    mixed_steps = False    # forward_tokens: prompt portions and decoded tokens in one batch
+    multi_device = False
+    _embed_head = False    # the step head resolves chained tokens on the device
+
+    def __init__(self, model, max_slots: int, max_len: int | None, use_graphs: bool | None, max_bans: int):
         self.model = model.eval()
-        cfg = model.cfg
-        self.cfg = cfg
+        self.cfg = cfg = model.cfg
         p = next(model.parameters())
         self.device, self.dtype = p.device, p.dtype
         self.max_len = max_len or cfg.max_pos
+        self.V = cfg.vocab_size
+        self.max_slots = max_slots
+        self.max_bans = max_bans
+        self.seen = torch.zeros(max_slots + 1, self.V, dtype=torch.uint8, device=self.device)
+        on_gpu = self.device.type == "cuda"
+        self.use_graphs = on_gpu if use_graphs is None else (use_graphs and on_gpu)
+        self._graphs: dict = {}
+        self._pool = None
+        self._static: dict = {}
+        self.step_launches: dict = {}
+        self._outbufs: dict = {}
+        self._packs = {}  # packed weight twins of the matrix-core layer (_packed_w)
+
+    @staticmethod
+    def default_page_size() -> int:
+        return int(os.environ.get("KCA_KV_PAGE_SIZE", "64"))
+
+    def _step_buffers(self, Bb: int, Kb: int) -> dict:
+        raise NotImplementedError
+
+    def _step_logits(self, st: dict, Bb: int, Kb: int) -> torch.Tensor:
+        raise NotImplementedError
+
+    def _eager_logits(self, tokens, pos, slots, kv_lens, max_kv) -> torch.Tensor:
+        raise NotImplementedError
+
+    def _desc_fields(self, Bb: int) -> dict:
+        return {}
+
+    def _fill_desc(self, a, Bb: int, pos, slots):
+        pass
+
+    def _packed_w(self, w):
+        """The packed stream twin of a weight the matrix-core layer reads (``skinny_mm.pack_weight``):
+        built once, on the first (eager) step that uses it -- the graph-capture warm-up -- and kept for the
+        runner's life (KCA_MM_PACK=0: none, the row-major weight streams). Keyed by storage address,
+        shape and version (an in-place weight update re-packs)."""
+        if not smm.PACK:
+            return None
+        key = (w.data_ptr(), tuple(w.shape), w._version)
+        p = self._packs.get(key)
+        if p is None and not torch.cuda.is_current_stream_capturing():
+            p = self._packs[key] = smm.pack_weight(w.detach())
+        return p
+
+    def _static_for(self, Bb: int, Kb: int):
+        key = (Bb, Kb)
+        st = self._static.get(key)
+        if st is not None:
+            return st
+        NB = self.max_bans
+        pk = _Packed({"tokens": (torch.int64, Bb), "seeds": (torch.int64, Bb), "pos": (torch.int32, Bb),
+                      "slots": (torch.int32, Bb), "kv_lens": (torch.int32, Bb), "top_k": (torch.int32, Bb),
+                      "temperature": (torch.float32, Bb), "top_p": (torch.float32, Bb),
+                      "rep": (torch.float32, Bb), "bans": (torch.int32, Bb * NB),
+                      "chain": (torch.int32, Bb), **self._desc_fields(Bb)}, self.device)
+        ob = self._outbuf(Bb)
+        st = {
+            "pk": pk,
+            **self._step_buffers(Bb, Kb),
+            "sws": torch.empty(Bb * self.V, device=self.device, dtype=torch.float32),
+            **ob,
+        }
+        self._static[key] = st
+        return st
+
+    def _outbuf(self, Bb: int):
+        """Sampled ids (int64) and log-probs (fp32) of a batch bucket in ONE device buffer shared by its
+        kv-length buckets -- one D2H copy per step, and a chained token (decode_async) is read by the
+        next step's embedding kernel from a fixed address whatever kv bucket that step lands in --
+        with two pinned landing buffers (one per host pk buffer)."""
+        ob = self._outbufs.get(Bb)
+        if ob is None:
+            pin = self.device.type == "cuda"
+            dev = torch.empty(3 * Bb, device=self.device, dtype=torch.int32)
+            hs = [torch.empty(3 * Bb, dtype=torch.int32, pin_memory=pin) for _ in range(2)]
+            # "flip": the landing buffer of the latest launch, counted per BATCH bucket (every kv bucket of
+            # this Bb copies into these two buffers, so consecutive launches must alternate here even when
+            # they land in different kv buckets -- a per-(Bb, Kb) counter could hand two in-flight steps
+            # the same buffer)
+            ob = {"out": dev, "ids": dev[:2 * Bb].view(torch.int64), "lps": dev[2 * Bb:].view(torch.float32),
+                  "flip": [0], "out_h": hs, "ids_h": [h[:2 * Bb].view(torch.int64) for h in hs],
+                  "lps_h": [h[2 * Bb:].view(torch.float32) for h in hs]}
+            self._outbufs[Bb] = ob
+        return ob
+
+    def _step_body(self, st, Bb, Kb, mc=False):
+        n0 = _lib.LAUNCHES[0]
+        try:
+            self._step_body_inner(st, Bb, Kb, mc)
+        finally:
+            # native launches one decode step issues (counted when the step is built: eager, or graph capture)
+            self.step_launches[Bb] = _lib.LAUNCHES[0] - n0
+
+    def _step_body_inner(self, st, Bb, Kb, mc=False):
+        pk = st["pk"]
+        logits = self._step_logits(st, Bb, Kb)
+        dops.sample_logits(logits, temperature=pk.d("temperature"), top_k=pk.d("top_k"), top_p=pk.d("top_p"),
+                           rep_penalty=pk.d("rep"), seen=self.seen, slots=pk.d("slots"),
+                           ban_ids=pk.d("bans").view(Bb, self.max_bans), seeds=pk.d("seeds"), step=0,
+                           ws=st["sws"], out_ids=st["ids"], out_logprobs=st["lps"], mwg_complete=mc)
+
+    # ----------------------------------------------------------- beam search
+    @torch.no_grad()
+    def decode_topk(self, tokens: list[int], positions: list[int], slots: list[int], k: int):
+        """Eager decode step returning the top-k next-token log-probs per row
+        (beam search; K30). -> (logprobs [n, k] fp32, ids [n, k] int64) on device."""
+        dev = self.device
+        for s_, p_ in zip(slots, positions):
+            self.cache.reserve(s_, p_ + 1)
+        self.cache.sync()
+        tok = torch.tensor(tokens, device=dev, dtype=torch.long)
+        pos = torch.tensor(positions, device=dev, dtype=torch.int32)
+        sl = torch.tensor(slots, device=dev, dtype=torch.int32)
+        kl = pos + 1
+        max_kv = max(positions) + 1
+        logits = self._eager_logits(tok, pos, sl, kl, max_kv)
+        lp = torch.log_softmax(logits.float(), dim=-1)
+        return lp.topk(k, dim=-1)
+
+    @torch.no_grad()
+    def copy_slots(self, dst: list[int], src: list[int], upto: int):
+        """KV cache (and seen mask) of ``src`` slots -> ``dst`` slots, positions
+        [0, upto) (paged: prefix pages shared, see ``KVCache.fork``)."""
+        if not dst:
+            return
+        self.cache.fork(dst, src, upto)
+        self.cache.sync()
+        d = torch.tensor(dst, device=self.device, dtype=torch.long)
+        s = torch.tensor(src, device=self.device, dtype=torch.long)
+        self.seen[d] = self.seen[s]
+
+    def release(self, slot: int):
+        """A finished sequence's KV pages go back to the pool."""
+        self.cache.release(slot)
+
+    @torch.no_grad()
+    def decode(self, rows: list[dict]):
+        """rows: [{token, pos, slot, temperature, top_k, top_p, rep, seed, bans}]
+        -> (ids list[int], logprobs list[float]) of the next token per row."""
+        return self.decode_async(rows).result()
+
+    @torch.no_grad()
+    def decode_async(self, rows: list[dict], prev: DecodeHandle | None = None) -> DecodeHandle:
+        """Launch one decode step without waiting for it. A row whose
+        ``token`` is None takes its input token from ``prev``'s output row
+        ``src`` on the device (the previous step's sample, not yet seen by the
+        host), so the engine can launch step t+1 before reading step t: the GPU
+        never idles on the host's bookkeeping between steps."""
+        n = len(rows)
+        Bb = _next_pow2(n)
+        max_kv = max(r["pos"] for r in rows) + 1
+        Kb = min(_next_pow2(max_kv, 256), self.max_len)
+        if self.device.type != "cuda":
+            Bb = n  # GPU eager keeps the graph buckets so both paths run identical shapes
+        st = self._static_for(Bb, Kb)
+        pk = st["pk"]
+        pk.flip()
+        NB = self.max_bans
+        for r in rows:
+            self.cache.reserve(r["slot"], r["pos"] + 1)
+        self.cache.sync()
+        a = pk.np
+        tok, sd, pos, sl, kl = a["tokens"], a["seeds"], a["pos"], a["slots"], a["kv_lens"]
+        tk, te, tp, rp, bans = a["top_k"], a["temperature"], a["top_p"], a["rep"], a["bans"]
+        bans.fill(-1)
+        ch = a["chain"]
+        ch.fill(-1)
+        chain_dst, chain_src = [], []
+        for i in range(Bb):
+            if i < n:
+                r = rows[i]
+                t = r["token"]
+                if t is None:
+                    chain_dst.append(i)
+                    chain_src.append(int(r["src"]))
+                    t = 0
+                tok[i], pos[i], sl[i], kl[i] = t, r["pos"], r["slot"], r["pos"] + 1
+                te[i], tk[i], tp[i], rp[i] = r["temperature"], r["top_k"], r["top_p"], r["rep"]
+                sd[i] = r["seed"]
+                b = r.get("bans") or ()
+                if len(b) > NB:
+                    raise ValueError(f"{len(b)} banned ids > max_bans={NB}")
+                for j, t in enumerate(b):
+                    bans[i * NB + j] = t
+            else:  # padding row -> scratch slot
+                tok[i], pos[i], sl[i], kl[i] = 0, 0, self.cache.scratch, 1
+                te[i], tk[i], tp[i], rp[i], sd[i] = 0.0, 0, 1.0, 1.0, 0
+        if "rcos" in pk.fields or "pages" in pk.fields:
+            self._fill_desc(a, Bb, pos, sl)
+        # every row (padding rows are greedy) on the multi-workgroup sampler: no closing kernel; the
+        # step graphs are keyed by it too
+        mc = bool(((~(te[:Bb] > 0)) | ((tk[:Bb] >= 1) & (tk[:Bb] <= dops.MWG_KMAX))).all())
+        gk = (Bb, Kb, mc)
+        if chain_dst and prev is None:
+            raise ValueError("rows chain their token from a previous launch, but prev is None")
+        # chained tokens read on the device by the step's first kernel: the previous step wrote them into
+        # this bucket's shared output buffer (same batch bucket); otherwise copied into `tokens` below
+        # (not on a step that captures its graph: the capture's eager warm-up runs would read the chained
+        # token from the output buffer their own first run already overwrote)
+        fold = (bool(chain_dst) and Bb == 1 and self._embed_head
+                and prev.ids_dev.data_ptr() == st["ids"].data_ptr()
+                and (not self.use_graphs or gk in self._graphs))
+        if fold:
+            for d_, s_ in zip(chain_dst, chain_src):
+                ch[d_] = s_
+        pk.upload()
+        if chain_dst and not fold:
+            dst = pk.d("tokens")
+            m = len(chain_dst)
+            if chain_dst == chain_src == list(range(m)):  # the common case: same rows, same order
+                dst[:m].copy_(prev.ids_dev[:m])
+            else:
+                di = torch.tensor(chain_dst, dtype=torch.long).to(self.device, non_blocking=True)
+                si = torch.tensor(chain_src, dtype=torch.long).to(self.device, non_blocking=True)
+                dst.index_copy_(0, di, prev.ids_dev.index_select(0, si))
+        if self.use_graphs:
+            g = self._graphs.get(gk)
+            if g is None:
+                g = self._capture(st, Bb, Kb, mc)
+            g.replay()
+        else:
+            self._step_body(st, Bb, Kb, mc)
+        fl = st["flip"]
+        fl[0] ^= 1
+        k = fl[0]
+        ids_h, lps_h = st["ids_h"][k], st["lps_h"][k]
+        if self.device.type == "cuda":
+            st["out_h"][k].copy_(st["out"], non_blocking=True)  # ids + log-probs, one copy
+            ev = torch.cuda.Event()
+            ev.record()
+        else:
+            st["out_h"][k].copy_(st["out"])
+            ev = None
+        return DecodeHandle(ids_h, lps_h, n, ev, st["ids"])
+
+    def _step_state(self) -> list:
+        """Tensors a step advances (beyond the cache rows it rewrites with the same values)."""
+        return [self.seen]
+
+    def _capture(self, st, Bb, Kb, mc=False):
+        saved = [t.clone() for t in self._step_state()]
+        s = torch.cuda.Stream()
+        s.wait_stream(torch.cuda.current_stream())
+        with torch.cuda.stream(s):
+            for _ in range(2):  # warm up (allocator, hipBLASLt heuristics)
+                self._step_body(st, Bb, Kb, mc)
+        torch.cuda.current_stream().wait_stream(s)
+        for t, old in zip(self._step_state(), saved):  # the warm-up runs advanced it
+            t.copy_(old)
+        if self._pool is None:
+            self._pool = torch.cuda.graph_pool_handle()
+        g = torch.cuda.CUDAGraph()
+        # thread-local capture: the RCCL process-group watchdog thread polls its work events while a
+        # capture runs; under the default global mode that query fails ("operation not permitted when
+        # stream is capturing") and the watchdog aborts the process
+        with torch.cuda.graph(g, pool=self._pool, capture_error_mode="thread_local"):
+            self._step_body(st, Bb, Kb, mc)
+        self._graphs[(Bb, Kb, mc)] = g
+        return g
+
+    @torch.no_grad()
+    def sample_first(self, logits: torch.Tensor, rows: list[dict]):
+        """Sample from prefill logits [n, V] (row params as in ``decode``)."""
+        n = logits.shape[0]
+        dev = self.device
+        NB = self.max_bans
+        bans = torch.full((n, NB), -1, dtype=torch.int32)
+        for i, r in enumerate(rows):
+            for j, t in enumerate((r.get("bans") or ())[:NB]):
+                bans[i, j] = t
+        f = lambda k, dt: torch.tensor([r[k] for r in rows], dtype=dt, device=dev)  # noqa: E731
+        ids, lps = dops.sample_logits(
+            logits.contiguous(), temperature=f("temperature", torch.float32), top_k=f("top_k", torch.int32),
+            top_p=f("top_p", torch.float32), rep_penalty=f("rep", torch.float32), seen=self.seen,
+            slots=f("slot", torch.int32), ban_ids=bans.to(dev), seeds=f("seed", torch.int64), step=0,
+            mwg_complete=dops.mwg_complete_rows([r["temperature"] for r in rows], [r["top_k"] for r in rows]))
+        return ids.tolist(), lps.tolist()
+
+
+class ModelRunner(StepRunner):
+    def __init__(self, model, max_slots: int = 32, max_len: int | None = None, use_graphs: bool | None = None,
+                 max_bans: int = 16, page_size: int | None = None, kv_pages: int | None = None):
+        super().__init__(model, max_slots, max_len, use_graphs, max_bans)
+        cfg = self.cfg
         # local heads: a tensor-parallel shard holds H/tp of them (parallel.tensor_parallel)
         self.H = model.h[0].attn.n_heads
         self.Hkv = self.H * cfg.kv_heads // cfg.n_heads
         self.D = cfg.head_dim
-        self.V = cfg.vocab_size
         if page_size is None:
-            page_size = int(os.environ.get("KCA_KV_PAGE_SIZE", "64"))
+            page_size = self.default_page_size()
         # layer-split placement (parallel.layer_split): per-layer devices, the head's device
         self.layer_devs = [blk.ln_1.weight.device for blk in model.h]
         self.head_dev = model.ln_f.weight.device
         self.multi_device = len({str(d) for d in self.layer_devs + [self.device, self.head_dev]}) > 1
         self.cache = KVCache(cfg.n_layers, max_slots, self.Hkv, self.max_len, self.D, self.device, self.dtype,
                              page_size=page_size, n_pages=kv_pages, layer_devices=self.layer_devs)
-        self.max_slots = max_slots
         self.rot = cfg.rotary_dim
         self._rope = {}
         for d in self.cache.devices:
@@ -339,18 +655,12 @@ class ModelRunner:
         self.cos, self.sin = self._rope[self.device]
         self._rope_h = (self.cos.cpu().numpy(), self.sin.cpu().numpy()) if self.rot > 0 else None
         self._step_desc = None
-        self.seen = torch.zeros(max_slots + 1, self.V, dtype=torch.uint8, device=self.device)
-        self.max_bans = max_bans
         on_gpu = self.device.type == "cuda"
         if on_gpu:  # MI355X-tuned hipBLASLt/rocBLAS choices for the batched decode GEMMs (utils/tunable.py)
             from ..utils import tunable
             tunable.ensure(tunable.DECODE_FILE)
-        self.use_graphs = on_gpu if use_graphs is None else (use_graphs and on_gpu)
         if self.multi_device:
             self.use_graphs = False  # one graph cannot span devices; the split path runs eagerly
-        self._graphs: dict = {}
-        self._pool = None
-        self._static: dict = {}
         # parallel-residual models (GPT-J, NeoX): the MLP branch does not depend on attention, so at
         # decode its two weight-streaming GEMVs run on a side stream while the latency-bound attention
         # chain (split-K attention, combine, out-proj) runs on the main one -- both captured into the
@@ -394,8 +704,6 @@ class ModelRunner:
                           and (self._layer_kind == "seq"
                                or (self.H == self.Hkv and self.D % 8 == 0 and 64 < self.D <= 256)))
         self._fz: dict = {}
-        self.step_launches: dict = {}
-        self._outbufs: dict = {}
         self._chain_src = None
         # the fused step head gathers the token embedding itself (no learned positions / scale / LN on
         # the embedding) and resolves chained tokens on the device: KCA_DECODE_EMBED_HEAD=0 keeps the
@@ -410,7 +718,6 @@ class ModelRunner:
         # out-proj + fc_out one K-concatenated launch). KCA_DECODE_FUSED_BATCHED=0: per-projection path.
         d_model = cfg.hidden
         self.batched_steps = 0
-        self._packs = {}  # packed weight twins of the matrix-core layer (_packed_w)
         self.fused_steps = 0  # batch-1 fused-layer steps built (eager runs and graph captures)
         # (real TP: sequential layers only -- each row-parallel projection closed by the custom all-reduce's
         # residual + row-statistics tail, parallel/custom_ar.py res_stats)
@@ -759,19 +1066,6 @@ class ModelRunner:
             logits = gather_last_dim(logits, grp)
         return logits
 
-    def _packed_w(self, w):
-        """The packed stream twin of a weight the matrix-core layer reads (``skinny_mm.pack_weight``):
-        built once, on the first (eager) step that uses it -- the graph-capture warm-up -- and kept for the
-        runner's life (KCA_MM_PACK=0: none, the row-major weight streams). Keyed by storage address,
-        shape and version (an in-place weight update re-packs)."""
-        if not smm.PACK:
-            return None
-        key = (w.data_ptr(), tuple(w.shape), w._version)
-        p = self._packs.get(key)
-        if p is None and not torch.cuda.is_current_stream_capturing():
-            p = self._packs[key] = smm.pack_weight(w.detach())
-        return p
-
     def _layers_decode(self, tokens, pos, slots, kv_lens, max_kv, ws, obuf):
         m, cfg = self.model, self.cfg
         if self._fused_ok and tokens.shape[0] == 1 and obuf is not None:
@@ -873,28 +1167,25 @@ class ModelRunner:
             return gather_last_dim(skinny_linear(x, mod.local_weight(), mod.bias), mod.group)
         return skinny_linear(x, mod.weight, mod.bias, act)
 
-    def _static_for(self, Bb: int, Kb: int):
-        key = (Bb, Kb)
-        st = self._static.get(key)
-        if st is not None:
-            return st
-        NB = self.max_bans
-        pk = _Packed({"tokens": (torch.int64, Bb), "seeds": (torch.int64, Bb), "pos": (torch.int32, Bb),
-                      "slots": (torch.int32, Bb), "kv_lens": (torch.int32, Bb), "top_k": (torch.int32, Bb),
-                      "temperature": (torch.float32, Bb), "top_p": (torch.float32, Bb),
-                      "rep": (torch.float32, Bb), "bans": (torch.int32, Bb * NB),
-                      "chain": (torch.int32, Bb), **self._desc_fields(Bb)}, self.device)
+    def _step_buffers(self, Bb: int, Kb: int) -> dict:
         ws_n = dops.decode_ws_floats(Bb, self.H, self.Hkv, self.D, Kb)
-        ob = self._outbuf(Bb)
-        st = {
-            "pk": pk,
-            "ws": torch.zeros(max(ws_n, 1), device=self.device, dtype=torch.float32),  # zeroed: fan-in counters
-            "obuf": torch.empty(Bb, self.H * self.D, device=self.device, dtype=self.dtype),
-            "sws": torch.empty(Bb * self.V, device=self.device, dtype=torch.float32),
-            **ob,
-        }
-        self._static[key] = st
-        return st
+        return {"ws": torch.zeros(max(ws_n, 1), device=self.device, dtype=torch.float32),  # zeroed: fan-in counters
+                "obuf": torch.empty(Bb, self.H * self.D, device=self.device, dtype=self.dtype)}
+
+    def _step_logits(self, st, Bb, Kb):
+        pk = st["pk"]
+        # chained tokens resolved on the device by the fused B = 1 step head (_layers_decode_fused)
+        self._chain_src = (pk.d("chain"), st["ids"]) if (Bb == 1 and self._embed_head) else None
+        if "rcos" in pk.fields or "pages" in pk.fields:
+            self._step_desc = self._desc_views(pk, Bb)
+        try:
+            return self._layers_decode(pk.d("tokens"), pk.d("pos"), pk.d("slots"), pk.d("kv_lens"), Kb,
+                                         st["ws"], st["obuf"])
+        finally:
+            self._step_desc = None
+
+    def _eager_logits(self, tokens, pos, slots, kv_lens, max_kv):
+        return self._layers_decode(tokens, pos, slots, kv_lens, max_kv, None, None)
 
     def _desc_on(self, Bb: int) -> bool:
         return (_STEP_DESC and (Bb == 1 or _STEP_DESC_BATCHED) and self.device.type == "cuda"
@@ -928,222 +1219,6 @@ class ModelRunner:
         return (pk.d("rcos") if "rcos" in f else None, pk.d("rsin") if "rsin" in f else None,
                 pk.d("pages").view(Bb, self.cache.blocks) if "pages" in f else None)
 
-    def _outbuf(self, Bb: int):
-        """Sampled ids (int64) and log-probs (fp32) of a batch bucket in ONE device buffer shared by its
-        kv-length buckets -- one D2H copy per step, and a chained token (decode_async) is read by the
-        next step's embedding kernel from a fixed address whatever kv bucket that step lands in --
-        with two pinned landing buffers (one per host pk buffer)."""
-        ob = self._outbufs.get(Bb)
-        if ob is None:
-            pin = self.device.type == "cuda"
-            dev = torch.empty(3 * Bb, device=self.device, dtype=torch.int32)
-            hs = [torch.empty(3 * Bb, dtype=torch.int32, pin_memory=pin) for _ in range(2)]
-            # "flip": the landing buffer of the latest launch, counted per BATCH bucket (every kv bucket of
-            # this Bb copies into these two buffers, so consecutive launches must alternate here even when
-            # they land in different kv buckets -- a per-(Bb, Kb) counter could hand two in-flight steps
-            # the same buffer)
-            ob = {"out": dev, "ids": dev[:2 * Bb].view(torch.int64), "lps": dev[2 * Bb:].view(torch.float32),
-                  "flip": [0], "out_h": hs, "ids_h": [h[:2 * Bb].view(torch.int64) for h in hs],
-                  "lps_h": [h[2 * Bb:].view(torch.float32) for h in hs]}
-            self._outbufs[Bb] = ob
-        return ob
-
-    def _step_body(self, st, Bb, Kb, mc=False):
-        n0 = _lib.LAUNCHES[0]
-        try:
-            self._step_body_inner(st, Bb, Kb, mc)
-        finally:
-            # native launches one decode step issues (counted when the step is built: eager, or graph capture)
-            self.step_launches[Bb] = _lib.LAUNCHES[0] - n0
-
-    def _step_body_inner(self, st, Bb, Kb, mc=False):
-        pk = st["pk"]
-        # chained tokens resolved on the device by the fused B = 1 step head (_layers_decode_fused)
-        self._chain_src = (pk.d("chain"), st["ids"]) if (Bb == 1 and self._embed_head) else None
-        if "rcos" in pk.fields or "pages" in pk.fields:
-            self._step_desc = self._desc_views(pk, Bb)
-        try:
-            logits = self._layers_decode(pk.d("tokens"), pk.d("pos"), pk.d("slots"), pk.d("kv_lens"), Kb,
-                                         st["ws"], st["obuf"])
-        finally:
-            self._step_desc = None
-        dops.sample_logits(logits, temperature=pk.d("temperature"), top_k=pk.d("top_k"), top_p=pk.d("top_p"),
-                           rep_penalty=pk.d("rep"), seen=self.seen, slots=pk.d("slots"),
-                           ban_ids=pk.d("bans").view(Bb, self.max_bans), seeds=pk.d("seeds"), step=0,
-                           ws=st["sws"], out_ids=st["ids"], out_logprobs=st["lps"], mwg_complete=mc)
-
-    # ----------------------------------------------------------- beam search
-    @torch.no_grad()
-    def decode_topk(self, tokens: list[int], positions: list[int], slots: list[int], k: int):
-        """Eager decode step returning the top-k next-token log-probs per row
-        (beam search; K30). -> (logprobs [n, k] fp32, ids [n, k] int64) on device."""
-        dev = self.device
-        for s_, p_ in zip(slots, positions):
-            self.cache.reserve(s_, p_ + 1)
-        self.cache.sync()
-        tok = torch.tensor(tokens, device=dev, dtype=torch.long)
-        pos = torch.tensor(positions, device=dev, dtype=torch.int32)
-        sl = torch.tensor(slots, device=dev, dtype=torch.int32)
-        kl = pos + 1
-        max_kv = max(positions) + 1
-        logits = self._layers_decode(tok, pos, sl, kl, max_kv, None, None)
-        lp = torch.log_softmax(logits.float(), dim=-1)
-        return lp.topk(k, dim=-1)
-
-    @torch.no_grad()
-    def copy_slots(self, dst: list[int], src: list[int], upto: int):
-        """KV cache (and seen mask) of ``src`` slots -> ``dst`` slots, positions
-        [0, upto) (paged: prefix pages shared, see ``KVCache.fork``)."""
-        if not dst:
-            return
-        self.cache.fork(dst, src, upto)
-        self.cache.sync()
-        d = torch.tensor(dst, device=self.device, dtype=torch.long)
-        s = torch.tensor(src, device=self.device, dtype=torch.long)
-        self.seen[d] = self.seen[s]
-
-    def release(self, slot: int):
-        """A finished sequence's KV pages go back to the pool."""
-        self.cache.release(slot)
-
-    pipelined = True  # supports decode_async (the TP CollectiveRunner does not)
-
-    @torch.no_grad()
-    def decode(self, rows: list[dict]):
-        """rows: [{token, pos, slot, temperature, top_k, top_p, rep, seed, bans}]
-        -> (ids list[int], logprobs list[float]) of the next token per row."""
-        return self.decode_async(rows).result()
-
-    @torch.no_grad()
-    def decode_async(self, rows: list[dict], prev: DecodeHandle | None = None) -> DecodeHandle:
-        """Launch one decode step without waiting for it. A row whose
-        ``token`` is None takes its input token from ``prev``'s output row
-        ``src`` on the device (the previous step's sample, not yet seen by the
-        host), so the engine can launch step t+1 before reading step t: the GPU
-        never idles on the host's bookkeeping between steps."""
-        n = len(rows)
-        Bb = _next_pow2(n)
-        max_kv = max(r["pos"] for r in rows) + 1
-        Kb = min(_next_pow2(max_kv, 256), self.max_len)
-        if self.device.type != "cuda":
-            Bb = n  # GPU eager keeps the graph buckets so both paths run identical shapes
-        st = self._static_for(Bb, Kb)
-        pk = st["pk"]
-        pk.flip()
-        NB = self.max_bans
-        for r in rows:
-            self.cache.reserve(r["slot"], r["pos"] + 1)
-        self.cache.sync()
-        a = pk.np
-        tok, sd, pos, sl, kl = a["tokens"], a["seeds"], a["pos"], a["slots"], a["kv_lens"]
-        tk, te, tp, rp, bans = a["top_k"], a["temperature"], a["top_p"], a["rep"], a["bans"]
-        bans.fill(-1)
-        ch = a["chain"]
-        ch.fill(-1)
-        chain_dst, chain_src = [], []
-        for i in range(Bb):
-            if i < n:
-                r = rows[i]
-                t = r["token"]
-                if t is None:
-                    chain_dst.append(i)
-                    chain_src.append(int(r["src"]))
-                    t = 0
-                tok[i], pos[i], sl[i], kl[i] = t, r["pos"], r["slot"], r["pos"] + 1
-                te[i], tk[i], tp[i], rp[i] = r["temperature"], r["top_k"], r["top_p"], r["rep"]
-                sd[i] = r["seed"]
-                b = r.get("bans") or ()
-                if len(b) > NB:
-                    raise ValueError(f"{len(b)} banned ids > max_bans={NB}")
-                for j, t in enumerate(b):
-                    bans[i * NB + j] = t
-            else:  # padding row -> scratch slot
-                tok[i], pos[i], sl[i], kl[i] = 0, 0, self.cache.scratch, 1
-                te[i], tk[i], tp[i], rp[i], sd[i] = 0.0, 0, 1.0, 1.0, 0
-        if "rcos" in pk.fields or "pages" in pk.fields:
-            self._fill_desc(a, Bb, pos, sl)
-        # every row (padding rows are greedy) on the multi-workgroup sampler: no closing kernel; the
-        # step graphs are keyed by it too
-        mc = bool(((~(te[:Bb] > 0)) | ((tk[:Bb] >= 1) & (tk[:Bb] <= dops.MWG_KMAX))).all())
-        gk = (Bb, Kb, mc)
-        if chain_dst and prev is None:
-            raise ValueError("rows chain their token from a previous launch, but prev is None")
-        # chained tokens read on the device by the step's first kernel: the previous step wrote them into
-        # this bucket's shared output buffer (same batch bucket); otherwise copied into `tokens` below
-        # (not on a step that captures its graph: the capture's eager warm-up runs would read the chained
-        # token from the output buffer their own first run already overwrote)
-        fold = (bool(chain_dst) and Bb == 1 and self._embed_head
-                and prev.ids_dev.data_ptr() == st["ids"].data_ptr()
-                and (not self.use_graphs or gk in self._graphs))
-        if fold:
-            for d_, s_ in zip(chain_dst, chain_src):
-                ch[d_] = s_
-        pk.upload()
-        if chain_dst and not fold:
-            dst = pk.d("tokens")
-            m = len(chain_dst)
-            if chain_dst == chain_src == list(range(m)):  # the common case: same rows, same order
-                dst[:m].copy_(prev.ids_dev[:m])
-            else:
-                di = torch.tensor(chain_dst, dtype=torch.long).to(self.device, non_blocking=True)
-                si = torch.tensor(chain_src, dtype=torch.long).to(self.device, non_blocking=True)
-                dst.index_copy_(0, di, prev.ids_dev.index_select(0, si))
-        if self.use_graphs:
-            g = self._graphs.get(gk)
-            if g is None:
-                g = self._capture(st, Bb, Kb, mc)
-            g.replay()
-        else:
-            self._step_body(st, Bb, Kb, mc)
-        fl = st["flip"]
-        fl[0] ^= 1
-        k = fl[0]
-        ids_h, lps_h = st["ids_h"][k], st["lps_h"][k]
-        if self.device.type == "cuda":
-            st["out_h"][k].copy_(st["out"], non_blocking=True)  # ids + log-probs, one copy
-            ev = torch.cuda.Event()
-            ev.record()
-        else:
-            st["out_h"][k].copy_(st["out"])
-            ev = None
-        return DecodeHandle(ids_h, lps_h, n, ev, st["ids"])
-
-    def _capture(self, st, Bb, Kb, mc=False):
-        s = torch.cuda.Stream()
-        s.wait_stream(torch.cuda.current_stream())
-        with torch.cuda.stream(s):
-            for _ in range(2):  # warm up (allocator, hipBLASLt heuristics)
-                self._step_body(st, Bb, Kb, mc)
-        torch.cuda.current_stream().wait_stream(s)
-        if self._pool is None:
-            self._pool = torch.cuda.graph_pool_handle()
-        g = torch.cuda.CUDAGraph()
-        # thread-local capture: the RCCL process-group watchdog thread polls its work events while a
-        # capture runs; under the default global mode that query fails ("operation not permitted when
-        # stream is capturing") and the watchdog aborts the process
-        with torch.cuda.graph(g, pool=self._pool, capture_error_mode="thread_local"):
-            self._step_body(st, Bb, Kb, mc)
-        self._graphs[(Bb, Kb, mc)] = g
-        return g
-
-    @torch.no_grad()
-    def sample_first(self, logits: torch.Tensor, rows: list[dict]):
-        """Sample from prefill logits [n, V] (row params as in ``decode``)."""
-        n = logits.shape[0]
-        dev = self.device
-        NB = self.max_bans
-        bans = torch.full((n, NB), -1, dtype=torch.int32)
-        for i, r in enumerate(rows):
-            for j, t in enumerate((r.get("bans") or ())[:NB]):
-                bans[i, j] = t
-        f = lambda k, dt: torch.tensor([r[k] for r in rows], dtype=dt, device=dev)  # noqa: E731
-        ids, lps = dops.sample_logits(
-            logits.contiguous(), temperature=f("temperature", torch.float32), top_k=f("top_k", torch.int32),
-            top_p=f("top_p", torch.float32), rep_penalty=f("rep", torch.float32), seen=self.seen,
-            slots=f("slot", torch.int32), ban_ids=bans.to(dev), seeds=f("seed", torch.int64), step=0,
-            mwg_complete=dops.mwg_complete_rows([r["temperature"] for r in rows], [r["top_k"] for r in rows]))
-        return ids.tolist(), lps.tolist()
-
 
 def mix_seed(seed: int, step: int) -> int:
     """Per-(request, token) 64-bit Philox key as a signed int64."""
@@ -1154,4 +1229,4 @@ def mix_seed(seed: int, step: int) -> int:
     return x - (1 << 64) if x >= (1 << 63) else x
 
 
-__all__ = ["KVCache", "KVCacheFull", "ModelRunner", "DecodeHandle", "mix_seed", "math"]
+__all__ = ["KVCache", "KVCacheFull", "SlotState", "StepRunner", "ModelRunner", "DecodeHandle", "mix_seed", "math"]

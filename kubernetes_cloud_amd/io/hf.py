@@ -16,7 +16,8 @@ import torch
 
 from ..models.causal_lm import CausalLM, build_model
 from ..models.config import LMConfig
-from ..models.hf_convert import hf_to_native, is_ignorable_hf_key, native_to_hf
+from ..models.hf_convert import is_ignorable_hf_key
+from ..models.registry import family_of
 
 SAFE_NAME = "model.safetensors"
 
@@ -51,12 +52,13 @@ def has_weights(path: str) -> bool:
 
 
 def load_pretrained(path: str, device="cpu", dtype=torch.bfloat16, random_init_if_missing=False,
-                    cfg: LMConfig | None = None) -> CausalLM:
+                    cfg=None):
+    """Model of the family ``config.json`` names (``models.registry``) with the directory's weights."""
     cfg = cfg or LMConfig.from_pretrained(path)
     model = build_model(cfg, device=device, dtype=dtype, seed=0)
     if has_weights(path):
         sd = read_hf_state_dict(path)
-        nat = hf_to_native(sd, cfg)
+        nat = family_of(cfg).to_native(sd, cfg)
         missing, unexpected = model.load_state_dict({k: v.to(dtype) for k, v in nat.items()},
                                                     strict=False)
         missing = [m for m in missing if not m.endswith("alibi")]
@@ -84,22 +86,31 @@ def load_tensorized(uri: str, config_dir: str | None = None, device="cpu", dtype
         if "config" not in meta:
             raise FileNotFoundError(f"{uri}: no config.json given and no config in the file metadata")
         cfg = LMConfig.from_hf(meta["config"])
-    with torch.device("meta"):
-        model = CausalLM(cfg)
-    model = model.to(dtype).to_empty(device=device)  # cast on meta: no fp32 materialisation
+    if isinstance(cfg, LMConfig):
+        with torch.device("meta"):
+            model = CausalLM(cfg)
+        model = model.to(dtype).to_empty(device=device)  # cast on meta: no fp32 materialisation
+    else:
+        model = family_of(cfg).build(cfg, device=device, dtype=dtype, seed=None)
     stats = load_into_module(model, uri, device=device, threads=threads)
-    if cfg.alibi:
+    if getattr(cfg, "alibi", False):
         for blk in model.h:
             blk.attn.alibi = alibi_slopes(cfg.n_heads).to(device)
     return model, stats
+
+
+def _config_dict(cfg) -> dict:
+    d = cfg.to_hf()
+    if isinstance(cfg, LMConfig):  # HF dicts follow a resized vocabulary
+        d["vocab_size"] = cfg.vocab_size
+    return d
 
 
 def serialize_causal_lm(model: CausalLM, path: str, dtype: torch.dtype | None = None) -> dict:
     """``.tensors`` of a causal LM with its HF config embedded (so a URI alone
     is enough to rebuild it), e.g. ``model.tensors`` / ``gptj.tensors``."""
     from .tensors import serialize
-    hf_cfg = model.cfg.to_hf()
-    hf_cfg["vocab_size"] = model.cfg.vocab_size
+    hf_cfg = _config_dict(model.cfg)
     sd = {k: v for k, v in model.state_dict().items() if not k.endswith("alibi")}
     return serialize(sd, path, dtype=dtype, metadata={"config": hf_cfg, "kind": "causal_lm"})
 
@@ -110,13 +121,13 @@ def save_pretrained(model: CausalLM, path: str, max_shard_bytes: int = 10 << 30)
 
     os.makedirs(path, exist_ok=True)
     cfg = model.cfg
-    hf_cfg = cfg.to_hf()
-    hf_cfg["vocab_size"] = cfg.vocab_size
-    hf_cfg.setdefault("torch_dtype", str(next(model.parameters()).dtype).replace("torch.", ""))
+    hf_cfg = _config_dict(cfg)
+    if isinstance(cfg, LMConfig):
+        hf_cfg.setdefault("torch_dtype", str(next(model.parameters()).dtype).replace("torch.", ""))
     with open(os.path.join(path, "config.json"), "w") as f:
         json.dump(hf_cfg, f, indent=2)
     sd = {k: v.detach() for k, v in model.state_dict().items() if not k.endswith("alibi")}
-    hf = native_to_hf(sd, cfg)
+    hf = family_of(cfg).from_native(sd, cfg)
     hf = {k: v.contiguous().cpu() for k, v in hf.items()}
     total = sum(v.numel() * v.element_size() for v in hf.values())
     if total <= max_shard_bytes:

@@ -342,7 +342,13 @@ class CausalLM(nn.Module):
         return sum(p.numel() for p in self.parameters())
 
 
-def build_model(cfg: LMConfig, device="cpu", dtype=torch.bfloat16, seed: int | None = 0) -> CausalLM:
+def build_model(cfg, device="cpu", dtype=torch.bfloat16, seed: int | None = 0):
+    """Randomly initialised model of any registered family (``models.registry``)."""
+    from .registry import family_of
+    return family_of(cfg).build(cfg, device=device, dtype=dtype, seed=seed)
+
+
+def build_causal_lm(cfg: LMConfig, device="cpu", dtype=torch.bfloat16, seed: int | None = 0) -> CausalLM:
     with torch.device("meta"):
         m = CausalLM(cfg)
     m = m.to_empty(device=device).to(dtype)

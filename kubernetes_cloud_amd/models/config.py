@@ -16,6 +16,7 @@ import os
 
 
 SUPPORTED_MODEL_TYPES = ("gpt2", "gpt_neo", "gptj", "gpt_neox", "bloom", "xglm")
+SUPPORTED_ARCHITECTURES = ("Megusun",)  # native designs (models.registry), config.json "architecture"
 
 
 class UnsupportedModel(ValueError):
@@ -27,7 +28,8 @@ class UnsupportedModel(ValueError):
     def __init__(self, model_type: str):
         super().__init__(
             f"unsupported model_type {model_type!r}: the MI355X-native model families are "
-            f"{', '.join(SUPPORTED_MODEL_TYPES)} (GPT-2, GPT-Neo, GPT-J, GPT-NeoX/Pythia, BLOOM, XGLM/fairseq-dense). "
+            f"{', '.join(SUPPORTED_MODEL_TYPES)} (GPT-2, GPT-Neo, GPT-J, GPT-NeoX/Pythia, BLOOM, XGLM/fairseq-dense) "
+            f"and {', '.join(SUPPORTED_ARCHITECTURES)}. "
             "--trust-remote-code cannot add an architecture: remote modeling code is not executed; "
             "convert the checkpoint to one of these families")
         self.model_type = model_type
@@ -95,7 +97,14 @@ class LMConfig:
         return 6.0 * n + 12.0 * self.n_layers * self.hidden * seq
 
     @classmethod
-    def from_hf(cls, cfg: dict) -> "LMConfig":
+    def from_hf(cls, cfg: dict):
+        """Parsed config of any registered family: an ``LMConfig`` for HF configs (``model_type``), the
+        design's own config class for native ones (``architecture``)."""
+        from .registry import family_of_dict
+        return family_of_dict(cfg).read_config(cfg)
+
+    @classmethod
+    def read_hf(cls, cfg: dict) -> "LMConfig":
         mt = cfg.get("model_type", "")
         if mt == "gptj":
             d = cfg["n_embd"]
@@ -173,7 +182,7 @@ class LMConfig:
         raise UnsupportedModel(mt)
 
     @classmethod
-    def from_pretrained(cls, path: str) -> "LMConfig":
+    def from_pretrained(cls, path: str):
         with open(os.path.join(path, "config.json")) as f:
             return cls.from_hf(json.load(f))
 

@@ -1,0 +1,104 @@
+"""Decoders whose layers mix tokens differently (``HybridConfig``): differential attention or a gated
+recurrence, beside a dense, routed or no feed-forward, on an fp32 residual stream.
+
+A layer is parallel: with h the normed stream and hs its token-shifted copy,
+
+    x <- x + m (mixer(hs) + ff(h))
+
+The modules hold weights laid out for the kernels; the step itself (cache, state, batching) is
+``engine.hybrid_runner``. Layout:
+
+* ``w_in``   every projection of the mixer in one matrix ([q | k | v] or [z | x | g])
+* ``w_out``  the mixer's output projection and the dense (or shared-expert) down projection side by side,
+  [d, mixer + ff]: both branches close in one product, summed in fp32 before its rounding
+* experts stacked: gate-and-up [E, 2F, d], down [E, d, F]
+"""
+from __future__ import annotations
+
+import torch
+import torch.nn as nn
+
+from .hybrid_config import DenseSpec, DiffAttentionSpec, HybridConfig, LayerSpec, MoESpec
+
+
+def _p(*shape):
+    return nn.Parameter(torch.empty(*shape), requires_grad=False)
+
+
+class HybridLayer(nn.Module):
+    def __init__(self, cfg: HybridConfig, spec: LayerSpec):
+        super().__init__()
+        d, mx, mlp = cfg.hidden, spec.mixer, spec.mlp
+        self.spec = spec
+        self.norm = nn.Parameter(torch.empty(()), requires_grad=False)
+        self.shift = _p(d)
+        self.w_in = _p(mx.in_rows, d)
+        self.attention = isinstance(mx, DiffAttentionSpec)
+        if self.attention:
+            self.lam = _p(4, mx.dim)          # rows lq1, lk1, lq2, lk2
+        else:
+            self.b_z, self.b_x = _p(mx.width), _p(mx.width)
+        self.moe = isinstance(mlp, MoESpec)
+        self.ff_cols = mlp.ff if isinstance(mlp, DenseSpec) else mlp.shared_ff if self.moe else 0
+        self.w_up = _p((2 if self.moe else 1) * self.ff_cols, d) if self.ff_cols else None
+        self.w_out = _p(d, mx.out_cols + self.ff_cols)
+        if self.moe:
+            self.router = _p(mlp.experts, d)
+            self.gate_up = _p(mlp.experts, 2 * mlp.ff, d)
+            self.down = _p(mlp.experts, d, mlp.ff)
+            self.shared_gate = _p(1, d) if mlp.shared_ff else None
+
+    def lam_value(self) -> float:
+        """lambda = exp(lq1 . lk1) - exp(lq2 . lk2) + diff, one number for the layer (fp32)."""
+        v = self.lam.float()
+        return float(torch.exp((v[0] * v[1]).sum()) - torch.exp((v[2] * v[3]).sum())) + self.spec.mixer.diff
+
+
+class HybridLM(nn.Module):
+    def __init__(self, cfg: HybridConfig):
+        super().__init__()
+        self.cfg = cfg
+        self.wte = _p(cfg.vocab_size, cfg.hidden)
+        self.layers = nn.ModuleList([HybridLayer(cfg, s) for s in cfg.layers])
+        self.final_norm = nn.Parameter(torch.empty(()), requires_grad=False)
+        self.head = _p(cfg.vocab_size, cfg.hidden)
+
+    @torch.no_grad()
+    def init_weights(self, std: float = 0.02, seed: int | None = None):
+        g = torch.Generator(device=self.wte.device)
+        if seed is not None:
+            g.manual_seed(seed)
+        for name, p in self.named_parameters():
+            if p.dim() >= 2:
+                p.normal_(0.0, std, generator=g)
+            elif "norm" in name:
+                p.fill_(1.0)
+            elif name.endswith("shift"):
+                p.fill_(0.5)
+            else:
+                p.zero_()
+        return self
+
+    def num_parameters(self) -> int:
+        return sum(p.numel() for p in self.parameters())
+
+    @torch.no_grad()
+    def forward(self, input_ids: torch.Tensor) -> torch.Tensor:
+        """Logits [B, S, V] of whole sequences: one step of a throw-away runner."""
+        from ..engine.hybrid_runner import HybridRunner
+        B, S = input_ids.shape
+        r = HybridRunner(self, max_slots=B, max_len=S, use_graphs=False)
+        out = r.forward_tokens([(b, row, 0, range(S)) for b, row in enumerate(input_ids.tolist())])
+        return out.view(B, S, -1)
+
+
+def build_hybrid(cfg: HybridConfig, device="cpu", dtype=torch.bfloat16, seed: int | None = 0) -> HybridLM:
+    with torch.device("meta"):
+        m = HybridLM(cfg)
+    m = m.to(dtype).to_empty(device=device)
+    if seed is not None:
+        m.init_weights(seed=seed)
+    return m
+
+
+__all__ = ["HybridLM", "HybridLayer", "build_hybrid"]

@@ -1,0 +1,76 @@
+"""Model families: which config class, module, weight names and step runner serve a ``config.json``.
+
+HF configs carry ``model_type`` and map onto ``CausalLM``; native designs carry ``architecture``. Everything
+that loads, serves or saves a model goes through the lookups here, so a design added to ``FAMILIES`` is
+available to all of them.
+"""
+from __future__ import annotations
+
+import dataclasses
+import json
+import os
+from typing import Callable
+
+
+@dataclasses.dataclass(frozen=True)
+class Family:
+    """``kernels``: the ``csrc/kernels`` sources a fresh checkout needs to run the family's step."""
+    name: str
+    read_config: Callable
+    build: Callable            # (cfg, device, dtype, seed) -> module
+    to_native: Callable        # (checkpoint tensors, cfg) -> module state
+    from_native: Callable
+    runner: Callable           # () -> StepRunner class
+    kernels: tuple = ()
+
+
+def _megusun() -> Family:
+    from . import megusun
+    from .hybrid_lm import build_hybrid
+
+    def runner():
+        from ..engine.hybrid_runner import HybridRunner
+        return HybridRunner
+    return Family("megusun", megusun.read_config, build_hybrid, megusun.to_native, megusun.from_native, runner,
+                  ("rms_shift", "gated_scan", "diff_attn", "moe", "act_rows", "gemv", "skinny_mfma"))
+
+
+def _causal_lm() -> Family:
+    from .causal_lm import build_causal_lm
+    from .config import LMConfig
+    from .hf_convert import hf_to_native, native_to_hf
+
+    def runner():
+        from ..engine.runner import ModelRunner
+        return ModelRunner
+    return Family("causal_lm", LMConfig.read_hf, build_causal_lm, hf_to_native, native_to_hf, runner)
+
+
+FAMILIES = {"Megusun": _megusun}   # config.json "architecture" -> family
+
+
+def family_of_dict(cfg: dict) -> Family:
+    arch = cfg.get("architecture")
+    if arch is None:
+        return _causal_lm()
+    if arch not in FAMILIES:
+        from .config import UnsupportedModel
+        raise UnsupportedModel(arch)
+    return FAMILIES[arch]()
+
+
+def family_of(cfg) -> Family:
+    """Family of a parsed config (``LMConfig`` / ``HybridConfig``)."""
+    for make in FAMILIES.values():
+        f = make()
+        if f.name == cfg.arch:
+            return f
+    return _causal_lm()
+
+
+def read_dict(path: str) -> dict:
+    with open(os.path.join(path, "config.json")) as f:
+        return json.load(f)
+
+
+__all__ = ["Family", "FAMILIES", "family_of", "family_of_dict", "read_dict"]

@@ -15,6 +15,7 @@ from __future__ import annotations
 
 import ctypes
 import os
+import sys
 import threading
 
 import torch
@@ -113,6 +114,18 @@ _SIGS = {
     "kca_sample_logits": [P, LL, I, I, I, P, P, P, P, P, P, P, I, P, LL, P, P, P, P, P, I, P],
 }
 
+# layers with an fp32 residual stream, token shift, recurrences and routed experts (first argument: 0 fp32,
+# 1 bf16); differential attention takes a descriptor (ops/diff_attention.py)
+_SIGS.update({
+    "kca_rms_shift": [I, P, P, P, P, LL, P, P, I, F, P, I, F, P, P, P, P, P, P, P, P, P, P, P, I, I, I, P],
+    "kca_gated_scan": [I, P, LL, P, P, P, LL, P, P, LL, P, I, I, I, P],
+    "kca_gated_step": [I, P, LL, P, P, P, LL, P, P, P, I, I, P],
+    "kca_moe_route": [I, P, P, P, P, P, P, I, I, I, I, P],
+    "kca_moe_group": [P, I, I, I, P, P, P, I, P, P],
+    "kca_moe_expert": [I, P, P, P, P, P, P, P, I, I, I, I, I, I, I, P],
+    "kca_act_rows": [I, I, P, LL, P, P, LL, I, I, P],
+})
+
 
 # fused decode layer (batch 1): kca_decode_prep_attn's arguments (minus the stream), then the fc_in
 # GEMV's x, W, bias, y, N, K, act, then the stream
@@ -147,6 +160,20 @@ def _load():
             fn.restype = ctypes.c_int
         _lib = lib
         return _lib
+
+
+def ensure_built(sources) -> None:
+    """Make the kernel library loadable in a checkout without built files: if the full library is missing,
+    compile only ``sources`` (names under ``csrc/kernels``) into a partial one and use that. Call before the
+    first kernel."""
+    global KERNEL_LIB
+    if os.path.exists(KERNEL_LIB) or not sources:
+        return
+    tools = os.path.join(os.path.dirname(os.path.dirname(_HERE)), "tools")
+    if tools not in sys.path:
+        sys.path.insert(0, tools)
+    import build_ext
+    KERNEL_LIB = build_ext.build_partial(sources)
 
 
 def available() -> bool:

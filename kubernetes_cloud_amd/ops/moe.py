@@ -1,0 +1,119 @@
+"""Mixture of gated experts (``csrc/kernels/moe.hip``): sigmoid top-k router, grouping by expert, expert
+products with the router weight on the expert's input (or output), and the strided feed-forward
+activations (``csrc/kernels/act_rows.hip``).
+
+Expert weights are stacked: gate-and-up [E, 2F, d] (gate rows first), down [E, d, F].
+"""
+from __future__ import annotations
+
+import dataclasses
+import math
+
+import torch
+
+from . import _lib
+from .rms_shift import native_dt
+
+GEMM_ROWS = 128
+
+
+def route(h: torch.Tensor, router: torch.Tensor, top: int, shared_gate: torch.Tensor | None = None):
+    """h [T, d] -> (ids int32 [T, top], weights fp32 [T, top], sigmoid of the shared expert's gate [T] | None)."""
+    code = native_dt(h, router, shared_gate)
+    T, d = h.shape
+    E = router.shape[0]
+    if code is None:
+        s = torch.sigmoid(h.float() @ router.float().t())
+        w, ids = s.topk(top, dim=-1)
+        sg = torch.sigmoid(h.float() @ shared_gate.float().reshape(-1)) if shared_gate is not None else None
+        return ids.to(torch.int32), w, sg
+    assert h.is_contiguous() and router.is_contiguous() and router.shape[1] == d
+    ids = torch.empty(T, top, device=h.device, dtype=torch.int32)
+    w = torch.empty(T, top, device=h.device, dtype=torch.float32)
+    sg = torch.empty(T, device=h.device, dtype=torch.float32) if shared_gate is not None else None
+    _lib.call("kca_moe_route", code, h.data_ptr(), router.data_ptr(), _lib.ptr(shared_gate), ids.data_ptr(),
+              w.data_ptr(), _lib.ptr(sg), T, d, E, top, _lib.stream())
+    return ids, w, sg
+
+
+@dataclasses.dataclass
+class Groups:
+    """Assignments sorted by expert, in tiles of at most ``mt`` rows of one expert."""
+    perm: torch.Tensor
+    inv: torch.Tensor     # [T, top]
+    tiles: torch.Tensor
+    ntiles: torch.Tensor
+    mt: int
+
+
+def tile_rows(T: int, top: int, E: int, d: int, F: int, dtype) -> int:
+    """Row limit of an expert tile: the matrix-core product (128) once an active expert expects enough rows
+    to be worth a tile, else a streaming product of 1 .. 8 rows."""
+    gemm = dtype == torch.bfloat16 and d % 8 == 0 and F % 8 == 0
+    if gemm and T * top > 16 * min(E, T * top):
+        return GEMM_ROWS
+    return 1 if T == 1 else 2 if T == 2 else 4 if T <= 4 else 8
+
+
+def group(ids: torch.Tensor, E: int, mt: int) -> Groups:
+    T, top = ids.shape
+    n = T * top
+    mx = min(E, n) + n // mt
+    z = dict(device=ids.device, dtype=torch.int32)
+    g = Groups(torch.empty(n, **z), torch.empty(T, top, **z), torch.empty(mx, 3, **z), torch.empty(1, **z), mt)
+    if not ids.is_cuda:
+        order = torch.argsort(ids.reshape(-1), stable=True)
+        g.perm.copy_(order)
+        g.inv.view(-1)[order] = torch.arange(n, dtype=torch.int32)
+        return g
+    _lib.call("kca_moe_group", ids.data_ptr(), n, E, mt, g.perm.data_ptr(), g.inv.data_ptr(), g.tiles.data_ptr(), mx,
+              g.ntiles.data_ptr(), _lib.stream())
+    return g
+
+
+def experts(h: torch.Tensor, ids: torch.Tensor, weights: torch.Tensor, gate_up: torch.Tensor, down: torch.Tensor,
+            g: Groups, scale_in: bool = True) -> torch.Tensor:
+    """Output rows [n, d] of the routed experts in ``g``'s sorted order."""
+    E, F2, d = gate_up.shape
+    F, top, n = F2 // 2, ids.shape[1], ids.numel()
+    code = native_dt(h, gate_up, down)
+    if code is None:
+        flat, wt = ids.reshape(-1).long(), weights.reshape(-1)
+        y = torch.empty(n, d, dtype=h.dtype)
+        for pos, a in enumerate(g.perm.tolist()):
+            x, e = h[a // top].float(), int(flat[a])
+            s_in, s_out = (float(wt[a]), 1.0) if scale_in else (1.0, float(wt[a]))
+            u = gate_up[e].float() @ (x * s_in)
+            y[pos] = (down[e].float() @ (torch.nn.functional.silu(u[:F]) * u[F:]) * s_out).to(h.dtype)
+        return y
+    assert h.is_contiguous() and gate_up.is_contiguous() and down.is_contiguous() and down.shape == (E, d, F)
+    act = torch.empty(n, F, device=h.device, dtype=h.dtype)
+    y = torch.empty(n, d, device=h.device, dtype=h.dtype)
+    mx = g.tiles.shape[0]
+    common = (g.perm.data_ptr(), weights.data_ptr(), g.tiles.data_ptr(), g.ntiles.data_ptr(), mx, g.mt, top)
+    _lib.call("kca_moe_expert", code, h.data_ptr(), gate_up.data_ptr(), act.data_ptr(), *common, F, d, 1,
+              int(scale_in), _lib.stream())
+    _lib.call("kca_moe_expert", code, act.data_ptr(), down.data_ptr(), y.data_ptr(), *common, d, F, 0,
+              int(not scale_in), _lib.stream())
+    return y
+
+
+def act_rows(x: torch.Tensor, out: torch.Tensor, gated: bool, row_scale: torch.Tensor | None = None) -> torch.Tensor:
+    """out = gelu(x) (exact), or silu(gate) * up * row_scale with x = [gate | up]; strided rows."""
+    T, F = out.shape
+    code = native_dt(x, out)
+    assert x.shape == (T, 2 * F if gated else F) and x.stride(1) == 1 and out.stride(1) == 1
+    if code is None:
+        if gated:
+            y = torch.nn.functional.silu(x[:, :F].float()) * x[:, F:].float()
+            out.copy_(y if row_scale is None else y * row_scale[:, None])
+        else:
+            xf = x.float()
+            out.copy_(0.5 * xf * (1 + torch.erf(xf / math.sqrt(2.0))))
+        return out
+    _lib.call("kca_act_rows", code, int(gated), x.data_ptr(), x.stride(0), _lib.ptr(row_scale), out.data_ptr(),
+              out.stride(0), T, F, _lib.stream())
+    return out
+
+
+__all__ = ["route", "group", "experts", "act_rows", "tile_rows", "Groups"]
