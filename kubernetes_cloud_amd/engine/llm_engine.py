@@ -24,6 +24,9 @@ prefilled over several steps (``ModelRunner.prefill(..., start=)`` continues
 its slot), each followed by the decode step of the running batch, so a
 2048-token admission no longer stalls every running stream for its whole
 prefill; with nothing decoding a prompt prefills in one pass.
+Mixed steps (a runner with ``mixed_steps``): with ``prefill_chunk`` set, the step's prompt portions and the
+running requests' tokens go through the model as ONE batch (``runner.forward_tokens``) instead of a prefill
+call per portion followed by a decode step.
 Admission reserves a request's worst-case page count (prompt + max_new_tokens)
 against the paged cache, so a running request never runs out of pages (no
 preemption needed); pages go back to the pool the step a request finishes.
@@ -113,10 +116,11 @@ class LLMEngine:
         self.prefill_chunk = int(prefill_chunk) if prefill_chunk else 0
         self.prefilling: list[Request] = []  # admitted, prompt partially in the cache (r.prefilled tokens)
         self.pipeline = bool(getattr(self.runner, "pipelined", False)) if pipeline is None else pipeline
+        self.mixed = bool(getattr(self.runner, "mixed_steps", False))
         self._inflight = None  # (DecodeHandle, [Request]) of the launched, not yet read decode step
         self.stats = {"steps": 0, "decode_tokens": 0, "prefill_tokens": 0, "finished": 0, "prefill_batches": 0,
                       "prefill_pad_tokens": 0, "prefill_chunks": 0, "max_step_prefill_tokens": 0,
-                      "decode_steps": 0}
+                      "decode_steps": 0, "mixed_steps": 0}
         cache = getattr(self.runner, "cache", None)
         self._paged = cache is not None and getattr(cache, "paged", False)
         self._page_budget = cache.n_pages if self._paged else 0
@@ -272,12 +276,51 @@ class LLMEngine:
                 self._first_token(r, logits, finished)
         return used
 
+    def _mixed_step(self, budget: int, finished: list) -> int:
+        """Up to ``budget`` prompt tokens of the prefilling requests and one token of every running one, as
+        one batch."""
+        self._drain(finished)  # the running rows' input tokens
+        self.running = [r for r in self.running if not r.done]
+        entries, sampled, used = [], [], 0
+        for r in self.prefilling:
+            n = min(budget - used, len(r.prompt) - r.prefilled)
+            if n <= 0:
+                break
+            last = r.prefilled + n == len(r.prompt)
+            entries.append((r.slot, r.prompt[r.prefilled:r.prefilled + n], r.prefilled, [n - 1] if last else []))
+            if last:
+                sampled.append((r, self._row(r, 0)))
+            r.prefilled += n
+            used += n
+            self.stats["prefill_chunks"] += 1
+        for r in self.running:
+            row = self._row(r)
+            entries.append((r.slot, [row["token"]], row["pos"], [0]))
+            sampled.append((r, row))
+        self.stats["prefill_tokens"] += used
+        self.stats["decode_tokens"] += len(self.running)
+        self.stats["mixed_steps"] += 1
+        logits = self.runner.forward_tokens(entries)
+        self.prefilling = [r for r in self.prefilling if r.prefilled < len(r.prompt)]
+        if sampled:
+            toks, lps = self.runner.sample_first(logits, [row for _, row in sampled])
+            reqs = [r for r, _ in sampled]
+            self.running += [r for r in reqs if not r.output]  # prompts that ended in this step
+            self._take(reqs, toks, lps, finished)
+            self.running = [r for r in self.running if not r.done]
+        return used
+
     def _step(self) -> list[Request]:
         finished = []
         chunked = self.prefill_chunk > 0 and (self.running or self.prefilling)
+        mixed = chunked and self.mixed
         budget = self.prefill_chunk if chunked else self.max_prefill_tokens
-        used = self._chunk_step(budget, finished) if self.prefilling else 0
-        budget -= used
+        used = 0
+        if mixed:
+            budget -= sum(len(r.prompt) - r.prefilled for r in self.prefilling)
+        elif self.prefilling:
+            used = self._chunk_step(budget, finished)
+            budget -= used
         with self._lock:
             admit = []
             while self.waiting and self.free and budget > 0 and (not admit or budget >= len(self.waiting[0].prompt)):
@@ -295,13 +338,23 @@ class LLMEngine:
                 r = self.waiting.pop(0)
                 r.slot = self.free.pop()
                 self._committed += need
+                if mixed:
+                    r.prefilled = 0
+                    self.prefilling.append(r)
+                    budget -= len(r.prompt)
+                    continue
                 if chunked and len(r.prompt) > budget:  # prefill this one chunk by chunk
                     r.prefilled = 0
                     self.prefilling.append(r)
                     break
                 budget -= len(r.prompt)
                 admit.append(r)
-        if self.prefilling and budget > 0 and chunked:
+        if mixed and self.prefilling:
+            used = self._mixed_step(self.prefill_chunk, finished)
+            self.stats["steps"] += 1
+            self.stats["max_step_prefill_tokens"] = max(self.stats["max_step_prefill_tokens"], used)
+            return finished
+        if self.prefilling and budget > 0 and chunked and not mixed:
             used += self._chunk_step(budget, finished)
         for group in _prefill_groups(admit):
             T = max(len(r.prompt) for r in group)

@@ -32,6 +32,8 @@ def build_parser():
     p.add_argument("--fp16", action=FuzzyBoolAction, default=False, help="Force evaluation in fp16")
     p.add_argument("--prompt", type=str, help="Prompt to use")
     p.add_argument("--prompt-file", type=val.optional_extant_file, help="File containing prompts")
+    p.add_argument("--prompt-ids", type=str, help="Prompt as token ids (\"5 17 3\"): no tokenizer is loaded and the "
+                   "response is printed as ids")
     p.add_argument("--prompt-tokens", type=val.non_negative(int), default=200, help="Number of tokens to generate")
     p.add_argument("--seed", type=val.at_most_32_bit(val.non_negative(int)), default=None, help="Random seed value")
     p.add_argument("--prompt-samples", type=val.non_negative(int), default=1, help="Number of samples to generate")
@@ -45,6 +47,10 @@ def build_parser():
 
 
 def read_prompts(parser, args) -> list[str]:
+    if args.prompt_ids:
+        if args.prompt or args.prompt_file:
+            parser.error("Cannot specify token ids beside a prompt or a prompt file")
+        return [args.prompt_ids.strip()]
     if args.prompt and args.prompt_file:
         parser.error("Cannot specify both a prompt and a prompt file")
     if not args.prompt and not args.prompt_file:
@@ -75,9 +81,9 @@ def main(argv=None, out=None):
     dtype = (torch.float16 if args.fp16 else torch.bfloat16) if dev.type == "cuda" else torch.float32
     print(MemoryUsage.now(), file=out)
     t0 = time.time()
-    tok = load_tokenizer(args.tokenizer, args.eot, args.pad)
+    tok = None if args.prompt_ids else load_tokenizer(args.tokenizer, args.eot, args.pad)
     model = load_pretrained(args.model, device=dev, dtype=dtype)
-    if len(tok) > model.cfg.vocab_size:
+    if tok is not None and len(tok) > model.cfg.vocab_size:
         model.resize_token_embeddings(len(tok))
     model.eval()
     print(f"Loaded model in {time.time() - t0:.2f}s", file=out)
@@ -87,14 +93,17 @@ def main(argv=None, out=None):
         print("=============================", file=out)
         print("PROMPT:", prompt, file=out)
         print("UTILIZATION:", MemoryUsage.now(), file=out)
-        ids = torch.tensor([tok.encode(prompt)])
+        ids = torch.tensor([[int(t) for t in prompt.replace(",", " ").split()] if tok is None else tok.encode(prompt)])
+        eos = tok.eos_token_id if tok is not None else model.cfg.eos_token_id
         res = generate(model, ids, GenerationConfig(
             max_new_tokens=args.prompt_tokens, do_sample=True, top_k=args.top_k, top_p=args.top_p,
             temperature=args.temperature, repetition_penalty=args.repetition_penalty,
-            num_return_sequences=args.prompt_samples, eos_token_id=tok.eos_token_id,
-            pad_token_id=tok.pad_token_id, bad_words_ids=[[tok.eos_token_id]],
+            num_return_sequences=args.prompt_samples, eos_token_id=eos,
+            pad_token_id=tok.pad_token_id if tok is not None else model.cfg.pad_token_id,
+            bad_words_ids=[[eos]] if eos is not None else None,
             seed=None if args.seed is None else args.seed + 7919 * i))
-        texts = [tok.decode(s[:int(n)].tolist(), skip_special_tokens=False)
+        texts = [" ".join(map(str, s[:int(n)].tolist())) if tok is None else
+                 tok.decode(s[:int(n)].tolist(), skip_special_tokens=False)
                  for s, n in zip(res.sequences, res.lengths)]
         results[prompt] = texts
         for t in texts:
