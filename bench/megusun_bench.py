@@ -260,12 +260,10 @@ def run_kernels(d=4096, heads=16, T=4096, cached=2048, batches=(1, 8, 32), ring=
     dn = [torch.randn(E, d, Fe, **bf) for _ in range(2)]
     for n in (T, 32, 8, 1):
         h = torch.randn(n, d, **bf)
-        us = _time([lambda: moe.route(h, rw, top, sgw) for _ in R])
-        rec(f"moe_route T={n} E={E}", us, n * d * 2 + E * d * 2, 2. * n * d * E, like="layer_norm")
-        ids, wt, _ = moe.route(h, rw, top, sgw)
         mt = moe.tile_rows(n, top, E, d, Fe, torch.bfloat16)
-        us = _time([lambda: moe.group(ids, E, mt) for _ in R])
-        rec(f"moe_group T={n}", us, n * top * 12)
+        us = _time([lambda: moe.route_group(h, rw, top, sgw, mt) for _ in R])
+        rec(f"moe_route_group T={n} E={E}", us, n * d * 2 + E * d * 2, 2. * n * d * E, like="layer_norm")
+        ids, wt, _ = moe.route(h, rw, top, sgw)
         g = moe.group(ids, E, mt)
         us = _time([lambda a=a, b=b: moe.experts(h, ids, wt, a, b, g) for a, b in zip(gu, dn)])
         active = int(ids.unique().numel())

@@ -84,6 +84,29 @@ __global__ void __launch_bounds__(256) kv_append_kernel(DiffArgs p, int T) {
 // a value row; a wave-private LDS array carries the 2 x RB x KT weights between the two layouts. The
 // waves, then the splits, merge at the end.
 
+// sum / maximum over N consecutive lanes (all of them get it): DPP steps within a row of 16
+template <int CTRL>
+__device__ __forceinline__ float dpp(float x) {
+  return __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(x), CTRL, 0xf, 0xf, true));
+}
+template <int N, typename F>
+__device__ __forceinline__ float lanes_reduce(float x, F f) {
+  static_assert(N == 4 || N == 8 || N == 16 || N == 32 || N == 64, "lanes");
+  x = f(x, dpp<0xB1>(x));  // lane ^ 1
+  x = f(x, dpp<0x4E>(x));  // lane ^ 2
+  if constexpr (N >= 8) x = f(x, dpp<0x141>(x));   // mirrored in 8: the other four
+  if constexpr (N >= 16) x = f(x, dpp<0x140>(x));  // mirrored in 16: the other eight
+  if constexpr (N >= 32) x = f(x, __shfl_xor(x, 16, 64));
+  if constexpr (N >= 64) x = f(x, __shfl_xor(x, 32, 64));
+  return x;
+}
+__device__ __forceinline__ void wave_sync() {  // orders one wave's LDS writes before its later reads
+  __builtin_amdgcn_fence(__ATOMIC_RELEASE, "wavefront");
+  __builtin_amdgcn_wave_barrier();
+  __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "wavefront");
+}
+constexpr int MAX_SPLITS = 256;
+
 // eight elements as loaded (converted where they are used); `left` of them exist
 template <typename E>
 struct Raw8 {
@@ -110,7 +133,8 @@ __global__ void __launch_bounds__(256) diff_rows_kernel(DiffArgs p) {
   constexpr int KPV = 64 / LPV, NPV = KT / KPV > 0 ? KT / KPV : 1;   // (values)
   static_assert(KPK <= KT && KPV <= KT, "a pass covers at most one tile");
   constexpr int NS = 2 * RB;                                         // score rows: [map][head]
-  __shared__ __attribute__((aligned(16))) float sc[4][KT][NS];
+  constexpr int NP = NS * KT, PPL = (NP + 63) / 64;                  // (score row, key) pairs, pairs per lane
+  __shared__ __attribute__((aligned(16))) float sc[4][KT][NS], als[4][NS];
   __shared__ float wm[4][NS], wl[4][NS];
   __shared__ int s_last;
   extern __shared__ __attribute__((aligned(16))) float merged[];     // [4][NS][vdim] then reused
@@ -145,15 +169,16 @@ __global__ void __launch_bounds__(256) diff_rows_kernel(DiffArgs p) {
 #pragma unroll
       for (int i = 0; i < 8; ++i) q[m][r][i] = x.f(i) * f;
     }
+  auto add = [](float x, float y) { return x + y; };
+  auto mxf = [](float x, float y) { return fmaxf(x, y); };
   float acc[NS][8];
-  float mx[NS], l[NS];
 #pragma unroll
-  for (int s = 0; s < NS; ++s) {
-    mx[s] = -INFINITY;
-    l[s] = 0.f;
+  for (int s = 0; s < NS; ++s)
 #pragma unroll
     for (int i = 0; i < 8; ++i) acc[s][i] = 0.f;
-  }
+  float mx[PPL], l[PPL];  // running maximum and sum of the score row this lane's pairs belong to
+#pragma unroll
+  for (int j = 0; j < PPL; ++j) mx[j] = -INFINITY, l[j] = 0.f;
   for (int k0 = lo + wv * KT; k0 < hi; k0 += 4 * KT) {
     Raw8<E> kx[NPK][2];
 #pragma unroll
@@ -186,39 +211,36 @@ __global__ void __launch_bounds__(256) diff_rows_kernel(DiffArgs p) {
           float d = 0.f;
 #pragma unroll
           for (int i = 0; i < 8; ++i) d = fmaf(q[m][r][i], kx[n][m].f(i), d);
-#pragma unroll
-          for (int o = LPK / 2; o > 0; o >>= 1) d += __shfl_xor(d, o, 64);
+          d = lanes_reduce<LPK>(d, add);
           const int kt = n * KPK + jk;
           if (lk == 0) sc[wv][kt][m * RB + r] = k0 + kt < hi ? d : -INFINITY;
         }
-    __builtin_amdgcn_fence(__ATOMIC_RELEASE, "wavefront");
-    __builtin_amdgcn_wave_barrier();
-    __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "wavefront");
-    float al[NS];
+    wave_sync();
+    float e[PPL];
 #pragma unroll
-    for (int s = 0; s < NS; ++s) {  // every lane: the tile's maximum and sum of score row s
-      const float x = sc[wv][lane & (KT - 1)][s];
-      float t = x;
-#pragma unroll
-      for (int o = KT / 2; o > 0; o >>= 1) t = fmaxf(t, __shfl_xor(t, o, 64));
-      const float mn = fmaxf(mx[s], t);
-      al[s] = El<E>::ex(mx[s] - mn);
-      const float e = El<E>::ex(x - mn);
-      float u = e;
-#pragma unroll
-      for (int o = KT / 2; o > 0; o >>= 1) u += __shfl_xor(u, o, 64);
-      l[s] = l[s] * al[s] + u;
-      mx[s] = mn;
-      __builtin_amdgcn_wave_barrier();
-      if (lane < KT) sc[wv][lane][s] = e;
+    for (int j = 0; j < PPL; ++j) {  // pair (score row, key): the KT lanes of a row reduce together
+      const int pr = min(lane + 64 * j, NP - KT + lane % KT), s = pr / KT, kt = pr % KT;
+      const float x = sc[wv][kt][s];
+      const float mn = fmaxf(mx[j], lanes_reduce<KT>(x, mxf));
+      const float al = El<E>::ex(mx[j] - mn);
+      e[j] = El<E>::ex(x - mn);
+      l[j] = l[j] * al + lanes_reduce<KT>(e[j], add);
+      mx[j] = mn;
+      if (kt == 0) als[wv][s] = al;
     }
-    __builtin_amdgcn_fence(__ATOMIC_RELEASE, "wavefront");
-    __builtin_amdgcn_wave_barrier();
-    __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "wavefront");
+    wave_sync();
 #pragma unroll
-    for (int s = 0; s < NS; ++s)
+    for (int j = 0; j < PPL; ++j) {
+      const int pr = min(lane + 64 * j, NP - KT + lane % KT);
+      sc[wv][pr % KT][pr / KT] = e[j];
+    }
+    wave_sync();
 #pragma unroll
-      for (int i = 0; i < 8; ++i) acc[s][i] *= al[s];
+    for (int s = 0; s < NS; ++s) {
+      const float al = als[wv][s];
+#pragma unroll
+      for (int i = 0; i < 8; ++i) acc[s][i] *= al;
+    }
 #pragma unroll
     for (int n = 0; n < NPV; ++n) {
       float w[NS];
@@ -229,7 +251,7 @@ __global__ void __launch_bounds__(256) diff_rows_kernel(DiffArgs p) {
 #pragma unroll
         for (int i = 0; i < 8; ++i) acc[s][i] = fmaf(w[s], vx[n].f(i), acc[s][i]);
     }
-    __builtin_amdgcn_wave_barrier();
+    wave_sync();
   }
   // the key lanes of a value row, then the four waves
 #pragma unroll
@@ -244,12 +266,14 @@ __global__ void __launch_bounds__(256) diff_rows_kernel(DiffArgs p) {
 #pragma unroll
       for (int i = 0; i < 8; ++i)
         if (lv * 8 + i < Vd) merged[(wv * NS + s) * Vd + lv * 8 + i] = acc[s][i];
-  if (lane == 0)
 #pragma unroll
-    for (int s = 0; s < NS; ++s) {
-      wm[wv][s] = mx[s];
-      wl[wv][s] = l[s];
+  for (int j = 0; j < PPL; ++j) {
+    const int pr = lane + 64 * j;
+    if (pr < NP && pr % KT == 0) {
+      wm[wv][pr / KT] = mx[j];
+      wl[wv][pr / KT] = l[j];
     }
+  }
   __syncthreads();
   if (p.append && hi == kv && sub == 0) {  // the split that holds the new token stores it
     const long long pg = tbl[pos >> p.shift];
@@ -303,33 +327,38 @@ __global__ void __launch_bounds__(256) diff_rows_kernel(DiffArgs p) {
     }
     __syncthreads();
     if (!s_last) return;
+    // weights of the splits first (a wave per score row), then every thread sums outputs, UZ splits' loads
+    // in flight
     const float* base = p.ws + blk * p.nsplit * stride;
+    __shared__ float wz[NS][MAX_SPLITS];
     for (int s = wv; s < NS; s += 4) {
-      float M = -INFINITY;
-      for (int z = lane; z < used; z += 64) M = fmaxf(M, base[(long long)z * stride + s * (Vd + 2)]);
+      const float* b = base + s * (Vd + 2);
+      float M = -INFINITY, L = 0.f;
+      for (int z = lane; z < used; z += 64) M = fmaxf(M, b[(long long)z * stride]);
       M = wave_max(M);
-      float L = 0.f;
       for (int z = lane; z < used; z += 64) {
-        const float* b = base + (long long)z * stride + s * (Vd + 2);
-        L += El<E>::ex(b[0] - M) * b[1];
+        const float c = El<E>::ex(b[(long long)z * stride] - M);
+        wz[s][z] = c;
+        L += c * b[(long long)z * stride + 1];
       }
-      L = wave_sum(L);
-      for (int i = lane; i < Vd; i += 64) {
-        float o = 0.f;
-        for (int z0 = 0; z0 < used; z0 += 4) {
-          float mm[4], oo[4];
+      L = 1.f / wave_sum(L);
+      for (int z = lane; z < used; z += 64) wz[s][z] *= L;
+    }
+    __syncthreads();
+    constexpr int UZ = 16;
+    for (int i = tid; i < NS * Vd; i += 256) {
+      const int s = i / Vd;
+      const float* b = base + i + 2 * s + 2;  // s * (Vd + 2) + 2 + i % Vd
+      float o = 0.f;
+      for (int z0 = 0; z0 < used; z0 += UZ) {
+        float x[UZ];
 #pragma unroll
-          for (int u = 0; u < 4; ++u) {
-            const float* b = base + (long long)min(z0 + u, used - 1) * stride + s * (Vd + 2);
-            mm[u] = b[0];
-            oo[u] = b[2 + i];
-          }
+        for (int u = 0; u < UZ; ++u) x[u] = b[(long long)min(z0 + u, used - 1) * stride];
 #pragma unroll
-          for (int u = 0; u < 4; ++u)
-            if (z0 + u < used) o += El<E>::ex(mm[u] - M) * oo[u];
-        }
-        merged[s * Vd + i] = o / L;
+        for (int u = 0; u < UZ; ++u)
+          if (z0 + u < used) o = fmaf(wz[s][z0 + u], x[u], o);
       }
+      merged[i] = o;
     }
   }
   __syncthreads();
@@ -663,7 +692,8 @@ KCA_API int kca_diff_rows_plan(const KcaDiffAttn* in, int* sub, int* rb) {
 KCA_API int kca_diff_rows(const KcaDiffAttn* in, int dtype, int rows, long long ws_floats, long long n_cnt, int max_kv,
                           hipStream_t s) {
   const DiffArgs& p = in->a;
-  if (!args_ok(p) || !p.pos || !p.slot || !p.out || rows < 1 || p.nsplit < 1 || p.chunk < 1 || p.nsplit > 65535) return 1;
+  if (!args_ok(p) || !p.pos || !p.slot || !p.out || rows < 1 || p.nsplit < 1 || p.chunk < 1 || p.nsplit > MAX_SPLITS)
+    return 1;
   if ((long long)p.nsplit * p.chunk < max_kv) return 2;
   const bool vec = vec_ok(p);
   const int rb = rb_for(p.H / p.G, vec), nsub = (p.H / p.G + rb - 1) / rb;

@@ -40,6 +40,13 @@ template <> struct Vec<float> {
   static __device__ __forceinline__ float sig(float x) { return 1.f / (1.f + expf(-x)); }
 };
 
+// V elements as loaded (converted at use), so that the next tokens' loads stay in flight in few registers
+template <typename E, int V>
+struct alignas(sizeof(E) * V) Raw {
+  E v[V];
+  __device__ __forceinline__ float f(int i) const { return Vec<E>::ld(v + i); }
+};
+
 template <typename E, int V>
 __device__ __forceinline__ void ldn(const E* p, float (&v)[V]) {
   if constexpr (V == 4 && sizeof(E) == 2) {
@@ -58,6 +65,8 @@ template <typename E, int V>
 __device__ __forceinline__ void stn(E* p, const float (&v)[V]) {
   if constexpr (V == 4 && sizeof(E) == 2)
     *reinterpret_cast<uint2*>(p) = make_uint2(pack_bf16x2(v[0], v[1]), pack_bf16x2(v[2], v[3]));
+  else if constexpr (V == 2 && sizeof(E) == 2)
+    *reinterpret_cast<uint32_t*>(p) = pack_bf16x2(v[0], v[1]);
   else if constexpr (V == 4)
     *reinterpret_cast<float4*>(p) = make_float4(v[0], v[1], v[2], v[3]);
   else
@@ -95,25 +104,32 @@ __global__ void __launch_bounds__(64) scan_sum_kernel(ScanArgs p) {
 #pragma unroll
   for (int e = 0; e < V; ++e) A[e] = 1.f, B[e] = 0.f;
   const E* base = reinterpret_cast<const E*>(p.zxg) + (long long)row0 * p.ld + w;
-  for (int t0 = 0; t0 < n; t0 += UN) {
-    float zv[UN][V], uv[UN][V];
+  Raw<E, V> zv[UN], uv[UN];
+  auto load = [&](int t0, Raw<E, V>(&z)[UN], Raw<E, V>(&u)[UN]) {
 #pragma unroll
     for (int i = 0; i < UN; ++i) {
-      const int t = min(t0 + i, n - 1);
-      ldn<E, V>(base + t * p.ld, zv[i]);
-      ldn<E, V>(base + t * p.ld + W, uv[i]);
+      const E* q = base + min(t0 + i, n - 1) * p.ld;
+      z[i] = *reinterpret_cast<const Raw<E, V>*>(q);
+      u[i] = *reinterpret_cast<const Raw<E, V>*>(q + W);
     }
+  };
+  load(0, zv, uv);
+  for (int t0 = 0; t0 < n; t0 += UN) {
+    Raw<E, V> zn[UN], un[UN];
+    load(t0 + UN, zn, un);
 #pragma unroll
     for (int i = 0; i < UN; ++i) {
       if (t0 + i >= n) break;
 #pragma unroll
       for (int e = 0; e < V; ++e) {
         float z, zc;
-        gate<E>(zv[i][e] + bz[e], uv[i][e] + bx[e], z, zc);
+        gate<E>(zv[i].f(e) + bz[e], uv[i].f(e) + bx[e], z, zc);
         A[e] *= 1.f - z;
         B[e] = fmaf(1.f - z, B[e], zc);
       }
     }
+#pragma unroll
+    for (int i = 0; i < UN; ++i) zv[i] = zn[i], uv[i] = un[i];
   }
   stn<float, V>(ws, A);
   stn<float, V>(ws + W, B);
@@ -153,15 +169,20 @@ __global__ void __launch_bounds__(64) scan_run_kernel(ScanArgs p) {
   ldn<E, V>(reinterpret_cast<const E*>(p.bx) + w, bx);
   const E* base = reinterpret_cast<const E*>(p.zxg) + (long long)row0 * p.ld + w;
   E* y = reinterpret_cast<E*>(p.y) + (long long)row0 * p.ldy + w;
-  for (int t0 = 0; t0 < n; t0 += UN) {
-    float zv[UN][V], uv[UN][V], gv[UN][V];
+  Raw<E, V> zv[UN], uv[UN], gv[UN];
+  auto load = [&](int t0, Raw<E, V>(&z)[UN], Raw<E, V>(&u)[UN], Raw<E, V>(&g)[UN]) {
 #pragma unroll
     for (int i = 0; i < UN; ++i) {
-      const int t = min(t0 + i, n - 1);
-      ldn<E, V>(base + t * p.ld, zv[i]);
-      ldn<E, V>(base + t * p.ld + W, uv[i]);
-      ldn<E, V>(base + t * p.ld + 2 * W, gv[i]);
+      const E* q = base + min(t0 + i, n - 1) * p.ld;
+      z[i] = *reinterpret_cast<const Raw<E, V>*>(q);
+      u[i] = *reinterpret_cast<const Raw<E, V>*>(q + W);
+      g[i] = *reinterpret_cast<const Raw<E, V>*>(q + 2 * W);
     }
+  };
+  load(0, zv, uv, gv);
+  for (int t0 = 0; t0 < n; t0 += UN) {
+    Raw<E, V> zn[UN], un[UN], gn[UN];
+    load(t0 + UN, zn, un, gn);
 #pragma unroll
     for (int i = 0; i < UN; ++i) {
       if (t0 + i >= n) break;
@@ -169,12 +190,15 @@ __global__ void __launch_bounds__(64) scan_run_kernel(ScanArgs p) {
 #pragma unroll
       for (int e = 0; e < V; ++e) {
         float z, zc;
-        gate<E>(zv[i][e] + bz[e], uv[i][e] + bx[e], z, zc);
+        gate<E>(zv[i].f(e) + bz[e], uv[i].f(e) + bx[e], z, zc);
         S[e] = fmaf(1.f - z, S[e], zc);
-        o[e] = S[e] * gv[i][e] * Vec<E>::sig(gv[i][e]);
+        const float g = gv[i].f(e);
+        o[e] = S[e] * g * Vec<E>::sig(g);
       }
       stn<E, V>(y + (t0 + i) * p.ldy, o);
     }
+#pragma unroll
+    for (int i = 0; i < UN; ++i) zv[i] = zn[i], uv[i] = un[i], gv[i] = gn[i];
   }
   if (ci == nc - 1) stn<float, V>(p.state + (long long)slot * W + w, S);
 }
@@ -230,9 +254,10 @@ KCA_API int kca_gated_scan(int dtype, const void* zxg, long long ld, const void*
   if (nchunk < 1 || nchunk > 65535 || W < 1 || !zxg || !bz || !bx || !y || !state || !chunks) return 1;
   if (multi && (!ws || ws_floats < (long long)nchunk * 3 * W)) return 2;
   const ScanArgs a{zxg, ld, bz, bx, y, ldy, (float*)state, (float*)ws, (const int*)chunks, W, nchunk};
-  const bool v4 = W % 4 == 0 && ld % 4 == 0 && ldy % 4 == 0 && (uintptr_t)y % 16 == 0;
-  if (dtype == 0) return v4 ? launch<float, 4>(a, multi, s) : launch<float, 1>(a, multi, s);
-  if (dtype == 1) return v4 ? launch<bf16_t, 4>(a, multi, s) : launch<bf16_t, 1>(a, multi, s);
+  // two channels a thread: the scan's waves are few, four would halve them again
+  const bool v2 = W % 2 == 0 && ld % 2 == 0 && ldy % 2 == 0 && (uintptr_t)y % 8 == 0 && (uintptr_t)zxg % 8 == 0;
+  if (dtype == 0) return v2 ? launch<float, 2>(a, multi, s) : launch<float, 1>(a, multi, s);
+  if (dtype == 1) return v2 ? launch<bf16_t, 2>(a, multi, s) : launch<bf16_t, 1>(a, multi, s);
   return 3;
 }
 

@@ -16,6 +16,8 @@
 // through `inv`.
 #include "common.h"
 
+#include <type_traits>
+
 namespace {
 
 typedef unsigned int u32x4 __attribute__((ext_vector_type(4)));
@@ -83,9 +85,68 @@ __global__ void __launch_bounds__(256) route_rows_kernel(RouteArgs p) {
   if (threadIdx.x == 64 && p.wsg) p.sg[t] = sigmoid(z[p.E]);
 }
 
-// bf16: 16 tokens per workgroup, the K range cut over 8 waves, 64 experts at a time
-__global__ void __launch_bounds__(512) route_mfma_kernel(RouteArgs p) {
-  extern __shared__ __attribute__((aligned(16))) float lds[];  // z[16][zs], part[8][16][64]
+struct GroupArgs {
+  const int* ids;      // [n]
+  int n, E, mt;
+  int *perm, *inv, *tiles, *ntiles;
+};
+
+// n assignments -> perm (sorted position -> assignment), inv (assignment -> sorted position), tiles
+// [ntiles][3] (expert, first sorted position, rows <= mt) and their count. One workgroup of NT threads;
+// sh: 3 E + 2 ints.
+template <int NT>
+__device__ __forceinline__ void group_rows(const GroupArgs& p, int* sh) {
+  const int E = p.E, n = p.n, mt = p.mt, tid = threadIdx.x;
+  int *cnt = sh, *off = sh + E, *toff = off + E + 1;
+  for (int e = tid; e < E; e += NT) cnt[e] = 0;
+  __syncthreads();
+  for (int i = tid; i < n; i += NT) atomicAdd(&cnt[p.ids[i]], 1);
+  __syncthreads();
+  if (tid < 64) {  // exclusive sums over the experts, 64 at a time
+    int co = 0, to = 0;
+    for (int e0 = 0; e0 < E; e0 += 64) {
+      const int e = e0 + tid, c = e < E ? cnt[e] : 0, t = (c + mt - 1) / mt;
+      int cs = c, ts = t;
+#pragma unroll
+      for (int o = 1; o < 64; o <<= 1) {
+        const int a = __shfl_up(cs, o, 64), b = __shfl_up(ts, o, 64);
+        if (tid >= o) cs += a, ts += b;
+      }
+      if (e < E) off[e] = co + cs - c, toff[e] = to + ts - t;
+      co += __shfl(cs, 63, 64);
+      to += __shfl(ts, 63, 64);
+    }
+    if (tid == 0) off[E] = co, toff[E] = to, *p.ntiles = to;
+  }
+  __syncthreads();
+  for (int e = tid; e < E; e += NT) {
+    const int c = cnt[e];
+    for (int j = 0; j * mt < c; ++j) {
+      int* t = p.tiles + (toff[e] + j) * 3;
+      t[0] = e;
+      t[1] = off[e] + j * mt;
+      t[2] = min(mt, c - j * mt);
+    }
+    cnt[e] = off[e];
+  }
+  __syncthreads();
+  for (int i = tid; i < n; i += NT) {  // (the order within an expert does not matter: rows are independent)
+    const int pos = atomicAdd(&cnt[p.ids[i]], 1);
+    p.perm[pos] = i;
+    p.inv[i] = pos;
+  }
+}
+
+__global__ void __launch_bounds__(1024) group_kernel(GroupArgs p) {
+  extern __shared__ int sh[];
+  group_rows<1024>(p, sh);
+}
+
+// bf16: 16 tokens per workgroup, the K range cut over NW waves, 64 experts at a time. GROUP: the launch is
+// one workgroup, which also groups its assignments (the decode step)
+template <int NW, bool GROUP>
+__global__ void __launch_bounds__(NW * 64) route_mfma_kernel(RouteArgs p, GroupArgs gr) {
+  extern __shared__ __attribute__((aligned(16))) float lds[];  // z[16][zs], part[NW][16][64] (then group_rows')
   const int n = p.E + (p.wsg ? 1 : 0), zs = (n + 63) / 64 * 64;
   float *z = lds, *part = lds + 16 * zs;
   const int tid = threadIdx.x, lane = tid & 63, wv = tid >> 6, r16 = lane & 15, g = lane >> 4;
@@ -103,84 +164,47 @@ __global__ void __launch_bounds__(512) route_mfma_kernel(RouteArgs p) {
     f32x4 acc[4];
 #pragma unroll
     for (int i = 0; i < 4; ++i) acc[i] = f32x4{0.f, 0.f, 0.f, 0.f};
-#pragma unroll 2
-    for (int k = wv; k < nk; k += 8) {
-      const int c = k * 32 + g * 8;
-      const u32x4 zero = {0u, 0u, 0u, 0u};
-      const u32x4 b = c < d ? *reinterpret_cast<const u32x4*>(h + c) : zero;
+    auto steps = [&](auto ntc) {
+      constexpr int NTC = decltype(ntc)::value;
+#pragma unroll 4
+      for (int k = wv; k < nk; k += NW) {
+        const int c = k * 32 + g * 8;
+        const u32x4 zero = {0u, 0u, 0u, 0u};
+        const u32x4 b = c < d ? *reinterpret_cast<const u32x4*>(h + c) : zero;
 #pragma unroll
-      for (int i = 0; i < 4; ++i)
-        if (i < nt) {
+        for (int i = 0; i < NTC; ++i) {
           const u32x4 a = c < d ? *reinterpret_cast<const u32x4*>(w[i] + c) : zero;
           acc[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8, a), __builtin_bit_cast(bf16x8, b),
                                                            acc[i], 0, 0, 0);
         }
-    }
+      }
+    };
+    if (nt == 1) steps(std::integral_constant<int, 1>{});
+    else if (nt == 2) steps(std::integral_constant<int, 2>{});
+    else steps(std::integral_constant<int, 4>{});
     __syncthreads();
 #pragma unroll
     for (int i = 0; i < 4; ++i)
 #pragma unroll
       for (int r = 0; r < 4; ++r) part[(wv * 16 + r16) * 64 + i * 16 + g * 4 + r] = acc[i][r];
     __syncthreads();
-    for (int i = tid; i < 1024; i += 512) {
+    for (int i = tid; i < 1024; i += NW * 64) {
       float s = 0.f;
 #pragma unroll
-      for (int w8 = 0; w8 < 8; ++w8) s += part[w8 * 1024 + i];
+      for (int w8 = 0; w8 < NW; ++w8) s += part[w8 * 1024 + i];
       z[(i >> 6) * zs + e0 + (i & 63)] = s;
     }
   }
   __syncthreads();
-  for (int r = wv; r < 16; r += 8) {
+  for (int r = wv; r < 16; r += NW) {
     if (t0 + r >= p.T) break;
     if (p.wsg && lane == 0) p.sg[t0 + r] = sigmoid(z[r * zs + p.E]);
     pick(p, z + r * zs, t0 + r, lane);
   }
-}
-
-// n assignments -> perm (sorted position -> assignment), inv (assignment -> sorted position), tiles
-// [ntiles][3] (expert, first sorted position, rows <= mt) and their count. One workgroup.
-__global__ void __launch_bounds__(1024) group_kernel(const int* ids, int n, int E, int mt, int* perm, int* inv,
-                                                     int* tiles, int* ntiles) {
-  extern __shared__ int sh[];  // cnt[E], off[E + 1], toff[E + 1]
-  int *cnt = sh, *off = sh + E, *toff = off + E + 1;
-  const int tid = threadIdx.x;
-  for (int e = tid; e < E; e += 1024) cnt[e] = 0;
-  __syncthreads();
-  for (int i = tid; i < n; i += 1024) atomicAdd(&cnt[ids[i]], 1);
-  __syncthreads();
-  if (tid < 64) {  // exclusive sums over the experts, 64 at a time
-    int co = 0, to = 0;
-    for (int e0 = 0; e0 < E; e0 += 64) {
-      const int e = e0 + tid, c = e < E ? cnt[e] : 0, t = (c + mt - 1) / mt;
-      int cs = c, ts = t;
-#pragma unroll
-      for (int o = 1; o < 64; o <<= 1) {
-        const int a = __shfl_up(cs, o, 64), b = __shfl_up(ts, o, 64);
-        if (tid >= o) cs += a, ts += b;
-      }
-      if (e < E) off[e] = co + cs - c, toff[e] = to + ts - t;
-      co += __shfl(cs, 63, 64);
-      to += __shfl(ts, 63, 64);
-    }
-    if (tid == 0) off[E] = co, toff[E] = to, *ntiles = to;
-  }
-  __syncthreads();
-  for (int e = tid; e < E; e += 1024) {
-    const int c = cnt[e];
-    for (int j = 0; j * mt < c; ++j) {
-      int* t = tiles + (toff[e] + j) * 3;
-      t[0] = e;
-      t[1] = off[e] + j * mt;
-      t[2] = min(mt, c - j * mt);
-    }
-  }
-  __syncthreads();
-  for (int e = tid; e < E; e += 1024) cnt[e] = off[e];
-  __syncthreads();
-  for (int i = tid; i < n; i += 1024) {  // (the order within an expert does not matter: rows are independent)
-    const int pos = atomicAdd(&cnt[ids[i]], 1);
-    perm[pos] = i;
-    inv[i] = pos;
+  if constexpr (GROUP) {  // (the ids just stored are this workgroup's own)
+    asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
+    __syncthreads();
+    group_rows<NW * 64>(gr, reinterpret_cast<int*>(part));
   }
 }
 
@@ -303,12 +327,19 @@ template <bool UP>
 __global__ void __launch_bounds__(256, 2) expert_gemm_kernel(ExpertArgs p) {
   constexpr int BK = 64;
   __shared__ __attribute__((aligned(16))) bf16_t sw[2][128 * BK], sx[2][128 * BK];
-  if ((int)blockIdx.y >= *p.ntiles) return;
+  // order: an XCD works a contiguous run of (group of TG row tiles, weight block, row tile), so the weight
+  // rows that row tiles of one expert share, and the activations its weight blocks share, meet in one L2
+  constexpr int TG = 4;
+  const int nt = *p.ntiles, nb = (p.N + (UP ? 63 : 127)) / (UP ? 64 : 128);
+  if ((int)blockIdx.x >= nt * nb) return;
+  const int id = xcd_remap(blockIdx.x, nt * nb);
+  const int grp = id / (TG * nb), gt = min(TG, nt - grp * TG), in = id - grp * TG * nb;
+  const int tile = grp * TG + in % gt, bn = in / gt;
   const int tid = threadIdx.x, lane = tid & 63, wv = tid >> 6, l32 = lane & 31, hh = lane >> 5;
   const int wn = wv >> 1, wm = wv & 1;
-  const int* tl = p.tiles + blockIdx.y * 3;
+  const int* tl = p.tiles + tile * 3;
   const int ex = tl[0], lo = tl[1], nr = tl[2], K = p.K, N = p.N;
-  const int n0 = blockIdx.x * (UP ? 64 : 128);
+  const int n0 = bn * (UP ? 64 : 128);
   // staging: thread tid owns 16-B chunk tid % 8 of rows tid / 8 + 32 i
   const int ch = tid & 7, sr = tid >> 3;
   const bf16_t *wp[4], *xp[4];
@@ -429,6 +460,16 @@ int gemv_go(const ExpertArgs& a, int mt, int max_tiles, hipStream_t s) {
 
 bool al16(const void* p) { return (uintptr_t)p % 16 == 0; }
 
+template <int NW, bool GROUP>
+int route_go(const RouteArgs& a, const GroupArgs& g, hipStream_t s) {
+  const int zs = (a.E + (a.wsg ? 1 : 0) + 63) / 64 * 64, lds = (16 * zs + NW * 1024) * 4;
+  auto kern = route_mfma_kernel<NW, GROUP>;
+  if (lds > 48 * 1024 && hipFuncSetAttribute((const void*)kern, hipFuncAttributeMaxDynamicSharedMemorySize, lds) != hipSuccess)
+    return 5;
+  hipLaunchKernelGGL(kern, dim3((a.T + 15) / 16), dim3(NW * 64), lds, s, a, g);
+  return hipGetLastError() == hipSuccess ? 0 : 4;
+}
+
 }  // namespace
 
 // dtype: 0 fp32, 1 bf16
@@ -436,30 +477,37 @@ KCA_API int kca_moe_route(int dtype, const void* h, const void* wr, const void* 
                           int T, int d, int E, int top, hipStream_t s) {
   if (T < 1 || d < 1 || E < 1 || E > 1024 || top < 1 || top > E || !h || !wr || !ids || !wts || (wsg && !sg)) return 1;
   const RouteArgs a{h, wr, wsg, (int*)ids, (float*)wts, (float*)sg, T, d, E, top};
-  if (dtype == 1 && d % 8 == 0 && al16(h) && al16(wr) && al16(wsg)) {
-    const int zs = (E + (wsg ? 1 : 0) + 63) / 64 * 64, lds = (16 * zs + 8 * 1024) * 4;
-    if (lds > 48 * 1024 && hipFuncSetAttribute((const void*)route_mfma_kernel, hipFuncAttributeMaxDynamicSharedMemorySize,
-                                               lds) != hipSuccess)
-      return 5;
-    hipLaunchKernelGGL(route_mfma_kernel, dim3((T + 15) / 16), dim3(512), lds, s, a);
-  } else if (dtype == 1) {
-    hipLaunchKernelGGL(route_rows_kernel<bf16_t>, dim3(T), dim3(256), (E + 1) * 4, s, a);
-  } else if (dtype == 0) {
-    hipLaunchKernelGGL(route_rows_kernel<float>, dim3(T), dim3(256), (E + 1) * 4, s, a);
-  } else {
-    return 3;
-  }
+  if (dtype == 1 && d % 8 == 0 && al16(h) && al16(wr) && al16(wsg)) return route_go<8, false>(a, GroupArgs{}, s);
+  if (dtype == 1) hipLaunchKernelGGL(route_rows_kernel<bf16_t>, dim3(T), dim3(256), (E + 1) * 4, s, a);
+  else if (dtype == 0) hipLaunchKernelGGL(route_rows_kernel<float>, dim3(T), dim3(256), (E + 1) * 4, s, a);
+  else return 3;
   return hipGetLastError() == hipSuccess ? 0 : 4;
+}
+
+static bool group_ok(const GroupArgs& g, int max_tiles) {
+  return g.n >= 1 && g.E >= 1 && g.E <= 1024 && g.mt >= 1 && g.ids && g.perm && g.inv && g.tiles && g.ntiles &&
+         max_tiles >= (g.E < g.n ? g.E : g.n) + g.n / g.mt;
 }
 
 // tiles: [max_tiles][3] with max_tiles >= min(E, n) + n / mt
 KCA_API int kca_moe_group(const void* ids, int n, int E, int mt, void* perm, void* inv, void* tiles, int max_tiles,
                           void* ntiles, hipStream_t s) {
-  if (n < 1 || E < 1 || E > 1024 || mt < 1 || !ids || !perm || !inv || !tiles || !ntiles) return 1;
-  if (max_tiles < (E < n ? E : n) + n / mt) return 2;
-  hipLaunchKernelGGL(group_kernel, dim3(1), dim3(1024), (3 * E + 2) * 4, s, (const int*)ids, n, E, mt, (int*)perm,
-                     (int*)inv, (int*)tiles, (int*)ntiles);
+  const GroupArgs g{(const int*)ids, n, E, mt, (int*)perm, (int*)inv, (int*)tiles, (int*)ntiles};
+  if (!group_ok(g, max_tiles)) return 1;
+  hipLaunchKernelGGL(group_kernel, dim3(1), dim3(1024), (3 * E + 2) * 4, s, g);
   return hipGetLastError() == hipSuccess ? 0 : 4;
+}
+
+// Both in one launch: bf16, at most 16 tokens (10: shape outside it)
+KCA_API int kca_moe_route_group(const void* h, const void* wr, const void* wsg, void* ids, void* wts, void* sg, int T,
+                                int d, int E, int top, int mt, void* perm, void* inv, void* tiles, int max_tiles,
+                                void* ntiles, hipStream_t s) {
+  if (T < 1 || d < 1 || E < 1 || E > 1024 || top < 1 || top > E || !h || !wr || !ids || !wts || (wsg && !sg)) return 1;
+  if (T > 16 || d % 8 || !al16(h) || !al16(wr) || !al16(wsg)) return 10;
+  const RouteArgs a{h, wr, wsg, (int*)ids, (float*)wts, (float*)sg, T, d, E, top};
+  const GroupArgs g{(const int*)ids, T * top, E, mt, (int*)perm, (int*)inv, (int*)tiles, (int*)ntiles};
+  if (!group_ok(g, max_tiles)) return 1;
+  return route_go<16, true>(a, g, s);
 }
 
 // One expert product of every tile. mt: the tiles' row limit (1, 2, 4, 8: gemv; 128: gemm, bf16 with
@@ -471,8 +519,8 @@ KCA_API int kca_moe_expert(int dtype, const void* x, const void* w, void* y, con
   const ExpertArgs a{x, w, y, (const int*)perm, (const float*)wts, (const int*)tiles, (const int*)ntiles, top, N, K, up, scale};
   if (mt == 128) {
     if (dtype != 1 || K % 8 || N % 4 || !al16(x) || !al16(w) || (uintptr_t)y % 8) return 10;
-    if (up) hipLaunchKernelGGL(expert_gemm_kernel<true>, dim3((N + 63) / 64, max_tiles), dim3(256), 0, s, a);
-    else hipLaunchKernelGGL(expert_gemm_kernel<false>, dim3((N + 127) / 128, max_tiles), dim3(256), 0, s, a);
+    if (up) hipLaunchKernelGGL(expert_gemm_kernel<true>, dim3((N + 63) / 64 * max_tiles), dim3(256), 0, s, a);
+    else hipLaunchKernelGGL(expert_gemm_kernel<false>, dim3((N + 127) / 128 * max_tiles), dim3(256), 0, s, a);
     return hipGetLastError() == hipSuccess ? 0 : 4;
   }
   const bool vec = K % (dtype == 1 ? 8 : 4) == 0 && al16(x) && al16(w);

@@ -148,8 +148,8 @@ class HybridRunner(StepRunner):
             y = inv = None
             if L.moe:
                 mlp = L.spec.mlp
-                ids, wts, sg = moe.route(h, L.router, mlp.top, L.shared_gate)
-                g = moe.group(ids, mlp.experts, moe.tile_rows(T, mlp.top, mlp.experts, d, mlp.ff, h.dtype))
+                ids, wts, sg, g = moe.route_group(h, L.router, mlp.top, L.shared_gate,
+                                                  moe.tile_rows(T, mlp.top, mlp.experts, d, mlp.ff, h.dtype))
                 y, inv = moe.experts(h, ids, wts, L.gate_up, L.down, g, mlp.scale_in), g.inv
                 if up is not None:
                     moe.act_rows(up, cat[:, cols:], gated=True, row_scale=sg)

@@ -20,7 +20,8 @@ from . import _lib
 from .decode import decode_chunk, gather_kv
 from .rms_shift import native_dt
 
-TILE = 128  # query rows of a matrix-core workgroup
+TILE = 128        # query rows of a matrix-core workgroup
+MAX_SPLITS = 256  # key splits the rows kernel merges
 
 
 class _Args(ctypes.Structure):
@@ -129,7 +130,7 @@ def rows_plan(sp: DiffHeads, rows: int, max_kv: int, dtype) -> tuple[int, int, i
     rb = 4 if vec and hg > 1 else 1
     sub = -(-hg // rb)
     blocks = rows * sp.kv_heads * sub
-    chunk = decode_chunk(rows, sp.kv_heads * sub, max_kv)
+    chunk = max(decode_chunk(rows, sp.kv_heads * sub, max_kv), -(-max_kv // MAX_SPLITS))
     n = -(-max_kv // chunk)
     return n, chunk, (blocks * n * 2 * rb * (sp.vdim + 2) if n > 1 else 0), blocks
 

@@ -55,12 +55,36 @@ def tile_rows(T: int, top: int, E: int, d: int, F: int, dtype) -> int:
     return 1 if T == 1 else 2 if T == 2 else 4 if T <= 4 else 8
 
 
+def _groups(T: int, top: int, E: int, mt: int, device) -> Groups:
+    n = T * top
+    z = dict(device=device, dtype=torch.int32)
+    return Groups(torch.empty(n, **z), torch.empty(T, top, **z), torch.empty(min(E, n) + n // mt, 3, **z),
+                  torch.empty(1, **z), mt)
+
+
+def route_group(h: torch.Tensor, router: torch.Tensor, top: int, shared_gate: torch.Tensor | None, mt: int):
+    """``route`` and ``group`` -> (ids, weights, shared gate, groups); one launch for up to 16 bf16 tokens."""
+    T, d = h.shape
+    E = router.shape[0]
+    if native_dt(h, router, shared_gate) == 1 and T <= 16 and d % 8 == 0:
+        g = _groups(T, top, E, mt, h.device)
+        ids = torch.empty(T, top, device=h.device, dtype=torch.int32)
+        w = torch.empty(T, top, device=h.device, dtype=torch.float32)
+        sg = torch.empty(T, device=h.device, dtype=torch.float32) if shared_gate is not None else None
+        assert h.is_contiguous() and router.is_contiguous() and router.shape[1] == d
+        _lib.call("kca_moe_route_group", h.data_ptr(), router.data_ptr(), _lib.ptr(shared_gate), ids.data_ptr(),
+                  w.data_ptr(), _lib.ptr(sg), T, d, E, top, mt, g.perm.data_ptr(), g.inv.data_ptr(),
+                  g.tiles.data_ptr(), g.tiles.shape[0], g.ntiles.data_ptr(), _lib.stream())
+        return ids, w, sg, g
+    ids, w, sg = route(h, router, top, shared_gate)
+    return ids, w, sg, group(ids, E, mt)
+
+
 def group(ids: torch.Tensor, E: int, mt: int) -> Groups:
     T, top = ids.shape
     n = T * top
-    mx = min(E, n) + n // mt
-    z = dict(device=ids.device, dtype=torch.int32)
-    g = Groups(torch.empty(n, **z), torch.empty(T, top, **z), torch.empty(mx, 3, **z), torch.empty(1, **z), mt)
+    g = _groups(T, top, E, mt, ids.device)
+    mx = g.tiles.shape[0]
     if not ids.is_cuda:
         order = torch.argsort(ids.reshape(-1), stable=True)
         g.perm.copy_(order)
@@ -116,4 +140,4 @@ def act_rows(x: torch.Tensor, out: torch.Tensor, gated: bool, row_scale: torch.T
     return out
 
 
-__all__ = ["route", "group", "experts", "act_rows", "tile_rows", "Groups"]
+__all__ = ["route", "group", "route_group", "experts", "act_rows", "tile_rows", "Groups"]

@@ -397,6 +397,10 @@ def test_routed_experts(device, dtype, T, d, E, top, F, shared):
     assert (s is None) == (not shared)
     if shared:
         assert rel(s, torch.sigmoid(h.double() @ sg.double().T)[:, 0]) < 2e-6
+    ids2, wt2, s2, g2 = moe.route_group(dv(h), dv(w["router"]), top, dv(sg) if shared else None, 8)
+    assert torch.equal(ids2, ids) and rel(wt2, wt.cpu()) < 1e-6 and (not shared or rel(s2, s.cpu()) < 1e-6)
+    order = [ids2.reshape(-1)[a] for a in g2.perm.tolist()]
+    assert order == sorted(order) and g2.inv.reshape(-1)[g2.perm.long()].tolist() == list(range(T * top))
     tol = 3e-6 if dtype == F32 else 1.2e-2
     sizes = {moe.tile_rows(T, top, E, d, F, dtype)} | ({1, 4, 8} if device == "cuda" else set())
     if device == "cuda" and dtype == BF16 and d % 8 == 0 and F % 8 == 0:
