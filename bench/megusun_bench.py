@@ -115,10 +115,8 @@ def run_models(sizes=None, batches=(1, 8, 32), prompt=1024, new_tokens=48, prefi
 def _time(fns, reps=5):
     """us per call of a ring of calls on distinct buffers (weights and caches are cold in L2), as one HIP
     graph so that host time between launches does not count."""
-    s = torch.cuda.Stream()
-    with torch.cuda.stream(s):
-        for f in fns:
-            f()
+    for f in fns:  # (on the stream that filled the operands)
+        f()
     torch.cuda.synchronize()
     g = torch.cuda.CUDAGraph()
     with torch.cuda.graph(g):
@@ -231,7 +229,7 @@ def run_kernels(d=4096, heads=16, T=4096, cached=2048, batches=(1, 8, 32), ring=
     # ---- decode attention over cold caches
     for G in (heads, heads // 4):
         sp = da.DiffHeads(heads, G, D // 2, D, (D // 2) ** -0.5, .5, .6, 1e-5, .1, 512.)
-        for B in batches:
+        for B in batches:  # (a grouped cache: GPT-J's kernel on the same group count)
             nb = cached // 64
             n = max(2, min(ring * 2, int(1.5e9 / (B * nb * 64 * G * 2 * D * 2))))
             ks = [torch.randn(B * nb + 1, 2 * G, 64, D // 2, **bf) for _ in range(n)]
@@ -244,14 +242,13 @@ def run_kernels(d=4096, heads=16, T=4096, cached=2048, batches=(1, 8, 32), ring=
             us = _time([lambda k=k, v=v: da.attend_rows(sp, qkv, k, v, tbl, pos, slot, o, cached, fused_append=True, ws=ws,
                                                         cnt=cnt) for k, v in zip(ks, vs)])
             rec(f"diff_rows B={B} cached={cached} H={heads} G={G}", us, B * cached * G * 2 * D * 2, like="decode_attention")
-            if G == heads:
-                ks = [k.view(-1)[:(B * nb + 1) * G * 64 * D].view(-1, G, 64, D) for k in ks]
-                q3, kl = torch.randn(B, 3 * heads * D, **bf), torch.full((B,), cached, **i32)
-                w2 = torch.zeros(max(1, dops.decode_ws_floats(B, heads, G, D, cached)), device=dev)
-                us = _time([lambda k=k, v=v: dops.decode_prep_attention(
-                    q3, heads, G, D, 0, True, None, None, pos, slot, k, v, kl, cached, out=o, ws=w2, block_table=tbl)
-                    for k, v in zip(ks, vs)])
-                rec(f"gptj decode_attention B={B} cached={cached}", us, B * cached * G * 2 * D * 2)
+            ks = [k.view(-1)[:(B * nb + 1) * G * 64 * D].view(-1, G, 64, D) for k in ks]
+            q3, kl = torch.randn(B, (heads + 2 * G) * D, **bf), torch.full((B,), cached, **i32)
+            w2 = torch.zeros(max(1, dops.decode_ws_floats(B, heads, G, D, cached)), device=dev)
+            us = _time([lambda k=k, v=v: dops.decode_prep_attention(
+                q3, heads, G, D, 0, True, None, None, pos, slot, k, v, kl, cached, out=o, ws=w2, block_table=tbl)
+                for k, v in zip(ks, vs)])
+            rec(f"gptj decode_attention B={B} cached={cached} G={G}", us, B * cached * G * 2 * D * 2)
             del ks, vs
     # ---- router, experts
     E, top, Fe = 16, 2, 4096

@@ -480,10 +480,19 @@ __global__ void __launch_bounds__(512, 2) diff_tile_kernel(DiffArgs p) {
       f32x16 s;
 #pragma unroll
       for (int r = 0; r < 16; ++r) s[r] = 0.f;
+      bf16x8 fk[3];  // K fragments two steps ahead of their products
+      fk[0] = lds_b128(buf, kb_e);
+      if constexpr (KS > 1) fk[1] = lds_b128(buf, kb_o);
+      __builtin_amdgcn_sched_group_barrier(0x100, KS > 1 ? 2 : 1, 0);
 #pragma unroll
-      for (int k = 0; k < KS; ++k)
-        s = __builtin_amdgcn_mfma_f32_32x32x16_bf16(lds_b128(buf, ((k & 1) ? kb_o : kb_e) + 512 * (k >> 1)), qf[k], s,
-                                                    0, 0, 0);
+      for (int k = 0; k < KS; ++k) {
+        if (k + 2 < KS) {
+          fk[(k + 2) % 3] = lds_b128(buf, ((k & 1) ? kb_o : kb_e) + 512 * ((k + 2) >> 1));
+          __builtin_amdgcn_sched_group_barrier(0x100, 1, 0);
+        }
+        s = __builtin_amdgcn_mfma_f32_32x32x16_bf16(fk[k % 3], qf[k], s, 0, 0, 0);
+        __builtin_amdgcn_sched_group_barrier(0x8, 1, 0);
+      }
       // s[r]: key k0 + (r & 3) + 8 (r >> 2) + 4 hh of this lane's query
       if (k0 + BN > pos0 + qg * 32) {
         const int lim = pos - k0 - 4 * hh;
@@ -529,12 +538,23 @@ __global__ void __launch_bounds__(512, 2) diff_tile_kernel(DiffArgs p) {
       ls += sum;
       const bf16x8 p0 = __builtin_bit_cast(bf16x8, u32x4{u[0], u[1], u[2], u[3]});
       const bf16x8 p1 = __builtin_bit_cast(bf16x8, u32x4{u[4], u[5], u[6], u[7]});
+      auto vfrag = [&](int b, int h2) {
+        return cat8(lds_tr4(buf, vb_1 + 32 * DV * h2 + 512 * b), lds_tr4(buf, vb_2 + 32 * DV * h2 + 512 * b));
+      };
+      bf16x8 v0[2], v1[2];  // V fragments one block ahead
+      v0[0] = vfrag(0, 0);
+      v1[0] = vfrag(0, 1);
+      __builtin_amdgcn_sched_group_barrier(0x100, 4, 0);
 #pragma unroll
       for (int b = 0; b < NB; ++b) {
-        const bf16x8 v0 = cat8(lds_tr4(buf, vb_1 + 512 * b), lds_tr4(buf, vb_2 + 512 * b));
-        const bf16x8 v1 = cat8(lds_tr4(buf, vb_1 + 32 * DV + 512 * b), lds_tr4(buf, vb_2 + 32 * DV + 512 * b));
-        o[b] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(v0, p0, o[b], 0, 0, 0);
-        o[b] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(v1, p1, o[b], 0, 0, 0);
+        if (b + 1 < NB) {
+          v0[(b + 1) & 1] = vfrag(b + 1, 0);
+          v1[(b + 1) & 1] = vfrag(b + 1, 1);
+          __builtin_amdgcn_sched_group_barrier(0x100, 4, 0);
+        }
+        o[b] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(v0[b & 1], p0, o[b], 0, 0, 0);
+        o[b] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(v1[b & 1], p1, o[b], 0, 0, 0);
+        __builtin_amdgcn_sched_group_barrier(0x8, 2, 0);
       }
     }
     if (more) store(st, smem + ((t + 1) & 1) * BUF);

@@ -77,9 +77,32 @@ __device__ __forceinline__ void stn(E* p, const float (&v)[V]) {
 // one element's gate and candidate
 template <typename E>
 __device__ __forceinline__ void gate(float zx, float ux, float& z, float& zc) {
+  if constexpr (Vec<E>::fast) {
+    const float ez = 1.f + __expf(fminf(-zx, 28.f)), eu = 1.f + __expf(fminf(-ux, 28.f));
+    const float r = __builtin_amdgcn_rcpf(ez * eu);
+    z = r * eu;
+    zc = z * (ux >= 0.f ? ux + 0.5f : r * ez);
+    return;
+  }
   z = Vec<E>::sig(zx);
   const float c = ux >= 0.f ? ux + 0.5f : Vec<E>::sig(ux);
   zc = z * c;
+}
+
+// ... and with the output gate's silu: fp32 as written; bf16 shares one reciprocal between the sigmoids
+// (inputs clamped at -28, where a sigmoid is below 1e-12), since the scan is bound by these as much as by memory
+template <typename E>
+__device__ __forceinline__ void gate_out(float zx, float ux, float g, float& z, float& zc, float& sg) {
+  if constexpr (Vec<E>::fast) {
+    const float ez = 1.f + __expf(fminf(-zx, 28.f)), eu = 1.f + __expf(fminf(-ux, 28.f)), eg = 1.f + __expf(fminf(-g, 28.f));
+    const float zu = ez * eu, r = __builtin_amdgcn_rcpf(zu * eg);
+    z = r * eu * eg;
+    zc = z * (ux >= 0.f ? ux + 0.5f : r * ez * eg);
+    sg = g * r * zu;
+  } else {
+    gate<E>(zx, ux, z, zc);
+    sg = g * Vec<E>::sig(g);
+  }
 }
 
 constexpr int UN = 8;  // tokens whose loads are in flight together
@@ -189,11 +212,10 @@ __global__ void __launch_bounds__(64) scan_run_kernel(ScanArgs p) {
       float o[V];
 #pragma unroll
       for (int e = 0; e < V; ++e) {
-        float z, zc;
-        gate<E>(zv[i].f(e) + bz[e], uv[i].f(e) + bx[e], z, zc);
+        float z, zc, sg;
+        gate_out<E>(zv[i].f(e) + bz[e], uv[i].f(e) + bx[e], gv[i].f(e), z, zc, sg);
         S[e] = fmaf(1.f - z, S[e], zc);
-        const float g = gv[i].f(e);
-        o[e] = S[e] * g * Vec<E>::sig(g);
+        o[e] = S[e] * sg;
       }
       stn<E, V>(y + (t0 + i) * p.ldy, o);
     }
@@ -221,10 +243,10 @@ __global__ void __launch_bounds__(64) scan_step_kernel(ScanArgs p, const int* po
   if (pos[b] > 0) ldn<float, V>(st, S);
 #pragma unroll
   for (int e = 0; e < V; ++e) {
-    float z, zc;
-    gate<E>(z4[e] + bz[e], u4[e] + bx[e], z, zc);
+    float z, zc, sg;
+    gate_out<E>(z4[e] + bz[e], u4[e] + bx[e], g4[e], z, zc, sg);
     S[e] = fmaf(1.f - z, S[e], zc);
-    o[e] = S[e] * g4[e] * Vec<E>::sig(g4[e]);
+    o[e] = S[e] * sg;
   }
   stn<float, V>(st, S);
   stn<E, V>(reinterpret_cast<E*>(p.y) + (long long)b * p.ldy + w, o);

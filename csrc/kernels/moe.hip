@@ -42,7 +42,7 @@ struct RouteArgs {
 };
 
 // One wave: the top experts of one token from its logits z[E] (LDS); ties go to the lower index.
-__device__ __forceinline__ void pick(const RouteArgs& p, float* z, int t, int lane) {
+__device__ __forceinline__ void pick(const RouteArgs& p, float* z, int t, int lane, int* ids_lds = nullptr) {
   for (int k = 0; k < p.top; ++k) {
     float best = -INFINITY;
     int bi = 0x7fffffff;
@@ -57,6 +57,7 @@ __device__ __forceinline__ void pick(const RouteArgs& p, float* z, int t, int la
     if (bi >= p.E) bi = 0;  // (no finite score left)
     if (lane == 0) {
       p.ids[(long long)t * p.top + k] = bi;
+      if (ids_lds) ids_lds[t * p.top + k] = bi;
       p.wts[(long long)t * p.top + k] = sigmoid(best);
       z[bi] = -INFINITY;
     }
@@ -146,9 +147,10 @@ __global__ void __launch_bounds__(1024) group_kernel(GroupArgs p) {
 // one workgroup, which also groups its assignments (the decode step)
 template <int NW, bool GROUP>
 __global__ void __launch_bounds__(NW * 64) route_mfma_kernel(RouteArgs p, GroupArgs gr) {
-  extern __shared__ __attribute__((aligned(16))) float lds[];  // z[16][zs], part[NW][16][64] (then group_rows')
+  extern __shared__ __attribute__((aligned(16))) float lds[];  // z[16][zs], part[NW][16][64] (then group_rows'), ids
   const int n = p.E + (p.wsg ? 1 : 0), zs = (n + 63) / 64 * 64;
   float *z = lds, *part = lds + 16 * zs;
+  int* sids = reinterpret_cast<int*>(part + NW * 1024);  // GROUP: [T * top]
   const int tid = threadIdx.x, lane = tid & 63, wv = tid >> 6, r16 = lane & 15, g = lane >> 4;
   const int t0 = blockIdx.x * 16, d = p.d;
   const bf16_t* h = reinterpret_cast<const bf16_t*>(p.h) + (long long)min(t0 + r16, p.T - 1) * d;
@@ -199,11 +201,11 @@ __global__ void __launch_bounds__(NW * 64) route_mfma_kernel(RouteArgs p, GroupA
   for (int r = wv; r < 16; r += NW) {
     if (t0 + r >= p.T) break;
     if (p.wsg && lane == 0) p.sg[t0 + r] = sigmoid(z[r * zs + p.E]);
-    pick(p, z + r * zs, t0 + r, lane);
+    pick(p, z + r * zs, t0 + r, lane, GROUP ? sids : nullptr);
   }
-  if constexpr (GROUP) {  // (the ids just stored are this workgroup's own)
-    asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
+  if constexpr (GROUP) {
     __syncthreads();
+    gr.ids = sids;
     group_rows<NW * 64>(gr, reinterpret_cast<int*>(part));
   }
 }
@@ -320,17 +322,20 @@ __global__ void __launch_bounds__(256) expert_gemv_kernel(ExpertArgs p) {
 }
 
 // ------------------------------------------------------------------------------------------------ gemm
-// bf16, 128 rows x 128 weight rows x 64 per step, 4 waves of 64 x 64 (32x32x16 tiles); weights are the A
-// operand, so a lane holds one activation row and runs of four outputs. up: a workgroup covers 64 gate
-// and the matching 64 up rows, each wave 32 of both.
+// bf16, 128 rows x 256 weight rows x 64 per step, 8 waves of 64 x 64 (32x32x16 tiles); weights are the A
+// operand, so a lane holds one activation row and runs of four outputs. up: a workgroup covers 128 gate
+// and the matching 128 up rows, each wave 32 of both.
+constexpr int GBK = 64, GN = 256, GM = 128, GEMM_LDS = 2 * (GN + GM) * GBK * 2;
+
 template <bool UP>
-__global__ void __launch_bounds__(256, 2) expert_gemm_kernel(ExpertArgs p) {
-  constexpr int BK = 64;
-  __shared__ __attribute__((aligned(16))) bf16_t sw[2][128 * BK], sx[2][128 * BK];
+__global__ void __launch_bounds__(512, 2) expert_gemm_kernel(ExpertArgs p) {
+  constexpr int BK = GBK;
+  extern __shared__ __attribute__((aligned(16))) bf16_t gl[];  // [2][GN + GM][BK]: weight rows, then activation rows
+  bf16_t *const sw[2] = {gl, gl + (GN + GM) * BK}, *const sx[2] = {gl + GN * BK, gl + (2 * GN + GM) * BK};
   // order: an XCD works a contiguous run of (group of TG row tiles, weight block, row tile), so the weight
   // rows that row tiles of one expert share, and the activations its weight blocks share, meet in one L2
   constexpr int TG = 4;
-  const int nt = *p.ntiles, nb = (p.N + (UP ? 63 : 127)) / (UP ? 64 : 128);
+  const int nt = *p.ntiles, nb = (p.N + (UP ? 127 : 255)) / (UP ? 128 : 256);
   if ((int)blockIdx.x >= nt * nb) return;
   const int id = xcd_remap(blockIdx.x, nt * nb);
   const int grp = id / (TG * nb), gt = min(TG, nt - grp * TG), in = id - grp * TG * nb;
@@ -339,37 +344,42 @@ __global__ void __launch_bounds__(256, 2) expert_gemm_kernel(ExpertArgs p) {
   const int wn = wv >> 1, wm = wv & 1;
   const int* tl = p.tiles + tile * 3;
   const int ex = tl[0], lo = tl[1], nr = tl[2], K = p.K, N = p.N;
-  const int n0 = bn * (UP ? 64 : 128);
-  // staging: thread tid owns 16-B chunk tid % 8 of rows tid / 8 + 32 i
+  const int n0 = bn * (UP ? 128 : 256);
+  // staging: thread tid owns 16-B chunk tid % 8 of rows tid / 8 + 64 i
   const int ch = tid & 7, sr = tid >> 3;
-  const bf16_t *wp[4], *xp[4];
+  const bf16_t *wp[4], *xp[2];
 #pragma unroll
   for (int i = 0; i < 4; ++i) {
-    const int r = sr + 32 * i;
+    const int r = sr + 64 * i;
     long long wr;
-    if constexpr (UP) wr = (r < 64 ? 0 : N) + min(n0 + (r & 63), N - 1);
+    if constexpr (UP) wr = (r < 128 ? 0 : N) + min(n0 + (r & 127), N - 1);
     else wr = min(n0 + r, N - 1);
     wp[i] = reinterpret_cast<const bf16_t*>(p.w) + ((long long)ex * (UP ? 2 * N : N) + wr) * K;
-    const int xr = lo + min(r, nr - 1);
+  }
+#pragma unroll
+  for (int i = 0; i < 2; ++i) {
+    const int r = sr + 64 * i, xr = lo + min(r, nr - 1);
     const long long src = UP ? p.perm[xr] / p.top : xr;
     xp[i] = reinterpret_cast<const bf16_t*>(p.x) + src * K;
   }
-  u32x4 rw[4], rx[4];
-  auto load = [&](int k0) {
-    const int k = k0 + ch * 8;
+  // Two k steps in flight in registers (a step's products alone do not cover a trip past L2). No load or
+  // store of the loop is conditional -- a branch between them would make every wait a full drain: loads
+  // past K repeat valid columns, and such columns of the activation are stored as zeros.
+  u32x4 ra[2][4], rb[2][2];
+  auto load = [&](int t, u32x4 (&rw)[4], u32x4 (&rx)[2]) {
+    const int k = min(t * BK + ch * 8, K - 8);
 #pragma unroll
-    for (int i = 0; i < 4; ++i) {
-      rw[i] = k < K ? *reinterpret_cast<const u32x4*>(wp[i] + k) : u32x4{0u, 0u, 0u, 0u};
-      rx[i] = k < K ? *reinterpret_cast<const u32x4*>(xp[i] + k) : u32x4{0u, 0u, 0u, 0u};
-    }
+    for (int i = 0; i < 4; ++i) rw[i] = *reinterpret_cast<const u32x4*>(wp[i] + k);
+#pragma unroll
+    for (int i = 0; i < 2; ++i) rx[i] = *reinterpret_cast<const u32x4*>(xp[i] + k);
   };
-  auto store = [&](int b) {
+  const int so = sr * BK + ((ch ^ (sr & 7)) << 3);
+  auto store = [&](int t, int b, const u32x4 (&rw)[4], const u32x4 (&rx)[2]) {
+    const uint32_t keep = t * BK + ch * 8 < K ? ~0u : 0u;
 #pragma unroll
-    for (int i = 0; i < 4; ++i) {
-      const int r = sr + 32 * i, o = r * BK + ((ch ^ (r & 7)) << 3);
-      *reinterpret_cast<u32x4*>(&sw[b][o]) = rw[i];
-      *reinterpret_cast<u32x4*>(&sx[b][o]) = rx[i];
-    }
+    for (int i = 0; i < 4; ++i) *reinterpret_cast<u32x4*>(sw[b] + so + 64 * i * BK) = rw[i];
+#pragma unroll
+    for (int i = 0; i < 2; ++i) *reinterpret_cast<u32x4*>(sx[b] + so + 64 * i * BK) = rx[i] & u32x4{keep, keep, keep, keep};
   };
   f32x16 acc[2][2];
 #pragma unroll
@@ -381,34 +391,52 @@ __global__ void __launch_bounds__(256, 2) expert_gemm_kernel(ExpertArgs p) {
   int ar[2], br[2];
 #pragma unroll
   for (int i = 0; i < 2; ++i) {
-    ar[i] = (UP ? i * 64 + wn * 32 : wn * 64 + i * 32) + l32;
+    ar[i] = (UP ? i * 128 + wn * 32 : wn * 64 + i * 32) + l32;
     br[i] = wm * 64 + i * 32 + l32;
   }
-  const int nk = (K + BK - 1) / BK;
-  const bool live = wm * 64 < nr;
-  load(0);
-  store(0);
-  __syncthreads();
-  for (int t = 0; t < nk; ++t) {
-    const int b = t & 1;
-    if (t + 1 < nk) load((t + 1) * BK);
+  const int nk = ((K + BK - 1) / BK + 1) & ~1;  // (an odd count's extra step multiplies zeros)
+  const bool live = __builtin_amdgcn_readfirstlane(wm) * 64 < nr;
+  // step t: LDS buffer t & 1 holds it, register set (t + 1) & 1 the next, the other set is requested
+  auto step = [&](int t, auto par) {
+    constexpr int b = decltype(par)::value;
+    load(t + 2, ra[b], rb[b]);
+    asm volatile("" ::: "memory");
     if (live) {
-#pragma unroll
-      for (int s = 0; s < BK / 16; ++s) {
-        bf16x8 a[2], x[2];
+      bf16x8 a[2][2], x[2][2];
+      auto frag = [&](int s, int f) {
 #pragma unroll
         for (int i = 0; i < 2; ++i) {
-          a[i] = *reinterpret_cast<const bf16x8*>(&sw[b][ar[i] * BK + (((2 * s + hh) ^ (ar[i] & 7)) << 3)]);
-          x[i] = *reinterpret_cast<const bf16x8*>(&sx[b][br[i] * BK + (((2 * s + hh) ^ (br[i] & 7)) << 3)]);
+          a[f][i] = *reinterpret_cast<const bf16x8*>(sw[b] + ar[i] * BK + (((2 * s + hh) ^ (ar[i] & 7)) << 3));
+          x[f][i] = *reinterpret_cast<const bf16x8*>(sx[b] + br[i] * BK + (((2 * s + hh) ^ (br[i] & 7)) << 3));
+        }
+      };
+      frag(0, 0);
+      __builtin_amdgcn_sched_group_barrier(0x100, 4, 0);
+#pragma unroll
+      for (int s = 0; s < BK / 16; ++s) {  // fragments one sub-step ahead of their products
+        if (s + 1 < BK / 16) {
+          frag(s + 1, (s + 1) & 1);
+          __builtin_amdgcn_sched_group_barrier(0x100, 4, 0);
         }
 #pragma unroll
         for (int i = 0; i < 2; ++i)
 #pragma unroll
-          for (int j = 0; j < 2; ++j) acc[i][j] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(a[i], x[j], acc[i][j], 0, 0, 0);
+          for (int j = 0; j < 2; ++j)
+            acc[i][j] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(a[s & 1][i], x[s & 1][j], acc[i][j], 0, 0, 0);
+        __builtin_amdgcn_sched_group_barrier(0x8, 4, 0);
       }
     }
-    if (t + 1 < nk) store(b ^ 1);
+    asm volatile("" ::: "memory");
+    store(t + 1, b ^ 1, ra[b ^ 1], rb[b ^ 1]);
     __syncthreads();
+  };
+  load(0, ra[0], rb[0]);
+  store(0, 0, ra[0], rb[0]);
+  load(1, ra[1], rb[1]);
+  __syncthreads();
+  for (int t = 0; t < nk; t += 2) {
+    step(t, std::integral_constant<int, 0>{});
+    step(t + 1, std::integral_constant<int, 1>{});
   }
 #pragma unroll
   for (int j = 0; j < 2; ++j) {
@@ -462,7 +490,7 @@ bool al16(const void* p) { return (uintptr_t)p % 16 == 0; }
 
 template <int NW, bool GROUP>
 int route_go(const RouteArgs& a, const GroupArgs& g, hipStream_t s) {
-  const int zs = (a.E + (a.wsg ? 1 : 0) + 63) / 64 * 64, lds = (16 * zs + NW * 1024) * 4;
+  const int zs = (a.E + (a.wsg ? 1 : 0) + 63) / 64 * 64, lds = (16 * zs + NW * 1024 + (GROUP ? a.T * a.top : 0)) * 4;
   auto kern = route_mfma_kernel<NW, GROUP>;
   if (lds > 48 * 1024 && hipFuncSetAttribute((const void*)kern, hipFuncAttributeMaxDynamicSharedMemorySize, lds) != hipSuccess)
     return 5;
@@ -503,7 +531,7 @@ KCA_API int kca_moe_route_group(const void* h, const void* wr, const void* wsg, 
                                 int d, int E, int top, int mt, void* perm, void* inv, void* tiles, int max_tiles,
                                 void* ntiles, hipStream_t s) {
   if (T < 1 || d < 1 || E < 1 || E > 1024 || top < 1 || top > E || !h || !wr || !ids || !wts || (wsg && !sg)) return 1;
-  if (T > 16 || d % 8 || !al16(h) || !al16(wr) || !al16(wsg)) return 10;
+  if (T > 16 || top > 64 || d % 8 || !al16(h) || !al16(wr) || !al16(wsg)) return 10;
   const RouteArgs a{h, wr, wsg, (int*)ids, (float*)wts, (float*)sg, T, d, E, top};
   const GroupArgs g{(const int*)ids, T * top, E, mt, (int*)perm, (int*)inv, (int*)tiles, (int*)ntiles};
   if (!group_ok(g, max_tiles)) return 1;
@@ -519,8 +547,10 @@ KCA_API int kca_moe_expert(int dtype, const void* x, const void* w, void* y, con
   const ExpertArgs a{x, w, y, (const int*)perm, (const float*)wts, (const int*)tiles, (const int*)ntiles, top, N, K, up, scale};
   if (mt == 128) {
     if (dtype != 1 || K % 8 || N % 4 || !al16(x) || !al16(w) || (uintptr_t)y % 8) return 10;
-    if (up) hipLaunchKernelGGL(expert_gemm_kernel<true>, dim3((N + 63) / 64 * max_tiles), dim3(256), 0, s, a);
-    else hipLaunchKernelGGL(expert_gemm_kernel<false>, dim3((N + 127) / 128 * max_tiles), dim3(256), 0, s, a);
+    const void* kern = up ? (const void*)expert_gemm_kernel<true> : (const void*)expert_gemm_kernel<false>;
+    if (hipFuncSetAttribute(kern, hipFuncAttributeMaxDynamicSharedMemorySize, GEMM_LDS) != hipSuccess) return 5;
+    if (up) hipLaunchKernelGGL(expert_gemm_kernel<true>, dim3((N + 127) / 128 * max_tiles), dim3(512), GEMM_LDS, s, a);
+    else hipLaunchKernelGGL(expert_gemm_kernel<false>, dim3((N + 255) / 256 * max_tiles), dim3(512), GEMM_LDS, s, a);
     return hipGetLastError() == hipSuccess ? 0 : 4;
   }
   const bool vec = K % (dtype == 1 ? 8 : 4) == 0 && al16(x) && al16(w);

@@ -66,7 +66,7 @@ def route_group(h: torch.Tensor, router: torch.Tensor, top: int, shared_gate: to
     """``route`` and ``group`` -> (ids, weights, shared gate, groups); one launch for up to 16 bf16 tokens."""
     T, d = h.shape
     E = router.shape[0]
-    if native_dt(h, router, shared_gate) == 1 and T <= 16 and d % 8 == 0:
+    if native_dt(h, router, shared_gate) == 1 and T <= 16 and top <= 64 and d % 8 == 0:
         g = _groups(T, top, E, mt, h.device)
         ids = torch.empty(T, top, device=h.device, dtype=torch.int32)
         w = torch.empty(T, top, device=h.device, dtype=torch.float32)
