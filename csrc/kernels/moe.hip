@@ -93,7 +93,8 @@ struct GroupArgs {
 };
 
 // n assignments -> perm (sorted position -> assignment), inv (assignment -> sorted position), tiles
-// [ntiles][3] (expert, first sorted position, rows <= mt) and their count. One workgroup of NT threads;
+// [ntiles][5] (expert, first sorted position, rows <= mt, first tile and tile count of the expert) and
+// their count. One workgroup of NT threads;
 // sh: 3 E + 2 ints.
 template <int NT>
 __device__ __forceinline__ void group_rows(const GroupArgs& p, int* sh) {
@@ -123,10 +124,12 @@ __device__ __forceinline__ void group_rows(const GroupArgs& p, int* sh) {
   for (int e = tid; e < E; e += NT) {
     const int c = cnt[e];
     for (int j = 0; j * mt < c; ++j) {
-      int* t = p.tiles + (toff[e] + j) * 3;
+      int* t = p.tiles + (toff[e] + j) * 5;
       t[0] = e;
       t[1] = off[e] + j * mt;
       t[2] = min(mt, c - j * mt);
+      t[3] = toff[e];
+      t[4] = (c + mt - 1) / mt;
     }
     cnt[e] = off[e];
   }
@@ -231,7 +234,7 @@ __global__ void __launch_bounds__(256) expert_gemv_kernel(ExpertArgs p) {
   E* xs = reinterpret_cast<E*>(raw);  // [MT][KC]
   if ((int)blockIdx.y >= *p.ntiles) return;
   const int tid = threadIdx.x, lane = tid & 63, wv = tid >> 6;
-  const int* tl = p.tiles + blockIdx.y * 3;
+  const int* tl = p.tiles + blockIdx.y * 5;
   const int ex = tl[0], lo = tl[1], nr = tl[2], K = p.K;
   const int n0 = p.up ? blockIdx.x * 4 + wv : (blockIdx.x * 4 + wv) * 2;
   const int rows = p.up ? 2 * p.N : p.N;
@@ -332,17 +335,16 @@ __global__ void __launch_bounds__(512, 2) expert_gemm_kernel(ExpertArgs p) {
   constexpr int BK = GBK;
   extern __shared__ __attribute__((aligned(16))) bf16_t gl[];  // [2][GN + GM][BK]: weight rows, then activation rows
   bf16_t *const sw[2] = {gl, gl + (GN + GM) * BK}, *const sx[2] = {gl + GN * BK, gl + (2 * GN + GM) * BK};
-  // order: an XCD works a contiguous run of (group of TG row tiles, weight block, row tile), so the weight
-  // rows that row tiles of one expert share, and the activations its weight blocks share, meet in one L2
-  constexpr int TG = 4;
+  // order: an XCD works a contiguous run of (expert, weight block, row tile), so the row tiles that share a
+  // weight block are on one XCD at one time
   const int nt = *p.ntiles, nb = (p.N + (UP ? 127 : 255)) / (UP ? 128 : 256);
   if ((int)blockIdx.x >= nt * nb) return;
   const int id = xcd_remap(blockIdx.x, nt * nb);
-  const int grp = id / (TG * nb), gt = min(TG, nt - grp * TG), in = id - grp * TG * nb;
-  const int tile = grp * TG + in % gt, bn = in / gt;
+  const int* t0 = p.tiles + id / nb * 5;
+  const int in = id - t0[3] * nb, tile = t0[3] + in % t0[4], bn = in / t0[4];
   const int tid = threadIdx.x, lane = tid & 63, wv = tid >> 6, l32 = lane & 31, hh = lane >> 5;
   const int wn = wv >> 1, wm = wv & 1;
-  const int* tl = p.tiles + tile * 3;
+  const int* tl = p.tiles + tile * 5;
   const int ex = tl[0], lo = tl[1], nr = tl[2], K = p.K, N = p.N;
   const int n0 = bn * (UP ? 128 : 256);
   // staging: thread tid owns 16-B chunk tid % 8 of rows tid / 8 + 64 i
@@ -373,7 +375,7 @@ __global__ void __launch_bounds__(512, 2) expert_gemm_kernel(ExpertArgs p) {
 #pragma unroll
     for (int i = 0; i < 2; ++i) rx[i] = *reinterpret_cast<const u32x4*>(xp[i] + k);
   };
-  const int so = sr * BK + ((ch ^ (sr & 7)) << 3);
+  const int so = sr * BK + ((ch ^ ((sr >> 1) & 7)) << 3);  // 16 rows x one chunk, or 2 x 8: all 64 banks
   auto store = [&](int t, int b, const u32x4 (&rw)[4], const u32x4 (&rx)[2]) {
     const uint32_t keep = t * BK + ch * 8 < K ? ~0u : 0u;
 #pragma unroll
@@ -406,8 +408,8 @@ __global__ void __launch_bounds__(512, 2) expert_gemm_kernel(ExpertArgs p) {
       auto frag = [&](int s, int f) {
 #pragma unroll
         for (int i = 0; i < 2; ++i) {
-          a[f][i] = *reinterpret_cast<const bf16x8*>(sw[b] + ar[i] * BK + (((2 * s + hh) ^ (ar[i] & 7)) << 3));
-          x[f][i] = *reinterpret_cast<const bf16x8*>(sx[b] + br[i] * BK + (((2 * s + hh) ^ (br[i] & 7)) << 3));
+          a[f][i] = *reinterpret_cast<const bf16x8*>(sw[b] + ar[i] * BK + (((2 * s + hh) ^ ((ar[i] >> 1) & 7)) << 3));
+          x[f][i] = *reinterpret_cast<const bf16x8*>(sx[b] + br[i] * BK + (((2 * s + hh) ^ ((br[i] >> 1) & 7)) << 3));
         }
       };
       frag(0, 0);
@@ -517,7 +519,7 @@ static bool group_ok(const GroupArgs& g, int max_tiles) {
          max_tiles >= (g.E < g.n ? g.E : g.n) + g.n / g.mt;
 }
 
-// tiles: [max_tiles][3] with max_tiles >= min(E, n) + n / mt
+// tiles: [max_tiles][5] with max_tiles >= min(E, n) + n / mt
 KCA_API int kca_moe_group(const void* ids, int n, int E, int mt, void* perm, void* inv, void* tiles, int max_tiles,
                           void* ntiles, hipStream_t s) {
   const GroupArgs g{(const int*)ids, n, E, mt, (int*)perm, (int*)inv, (int*)tiles, (int*)ntiles};

@@ -58,7 +58,7 @@ def tile_rows(T: int, top: int, E: int, d: int, F: int, dtype) -> int:
 def _groups(T: int, top: int, E: int, mt: int, device) -> Groups:
     n = T * top
     z = dict(device=device, dtype=torch.int32)
-    return Groups(torch.empty(n, **z), torch.empty(T, top, **z), torch.empty(min(E, n) + n // mt, 3, **z),
+    return Groups(torch.empty(n, **z), torch.empty(T, top, **z), torch.empty(min(E, n) + n // mt, 5, **z),
                   torch.empty(1, **z), mt)
 
 
