@@ -42,6 +42,9 @@ the headline always prints):
                             req/s, p50/p99, tokens/s at concurrency 1/8/32, and
                             the same requests without the HTTP layer.
 
+``--megusun`` runs none of this: it prints one line with Megusun's prefill / decode throughput beside
+GPT-J of equal size and each kernel's distance from its roofline (bench/megusun_bench.py).
+
 ``KCA_BENCH_SHARED_GPU=1`` (rehearsal only, parallel/shared_gpu.py): N ranks
 share cuda:0 with gloo collectives staged through the host, so the N > 1 paths
 run on a one-GPU box; pair it with ``--layers/--hidden`` shrink flags, which
@@ -93,6 +96,9 @@ def main():
                          "'auto' = when N == 1")
     ap.add_argument("--extra-timeout", type=float, default=600.0,
                     help="seconds for all N=1 secondaries together; on overrun the line prints with what finished")
+    ap.add_argument("--megusun", choices=["models", "kernels", "all"], default=None,
+                    help="instead of the headline: Megusun prefill / decode throughput beside GPT-J of equal size "
+                         "('models') and kernel rooflines ('kernels'), random weights, one GPU (bench/megusun_bench.py)")
     # rehearsal shrink flags (tests/test_bench_shared_gpu.py): NOT the BASELINE config
     ap.add_argument("--layers", type=int, default=0)
     ap.add_argument("--hidden", type=int, default=0)
@@ -109,6 +115,16 @@ def main():
     if os.environ.get("KCA_BENCH_DRYRUN") == "1":  # CPU test of the launch contract (tests/test_launch_cpu.py)
         print(f"[bench] dryrun rank {os.environ.get('RANK', '0')} "
               + json.dumps({"world_size": int(os.environ.get("WORLD_SIZE", "1"))}), flush=True)
+        return
+
+    if args.megusun:
+        mb = _load_bench("megusun_bench")
+        rec = {"bench": "megusun", "dtype": "bf16", "data": "synthetic"}
+        if args.megusun != "kernels":
+            rec["models"] = mb.run_models()
+        if args.megusun != "models":
+            rec["kernels"] = mb.run_kernels()
+        print(json.dumps(rec), flush=True)
         return
 
     import torch

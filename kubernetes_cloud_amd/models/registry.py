@@ -68,9 +68,17 @@ def family_of(cfg) -> Family:
     return _causal_lm()
 
 
+def require_causal_lm(cfg, what: str):
+    """``cfg`` if it is an HF family's ``LMConfig``; the paths that handle those alone name the limit."""
+    from .config import LMConfig
+    if not isinstance(cfg, LMConfig):
+        raise NotImplementedError(f"{what} supports the HF causal-LM families, not {cfg.arch} (which serves on one GPU)")
+    return cfg
+
+
 def read_dict(path: str) -> dict:
     with open(os.path.join(path, "config.json")) as f:
         return json.load(f)
 
 
-__all__ = ["Family", "FAMILIES", "family_of", "family_of_dict", "read_dict"]
+__all__ = ["Family", "FAMILIES", "family_of", "family_of_dict", "read_dict", "require_causal_lm"]

@@ -128,7 +128,8 @@ def load_layer_split(path: str, max_memory, dtype: torch.dtype = torch.bfloat16,
     from ..models.config import LMConfig
     from ..models.hf_convert import hf_to_native_plan, prefixed_getter
     from .tensor_parallel import _LazySafetensors
-    cfg = LMConfig.from_pretrained(path)
+    from ..models.registry import require_causal_lm
+    cfg = require_causal_lm(LMConfig.from_pretrained(path), "layer splitting")
     with torch.device("meta"):
         m = CausalLM(cfg)
     m = m.to(dtype)

@@ -310,7 +310,8 @@ def load_tp_model(path: str, rank: int, world: int, group=None, device=None, dty
     from ..models.causal_lm import CausalLM, alibi_slopes
     from ..models.config import LMConfig
     from ..models.hf_convert import hf_to_native_plan, prefixed_getter
-    cfg = LMConfig.from_pretrained(path) if isinstance(path, str) else path
+    from ..models.registry import require_causal_lm
+    cfg = require_causal_lm(LMConfig.from_pretrained(path) if isinstance(path, str) else path, "tensor parallelism")
     with torch.device("meta"):
         m = CausalLM(cfg)
     tp_convert_(m, rank, world, group)

@@ -205,6 +205,8 @@ def main(argv=None):
         cfg = LMConfig.from_hf(metadata(tz_uri)["config"])
     else:
         cfg = LMConfig.from_pretrained(args.model)
+    from ..models.registry import require_causal_lm
+    require_causal_lm(cfg, "finetuning")
     eos_id = tokenizer.eos_token_id if tokenizer is not None else cfg.eos_token_id
     pad_id = tokenizer.pad_token_id if tokenizer is not None else (cfg.pad_token_id if cfg.pad_token_id is not None else eos_id)
 

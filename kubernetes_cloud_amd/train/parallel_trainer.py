@@ -124,6 +124,8 @@ def build_model_shard(args, topo: Topology, device, dtype):
     from ..models.causal_lm import CausalLM, alibi_slopes
     from ..models.config import LMConfig, preset
     cfg = preset(args.model) if args.random_init else LMConfig.from_pretrained(args.model)
+    from ..models.registry import require_causal_lm
+    require_causal_lm(cfg, "training")
     if args.layers:
         cfg.n_layers = args.layers
     if cfg.tie_embeddings and topo.tp > 1 and topo.pp > 1:

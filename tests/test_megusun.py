@@ -637,6 +637,15 @@ def test_checkpoint_round_trip(tmp_path):
         LMConfig.from_hf(config(16, 20, [({"type": "rnn", "mixer": {}}, None)]))
 
 
+def test_paths_for_other_families_name_the_limit(tmp_path):
+    from kubernetes_cloud_amd.parallel.tensor_parallel import load_tp_model
+    path = write_dir(tmp_path / "m", CFGS["odd"], mo.random_weights(CFGS["odd"], 3))
+    with pytest.raises(NotImplementedError, match="tensor parallelism.*megusun"):
+        load_tp_model(path, 0, 1)
+    with pytest.raises(TypeError, match="bf16 or fp32"):
+        runner_of(build_model(LMConfig.from_hf(CFGS["odd"]), dtype=torch.float16))
+
+
 def test_tensorized_round_trip(tmp_path):
     from kubernetes_cloud_amd.io.hf import load_tensorized, serialize_causal_lm
     cfg = CFGS["grouped"]
