@@ -30,6 +30,7 @@ from ..ops.gemv import skinny_linear
 from ..ops.rms_shift import Branch, rms_shift
 from .runner import KVCache, SlotState, StepRunner
 
+SPLIT_CLOSE = (1024, 4096)  # rows between which the closing product runs as two (HybridRunner._close)
 SKINNY_M = 16   # rows up to which projections stream on the skinny matrix-core kernel
 
 
@@ -120,6 +121,15 @@ class HybridRunner(StepRunner):
             return mix, None
         return mix, self._linear(h, w2)
 
+    def _close(self, cat, w, cols: int):
+        """The layer's closing product [mixer | ff] W_out^T. A mid-sized prompt's long K falls to a library
+        kernel at half speed (2048 x 20480 x 4096: 440 us as one product, 283 us as two), so those accumulate
+        the two column blocks in turn."""
+        if cat.is_cuda and SPLIT_CLOSE[0] <= cat.shape[0] < SPLIT_CLOSE[1] and cat.dtype == torch.bfloat16 \
+                and 0 < cols < cat.shape[1] and cols % 8 == 0 and cat.shape[1] % 8 == 0:
+            return F.linear(cat[:, :cols], w[:, :cols]).addmm_(cat[:, cols:], w[:, cols:].t())
+        return self._linear(cat, w)
+
     # ------------------------------------------------------------------ step
     def _forward(self, b: _Batch, want: torch.Tensor | None, layers_out: list | None = None) -> torch.Tensor:
         """Logits of the rows in ``want`` (None: every row)."""
@@ -153,7 +163,7 @@ class HybridRunner(StepRunner):
                 y, inv = moe.experts(h, ids, wts, L.gate_up, L.down, g, mlp.scale_in), g.inv
                 if up is not None:
                     moe.act_rows(up, cat[:, cols:], gated=True, row_scale=sg)
-            branch = Branch(self._linear(cat, L.w_out), y, inv)
+            branch = Branch(self._close(cat, L.w_out, cols), y, inv)
         if layers_out is not None:
             layers_out.append(rms_shift(x, branch, cfg.residual_mult, m.final_norm, cfg.norm_eps)[0])
         _, h, _ = rms_shift(x, branch, cfg.residual_mult, m.final_norm, cfg.norm_eps, rows=want, keep_x=False)

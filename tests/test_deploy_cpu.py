@@ -49,7 +49,7 @@ def _ref_params(path):
     return out
 
 
-@pytest.mark.skipif(not os.path.isdir(REF), reason="reference tree not mounted")
+@pytest.mark.skipif(not os.path.isdir(REF) or not os.listdir(REF), reason="reference tree not mounted")
 @pytest.mark.parametrize("ref,ours", [
     ("finetuner-workflow/finetune-workflow.yaml", workflows.FINETUNE_PARAMS),
     ("sd-finetuner-workflow/sd-finetune-workflow-template.yaml", workflows.SD_PARAMS),

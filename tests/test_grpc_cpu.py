@@ -39,7 +39,9 @@ def _sample_request(prompt_ids, out_len=8):
     if os.path.exists(SAMPLE):
         fields = json.load(open(SAMPLE))["request"]
     else:
-        fields = [{"name": "request_output_len", "data": [[64]], "dtype": "int32"},
+        fields = [{"name": "input_ids", "data": [[0]], "dtype": "uint32"},
+                  {"name": "input_lengths", "data": [[0]], "dtype": "uint32"},
+                  {"name": "request_output_len", "data": [[64]], "dtype": "int32"},
                   {"name": "runtime_top_k", "data": [[10]], "dtype": "int32"},
                   {"name": "random_seed", "data": [[0]], "dtype": "uint64"}]
     req = pb.ModelInferRequest(model_name="fastertransformer", id="r1")
@@ -53,9 +55,9 @@ def _sample_request(prompt_ids, out_len=8):
             data = [[out_len]]
         elif f["name"] == "runtime_top_k":
             data = [[0]]  # greedy (top_k == top_p == 0) so streamed == unary
-        a = np.array(data, dtype=np.dtype({"int32": np.int32, "float32": np.float32, "uint64": np.uint64,
+        a = np.array(data, dtype=np.dtype({"int32": np.int32, "uint32": np.uint32, "float32": np.float32, "uint64": np.uint64,
                                            "bool": np.bool_}[f["dtype"]]))
-        t = req.inputs.add(name=f["name"], datatype={"int32": "INT32", "float32": "FP32", "uint64": "UINT64",
+        t = req.inputs.add(name=f["name"], datatype={"int32": "INT32", "uint32": "UINT32", "float32": "FP32", "uint64": "UINT64",
                                                       "bool": "BOOL"}[f["dtype"]])
         t.shape.extend(a.shape)
         req.raw_input_contents.append(a.tobytes())  # tritonclient's wire form
