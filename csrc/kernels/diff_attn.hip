@@ -58,23 +58,20 @@ __device__ __forceinline__ float row_scale(const DiffArgs& p, int pos) {
   return p.scale * (1.f + p.coef * logf((float)floor((double)(pos + 1) / p.every) + 1.f));
 }
 
-template <typename E>
+// V elements per access (V > 1: head sizes, rows and pools are multiples of V)
+template <typename E, int V>
 __global__ void __launch_bounds__(256) kv_append_kernel(DiffArgs p, int T) {
-  const int nk = 2 * p.G * p.dim, nv = p.G * p.vdim, n = nk + nv;
-  const int t = blockIdx.x;
-  const int ps = p.pos[t], in_page = ps & ((1 << p.shift) - 1);
-  const long long pg = p.table[(long long)p.slot[t] * p.tstride + (ps >> p.shift)];
-  const E* src = reinterpret_cast<const E*>(p.qkv) + t * p.ld + 2 * p.H * p.dim;
-  E* kd = reinterpret_cast<E*>(p.kc) + pg * p.k_sp;
-  E* vd = reinterpret_cast<E*>(p.vc) + pg * p.v_sp;
-  for (int i = threadIdx.x; i < n; i += 256) {
-    if (i < nk) {
-      const int hd = i / p.dim, c = i - hd * p.dim;
-      kd[(((long long)hd << p.shift) + in_page) * p.dim + c] = src[i];
-    } else {
-      const int j = i - nk, hd = j / p.vdim, c = j - hd * p.vdim;
-      vd[(((long long)hd << p.shift) + in_page) * p.vdim + c] = src[i];
-    }
+  struct alignas(sizeof(E) * V) Pack { E v[V]; };
+  const int nk = 2 * p.G * p.dim, n = nk + p.G * p.vdim, per = n / V;
+  for (long long i = (long long)blockIdx.x * 256 + threadIdx.x; i < (long long)T * per; i += (long long)gridDim.x * 256) {
+    const int t = (int)(i / per), e = (int)(i - (long long)t * per) * V;
+    const int ps = p.pos[t], in_page = ps & ((1 << p.shift) - 1);
+    const long long pg = p.table[(long long)p.slot[t] * p.tstride + (ps >> p.shift)];
+    const bool key = e < nk;
+    const int j = key ? e : e - nk, sz = key ? p.dim : p.vdim, hd = j / sz, c = j - hd * sz;
+    E* dst = key ? reinterpret_cast<E*>(p.kc) + pg * p.k_sp : reinterpret_cast<E*>(p.vc) + pg * p.v_sp;
+    *reinterpret_cast<Pack*>(dst + (((long long)hd << p.shift) + in_page) * sz + c) =
+        *reinterpret_cast<const Pack*>(reinterpret_cast<const E*>(p.qkv) + t * p.ld + 2 * p.H * p.dim + e);
   }
 }
 
@@ -693,9 +690,14 @@ KCA_API int kca_diff_attn_abi() { return (int)sizeof(KcaDiffAttn); }
 KCA_API int kca_diff_append(const KcaDiffAttn* in, int dtype, int T, hipStream_t s) {
   const DiffArgs& p = in->a;
   if (!args_ok(p) || !p.pos || !p.slot || T < 1) return 1;
-  if (dtype == 0) hipLaunchKernelGGL(kv_append_kernel<float>, dim3(T), dim3(256), 0, s, p, T);
-  else if (dtype == 1) hipLaunchKernelGGL(kv_append_kernel<bf16_t>, dim3(T), dim3(256), 0, s, p, T);
-  else return 3;
+  if (dtype != 0 && dtype != 1) return 3;
+  const bool vec = vec_ok(p);
+  const long long work = (long long)T * (2 * p.G * p.dim + p.G * p.vdim) / (vec ? (dtype ? 8 : 4) : 1);
+  const dim3 g(kca_grid(work, 256, 8192));
+  if (dtype == 0 && vec) hipLaunchKernelGGL((kv_append_kernel<float, 4>), g, dim3(256), 0, s, p, T);
+  else if (dtype == 0) hipLaunchKernelGGL((kv_append_kernel<float, 1>), g, dim3(256), 0, s, p, T);
+  else if (vec) hipLaunchKernelGGL((kv_append_kernel<bf16_t, 8>), g, dim3(256), 0, s, p, T);
+  else hipLaunchKernelGGL((kv_append_kernel<bf16_t, 1>), g, dim3(256), 0, s, p, T);
   return hipGetLastError() == hipSuccess ? 0 : 4;
 }
 

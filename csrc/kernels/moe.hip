@@ -171,18 +171,20 @@ __global__ void __launch_bounds__(NW * 64) route_mfma_kernel(RouteArgs p, GroupA
     for (int i = 0; i < 4; ++i) acc[i] = f32x4{0.f, 0.f, 0.f, 0.f};
     auto steps = [&](auto ntc) {
       constexpr int NTC = decltype(ntc)::value;
-#pragma unroll 4
-      for (int k = wv; k < nk; k += NW) {
-        const int c = k * 32 + g * 8;
-        const u32x4 zero = {0u, 0u, 0u, 0u};
-        const u32x4 b = c < d ? *reinterpret_cast<const u32x4*>(h + c) : zero;
+#pragma unroll 2
+      for (int k2 = wv * 2; k2 < nk; k2 += NW * 2)  // 64 columns at a time: whole cache lines of every row
 #pragma unroll
-        for (int i = 0; i < NTC; ++i) {
-          const u32x4 a = c < d ? *reinterpret_cast<const u32x4*>(w[i] + c) : zero;
-          acc[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8, a), __builtin_bit_cast(bf16x8, b),
-                                                           acc[i], 0, 0, 0);
+        for (int u = 0; u < 2; ++u) {
+          const int c = (k2 + u) * 32 + g * 8;
+          const u32x4 zero = {0u, 0u, 0u, 0u};
+          const u32x4 b = c < d ? *reinterpret_cast<const u32x4*>(h + c) : zero;
+#pragma unroll
+          for (int i = 0; i < NTC; ++i) {
+            const u32x4 a = c < d ? *reinterpret_cast<const u32x4*>(w[i] + c) : zero;
+            acc[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8, a), __builtin_bit_cast(bf16x8, b),
+                                                             acc[i], 0, 0, 0);
+          }
         }
-      }
     };
     if (nt == 1) steps(std::integral_constant<int, 1>{});
     else if (nt == 2) steps(std::integral_constant<int, 2>{});
