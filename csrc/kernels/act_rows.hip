@@ -1,6 +1,6 @@
-// Feed-forward activations over strided rows (the producer's and the consumer's buffers are column slices
-// of wider ones): y = gelu(u), exact (erf) form, or y = silu(g) * u * s with [g | u] side by side in a row
-// and an optional number s per row.
+// Activations over strided rows (the producer's and the consumer's buffers are column slices of wider ones).
+// MODE 0: y = gelu(x), exact (erf) form; 1: y = silu(g) * u * s with [g | u] side by side in a row and an
+// optional number s per row; 2: y = gelu_tanh(g) * u; 3: y = tanh(x). An optional bias per input column.
 #include "common.h"
 
 namespace {
@@ -15,9 +15,16 @@ template <> __device__ __forceinline__ bf16_t from_f<bf16_t>(float v) { return f
 template <typename E, int V>
 struct alignas(sizeof(E) * V) Pack { E v[V]; };
 
-template <typename E, int V, bool GATED>
-__global__ void __launch_bounds__(256) act_rows_kernel(const E* x, long long ldx, const float* rs, E* y, long long ldy,
-                                                       int T, int F) {
+template <typename E>
+__device__ __forceinline__ float tanh_t(float u) {
+  if constexpr (sizeof(E) == 4) return tanhf(u);
+  else return fast_tanh(u);
+}
+
+template <typename E, int V, int MODE>
+__global__ void __launch_bounds__(256) act_rows_kernel(const E* x, long long ldx, const float* rs, const E* bias, E* y,
+                                                       long long ldy, int T, int F) {
+  constexpr bool GATED = MODE == 1 || MODE == 2;
   const int per = F / V;
   const long long n = (long long)T * per;
   for (long long i = (long long)blockIdx.x * 256 + threadIdx.x; i < n; i += (long long)gridDim.x * 256) {
@@ -25,47 +32,67 @@ __global__ void __launch_bounds__(256) act_rows_kernel(const E* x, long long ldx
     const E* src = x + t * ldx + c;
     const Pack<E, V> a = *reinterpret_cast<const Pack<E, V>*>(src);
     Pack<E, V> o;
+    float g[V], u[V];
+#pragma unroll
+    for (int e = 0; e < V; ++e) g[e] = to_f<E>(a.v[e]);
     if constexpr (GATED) {
-      const Pack<E, V> u = *reinterpret_cast<const Pack<E, V>*>(src + F);
-      const float s = rs ? rs[t] : 1.f;
+      const Pack<E, V> w = *reinterpret_cast<const Pack<E, V>*>(src + F);
 #pragma unroll
-      for (int e = 0; e < V; ++e) {
-        const float g = to_f<E>(a.v[e]);
-        o.v[e] = from_f<E>(g / (1.f + (sizeof(E) == 4 ? expf(-g) : __expf(-g))) * to_f<E>(u.v[e]) * s);
-      }
-    } else {
+      for (int e = 0; e < V; ++e) u[e] = to_f<E>(w.v[e]);
+    }
+    if (bias) {
+      const Pack<E, V> b = *reinterpret_cast<const Pack<E, V>*>(bias + c);
 #pragma unroll
-      for (int e = 0; e < V; ++e) {
-        const float g = to_f<E>(a.v[e]);
-        o.v[e] = from_f<E>(0.5f * g * (1.f + erff(g * 0.70710678118654752f)));
+      for (int e = 0; e < V; ++e) g[e] += to_f<E>(b.v[e]);
+      if constexpr (GATED) {
+        const Pack<E, V> w = *reinterpret_cast<const Pack<E, V>*>(bias + F + c);
+#pragma unroll
+        for (int e = 0; e < V; ++e) u[e] += to_f<E>(w.v[e]);
       }
+    }
+    const float s = GATED && rs ? rs[t] : 1.f;
+#pragma unroll
+    for (int e = 0; e < V; ++e) {
+      float v;
+      if constexpr (MODE == 0) v = 0.5f * g[e] * (1.f + erff(g[e] * 0.70710678118654752f));
+      else if constexpr (MODE == 1) v = g[e] / (1.f + (sizeof(E) == 4 ? expf(-g[e]) : __expf(-g[e]))) * u[e] * s;
+      else if constexpr (MODE == 2)
+        v = 0.5f * g[e] * (1.f + tanh_t<E>(0.7978845608028654f * (g[e] + 0.044715f * g[e] * g[e] * g[e]))) * u[e] * s;
+      else v = tanh_t<E>(g[e]);
+      o.v[e] = from_f<E>(v);
     }
     *reinterpret_cast<Pack<E, V>*>(y + t * ldy + c) = o;
   }
 }
 
 template <typename E, int V>
-void go(int gated, const void* x, long long ldx, const void* rs, void* y, long long ldy, int T, int F, hipStream_t s) {
+void go(int mode, const void* x, long long ldx, const void* rs, const void* bias, void* y, long long ldy, int T, int F,
+        hipStream_t s) {
   const int g = kca_grid((long long)T * (F / V), 256);
-  if (gated)
-    hipLaunchKernelGGL((act_rows_kernel<E, V, true>), dim3(g), dim3(256), 0, s, (const E*)x, ldx, (const float*)rs,
-                       (E*)y, ldy, T, F);
-  else
-    hipLaunchKernelGGL((act_rows_kernel<E, V, false>), dim3(g), dim3(256), 0, s, (const E*)x, ldx, (const float*)rs,
-                       (E*)y, ldy, T, F);
+#define GO(M)                                                                                                          \
+  hipLaunchKernelGGL((act_rows_kernel<E, V, M>), dim3(g), dim3(256), 0, s, (const E*)x, ldx, (const float*)rs,         \
+                     (const E*)bias, (E*)y, ldy, T, F)
+  if (mode == 0) GO(0);
+  else if (mode == 1) GO(1);
+  else if (mode == 2) GO(2);
+  else GO(3);
+#undef GO
 }
 
 }  // namespace
 
 // dtype: 0 fp32, 1 bf16
-KCA_API int kca_act_rows(int dtype, int gated, const void* x, long long ldx, const void* rs, void* y, long long ldy,
-                         int T, int F, hipStream_t s) {
+KCA_API int kca_act_rows(int dtype, int mode, const void* x, long long ldx, const void* rs, const void* bias, void* y,
+                         long long ldy, int T, int F, hipStream_t s) {
+  if (mode < 0 || mode > 3) return 1;
+  const bool gated = mode == 1 || mode == 2;
   if (T < 1 || F < 1 || !x || !y || ldx < (gated ? 2LL : 1LL) * F || ldy < F) return 1;
   const int V = dtype == 0 ? 4 : 8;
-  const bool v = F % V == 0 && ldx % V == 0 && ldy % V == 0 && (uintptr_t)x % 16 == 0 && (uintptr_t)y % 16 == 0;
-  if (dtype == 0) v ? go<float, 4>(gated, x, ldx, rs, y, ldy, T, F, s) : go<float, 1>(gated, x, ldx, rs, y, ldy, T, F, s);
+  const bool v = F % V == 0 && ldx % V == 0 && ldy % V == 0 && (uintptr_t)x % 16 == 0 && (uintptr_t)y % 16 == 0 &&
+                 (uintptr_t)bias % 16 == 0;
+  if (dtype == 0) v ? go<float, 4>(mode, x, ldx, rs, bias, y, ldy, T, F, s) : go<float, 1>(mode, x, ldx, rs, bias, y, ldy, T, F, s);
   else if (dtype == 1)
-    v ? go<bf16_t, 8>(gated, x, ldx, rs, y, ldy, T, F, s) : go<bf16_t, 1>(gated, x, ldx, rs, y, ldy, T, F, s);
+    v ? go<bf16_t, 8>(mode, x, ldx, rs, bias, y, ldy, T, F, s) : go<bf16_t, 1>(mode, x, ldx, rs, bias, y, ldy, T, F, s);
   else return 3;
   return hipGetLastError() == hipSuccess ? 0 : 4;
 }

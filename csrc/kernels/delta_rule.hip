@@ -1,0 +1,300 @@
+// Delta-rule mixers (delta_rule.h) token by token: the decode step, and the scan of prompt portions in any
+// size or type (bf16 portions of usual head sizes run in chunks on the matrix cores: delta_chunk.hip).
+//
+//   step kernel   one token per row: projections -> vectors -> state update -> normed, gated output, one launch
+//   prep kernel   vectors of every (token, head) of a batch of portions
+//   scan kernel   an entry's tokens in order, state in registers; a wave owns 16 value columns of a head
+//   gate kernel   head norm, gain and gate of every (token, head); convolution inputs into the slots' rings
+//
+// The carried state of a sequence lives in its slot and counts as zero at position 0.
+#include "delta_rule.h"
+
+namespace {
+using namespace delta;
+
+// A wave's part of the state: CW columns from 4 column groups (lane >> 4), rows lane & 15 + 16 i.
+template <int R, int CW>
+struct Cols {
+  float s[R][CW];
+  __device__ __forceinline__ void load(const float* S, int dk, int dv, int rg, int col, bool live) {
+#pragma unroll
+    for (int i = 0; i < R; ++i) {
+      const int r = rg + 16 * i;
+#pragma unroll
+      for (int e = 0; e < CW; ++e) s[i][e] = 0.f;
+      if (live && r < dk && col < dv) {
+        const float* q = S + (long long)r * dv + col;
+        if constexpr (CW == 4) {
+          const float4 v = *reinterpret_cast<const float4*>(q);
+          s[i][0] = v.x; s[i][1] = v.y; s[i][2] = v.z; s[i][3] = v.w;
+        } else {
+          s[i][0] = *q;
+        }
+      }
+    }
+  }
+  __device__ __forceinline__ void store(float* S, int dk, int dv, int rg, int col) const {
+#pragma unroll
+    for (int i = 0; i < R; ++i) {
+      const int r = rg + 16 * i;
+      if (r < dk && col < dv) {
+        float* q = S + (long long)r * dv + col;
+        if constexpr (CW == 4) *reinterpret_cast<float4*>(q) = make_float4(s[i][0], s[i][1], s[i][2], s[i][3]);
+        else *q = s[i][0];
+      }
+    }
+  }
+  // one token: the vectors at rows rg + 16 i (zero past dk), v at the lane's columns -> read-out
+  __device__ __forceinline__ void token(const float (&w)[R], const float (&z)[R], const float (&p)[R], const float (&k)[R],
+                                        const float (&q)[R], const float (&v)[CW], float qp, float qk, float (&o)[CW]) {
+    float zs[CW], qs[CW];
+#pragma unroll
+    for (int e = 0; e < CW; ++e) zs[e] = qs[e] = 0.f;
+#pragma unroll
+    for (int i = 0; i < R; ++i) {
+      const float qw = q[i] * w[i];
+#pragma unroll
+      for (int e = 0; e < CW; ++e) {
+        zs[e] = fmaf(z[i], s[i][e], zs[e]);
+        qs[e] = fmaf(qw, s[i][e], qs[e]);
+      }
+    }
+    auto add = [](float x, float y) { return x + y; };
+#pragma unroll
+    for (int e = 0; e < CW; ++e) {
+      zs[e] = lanes_reduce<16>(zs[e], add);
+      qs[e] = lanes_reduce<16>(qs[e], add);
+      o[e] = qs[e] + qp * zs[e] + qk * v[e];  // q^T (w S + p s + k v)
+    }
+#pragma unroll
+    for (int i = 0; i < R; ++i)
+#pragma unroll
+      for (int e = 0; e < CW; ++e) s[i][e] = fmaf(w[i], s[i][e], fmaf(p[i], zs[e], k[i] * v[e]));
+  }
+};
+
+template <int R>
+__device__ __forceinline__ void rows_of(const float* src, int dk, int rg, float (&x)[R]) {
+#pragma unroll
+  for (int i = 0; i < R; ++i) x[i] = rg + 16 * i < dk ? src[rg + 16 * i] : 0.f;
+}
+
+template <typename E, int KIND, int R, int CW>
+__global__ void __launch_bounds__(1024) delta_step_kernel(DeltaArgs a) {
+  extern __shared__ float smem[];
+  const int b = blockIdx.x, h = blockIdx.y, tid = threadIdx.x, wv = tid >> 6, lane = tid & 63, nw = blockDim.x >> 6;
+  const int dk = a.dk, dv = a.dv, rg = lane & 15, cg = lane >> 4;
+  const int nblk = (dv + 4 * CW - 1) / (4 * CW);
+  float* S = a.state + ((long long)a.slot[b] * a.H + h) * dk * dv;
+  const bool live = a.pos[b] > 0;
+  Cols<R, CW> st;
+  st.load(S, dk, dv, rg, wv * 4 * CW + cg * CW, live);  // in flight while the vectors are made
+  Head hd(smem, dk, dv, a.rank_w, a.rank_g);
+  prep_head<E, KIND>(a, b, h, hd);
+  if constexpr (KIND == 1) ring_store<E>(a, b, h, tid, blockDim.x);
+  float w[R], z[R], p[R], k[R], q[R];
+  rows_of<R>(hd.w, dk, rg, w);
+  rows_of<R>(hd.z, dk, rg, z);
+  rows_of<R>(hd.p, dk, rg, p);
+  rows_of<R>(hd.k, dk, rg, k);
+  rows_of<R>(hd.q, dk, rg, q);
+  float ss = 0.f;
+  for (int cb = wv; cb < nblk; cb += nw) {
+    const int col = cb * 4 * CW + cg * CW;
+    if (cb != wv) st.load(S, dk, dv, rg, col, live);
+    float v[CW], o[CW];
+#pragma unroll
+    for (int e = 0; e < CW; ++e) v[e] = col + e < dv ? hd.v[col + e] : 0.f;
+    st.token(w, z, p, k, q, v, hd.qp, hd.qk, o);
+    st.store(S, dk, dv, rg, col);
+    if (rg == 0)
+#pragma unroll
+      for (int e = 0; e < CW; ++e)
+        if (col + e < dv) {  // (this wave alone reads and writes these columns of v)
+          hd.v[col + e] = o[e];
+          ss = fmaf(o[e], o[e], ss);
+        }
+  }
+  const float n = 1.f / sqrtf(block_sum(ss, hd.red) / (float)dv + a.eps);
+  E* out = reinterpret_cast<E*>(a.out) + (long long)b * a.ldo + h * dv;
+  const E* gain = reinterpret_cast<const E*>(a.gain) + (KIND == 0 ? h * dv : 0);
+  for (int c = tid; c < dv; c += blockDim.x) delta::st<E>(out + c, hd.v[c] * n * delta::ld<E>(gain + c) * hd.gate[c]);
+}
+
+template <typename E, int KIND>
+__global__ void __launch_bounds__(128) delta_prep_kernel(DeltaArgs a) {
+  extern __shared__ float smem[];
+  const int t = blockIdx.x, h = blockIdx.y, tid = threadIdx.x, dk = a.dk, dv = a.dv;
+  Head hd(smem, dk, dv, a.rank_w, a.rank_g);
+  prep_head<E, KIND>(a, t, h, hd);
+  float* pk = a.pk + ((long long)t * a.H + h) * pk_stride(dk, dv);
+  for (int c = tid; c < 5 * dk + dv; c += 128) pk[c] = smem[c];  // w z p k q v lie in this order
+  if (tid == 0) {
+    pk[5 * dk + dv] = hd.qp;
+    pk[5 * dk + dv + 1] = hd.qk;
+  }
+}
+
+template <int R, int CW>
+__global__ void __launch_bounds__(256) delta_scan_kernel(DeltaArgs a) {
+  const int* en = a.ent + blockIdx.x * 4;
+  const int row0 = en[0], n = en[1], pos0 = en[2], slot = en[3], h = blockIdx.y;
+  const int wv = threadIdx.x >> 6, lane = threadIdx.x & 63, rg = lane & 15, cg = lane >> 4;
+  const int dk = a.dk, dv = a.dv, col = (blockIdx.z * 4 + wv) * 4 * CW + cg * CW;
+  if ((int)(blockIdx.z * 4 + wv) * 4 * CW >= dv) return;
+  float* S = a.state + ((long long)slot * a.H + h) * dk * dv;
+  const int ps = pk_stride(dk, dv);
+  const long long step = (long long)a.H * ps;
+  const float* pk = a.pk + ((long long)row0 * a.H + h) * ps;
+  float* o = a.o + (long long)row0 * a.H * dv + h * dv + col;
+  Cols<R, CW> st;
+  st.load(S, dk, dv, rg, col, pos0 > 0);
+  float w[R], z[R], p[R], k[R], q[R], v[CW], qp, qk;
+  auto fetch = [&](const float* s) {
+    rows_of<R>(s, dk, rg, w);
+    rows_of<R>(s + dk, dk, rg, z);
+    rows_of<R>(s + 2 * dk, dk, rg, p);
+    rows_of<R>(s + 3 * dk, dk, rg, k);
+    rows_of<R>(s + 4 * dk, dk, rg, q);
+#pragma unroll
+    for (int e = 0; e < CW; ++e) v[e] = col + e < dv ? s[5 * dk + col + e] : 0.f;
+    qp = s[5 * dk + dv];
+    qk = s[5 * dk + dv + 1];
+  };
+  fetch(pk);
+  for (int t = 0; t < n; ++t) {
+    float wn[R], zn[R], pn[R], kn[R], qn[R], vn[CW];
+    const float qpn = qp, qkn = qk;
+#pragma unroll
+    for (int i = 0; i < R; ++i) wn[i] = w[i], zn[i] = z[i], pn[i] = p[i], kn[i] = k[i], qn[i] = q[i];
+#pragma unroll
+    for (int e = 0; e < CW; ++e) vn[e] = v[e];
+    pk += step;
+    if (t + 1 < n) fetch(pk);  // the next token's loads fly under this one's products
+    float y[CW];
+    st.token(wn, zn, pn, kn, qn, vn, qpn, qkn, y);
+    if (rg == 0)
+#pragma unroll
+      for (int e = 0; e < CW; ++e)
+        if (col + e < dv) o[e] = y[e];
+    o += (long long)a.H * dv;
+  }
+  st.store(S, dk, dv, rg, col);
+}
+
+// a wave per (token, head)
+template <typename E, int KIND>
+__global__ void __launch_bounds__(256) delta_gate_kernel(DeltaArgs a, int T) {
+  const long long i = (long long)blockIdx.x * 4 + (threadIdx.x >> 6);
+  if (i >= (long long)T * a.H) return;
+  const int t = (int)(i / a.H), h = (int)(i - (long long)t * a.H), lane = threadIdx.x & 63, dv = a.dv;
+  const float* o = a.o + ((long long)t * a.H + h) * dv;
+  float ss = 0.f;
+  for (int c = lane; c < dv; c += 64) ss = fmaf(o[c], o[c], ss);
+  const float n = 1.f / sqrtf(wave_sum(ss) / (float)dv + a.eps);
+  const E* gain = reinterpret_cast<const E*>(a.gain) + (KIND == 0 ? h * dv : 0);
+  const E* gt = KIND == 0 ? reinterpret_cast<const E*>(a.x) + (long long)t * a.ld + a.o_g + h * dv
+                          : reinterpret_cast<const E*>(a.dg) + (long long)t * a.ldg + h * dv;
+  E* out = reinterpret_cast<E*>(a.out) + (long long)t * a.ldo + h * dv;
+  for (int c = lane; c < dv; c += 64) delta::st<E>(out + c, o[c] * n * delta::ld<E>(gain + c) * sigmoid(delta::ld<E>(gt + c)));
+  if constexpr (KIND == 1)
+    if (a.e1[t] - t <= a.taps) ring_store<E>(a, t, h, lane, 64);
+}
+
+int rows_r(int dk) {  // rows a lane holds: 16 row groups
+  const int n = (dk + 15) / 16;
+  return n <= 1 ? 1 : n <= 2 ? 2 : n <= 3 ? 3 : n <= 4 ? 4 : n <= 6 ? 6 : n <= 8 ? 8 : n <= 12 ? 12 : 16;
+}
+
+#define DELTA_R(F)                  \
+  switch (rows_r(a.dk)) {           \
+    case 1: return F(1);            \
+    case 2: return F(2);            \
+    case 3: return F(3);            \
+    case 4: return F(4);            \
+    case 6: return F(6);            \
+    case 8: return F(8);            \
+    case 12: return F(12);          \
+    default: return F(16);          \
+  }
+
+bool wide(const DeltaArgs& a) { return a.dv % 4 == 0 && (uintptr_t)a.state % 16 == 0; }
+
+template <typename E, int KIND, int R, int CW>
+int step_go(const DeltaArgs& a, int B, hipStream_t s) {
+  int nw = (a.dv + 4 * CW - 1) / (4 * CW);
+  nw = nw < 4 ? 4 : nw > 16 ? 16 : nw;
+  const size_t lds = (size_t)prep_floats(a.dk, a.dv, a.rank_w, a.rank_g) * 4;
+  if (lds > 64 * 1024) return 10;
+  hipLaunchKernelGGL((delta_step_kernel<E, KIND, R, CW>), dim3(B, a.H), dim3(64 * nw), lds, s, a);
+  return hipGetLastError() == hipSuccess ? 0 : 4;
+}
+template <typename E, int KIND>
+int step_r(const DeltaArgs& a, int B, hipStream_t s) {
+#define F(R) (wide(a) ? step_go<E, KIND, R, 4>(a, B, s) : step_go<E, KIND, R, 1>(a, B, s))
+  DELTA_R(F)
+#undef F
+}
+
+template <int R, int CW>
+int scan_go(const DeltaArgs& a, int nent, hipStream_t s) {
+  const int nblk = (a.dv + 4 * CW - 1) / (4 * CW);
+  hipLaunchKernelGGL((delta_scan_kernel<R, CW>), dim3(nent, a.H, (nblk + 3) / 4), dim3(256), 0, s, a);
+  return hipGetLastError() == hipSuccess ? 0 : 4;
+}
+int scan_r(const DeltaArgs& a, int nent, hipStream_t s) {
+#define F(R) (wide(a) ? scan_go<R, 4>(a, nent, s) : scan_go<R, 1>(a, nent, s))
+  DELTA_R(F)
+#undef F
+}
+
+template <typename E, int KIND>
+int prep_go(const DeltaArgs& a, int T, hipStream_t s) {
+  const size_t lds = (size_t)prep_floats(a.dk, a.dv, a.rank_w, a.rank_g) * 4;
+  if (lds > 64 * 1024) return 10;
+  hipLaunchKernelGGL((delta_prep_kernel<E, KIND>), dim3(T, a.H), dim3(128), lds, s, a);
+  return hipGetLastError() == hipSuccess ? 0 : 4;
+}
+template <typename E, int KIND>
+int gate_go(const DeltaArgs& a, int T, hipStream_t s) {
+  hipLaunchKernelGGL((delta_gate_kernel<E, KIND>), dim3((unsigned)(((long long)T * a.H + 3) / 4)), dim3(256), 0, s, a, T);
+  return hipGetLastError() == hipSuccess ? 0 : 4;
+}
+
+}  // namespace
+
+// Mirrored by ops/delta_rule.py
+KCA_API int kca_delta_abi() { return (int)sizeof(DeltaArgs); }
+
+#define DELTA_DISPATCH(FN, N)                                                                 \
+  if (dtype == 0) return kind == 0 ? FN<float, 0>(a, N, s) : FN<float, 1>(a, N, s);           \
+  if (dtype == 1) return kind == 0 ? FN<bf16_t, 0>(a, N, s) : FN<bf16_t, 1>(a, N, s);         \
+  return 3;
+
+// one token per row
+KCA_API int kca_delta_step(const DeltaArgs* in, int dtype, int kind, int B, hipStream_t s) {
+  const DeltaArgs& a = *in;
+  if (!delta_args_ok(a, kind) || B < 1 || a.H > 65535 || a.e0) return 1;
+  DELTA_DISPATCH(step_r, B)
+}
+
+// a.pk of every (token, head)
+KCA_API int kca_delta_prep(const DeltaArgs* in, int dtype, int kind, int T, hipStream_t s) {
+  const DeltaArgs& a = *in;
+  if (!delta_args_ok(a, kind) || T < 1 || a.H > 65535 || !a.pk || !a.e0 || !a.e1) return 1;
+  DELTA_DISPATCH(prep_go, T)
+}
+
+// a.o of nent entries from a.pk; the slots' states advance
+KCA_API int kca_delta_scan(const DeltaArgs* in, int nent, hipStream_t s) {
+  const DeltaArgs& a = *in;
+  if (nent < 1 || !a.pk || !a.o || !a.ent || !a.state || a.H < 1 || a.H > 65535 || a.dk < 1 || a.dk > 256 || a.dv < 1) return 1;
+  return scan_r(a, nent, s);
+}
+
+// a.out of every (token, head) from a.o
+KCA_API int kca_delta_gate(const DeltaArgs* in, int dtype, int kind, int T, hipStream_t s) {
+  const DeltaArgs& a = *in;
+  if (!delta_args_ok(a, kind) || T < 1 || !a.o || !a.e0 || !a.e1 || (kind == 1 && !a.dg)) return 1;
+  DELTA_DISPATCH(gate_go, T)
+}

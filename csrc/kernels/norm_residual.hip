@@ -1,0 +1,213 @@
+// Sandwich norms around a sublayer, in one pass over the residual stream. Per token t:
+//   x_t = x_in_t (or the embedding row of its token) + ls * N(a_t + b; gb)
+//   h_t = N(x_t; g)
+// N(v; g) is a layer norm (v - mean) / sqrt(var + eps) * g or an RMS norm v / sqrt(mean v^2 + eps) * g.
+// a: the sublayer's output rows, b its bias (optional), ls a per-coordinate scale. The stream x is fp32 and
+// double buffered; statistics are two-pass fp32 over registers; h is rounded once.
+#include "common.h"
+
+namespace {
+
+struct NormArgs {
+  const float* x_in;
+  const void* embed;          // x_in null: embedding rows
+  const long long* tokens;
+  const void* a;              // sublayer output (nullable)
+  long long lda;
+  const void* bias;           // [d] (nullable)
+  const void* gb;             // [d] gain of the output norm
+  const void* ls;             // [d] layer scale (nullable: 1)
+  const void* g;              // [d] gain of the next norm
+  float eps;
+  const int* rows;            // output row i reads token rows[i] (nullable)
+  float* x_out;               // nullable
+  void* h;                    // nullable
+  int T, d, layer;            // layer: 1 layer norm, 0 RMS norm
+};
+
+template <typename E> __device__ __forceinline__ float ldf(const E* p);
+template <> __device__ __forceinline__ float ldf<float>(const float* p) { return *p; }
+template <> __device__ __forceinline__ float ldf<bf16_t>(const bf16_t* p) { return bf2f(*p); }
+
+template <typename E, int VEC>
+__device__ __forceinline__ void ldv(const E* p, float (&v)[VEC]) {
+  if constexpr (VEC == 4 && sizeof(E) == 4) {
+    const float4 q = *reinterpret_cast<const float4*>(p);
+    v[0] = q.x; v[1] = q.y; v[2] = q.z; v[3] = q.w;
+  } else if constexpr (VEC == 4) {
+    const U16x4 q = *reinterpret_cast<const U16x4*>(p);
+#pragma unroll
+    for (int i = 0; i < 4; ++i) v[i] = bf2f(q.v[i]);
+  } else {
+#pragma unroll
+    for (int i = 0; i < VEC; ++i) v[i] = ldf<E>(p + i);
+  }
+}
+template <int VEC>
+__device__ __forceinline__ void stv(float* p, const float (&v)[VEC]) {
+  if constexpr (VEC == 4) *reinterpret_cast<float4*>(p) = make_float4(v[0], v[1], v[2], v[3]);
+  else
+#pragma unroll
+    for (int i = 0; i < VEC; ++i) p[i] = v[i];
+}
+template <int VEC>
+__device__ __forceinline__ void stv(bf16_t* p, const float (&v)[VEC]) {
+  if constexpr (VEC == 4)
+    *reinterpret_cast<uint2*>(p) = make_uint2(pack_bf16x2(v[0], v[1]), pack_bf16x2(v[2], v[3]));
+  else
+#pragma unroll
+    for (int i = 0; i < VEC; ++i) p[i] = f2bf(v[i]);
+}
+
+// sum over the NT threads of a row; `red` holds NT / 64 floats of this reduction alone (no barrier before
+// the writes is needed as every reduction of a row has its own)
+template <int NT>
+__device__ __forceinline__ float row_sum(float v, float* red) {
+  v = wave_sum(v);
+  if constexpr (NT == 64) return v;
+  if ((threadIdx.x & 63) == 0) red[threadIdx.x >> 6] = v;
+  __syncthreads();
+  float t = 0.f;
+#pragma unroll
+  for (int i = 0; i < NT / 64; ++i) t += red[i];
+  return t;
+}
+
+template <typename E, int VEC, int NCH, int NT>
+__global__ void __launch_bounds__(256) norm_residual_kernel(NormArgs p) {
+  constexpr int RPB = 256 / NT;  // rows of a workgroup (one wave each when NT == 64)
+  static_assert(RPB == 1 || NT == 64, "a row is a wave or the workgroup");
+  __shared__ float red[4][NT / 64];
+  const int tid = threadIdx.x % NT, d = p.d;
+  const int r = blockIdx.x * RPB + threadIdx.x / NT;
+  if (r >= p.T) return;  // (whole waves; RPB == 1: never)
+  const int t = p.rows ? p.rows[r] : r;
+  const float inv = 1.f / (float)d;
+  float x[NCH][VEC], v[NCH][VEC];
+  const E* a = reinterpret_cast<const E*>(p.a);
+  const long long tok = p.x_in ? 0 : p.tokens[t];
+#pragma unroll
+  for (int c = 0; c < NCH; ++c) {
+    const int i = (c * NT + tid) * VEC;
+    if (i < d) {
+      if (p.x_in) ldv<float, VEC>(p.x_in + (long long)t * d + i, x[c]);
+      else ldv<E, VEC>(reinterpret_cast<const E*>(p.embed) + tok * d + i, x[c]);
+      if (a) ldv<E, VEC>(a + (long long)t * p.lda + i, v[c]);
+    } else {
+#pragma unroll
+      for (int e = 0; e < VEC; ++e) x[c][e] = 0.f;
+    }
+  }
+  auto stats = [&](float (&q)[NCH][VEC], float* r0, float* r1, float& mean, float& rstd) {
+    mean = 0.f;
+    if (p.layer) {
+      float s = 0.f;
+#pragma unroll
+      for (int c = 0; c < NCH; ++c)
+#pragma unroll
+        for (int e = 0; e < VEC; ++e) s += (c * NT + tid) * VEC < d ? q[c][e] : 0.f;
+      mean = row_sum<NT>(s, r0) * inv;
+    }
+    float ss = 0.f;
+#pragma unroll
+    for (int c = 0; c < NCH; ++c)
+#pragma unroll
+      for (int e = 0; e < VEC; ++e) {
+        const float y = (c * NT + tid) * VEC < d ? q[c][e] - mean : 0.f;
+        ss = fmaf(y, y, ss);
+      }
+    rstd = 1.f / sqrtf(row_sum<NT>(ss, r1) * inv + p.eps);
+  };
+  if (a) {
+    if (p.bias) {
+#pragma unroll
+      for (int c = 0; c < NCH; ++c) {
+        const int i = (c * NT + tid) * VEC;
+        if (i >= d) continue;
+        float b[VEC];
+        ldv<E, VEC>(reinterpret_cast<const E*>(p.bias) + i, b);
+#pragma unroll
+        for (int e = 0; e < VEC; ++e) v[c][e] += b[e];
+      }
+    }
+    float mean, rstd;
+    stats(v, red[0], red[1], mean, rstd);
+#pragma unroll
+    for (int c = 0; c < NCH; ++c) {
+      const int i = (c * NT + tid) * VEC;
+      if (i >= d) continue;
+      float g[VEC], s[VEC];
+      ldv<E, VEC>(reinterpret_cast<const E*>(p.gb) + i, g);
+      if (p.ls) ldv<E, VEC>(reinterpret_cast<const E*>(p.ls) + i, s);
+#pragma unroll
+      for (int e = 0; e < VEC; ++e) {
+        const float n = (v[c][e] - mean) * rstd * g[e];
+        x[c][e] = p.ls ? fmaf(s[e], n, x[c][e]) : x[c][e] + n;
+      }
+    }
+  }
+  if (p.x_out) {
+#pragma unroll
+    for (int c = 0; c < NCH; ++c) {
+      const int i = (c * NT + tid) * VEC;
+      if (i < d) stv<VEC>(p.x_out + (long long)r * d + i, x[c]);
+    }
+  }
+  if (!p.h) return;
+  float mean, rstd;
+  stats(x, red[2], red[3], mean, rstd);
+#pragma unroll
+  for (int c = 0; c < NCH; ++c) {
+    const int i = (c * NT + tid) * VEC;
+    if (i >= d) continue;
+    float g[VEC];
+    ldv<E, VEC>(reinterpret_cast<const E*>(p.g) + i, g);
+#pragma unroll
+    for (int e = 0; e < VEC; ++e) g[e] = (x[c][e] - mean) * rstd * g[e];
+    stv<VEC>(reinterpret_cast<E*>(p.h) + (long long)r * d + i, g);
+  }
+}
+
+template <typename E>
+int launch(const NormArgs& a, hipStream_t s) {
+  const bool v4 = a.d % 4 == 0 && a.lda % 4 == 0;
+#define GO(V, N, NT)                                                                                               \
+  hipLaunchKernelGGL((norm_residual_kernel<E, V, N, NT>), dim3((a.T + 256 / NT - 1) / (256 / NT)), dim3(256), 0, s, a)
+  if (v4 && a.T >= 512 && a.d <= 1024) {  // many short rows: a wave each, no barriers
+    if (a.d <= 256) GO(4, 1, 64);
+    else if (a.d <= 512) GO(4, 2, 64);
+    else GO(4, 4, 64);
+  } else if (v4) {
+    const int n = (a.d + 1023) / 1024;
+    if (n <= 1) GO(4, 1, 256);
+    else if (n <= 2) GO(4, 2, 256);
+    else if (n <= 4) GO(4, 4, 256);
+    else if (n <= 8) GO(4, 8, 256);
+    else if (n <= 16) GO(4, 16, 256);
+    else return 10;
+  } else {
+    const int n = (a.d + 255) / 256;
+    if (n <= 1) GO(1, 1, 256);
+    else if (n <= 4) GO(1, 4, 256);
+    else if (n <= 16) GO(1, 16, 256);
+    else return 10;
+  }
+#undef GO
+  return hipGetLastError() == hipSuccess ? 0 : 4;
+}
+
+}  // namespace
+
+// dtype: 0 fp32, 1 bf16 (of embed, a, bias, gains, ls, h)
+KCA_API int kca_norm_residual(int dtype, const void* x_in, const void* embed, const void* tokens, const void* a,
+                              long long lda, const void* bias, const void* gb, const void* ls, const void* g,
+                              float eps, const void* rows, void* x_out, void* h, int T, int d, int layer,
+                              hipStream_t s) {
+  if (T < 1 || d < 1 || (!x_in && (!embed || !tokens)) || (a && !gb) || (h && !g) || (!h && !x_out)) return 1;
+  if (x_in && x_in == x_out && rows) return 2;
+  const NormArgs p{(const float*)x_in, embed, (const long long*)tokens, a, lda, bias, gb, ls, g, eps, (const int*)rows,
+                   (float*)x_out, h, T, d, layer};
+  if (dtype == 0) return launch<float>(p, s);
+  if (dtype == 1) return launch<bf16_t>(p, s);
+  return 3;
+}

@@ -7,13 +7,16 @@ portion of its prompt or one decoded token.
 * ``prefill``         the engine's prompt call: the same step, without padding
 * ``decode_async``    (``StepRunner``) single tokens only, captured per bucket as a HIP graph
 
-A layer is three or four launches around the vendor (or skinny matrix-core) products: residual + norm +
-token shift, the mixer's core (attention over the paged cache, or the scan), the feed-forward's activation
-or experts; mixer and feed-forward close in one product.
+A layer's token mixer is an object of ``mixers`` (attention over the paged cache, a recurrence over the slots'
+state); around it a parallel layer takes three or four launches beside the vendor (or skinny matrix-core)
+products -- residual + norm + token shift, the mixer's core, the feed-forward's activation or experts; mixer and
+feed-forward close in one product -- and a sandwich layer one norm launch per sublayer (output norm, layer scale,
+residual and the next norm together). Layers may run several times in a row (``cfg.runs``); every run has its own
+cache or state.
 
-What a sequence owns besides its KV pages lives in ``SlotState``: the last normed row of every layer (token
-shift) and the fp32 recurrent state. A batch with multi-token portions reads the carried rows from a copy
-taken at its start, because a portion's first and last rows are handled by different workgroups.
+What a sequence owns besides its KV pages lives in ``SlotState``: the last normed row of every parallel layer
+(token shift) and the recurrent states. A batch with multi-token portions reads carried rows from a copy taken at
+its start, because a portion's first and last rows are handled by different workgroups.
 """
 from __future__ import annotations
 
@@ -21,13 +24,15 @@ import numpy as np
 import torch
 import torch.nn.functional as F
 
-from ..models.hybrid_config import DiffAttentionSpec
 from ..ops import diff_attention as da
 from ..ops import gated_scan as gs
 from ..ops import moe
 from ..ops import skinny_mm as smm
+from ..ops.delta_rule import Portions
 from ..ops.gemv import skinny_linear
+from ..ops.norm_residual import NormedBranch, norm_residual
 from ..ops.rms_shift import Branch, rms_shift
+from .mixers import make_mixer
 from .runner import KVCache, SlotState, StepRunner
 
 SPLIT_CLOSE = (1024, 4096)  # rows between which the closing product runs as two (HybridRunner._close)
@@ -41,7 +46,7 @@ class _Batch:
         self.tokens, self.pos, self.slots, self.max_kv = tokens, pos, slots, max_kv
         self.T = tokens.shape[0]
         self.single = True
-        self.flags = self.entry = self.tiles = self.row_of = self.rows_all = self.chunks = self.entry_slots = None
+        self.flags = self.entry = self.tiles = self.row_of = self.portions = self.chunks = self.entry_slots = None
         self.multi = False
         self.row_kv = 0
         self.bufs = {}
@@ -61,19 +66,23 @@ class HybridRunner(StepRunner):
             raise ValueError("these layers need the paged cache (page_size >= 16)")
         if self.dtype == torch.float32 and self.device.type == "cuda":
             torch.backends.cuda.matmul.allow_tf32 = False
-        self.heads, shapes, widths = {}, [], {"shift": (cfg.n_layers, d)}
-        for i, L in enumerate(model.layers):  # layer -> its cache index / its state's name
-            if L.attention:
-                mx = L.spec.mixer
-                sp = da.DiffHeads(mx.heads, mx.kv_heads, mx.dim, mx.vdim, mx.scale, L.lam_value(), 1.0 - mx.diff,
-                                  cfg.norm_eps, mx.temp_coef, mx.temp_every)
-                self.heads[i] = (len(shapes), sp)
-                shapes.append((2 * mx.kv_heads, mx.dim, mx.kv_heads, mx.vdim))
-            else:
-                widths[f"scan{i}"] = (1, L.spec.mixer.width)
+        self.mixers, first = [], {}  # one per layer run
+        for r, i in enumerate(cfg.runs):
+            self.mixers.append(make_mixer(model.layers[i], cfg, r, self._linear, first.get(i)))
+            first.setdefault(i, self.mixers[-1])
+        shapes, widths = [], {"shift": (len(cfg.runs), d)} if cfg.block == "parallel" else {}
+        for mx in self.mixers:
+            shape = mx.cache_shape()
+            if shape is not None:
+                mx.index = len(shapes)
+                shapes.append(shape)
+            widths.update(mx.state_widths())
         self.cache = KVCache(len(shapes), max_slots, 0, self.max_len, 0, self.device, self.dtype, page_size=page_size,
                              n_pages=kv_pages, layer_shapes=shapes)
         self.state = SlotState(max_slots, widths, self.device)
+        for mx in self.mixers:
+            mx.cache, mx.state = self.cache, self.state
+        self._forward_layers = {"parallel": self._parallel, "sandwich": self._sandwich}[cfg.block]
         if self.device.type == "cuda":
             from ..utils import tunable
             tunable.ensure(tunable.DECODE_FILE)
@@ -132,29 +141,29 @@ class HybridRunner(StepRunner):
 
     # ------------------------------------------------------------------ step
     def _forward(self, b: _Batch, want: torch.Tensor | None, layers_out: list | None = None) -> torch.Tensor:
-        """Logits of the rows in ``want`` (None: every row)."""
+        """Logits of the rows in ``want`` (None: every row). ``layers_out`` collects the residual stream after
+        every layer run."""
+        return self._linear(self._forward_layers(b, want, layers_out), self.model.head)
+
+    def _parallel(self, b, want, layers_out):
+        """One norm and token shift a layer feed mixer and feed-forward side by side."""
         m, cfg = self.model, self.cfg
         T, d = b.T, cfg.hidden
         x, branch = None, None
         shift = self.state["shift"]
         carry = None if b.single else shift[:, b.entry_slots]
-        for i, L in enumerate(m.layers):
-            src = {"embed": m.wte, "tokens": b.tokens} if i == 0 else {}
+        for r, i in enumerate(cfg.runs):
+            L = m.layers[i]
+            src = {"embed": m.wte, "tokens": b.tokens} if r == 0 else {}
             x, h, hs = rms_shift(x, branch, cfg.residual_mult, L.norm, cfg.norm_eps, shift=L.shift,
-                                 prev=shift[i] if b.single else carry[i], prev_idx=b.slots if b.single else b.entry,
-                                 pos=b.pos, flags=b.flags, state=shift[i], slots=b.slots, **src)
-            if layers_out is not None and i:
+                                 prev=shift[r] if b.single else carry[r], prev_idx=b.slots if b.single else b.entry,
+                                 pos=b.pos, flags=b.flags, state=shift[r], slots=b.slots, **src)
+            if layers_out is not None and r:
                 layers_out.append(x.clone())
-            mx = L.spec.mixer
-            cols = mx.out_cols
+            cols = L.spec.mixer.out_cols
             cat = torch.empty(T, cols + L.ff_cols, device=h.device, dtype=h.dtype)
             mix, up = self._mix_and_up(L, h, hs, cat[:, cols:])
-            if L.attention:
-                self._attention(i, mix, cat[:, :cols], b)
-            elif b.single:
-                gs.gated_step(mix, L.b_z, L.b_x, self.state[f"scan{i}"][0], cat[:, :cols], b.pos, b.slots)
-            else:
-                gs.gated_scan(mix, L.b_z, L.b_x, self.state[f"scan{i}"][0], cat[:, :cols], b.chunks, b.multi)
+            self.mixers[r](mix, cat[:, :cols], b)
             y = inv = None
             if L.moe:
                 mlp = L.spec.mlp
@@ -166,24 +175,30 @@ class HybridRunner(StepRunner):
             branch = Branch(self._close(cat, L.w_out, cols), y, inv)
         if layers_out is not None:
             layers_out.append(rms_shift(x, branch, cfg.residual_mult, m.final_norm, cfg.norm_eps)[0])
-        _, h, _ = rms_shift(x, branch, cfg.residual_mult, m.final_norm, cfg.norm_eps, rows=want, keep_x=False)
-        return self._linear(h, m.head)
+        return rms_shift(x, branch, cfg.residual_mult, m.final_norm, cfg.norm_eps, rows=want, keep_x=False)[1]
 
-    def _attention(self, i, qkv, out, b: _Batch):
-        ci, sp = self.heads[i]
-        kc, vc, tbl = self.cache.k[ci], self.cache.v[ci], self.cache.table
-        a = (sp, qkv, kc, vc, tbl, b.pos, b.slots)
-        if b.single:
-            da.attend_rows(*a, out, b.max_kv, fused_append=True, ws=b.bufs.get("ws"), cnt=b.bufs.get("cnt"))
-            return
-        da.append(*a)
-        if out.is_cuda and da.tiles_ok(sp, out.dtype, self.cache.page_size, out.stride(0)):
-            if b.tiles is not None:
-                da.attend_tiles(*a, out, b.tiles)
-            if b.row_of is not None:
-                da.attend_rows(*a, out, b.row_kv, fused_append=False, row_of=b.row_of)
-        else:
-            da.attend_rows(*a, out, b.max_kv, fused_append=False)
+    def _sandwich(self, b, want, layers_out):
+        """Mixer and feed-forward in turn, each normed before and after and scaled per coordinate."""
+        m, eps, T = self.model, self.cfg.norm_eps, b.T
+        x, branch = None, None
+        src = {"embed": m.wte, "tokens": b.tokens}
+        for r, i in enumerate(self.cfg.runs):
+            L = m.layers[i]
+            x, h = norm_residual(x, branch, L.norm, eps, **src)
+            if layers_out is not None and r:
+                layers_out.append(x.clone())
+            src = {}
+            y = torch.empty(T, L.spec.mixer.out_cols, device=h.device, dtype=h.dtype)
+            self.mixers[r](self._linear(h, L.w_in), y, b)
+            branch = NormedBranch(self._linear(y, L.w_out), L.norm_b, L.scale)
+            if L.spec.mlp is not None:
+                x, h = norm_residual(x, branch, L.norm2, eps)
+                y = torch.empty(T, L.spec.mlp.ff, device=h.device, dtype=h.dtype)
+                moe.act_rows(self._linear(h, L.w_up), y, True, act="gelu_tanh_gated", bias=L.b_up)
+                branch = NormedBranch(self._linear(y, L.w_down), L.norm2_b, L.scale2, L.b_down)
+        if layers_out is not None:
+            layers_out.append(norm_residual(x, branch, None, eps, **src)[0])
+        return norm_residual(x, branch, m.final_norm, eps, rows=want, keep_x=False, **src)[1]
 
     # ------------------------------------------------------- portions + tokens
     def _plan(self, entries, want_rows) -> tuple[_Batch, torch.Tensor | None]:
@@ -207,6 +222,10 @@ class HybridRunner(StepRunner):
             parts["flags"] = fl
             parts["entry"] = np.repeat(np.arange(len(ent)), [e[1] for e in ent])
             parts["entry_slots"] = np.asarray([e[3] for e in ent])
+            parts["ent"] = np.asarray(ent).reshape(-1)
+            n_of = [e[1] for e in ent]
+            parts["e0"] = np.repeat([e[0] for e in ent], n_of)
+            parts["e1"] = np.repeat([e[0] + e[1] for e in ent], n_of)
             chunks, multi = gs.plan_chunks(ent)
             parts["chunks"] = chunks.reshape(-1)
             parts["tiles"] = da.plan_tiles([e for e in ent if e[1] > 1]).reshape(-1)
@@ -223,6 +242,7 @@ class HybridRunner(StepRunner):
         if not single:
             b.single, b.multi = False, multi
             b.flags, b.entry, b.entry_slots = dev["flags"], dev["entry"], dev["entry_slots"].long()
+            b.portions = Portions(b.pos, b.slots, dev["e0"], dev["e1"], dev["ent"].view(-1, 4))
             b.chunks = dev["chunks"].view(-1, 6)
             b.tiles = dev["tiles"].view(-1, 4) if dev["tiles"].numel() else None
             if ones:
@@ -272,12 +292,11 @@ class HybridRunner(StepRunner):
 
     # ---------------------------------------------------------------- decode
     def _step_buffers(self, Bb: int, Kb: int) -> dict:
-        wsf = cnt = 1
-        for _, sp in self.heads.values():
-            _, _, w, c = da.rows_plan(sp, Bb, Kb, self.dtype)
-            wsf, cnt = max(wsf, w), max(cnt, c)
-        return {"ws": torch.empty(wsf, device=self.device, dtype=torch.float32),
-                "cnt": torch.zeros(cnt, device=self.device, dtype=torch.int32)}
+        need = {"ws": (1, torch.float32), "cnt": (1, torch.int32)}
+        for mx in self.mixers:
+            for k, (n, dt) in mx.buffers(Bb, Kb, self.dtype).items():
+                need[k] = (max(n, need.get(k, (1, dt))[0]), dt)
+        return {k: torch.zeros(n, device=self.device, dtype=dt) for k, (n, dt) in need.items()}
 
     def _step_logits(self, st, Bb, Kb):
         pk = st["pk"]

@@ -1,0 +1,152 @@
+"""Token mixers of per-layer mixed decoders on the serving engine's cache and slot state.
+
+A mixer belongs to one run of a layer (a looped layer has one per pass): it names what it keeps -- KV pages
+(``cache_shape``) and / or fp32 slot state (``state_widths``) -- and turns the layer's projection rows of a
+batch (``hybrid_runner._Batch``) into the rows that the output projection reads.
+"""
+from __future__ import annotations
+
+import torch
+
+from ..models.hybrid_config import (ChannelDeltaSpec, DiffAttentionSpec, GatedRecurrenceSpec, GeneralDeltaSpec,
+                                    LatentAttentionSpec)
+from ..ops import delta_rule as dr
+from ..ops import diff_attention as da
+from ..ops import gated_scan as gs
+from ..ops import latent_attention as la
+from ..ops import moe
+
+
+class Mixer:
+    """``run``: index of the layer run; ``linear``: the runner's projection; ``twin``: the mixer of an earlier
+    pass over the same layer (shares what is derived from the weights). ``cache`` / ``index`` (the layer's
+    place in it) and ``state`` are set once the runner has made them."""
+
+    def __init__(self, layer, cfg, run: int, linear, twin: Mixer | None = None):
+        self.layer, self.run, self.linear = layer, run, linear
+        self.cache = self.index = self.state = None
+
+    def cache_shape(self):
+        """(key heads, key size, value heads, value size) of the layer's pages, None without a cache."""
+        return None
+
+    def state_widths(self) -> dict:
+        return {}
+
+    def buffers(self, rows: int, max_kv: int, dtype) -> dict:
+        """Static workspaces of a decode bucket: name -> (elements, dtype); shared by the layers."""
+        return {}
+
+    def __call__(self, x, out, b):
+        raise NotImplementedError
+
+
+class DiffAttentionMixer(Mixer):
+    def __init__(self, layer, cfg, run, linear, twin=None):
+        super().__init__(layer, cfg, run, linear)
+        mx = layer.spec.mixer
+        self.sp = da.DiffHeads(mx.heads, mx.kv_heads, mx.dim, mx.vdim, mx.scale, layer.lam_value(), 1.0 - mx.diff,
+                               cfg.norm_eps, mx.temp_coef, mx.temp_every)
+
+    def cache_shape(self):
+        mx = self.layer.spec.mixer
+        return 2 * mx.kv_heads, mx.dim, mx.kv_heads, mx.vdim
+
+    def buffers(self, rows, max_kv, dtype):
+        _, _, w, c = da.rows_plan(self.sp, rows, max_kv, dtype)
+        return {"ws": (w, torch.float32), "cnt": (c, torch.int32)}
+
+    def __call__(self, qkv, out, b):
+        sp, kc, vc, tbl = self.sp, self.cache.k[self.index], self.cache.v[self.index], self.cache.table
+        a = (sp, qkv, kc, vc, tbl, b.pos, b.slots)
+        if b.single:
+            da.attend_rows(*a, out, b.max_kv, fused_append=True, ws=b.bufs.get("ws"), cnt=b.bufs.get("cnt"))
+            return
+        da.append(*a)
+        if out.is_cuda and da.tiles_ok(sp, out.dtype, self.cache.page_size, out.stride(0)):
+            if b.tiles is not None:
+                da.attend_tiles(*a, out, b.tiles)
+            if b.row_of is not None:
+                da.attend_rows(*a, out, b.row_kv, fused_append=False, row_of=b.row_of)
+        else:
+            da.attend_rows(*a, out, b.max_kv, fused_append=False)
+
+
+class GatedRecurrenceMixer(Mixer):
+    def state_widths(self):
+        return {f"scan{self.run}": (1, self.layer.spec.mixer.width)}
+
+    def __call__(self, zxg, out, b):
+        L, st = self.layer, self.state[f"scan{self.run}"][0]
+        if b.single:
+            gs.gated_step(zxg, L.b_z, L.b_x, st, out, b.pos, b.slots)
+        else:
+            gs.gated_scan(zxg, L.b_z, L.b_x, st, out, b.chunks, b.multi)
+
+
+class LatentAttentionMixer(Mixer):
+    def __init__(self, layer, cfg, run, linear, twin=None):
+        super().__init__(layer, cfg, run, linear)
+        mx, L = layer.spec.mixer, layer
+        self.sp = sp = la.LatentHeads(mx.heads, mx.dim, mx.rot_dim, mx.vdim, mx.q_rank, mx.kv_rank, mx.scale,
+                                      cfg.norm_eps, mx.rot_base, mx.rot_dims, (mx.parts["dq"][0], mx.parts["dkv"][0]))
+        nk = sp.heads * sp.dim
+        self.wt = twin.wt if twin is not None else la.LatentWeights(L.q_norm, L.kv_norm, L.sink,
+                                   L.ukv[:nk].view(sp.heads, sp.dim, sp.kv_rank).transpose(1, 2).contiguous(),
+                                   L.ukv[nk:].view(sp.heads, sp.vdim, sp.kv_rank), sp.frequencies().to(L.ukv.device))
+
+    def cache_shape(self):
+        return 1, self.sp.row, 0, 0
+
+    def buffers(self, rows, max_kv, dtype):
+        return {"part": (la.rows_plan(self.sp, rows, max_kv)[2], torch.float32)}
+
+    def __call__(self, x, out, b):
+        sp, wt, pages, tbl = self.sp, self.wt, self.cache.k[self.index], self.cache.table
+        a = (pages, tbl, b.pos, b.slots)
+        q = self.linear(la.latent_append(sp, wt, x, *a), self.layer.uq)
+        la.attend_rows(sp, wt, q, *a, out, b.max_kv, part=b.bufs.get("part"))
+
+
+class DeltaRuleMixer(Mixer):
+    def __init__(self, layer, cfg, run, linear, twin=None):
+        super().__init__(layer, cfg, run, linear)
+        mx, L = layer.spec.mixer, layer
+        at = lambda *names: tuple(mx.parts[n][0] for n in names)  # noqa: E731
+        if mx.general:
+            self.sp = dr.DeltaHeads(True, mx.heads, mx.heads, mx.dim, mx.dim, at("r", "k", "v", "a", "g", "w1"),
+                                    mx.rank_w, cfg.norm_eps)
+            self.wt = dr.DeltaWeights(L.w2, L.w0, L.a_bias, L.gain)
+        else:
+            self.sp = dr.DeltaHeads(False, mx.heads, mx.kv_heads, mx.dim, mx.vdim, at("q", "k", "v", "b", "g1", "a1"),
+                                    mx.rank_w, cfg.norm_eps, mx.taps, mx.rank_g)
+            self.wt = dr.DeltaWeights(L.a2, L.dt_bias, L.a_log, L.gain, L.g2, L.conv)
+
+    def state_widths(self):
+        w = {f"delta{self.run}": (1, self.sp.state_width)}
+        if not self.sp.general:
+            w[f"ring{self.run}"] = (1, self.sp.taps * self.sp.conv_channels)
+        return w
+
+    def __call__(self, x, out, b):
+        sp, wt = self.sp, self.wt
+        S = self.state[f"delta{self.run}"][0]
+        ring = None if sp.general else self.state[f"ring{self.run}"][0]
+        if b.single:
+            dr.delta_step(sp, wt, x, S, ring, b.pos, b.slots, out)
+            return
+        tanh = lambda t: moe.act_rows(t, torch.empty_like(t, memory_format=torch.contiguous_format), False, act="tanh")  # noqa: E731
+        inner, gate = dr.low_rank_inner(sp, x, tanh)
+        dr.delta_portions(sp, wt, x, S, ring, b.portions, out, self.linear(inner, wt.lo_w),
+                          None if gate is None else self.linear(gate, wt.lo_g))
+
+
+MIXERS = {DiffAttentionSpec: DiffAttentionMixer, GatedRecurrenceSpec: GatedRecurrenceMixer,
+          LatentAttentionSpec: LatentAttentionMixer, GeneralDeltaSpec: DeltaRuleMixer, ChannelDeltaSpec: DeltaRuleMixer}
+
+
+def make_mixer(layer, cfg, run: int, linear, twin: Mixer | None = None) -> Mixer:
+    return MIXERS[type(layer.spec.mixer)](layer, cfg, run, linear, twin)
+
+
+__all__ = ["Mixer", "MIXERS", "make_mixer"]

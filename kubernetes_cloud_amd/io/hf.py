@@ -55,10 +55,13 @@ def load_pretrained(path: str, device="cpu", dtype=torch.bfloat16, random_init_i
                     cfg=None):
     """Model of the family ``config.json`` names (``models.registry``) with the directory's weights."""
     cfg = cfg or LMConfig.from_pretrained(path)
+    fam = family_of(cfg)
+    sd = read_hf_state_dict(path) if has_weights(path) else None
+    if sd is not None and fam.with_shapes is not None:
+        cfg = fam.with_shapes(cfg, {k: tuple(v.shape) for k, v in sd.items()})
     model = build_model(cfg, device=device, dtype=dtype, seed=0)
-    if has_weights(path):
-        sd = read_hf_state_dict(path)
-        nat = family_of(cfg).to_native(sd, cfg)
+    if sd is not None:
+        nat = fam.to_native(sd, cfg)
         missing, unexpected = model.load_state_dict({k: v.to(dtype) for k, v in nat.items()},
                                                     strict=False)
         missing = [m for m in missing if not m.endswith("alibi")]

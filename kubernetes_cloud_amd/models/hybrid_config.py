@@ -5,6 +5,19 @@ from __future__ import annotations
 import dataclasses
 
 
+def _up8(n: int) -> int:
+    return -(-n // 8) * 8
+
+
+def aligned_parts(sizes: dict) -> tuple[dict, int]:
+    """Row (or column) blocks side by side, each starting at a multiple of 8: {name: (offset, size)}, total."""
+    out, o = {}, 0
+    for name, n in sizes.items():
+        out[name] = (o, n)
+        o = _up8(o + n)
+    return out, o
+
+
 @dataclasses.dataclass(frozen=True)
 class DiffAttentionSpec:
     """Differential attention: two softmax maps of size ``dim`` per head over shared values of size ``vdim``."""
@@ -29,6 +42,11 @@ class DiffAttentionSpec:
     def out_cols(self) -> int:
         return self.heads * self.vdim
 
+    @property
+    def extra(self) -> dict:
+        """Parameters beside the in and out projections: name -> shape."""
+        return {"lam": (4, self.dim)}
+
 
 @dataclasses.dataclass(frozen=True)
 class GatedRecurrenceSpec:
@@ -43,9 +61,158 @@ class GatedRecurrenceSpec:
     def out_cols(self) -> int:
         return self.width
 
+    @property
+    def extra(self) -> dict:
+        return {"b_z": (self.width,), "b_x": (self.width,)}
+
+
+@dataclasses.dataclass(frozen=True)
+class LatentAttentionSpec:
+    """Attention whose queries come from a normed latent of size ``q_rank`` and whose keys and values come from
+    a cached, normed latent of size ``kv_rank`` plus one rotated key part of size ``rot_dim`` shared by all
+    heads; a learned sink joins each head's softmax."""
+    heads: int
+    dim: int
+    vdim: int
+    rot_dim: int
+    q_rank: int
+    kv_rank: int
+    scale: float
+    rot_base: float
+    rot_dims: int               # of rot_dim, rotated in interleaved pairs
+
+    def __post_init__(self):
+        if self.rot_dims % 2 or not 0 <= self.rot_dims <= self.rot_dim:
+            raise ValueError(f"{self.rot_dims} of {self.rot_dim} dimensions rotate in pairs")
+
+    @property
+    def parts(self) -> dict:
+        return aligned_parts({"dq": self.q_rank, "dkv": self.kv_rank + self.rot_dim})[0]
+
+    @property
+    def in_rows(self) -> int:
+        return aligned_parts({"dq": self.q_rank, "dkv": self.kv_rank + self.rot_dim})[1]
+
+    @property
+    def out_cols(self) -> int:
+        return self.heads * self.vdim
+
+    @property
+    def extra(self) -> dict:
+        H, C = self.heads, self.kv_rank
+        return {"q_norm": (self.q_rank,), "kv_norm": (C,), "uq": (H * (self.dim + self.rot_dim), self.q_rank),
+                "ukv": (H * (self.dim + self.vdim), C), "sink": (H,)}
+
+
+@dataclasses.dataclass(frozen=True)
+class GeneralDeltaSpec:
+    """Generalised delta rule: a decay and a removal rate per head and key channel, unit removal keys.
+    ``decay_rank``: inner size of the two-step decay projection (None: the head size)."""
+    heads: int
+    dim: int
+    decay_rank: int | None = None
+
+    general = True
+    taps = 0
+
+    @property
+    def kv_heads(self) -> int:
+        return self.heads
+
+    @property
+    def vdim(self) -> int:
+        return self.dim
+
+    @property
+    def rank_w(self) -> int:
+        return self.decay_rank or self.dim
+
+    @property
+    def _sizes(self) -> dict:
+        n = self.heads * self.dim
+        return {"r": n, "k": n, "v": n, "g": n, "a": n, "w1": self.rank_w}
+
+    @property
+    def parts(self) -> dict:
+        return aligned_parts(self._sizes)[0]
+
+    @property
+    def in_rows(self) -> int:
+        return aligned_parts(self._sizes)[1]
+
+    @property
+    def out_cols(self) -> int:
+        return self.heads * self.dim
+
+    @property
+    def extra(self) -> dict:
+        n = self.heads * self.dim
+        return {"w2": (n, self.rank_w), "w0": (n,), "a_bias": (n,), "gain": (n,)}
+
+
+@dataclasses.dataclass(frozen=True)
+class ChannelDeltaSpec:
+    """Gated delta rule with a decay per head and key channel: q / k heads shared by groups of value heads,
+    short causal convolutions before unit keys and queries, two-step decay and gate projections (inner sizes
+    ``decay_rank`` / ``gate_rank``, None: the value head size)."""
+    heads: int
+    kv_heads: int
+    dim: int
+    vdim: int
+    taps: int
+    decay_rank: int | None = None
+    gate_rank: int | None = None
+
+    general = False
+
+    def __post_init__(self):
+        if self.heads % self.kv_heads:
+            raise ValueError(f"{self.heads} heads over {self.kv_heads} query/key heads")
+
+    @property
+    def rank_w(self) -> int:
+        return self.decay_rank or self.vdim
+
+    @property
+    def rank_g(self) -> int:
+        return self.gate_rank or self.vdim
+
+    @property
+    def conv_channels(self) -> int:
+        return 2 * self.kv_heads * self.dim + self.heads * self.vdim
+
+    @property
+    def _sizes(self) -> dict:
+        n = self.kv_heads * self.dim
+        return {"q": n, "k": n, "v": self.heads * self.vdim, "a1": self.rank_w, "g1": self.rank_g, "b": self.heads}
+
+    @property
+    def parts(self) -> dict:
+        return aligned_parts(self._sizes)[0]
+
+    @property
+    def in_rows(self) -> int:
+        return aligned_parts(self._sizes)[1]
+
+    @property
+    def out_cols(self) -> int:
+        return self.heads * self.vdim
+
+    @property
+    def extra(self) -> dict:
+        H = self.heads
+        return {"conv": (self.conv_channels, self.taps), "a2": (H * self.dim, self.rank_w), "dt_bias": (H * self.dim,),
+                "a_log": (H,), "g2": (H * self.vdim, self.rank_g), "gain": (self.vdim,)}
+
 
 @dataclasses.dataclass(frozen=True)
 class DenseSpec:
+    ff: int
+
+
+@dataclasses.dataclass(frozen=True)
+class GatedDenseSpec:
+    """W_down (gelu_tanh(W_gate h + b) * (W_up h + b)) + b."""
     ff: int
 
 
@@ -64,8 +231,17 @@ class MoESpec:
 
 @dataclasses.dataclass(frozen=True)
 class LayerSpec:
-    mixer: DiffAttentionSpec | GatedRecurrenceSpec
-    mlp: DenseSpec | MoESpec | None
+    mixer: (DiffAttentionSpec | GatedRecurrenceSpec | LatentAttentionSpec | GeneralDeltaSpec | ChannelDeltaSpec)
+    mlp: DenseSpec | GatedDenseSpec | MoESpec | None
+
+
+@dataclasses.dataclass(frozen=True)
+class LoopSpec:
+    """Layers ``start`` .. ``stop - 1`` run ``times`` times in a row with the same weights; every pass has its
+    own cache or state."""
+    start: int
+    stop: int
+    times: int
 
 
 @dataclasses.dataclass
@@ -76,6 +252,8 @@ class HybridConfig:
     layers: tuple
     norm_eps: float = 1e-5
     residual_mult: float = 1.0
+    block: str = "parallel"      # one norm feeds mixer and feed-forward | "sandwich": in turn, normed before and after
+    loop: LoopSpec | None = None
     max_pos: int = 8192          # serving default; the design itself sets no limit
     bos_token_id: int | None = None
     eos_token_id: int | None = None
@@ -86,20 +264,40 @@ class HybridConfig:
     def n_layers(self) -> int:
         return len(self.layers)
 
+    @property
+    def runs(self) -> tuple:
+        """Layer indices in the order they run."""
+        n, lp = len(self.layers), self.loop
+        if lp is None:
+            return tuple(range(n))
+        if not 0 <= lp.start <= lp.stop <= n or lp.times < 0:
+            raise ValueError(f"loop {lp} over {n} layers")
+        return (*range(lp.start), *(tuple(range(lp.start, lp.stop)) * lp.times), *range(lp.stop, n))
+
     def to_hf(self) -> dict:
         return dict(self.hf)
 
     def n_params(self) -> int:
-        d, n = self.hidden, 2 * self.vocab_size * self.hidden + 1
+        def numel(shape):
+            n = 1
+            for x in shape:
+                n *= x
+            return n
+
+        d = self.hidden
+        n = 2 * self.vocab_size * d + (1 if self.block == "parallel" else d)
         for L in self.layers:
-            n += 1 + d + (L.mixer.in_rows + L.mixer.out_cols) * d
-            n += 4 * L.mixer.dim if isinstance(L.mixer, DiffAttentionSpec) else 2 * L.mixer.width
+            n += (L.mixer.in_rows + L.mixer.out_cols) * d + sum(numel(s) for s in L.mixer.extra.values())
+            n += 1 + d if self.block == "parallel" else 3 * d
             if isinstance(L.mlp, DenseSpec):
                 n += 2 * d * L.mlp.ff
+            elif isinstance(L.mlp, GatedDenseSpec):
+                n += 3 * d * L.mlp.ff + 2 * L.mlp.ff + 4 * d
             elif L.mlp is not None:
                 n += d * (L.mlp.experts + 3 * L.mlp.experts * L.mlp.ff)
                 n += d * (3 * L.mlp.shared_ff + 1) if L.mlp.shared_ff else 0
         return n
 
 
-__all__ = ["HybridConfig", "LayerSpec", "DiffAttentionSpec", "GatedRecurrenceSpec", "DenseSpec", "MoESpec"]
+__all__ = ["HybridConfig", "LayerSpec", "LoopSpec", "DiffAttentionSpec", "GatedRecurrenceSpec", "LatentAttentionSpec",
+           "GeneralDeltaSpec", "ChannelDeltaSpec", "DenseSpec", "GatedDenseSpec", "MoESpec", "aligned_parts"]

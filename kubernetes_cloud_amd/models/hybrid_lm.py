@@ -1,16 +1,22 @@
-"""Decoders whose layers mix tokens differently (``HybridConfig``): differential attention or a gated
-recurrence, beside a dense, routed or no feed-forward, on an fp32 residual stream.
+"""Decoders whose layers mix tokens differently (``HybridConfig``): differential or latent attention, a gated
+recurrence or a delta rule, beside a dense, gated, routed or no feed-forward, on an fp32 residual stream.
 
-A layer is parallel: with h the normed stream and hs its token-shifted copy,
+``block`` "parallel": with h the normed stream and hs its token-shifted copy,
 
     x <- x + m (mixer(hs) + ff(h))
+
+"sandwich": two sublayers in turn, each normed before and after and scaled per coordinate,
+
+    x <- x + scale * N(mixer(N(x))),   x <- x + scale2 * N(ff(N(x)))
 
 The modules hold weights laid out for the kernels; the step itself (cache, state, batching) is
 ``engine.hybrid_runner``. Layout:
 
-* ``w_in``   every projection of the mixer in one matrix ([q | k | v] or [z | x | g])
-* ``w_out``  the mixer's output projection and the dense (or shared-expert) down projection side by side,
-  [d, mixer + ff]: both branches close in one product, summed in fp32 before its rounding
+* ``w_in``   every projection of the mixer's input in one matrix ([q | k | v], [z | x | g], ...; ``spec.parts``:
+  blocks start at multiples of 8 rows)
+* ``w_out``  the mixer's output projection; parallel layers put the dense (or shared-expert) down projection
+  beside it, [d, mixer + ff]: both branches close in one product, summed in fp32 before its rounding
+* ``w_up``   gate and up projections of a gated feed-forward, one above the other
 * experts stacked: gate-and-up [E, 2F, d], down [E, d, F]
 """
 from __future__ import annotations
@@ -18,7 +24,7 @@ from __future__ import annotations
 import torch
 import torch.nn as nn
 
-from .hybrid_config import DenseSpec, DiffAttentionSpec, HybridConfig, LayerSpec, MoESpec
+from .hybrid_config import DenseSpec, GatedDenseSpec, HybridConfig, LayerSpec, MoESpec
 
 
 def _p(*shape):
@@ -30,15 +36,24 @@ class HybridLayer(nn.Module):
         super().__init__()
         d, mx, mlp = cfg.hidden, spec.mixer, spec.mlp
         self.spec = spec
+        self.w_in = _p(mx.in_rows, d)
+        for name, shape in mx.extra.items():
+            setattr(self, name, _p(*shape))
+        self.moe = isinstance(mlp, MoESpec)
+        if cfg.block == "sandwich":
+            if mlp is not None and not isinstance(mlp, GatedDenseSpec):
+                raise ValueError(f"sandwich layers take a gated feed-forward or none, not {type(mlp).__name__}")
+            self.norm, self.norm_b, self.scale = _p(d), _p(d), _p(d)
+            self.w_out = _p(d, mx.out_cols)
+            if mlp is not None:
+                self.norm2, self.norm2_b, self.scale2 = _p(d), _p(d), _p(d)
+                self.w_up, self.b_up = _p(2 * mlp.ff, d), _p(2 * mlp.ff)
+                self.w_down, self.b_down = _p(d, mlp.ff), _p(d)
+            return
+        if isinstance(mlp, GatedDenseSpec):
+            raise ValueError("parallel layers take a dense or routed feed-forward, not a gated one")
         self.norm = nn.Parameter(torch.empty(()), requires_grad=False)
         self.shift = _p(d)
-        self.w_in = _p(mx.in_rows, d)
-        self.attention = isinstance(mx, DiffAttentionSpec)
-        if self.attention:
-            self.lam = _p(4, mx.dim)          # rows lq1, lk1, lq2, lk2
-        else:
-            self.b_z, self.b_x = _p(mx.width), _p(mx.width)
-        self.moe = isinstance(mlp, MoESpec)
         self.ff_cols = mlp.ff if isinstance(mlp, DenseSpec) else mlp.shared_ff if self.moe else 0
         self.w_up = _p((2 if self.moe else 1) * self.ff_cols, d) if self.ff_cols else None
         self.w_out = _p(d, mx.out_cols + self.ff_cols)
@@ -49,7 +64,8 @@ class HybridLayer(nn.Module):
             self.shared_gate = _p(1, d) if mlp.shared_ff else None
 
     def lam_value(self) -> float:
-        """lambda = exp(lq1 . lk1) - exp(lq2 . lk2) + diff, one number for the layer (fp32)."""
+        """Differential attention: lambda = exp(lq1 . lk1) - exp(lq2 . lk2) + diff, one number
+        for the layer (fp32); ``lam`` holds the rows lq1, lk1, lq2, lk2."""
         v = self.lam.float()
         return float(torch.exp((v[0] * v[1]).sum()) - torch.exp((v[2] * v[3]).sum())) + self.spec.mixer.diff
 
@@ -60,7 +76,7 @@ class HybridLM(nn.Module):
         self.cfg = cfg
         self.wte = _p(cfg.vocab_size, cfg.hidden)
         self.layers = nn.ModuleList([HybridLayer(cfg, s) for s in cfg.layers])
-        self.final_norm = nn.Parameter(torch.empty(()), requires_grad=False)
+        self.final_norm = _p(cfg.hidden) if cfg.block == "sandwich" else nn.Parameter(torch.empty(()), requires_grad=False)
         self.head = _p(cfg.vocab_size, cfg.hidden)
 
     @torch.no_grad()
@@ -71,7 +87,7 @@ class HybridLM(nn.Module):
         for name, p in self.named_parameters():
             if p.dim() >= 2:
                 p.normal_(0.0, std, generator=g)
-            elif "norm" in name:
+            elif any(k in name for k in ("norm", "scale", "gain")):
                 p.fill_(1.0)
             elif name.endswith("shift"):
                 p.fill_(0.5)

@@ -22,6 +22,7 @@ class Family:
     from_native: Callable
     runner: Callable           # () -> StepRunner class
     kernels: tuple = ()
+    with_shapes: Callable | None = None  # (cfg, {checkpoint tensor: shape}) -> cfg with the sizes only they give
 
 
 def _megusun() -> Family:
@@ -35,6 +36,18 @@ def _megusun() -> Family:
                   ("rms_shift", "gated_scan", "diff_attn", "moe", "act_rows", "gemv", "skinny_mfma"))
 
 
+def _rezusun() -> Family:
+    from . import rezusun
+    from .hybrid_lm import build_hybrid
+
+    def runner():
+        from ..engine.hybrid_runner import HybridRunner
+        return HybridRunner
+    return Family("rezusun", rezusun.read_config, build_hybrid, rezusun.to_native, rezusun.from_native, runner,
+                  ("norm_residual", "delta_rule", "latent_attn", "act_rows", "gemv", "skinny_mfma"),
+                  rezusun.with_shapes)
+
+
 def _causal_lm() -> Family:
     from .causal_lm import build_causal_lm
     from .config import LMConfig
@@ -46,7 +59,7 @@ def _causal_lm() -> Family:
     return Family("causal_lm", LMConfig.read_hf, build_causal_lm, hf_to_native, native_to_hf, runner)
 
 
-FAMILIES = {"Megusun": _megusun}   # config.json "architecture" -> family
+FAMILIES = {"Megusun": _megusun, "Rezusun": _rezusun}   # config.json "architecture" -> family
 
 
 def family_of_dict(cfg: dict) -> Family:

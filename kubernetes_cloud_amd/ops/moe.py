@@ -122,21 +122,31 @@ def experts(h: torch.Tensor, ids: torch.Tensor, weights: torch.Tensor, gate_up: 
     return y
 
 
-def act_rows(x: torch.Tensor, out: torch.Tensor, gated: bool, row_scale: torch.Tensor | None = None) -> torch.Tensor:
-    """out = gelu(x) (exact), or silu(gate) * up * row_scale with x = [gate | up]; strided rows."""
+ACT_ROWS = {"gelu": 0, "silu_gated": 1, "gelu_tanh_gated": 2, "tanh": 3}
+
+
+def act_rows(x: torch.Tensor, out: torch.Tensor, gated: bool, row_scale: torch.Tensor | None = None, *,
+             act: str | None = None, bias: torch.Tensor | None = None) -> torch.Tensor:
+    """out = gelu(x) (exact), or silu(gate) * up * row_scale with x = [gate | up]; strided rows. ``act`` names
+    another form (``ACT_ROWS``); ``bias`` is added to x first."""
     T, F = out.shape
-    code = native_dt(x, out)
+    act = act or ("silu_gated" if gated else "gelu")
+    gated = act.endswith("_gated")
+    code = native_dt(x, out, bias)
     assert x.shape == (T, 2 * F if gated else F) and x.stride(1) == 1 and out.stride(1) == 1
+    assert bias is None or (bias.is_contiguous() and bias.numel() == x.shape[1])
     if code is None:
+        xf = x.float() if bias is None else x.float() + bias.float()
         if gated:
-            y = torch.nn.functional.silu(x[:, :F].float()) * x[:, F:].float()
+            g = xf[:, :F]
+            y = (torch.nn.functional.silu(g) if act == "silu_gated" else
+                 0.5 * g * (1 + torch.tanh(math.sqrt(2 / math.pi) * (g + 0.044715 * g ** 3)))) * xf[:, F:]
             out.copy_(y if row_scale is None else y * row_scale[:, None])
         else:
-            xf = x.float()
-            out.copy_(0.5 * xf * (1 + torch.erf(xf / math.sqrt(2.0))))
+            out.copy_(torch.tanh(xf) if act == "tanh" else 0.5 * xf * (1 + torch.erf(xf / math.sqrt(2.0))))
         return out
-    _lib.call("kca_act_rows", code, int(gated), x.data_ptr(), x.stride(0), _lib.ptr(row_scale), out.data_ptr(),
-              out.stride(0), T, F, _lib.stream())
+    _lib.call("kca_act_rows", code, ACT_ROWS[act], x.data_ptr(), x.stride(0), _lib.ptr(row_scale), _lib.ptr(bias),
+              out.data_ptr(), out.stride(0), T, F, _lib.stream())
     return out
 
 
