@@ -35,9 +35,10 @@ struct DeltaArgs {
   const int* e1;            // [T] one past its last row
   void* out;                // rows [H dv], row stride ldo
   long long ldo;
-  float* pk;                // prepared vectors [T][H][pk_stride]: w z p k q [dk], v [dv], q.p, q.k
+  const int* rows;          // prep kernel: token row of prepared row b (nullable: b)
+  float* pk;                // prepared vectors [rows][H][pk_stride]: w z p k q [dk], v [dv], q.p, q.k
   float* o;                 // read-outs [T][H dv]
-  const int* ent;           // [n][4]: first row, rows, position of the first row, slot
+  const int* ent;           // scan kernel: [n][5]: first row, rows, position of the first row, slot, first prepared row
 };
 
 namespace delta {

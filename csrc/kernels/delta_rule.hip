@@ -124,10 +124,10 @@ __global__ void __launch_bounds__(1024) delta_step_kernel(DeltaArgs a) {
 template <typename E, int KIND>
 __global__ void __launch_bounds__(128) delta_prep_kernel(DeltaArgs a) {
   extern __shared__ float smem[];
-  const int t = blockIdx.x, h = blockIdx.y, tid = threadIdx.x, dk = a.dk, dv = a.dv;
+  const int t = a.rows ? a.rows[blockIdx.x] : (int)blockIdx.x, h = blockIdx.y, tid = threadIdx.x, dk = a.dk, dv = a.dv;
   Head hd(smem, dk, dv, a.rank_w, a.rank_g);
   prep_head<E, KIND>(a, t, h, hd);
-  float* pk = a.pk + ((long long)t * a.H + h) * pk_stride(dk, dv);
+  float* pk = a.pk + ((long long)blockIdx.x * a.H + h) * pk_stride(dk, dv);
   for (int c = tid; c < 5 * dk + dv; c += 128) pk[c] = smem[c];  // w z p k q v lie in this order
   if (tid == 0) {
     pk[5 * dk + dv] = hd.qp;
@@ -137,15 +137,15 @@ __global__ void __launch_bounds__(128) delta_prep_kernel(DeltaArgs a) {
 
 template <int R, int CW>
 __global__ void __launch_bounds__(256) delta_scan_kernel(DeltaArgs a) {
-  const int* en = a.ent + blockIdx.x * 4;
-  const int row0 = en[0], n = en[1], pos0 = en[2], slot = en[3], h = blockIdx.y;
+  const int* en = a.ent + blockIdx.x * 5;
+  const int row0 = en[0], n = en[1], pos0 = en[2], slot = en[3], pk0 = en[4], h = blockIdx.y;
   const int wv = threadIdx.x >> 6, lane = threadIdx.x & 63, rg = lane & 15, cg = lane >> 4;
   const int dk = a.dk, dv = a.dv, col = (blockIdx.z * 4 + wv) * 4 * CW + cg * CW;
   if ((int)(blockIdx.z * 4 + wv) * 4 * CW >= dv) return;
   float* S = a.state + ((long long)slot * a.H + h) * dk * dv;
   const int ps = pk_stride(dk, dv);
   const long long step = (long long)a.H * ps;
-  const float* pk = a.pk + ((long long)row0 * a.H + h) * ps;
+  const float* pk = a.pk + ((long long)pk0 * a.H + h) * ps;
   float* o = a.o + (long long)row0 * a.H * dv + h * dv + col;
   Cols<R, CW> st;
   st.load(S, dk, dv, rg, col, pos0 > 0);
@@ -278,7 +278,7 @@ KCA_API int kca_delta_step(const DeltaArgs* in, int dtype, int kind, int B, hipS
   DELTA_DISPATCH(step_r, B)
 }
 
-// a.pk of every (token, head)
+// a.pk of T token rows (a.rows)
 KCA_API int kca_delta_prep(const DeltaArgs* in, int dtype, int kind, int T, hipStream_t s) {
   const DeltaArgs& a = *in;
   if (!delta_args_ok(a, kind) || T < 1 || a.H > 65535 || !a.pk || !a.e0 || !a.e1) return 1;

@@ -28,7 +28,7 @@ from ..ops import diff_attention as da
 from ..ops import gated_scan as gs
 from ..ops import moe
 from ..ops import skinny_mm as smm
-from ..ops.delta_rule import Portions
+from ..ops.delta_rule import Portions, plan_portions
 from ..ops.gemv import skinny_linear
 from ..ops.norm_residual import NormedBranch, norm_residual
 from ..ops.rms_shift import Branch, rms_shift
@@ -222,10 +222,8 @@ class HybridRunner(StepRunner):
             parts["flags"] = fl
             parts["entry"] = np.repeat(np.arange(len(ent)), [e[1] for e in ent])
             parts["entry_slots"] = np.asarray([e[3] for e in ent])
-            parts["ent"] = np.asarray(ent).reshape(-1)
-            n_of = [e[1] for e in ent]
-            parts["e0"] = np.repeat([e[0] for e in ent], n_of)
-            parts["e1"] = np.repeat([e[0] + e[1] for e in ent], n_of)
+            portions = plan_portions(ent)
+            parts.update(("p_" + k, v.reshape(-1)) for k, v in portions.items())
             chunks, multi = gs.plan_chunks(ent)
             parts["chunks"] = chunks.reshape(-1)
             parts["tiles"] = da.plan_tiles([e for e in ent if e[1] > 1]).reshape(-1)
@@ -242,7 +240,7 @@ class HybridRunner(StepRunner):
         if not single:
             b.single, b.multi = False, multi
             b.flags, b.entry, b.entry_slots = dev["flags"], dev["entry"], dev["entry_slots"].long()
-            b.portions = Portions(b.pos, b.slots, dev["e0"], dev["e1"], dev["ent"].view(-1, 4))
+            b.portions = Portions(b.pos, b.slots, **{k: dev["p_" + k].view(v.shape) for k, v in portions.items()})
             b.chunks = dev["chunks"].view(-1, 6)
             b.tiles = dev["tiles"].view(-1, 4) if dev["tiles"].numel() else None
             if ones:

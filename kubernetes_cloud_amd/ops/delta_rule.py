@@ -21,6 +21,7 @@ import ctypes
 import dataclasses
 import math
 
+import numpy as np
 import torch
 
 from . import _lib
@@ -35,7 +36,15 @@ class _Args(ctypes.Structure):
                 *[(n, _I) for n in ("H", "G", "dk", "dv", "taps", "rank_w", "rank_g")], ("lo_w", _P), ("lo_g", _P),
                 ("dw", _P), ("ldw", _LL), ("dg", _P), ("ldg", _LL), ("w0", _P), ("ab", _P), ("conv", _P), ("gain", _P),
                 ("eps", _F), ("qscale", _F), ("state", _P), ("ring", _P), ("pos", _P), ("slot", _P), ("e0", _P),
-                ("e1", _P), ("out", _P), ("ldo", _LL), ("pk", _P), ("o", _P), ("ent", _P)]
+                ("e1", _P), ("out", _P), ("ldo", _LL), ("rows", _P), ("pk", _P), ("o", _P), ("ent", _P)]
+
+
+class _ChunkArgs(ctypes.Structure):
+    _fields_ = [("d", _Args), ("ck", _P), ("en", _P), ("m", _P), ("b", _P), ("q", _P), ("oo", _P), ("e", _P)]
+
+
+CHUNK = 64       # tokens of a matrix-core chunk
+CHUNK_MIN = 16   # shorter portions go token by token
 
 
 @dataclasses.dataclass(frozen=True)
@@ -75,13 +84,43 @@ class DeltaWeights:
 
 @dataclasses.dataclass
 class Portions:
-    """Device arrays of a batch of portions: per row its position, slot, and the first and one-past-last row of
-    its entry; ``ent`` [n, 4]: first row, rows, position of the first row, slot."""
+    """Device arrays of a batch of portions (``plan_portions``): per row its position, slot, and the first and
+    one-past-last row of its entry; ``ent`` [n, 5] every entry, ``short`` / ``rows`` the short entries and their
+    token rows, ``chunked`` [n, 6] / ``chunks`` [n, 4] the longer entries and their chunks."""
     pos: torch.Tensor
     slots: torch.Tensor
     e0: torch.Tensor
     e1: torch.Tensor
     ent: torch.Tensor
+    short: torch.Tensor
+    rows: torch.Tensor
+    chunked: torch.Tensor
+    chunks: torch.Tensor
+
+
+def plan_portions(entries) -> dict:
+    """[(first row, rows, position, slot)] -> host arrays of ``Portions`` (pos and slots aside), int32."""
+    n_of = [e[1] for e in entries]
+    out = {"e0": np.repeat([e[0] for e in entries], n_of), "e1": np.repeat([e[0] + e[1] for e in entries], n_of)}
+    ent, short, rows, chunked, chunks = [], [], [], [], []
+    for r0, n, pos, slot in entries:
+        ent.append((r0, n, pos, slot, r0))
+        if n < CHUNK_MIN:
+            short.append((r0, n, pos, slot, len(rows)))
+            rows += range(r0, r0 + n)
+        else:
+            nc = -(-n // CHUNK)
+            chunked.append((r0, n, pos, slot, len(chunks), nc))
+            chunks += [(r0 + i * CHUNK, min(CHUNK, n - i * CHUNK), r0, pos + i * CHUNK) for i in range(nc)]
+    for k, v, w in (("ent", ent, 5), ("short", short, 5), ("rows", rows, 0), ("chunked", chunked, 6), ("chunks", chunks, 4)):
+        v = np.asarray(v, dtype=np.int32)
+        out[k] = v.reshape(-1, w) if w else v
+    return {k: v.astype(np.int32) for k, v in out.items()}
+
+
+def chunks_ok(sp: DeltaHeads, dtype) -> bool:
+    """Sizes the chunked matrix-core kernels take (others, and fp32, run token by token)."""
+    return dtype == torch.bfloat16 and sp.dim % 8 == 0 and sp.vdim % 8 == 0 and max(sp.dim, sp.vdim) <= 128 and sp.taps <= 4
 
 
 def _args(sp: DeltaHeads, wt: DeltaWeights, x, state, ring, pos, slots, out) -> tuple[_Args, int]:
@@ -151,21 +190,38 @@ def delta_portions(sp: DeltaHeads, wt: DeltaWeights, x, state, ring, b: Portions
     a, code = _args(sp, wt, x, state, ring, b.pos, b.slots, out)
     T = x.shape[0]
     if code is None:
-        return _reference(sp, wt, x, state, ring, b.ent.tolist(), out, dw, dg)
+        return _reference(sp, wt, x, state, ring, b.ent[:, :4].tolist(), out, dw, dg)
     assert dw.stride(1) == 1 and dw.shape == (T, sp.heads * sp.dim) and dw.dtype == x.dtype
     a.dw, a.ldw = dw.data_ptr(), dw.stride(0)
     if not sp.general:
         assert dg.stride(1) == 1 and dg.shape == (T, sp.heads * sp.vdim) and dg.dtype == x.dtype
         a.dg, a.ldg = dg.data_ptr(), dg.stride(0)
-    assert b.ent.dtype == torch.int32 and b.ent.is_contiguous() and all(t.dtype == torch.int32 for t in (b.e0, b.e1))
-    a.e0, a.e1, a.ent = b.e0.data_ptr(), b.e1.data_ptr(), b.ent.data_ptr()
-    kind = 0 if sp.general else 1
-    per = -(-(5 * sp.dim + sp.vdim + 2) // 4) * 4
-    pk = torch.empty(T * sp.heads * per, device=x.device, dtype=torch.float32)
-    o = torch.empty(T, sp.heads * sp.vdim, device=x.device, dtype=torch.float32)
-    a.pk, a.o = pk.data_ptr(), o.data_ptr()
-    _call("kca_delta_prep", a, code, kind, T)
-    _call("kca_delta_scan", a, b.ent.shape[0])
+    assert all(t.dtype == torch.int32 and t.is_contiguous() for t in (b.e0, b.e1, b.ent, b.short, b.rows, b.chunked, b.chunks))
+    a.e0, a.e1 = b.e0.data_ptr(), b.e1.data_ptr()
+    kind, dev, H = 0 if sp.general else 1, x.device, sp.heads
+    o = torch.empty(T, H * sp.vdim, device=dev, dtype=torch.float32)
+    a.o = o.data_ptr()
+    chunked = chunks_ok(sp, x.dtype) and b.chunks.shape[0] > 0
+    if chunked:
+        nc, DK, DV = b.chunks.shape[0], (64 if sp.dim <= 64 else 128), (64 if sp.vdim <= 64 else 128)
+        sizes = (DK * DK, DV * DK, CHUNK * DK, DV * CHUNK)
+        ws = [torch.empty(nc * H * n, device=dev, dtype=torch.bfloat16) for n in sizes]
+        e = torch.empty(nc * H * DK, device=dev, dtype=torch.float32)
+        if _lib.require().kca_delta_chunk_abi() != ctypes.sizeof(_ChunkArgs):
+            raise RuntimeError("kca_delta_chunk descriptor: C and ctypes sizes differ")
+        c = _ChunkArgs()
+        c.d, c.ck, c.en = a, b.chunks.data_ptr(), b.chunked.data_ptr()
+        c.m, c.b, c.q, c.oo = (t.data_ptr() for t in ws)
+        c.e = e.data_ptr()
+        _call("kca_delta_map", c, kind, nc)
+        _call("kca_delta_run", c, kind, b.chunked.shape[0])
+    ent, rows = (b.short, b.rows) if chunked else (b.ent, None)
+    if ent.shape[0]:
+        n = T if rows is None else rows.shape[0]
+        pk = torch.empty(n * H * (-(-(5 * sp.dim + sp.vdim + 2) // 4) * 4), device=dev, dtype=torch.float32)
+        a.pk, a.rows, a.ent = pk.data_ptr(), _lib.ptr(rows), ent.data_ptr()
+        _call("kca_delta_prep", a, code, kind, n)
+        _call("kca_delta_scan", a, ent.shape[0])
     _call("kca_delta_gate", a, code, kind, T)
     return out
 
@@ -221,4 +277,5 @@ def _reference(sp, wt, x, state, ring, entries, out, dw, dg):
     return out
 
 
-__all__ = ["DeltaHeads", "DeltaWeights", "Portions", "delta_step", "delta_portions", "low_rank_inner"]
+__all__ = ["DeltaHeads", "DeltaWeights", "Portions", "plan_portions", "chunks_ok", "delta_step", "delta_portions",
+           "low_rank_inner"]
