@@ -30,6 +30,7 @@ from ..ops import moe
 from ..ops import skinny_mm as smm
 from ..ops.delta_rule import Portions, plan_portions
 from ..ops.gemv import skinny_linear
+from ..ops.latent_attention import Prompts, plan_prompts
 from ..ops.norm_residual import NormedBranch, norm_residual
 from ..ops.rms_shift import Branch, rms_shift
 from .mixers import make_mixer
@@ -46,7 +47,7 @@ class _Batch:
         self.tokens, self.pos, self.slots, self.max_kv = tokens, pos, slots, max_kv
         self.T = tokens.shape[0]
         self.single = True
-        self.flags = self.entry = self.tiles = self.row_of = self.portions = self.chunks = self.entry_slots = None
+        self.flags = self.entry = self.tiles = self.row_of = self.portions = self.prompts = self.chunks = self.entry_slots = None
         self.multi = False
         self.row_kv = 0
         self.bufs = {}
@@ -224,6 +225,8 @@ class HybridRunner(StepRunner):
             parts["entry_slots"] = np.asarray([e[3] for e in ent])
             portions = plan_portions(ent)
             parts.update(("p_" + k, v.reshape(-1)) for k, v in portions.items())
+            prompts, sizes = plan_prompts(ent)
+            parts.update(("l_" + k, v.reshape(-1)) for k, v in prompts.items())
             chunks, multi = gs.plan_chunks(ent)
             parts["chunks"] = chunks.reshape(-1)
             parts["tiles"] = da.plan_tiles([e for e in ent if e[1] > 1]).reshape(-1)
@@ -241,6 +244,7 @@ class HybridRunner(StepRunner):
             b.single, b.multi = False, multi
             b.flags, b.entry, b.entry_slots = dev["flags"], dev["entry"], dev["entry_slots"].long()
             b.portions = Portions(b.pos, b.slots, **{k: dev["p_" + k].view(v.shape) for k, v in portions.items()})
+            b.prompts = Prompts(**{k: dev["l_" + k].view(v.shape) for k, v in prompts.items()}, **sizes)
             b.chunks = dev["chunks"].view(-1, 6)
             b.tiles = dev["tiles"].view(-1, 4) if dev["tiles"].numel() else None
             if ones:

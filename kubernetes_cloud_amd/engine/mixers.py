@@ -105,7 +105,13 @@ class LatentAttentionMixer(Mixer):
         sp, wt, pages, tbl = self.sp, self.wt, self.cache.k[self.index], self.cache.table
         a = (pages, tbl, b.pos, b.slots)
         q = self.linear(la.latent_append(sp, wt, x, *a), self.layer.uq)
-        la.attend_rows(sp, wt, q, *a, out, b.max_kv, part=b.bufs.get("part"))
+        pr = b.prompts
+        if pr is None or not pr.tiles.shape[0] or not (out.is_cuda and la.tiles_ok(sp, out.dtype, out.stride(0))):
+            la.attend_rows(sp, wt, q, *a, out, b.max_kv, part=b.bufs.get("part"))
+            return
+        la.attend_prompts(sp, wt, q, *a, out, self.layer.ukv, pr, self.linear)
+        if pr.rows.shape[0]:
+            la.attend_rows(sp, wt, q, *a, out, pr.rows_kv, row_of=pr.rows)
 
 
 class DeltaRuleMixer(Mixer):

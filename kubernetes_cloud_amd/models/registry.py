@@ -44,7 +44,7 @@ def _rezusun() -> Family:
         from ..engine.hybrid_runner import HybridRunner
         return HybridRunner
     return Family("rezusun", rezusun.read_config, build_hybrid, rezusun.to_native, rezusun.from_native, runner,
-                  ("norm_residual", "delta_rule", "delta_chunk", "latent_attn", "act_rows", "gemv", "skinny_mfma"),
+                  ("norm_residual", "delta_rule", "delta_chunk", "latent_attn", "latent_mfma", "act_rows", "gemv", "skinny_mfma"),
                   rezusun.with_shapes)
 
 

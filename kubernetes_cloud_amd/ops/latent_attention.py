@@ -1,5 +1,9 @@
 """Latent attention over the paged cache (``csrc/kernels/latent_attn.h``).
 
+Few query tokens attend over the latents themselves (``attend_rows``); prompt portions expand their context's
+keys and values once and run as tiles of queries (``attend_prompts``). bf16 takes the matrix-core kernels of
+``latent_mfma.hip`` wherever the sizes allow, everything else ``latent_attn.hip``.
+
 The cache holds one row per token, [c (kv_rank, normed) | r (rot_dim, rotated key part)], shared by all heads:
 pages [n, 1, PS, kv_rank + rot_dim]. A head's key is [W_uk c | r], its value W_uv c, so a score is
 (W_uk^T q) . c + rot(q) . r and an output W_uv (sum_j weight_j c_j); exp(sink) joins the softmax's denominator.
@@ -9,6 +13,7 @@ from __future__ import annotations
 import ctypes
 import dataclasses
 
+import numpy as np
 import torch
 
 from . import _lib
@@ -25,6 +30,11 @@ class _Args(ctypes.Structure):
                 ("table", _P), ("tstride", _I), ("shift", _I), ("pos", _P), ("slot", _P), ("freq", _P), ("q", _P),
                 ("qa", _P), ("sink", _P), ("part", _P), ("nsplit", _I), ("chunk", _I), ("row_of", _P), ("wuv", _P),
                 ("out", _P), ("ldo", _LL), ("kv", _P), ("ldkv", _LL), ("kr", _P), ("tiles", _P)]
+
+
+TILE = 128        # query rows of a prompt tile
+PROMPT_MIN = 32   # shorter portions run row by row
+MAX_SPLITS = 256
 
 
 @dataclasses.dataclass(frozen=True)
@@ -93,16 +103,20 @@ def _base(sp: LatentHeads, wt: LatentWeights, pages, table, pos, slots, T) -> _A
     return a
 
 
-def _call(name, a, *args):
+def _call(name, a, *args, other: bool = False) -> bool:
+    """``other``: status 10 (sizes for another kernel) returns False instead of raising."""
     fn = getattr(_lib.require(), name)
     fn.argtypes = [ctypes.c_void_p] + [ctypes.c_int] * len(args) + [ctypes.c_void_p]
     fn.restype = ctypes.c_int
     rc = fn(ctypes.addressof(a), *args, _lib.stream())
+    if rc == 10 and other:
+        return False
     if rc != 0:
         raise RuntimeError(f"{name} returned status {rc} (unsupported shape/arguments)")
     _lib.LAUNCHES[0] += 1
     if _lib.SYNC_LAUNCH:
         torch.cuda.synchronize()
+    return True
 
 
 def latent_append(sp: LatentHeads, wt: LatentWeights, x, pages, table, pos, slots) -> torch.Tensor:
@@ -131,6 +145,7 @@ def latent_append(sp: LatentHeads, wt: LatentWeights, x, pages, table, pos, slot
 def rows_plan(sp: LatentHeads, rows: int, max_kv: int) -> tuple[int, int, int]:
     """(splits, keys per split, partial floats)."""
     chunk = -(-(max_kv if rows * sp.heads >= 4096 else decode_chunk(rows, max(1, sp.heads // 16), max_kv)) // 64) * 64
+    chunk = max(chunk, -(-max_kv // (64 * MAX_SPLITS)) * 64)
     n = -(-max_kv // chunk)
     return n, chunk, rows * sp.heads * n * (sp.kv_rank + 2)
 
@@ -157,8 +172,71 @@ def attend_rows(sp: LatentHeads, wt: LatentWeights, q, pages, table, pos, slots,
     a.q, a.qa, a.part, a.nsplit, a.chunk = q.data_ptr(), qa.data_ptr(), part.data_ptr(), splits, chunk
     a.row_of, a.sink, a.wuv = _lib.ptr(row_of), wt.sink.data_ptr(), wt.wuv.data_ptr()
     a.out, a.ldo = out.data_ptr(), out.stride(0)
-    _call("kca_latent_rows", a, code, n, int(max_kv))
-    _call("kca_latent_merge", a, code, n)
+    if code != 1 or not _call("kca_latent_rows_mfma", a, n, int(max_kv), other=True):
+        _call("kca_latent_rows", a, code, n, int(max_kv))
+    if code != 1 or not _call("kca_latent_merge_mfma", a, n, other=True):
+        _call("kca_latent_merge", a, code, n)
+    return out
+
+
+@dataclasses.dataclass
+class Prompts:
+    """Device arrays of the portions that run as tiles (``plan_prompts``): ``tiles`` [n, 4] first row, rows,
+    position of the first row, context row of position 0 (longest key ranges first); ``ctx`` [m, 3] first context
+    row, length, slot; ``rows`` the token rows of all other entries."""
+    tiles: torch.Tensor
+    ctx: torch.Tensor
+    rows: torch.Tensor
+    n_ctx: int      # context rows
+    max_ctx: int    # longest context
+    rows_kv: int    # keys the longest of the other rows sees
+
+
+def plan_prompts(entries, min_rows: int = PROMPT_MIN) -> tuple[dict, dict]:
+    """[(first row, rows, position, slot)] -> (host arrays, host numbers) of ``Prompts``."""
+    tiles, ctx, rows, at, kv = [], [], [], 0, 0
+    for r0, n, p0, slot in entries:
+        if n < min_rows:
+            rows += range(r0, r0 + n)
+            kv = max(kv, p0 + n)
+            continue
+        ctx.append((at, p0 + n, slot))
+        tiles += [(r0 + i, min(TILE, n - i), p0 + i, at) for i in range(0, n, TILE)]
+        at += p0 + n
+    tiles.sort(key=lambda t: -(t[2] + t[1]))
+    arr = {"tiles": np.asarray(tiles, dtype=np.int32).reshape(-1, 4), "ctx": np.asarray(ctx, dtype=np.int32).reshape(-1, 3),
+           "rows": np.asarray(rows, dtype=np.int32)}
+    return arr, {"n_ctx": at, "max_ctx": max((c[1] for c in ctx), default=0), "rows_kv": kv}
+
+
+def tiles_ok(sp: LatentHeads, dtype, ldo: int) -> bool:
+    """Sizes the prompt tiles take (others run row by row)."""
+    return (dtype == torch.bfloat16 and not any(n % 8 for n in (sp.dim, sp.rot_dim, sp.vdim, sp.kv_rank))
+            and sp.dim + sp.rot_dim <= 256 and sp.vdim <= 256 and ldo % 4 == 0 and sp.scale > 0)
+
+
+def attend_prompts(sp: LatentHeads, wt: LatentWeights, q, pages, table, pos, slots, out, ukv, b: Prompts, linear):
+    """The portions of ``b.tiles`` over keys and values expanded from their contexts (which the pages hold):
+    ``ukv`` [H (dim + vdim), kv_rank] = W_uk over W_uv, through ``linear(x, w)``."""
+    T, H = q.shape[0], sp.heads
+    assert native_dt(q, pages, wt.sink, out, ukv) == 1 and q.is_contiguous() and q.shape[1] == H * (sp.dim + sp.rot_dim)
+    assert out.stride(1) == 1 and out.shape == (T, H * sp.vdim) and ukv.shape == (H * (sp.dim + sp.vdim), sp.kv_rank)
+    assert b.tiles.dtype == b.ctx.dtype == torch.int32 and b.tiles.is_contiguous() and b.ctx.is_contiguous()
+    a = _base(sp, wt, pages, table, pos, slots, T)
+    rows = torch.empty(b.n_ctx, sp.row, device=q.device, dtype=q.dtype)
+    P, LL, I = ctypes.c_void_p, ctypes.c_longlong, ctypes.c_int
+    fn = _lib.require().kca_latent_gather
+    fn.argtypes, fn.restype = [P, LL, P, I, I, I, P, I, I, P, P], I
+    rc = fn(a.kc, a.k_sp, a.table, a.tstride, a.shift, sp.row, b.ctx.data_ptr(), b.ctx.shape[0], b.max_ctx, rows.data_ptr(),
+            _lib.stream())
+    if rc != 0:
+        raise RuntimeError(f"kca_latent_gather returned status {rc} (unsupported shape/arguments)")
+    _lib.LAUNCHES[0] += 1
+    kv = linear(rows[:, :sp.kv_rank], ukv)
+    assert kv.stride(1) == 1
+    a.q, a.kv, a.ldkv, a.kr, a.tiles = q.data_ptr(), kv.data_ptr(), kv.stride(0), rows.data_ptr(), b.tiles.data_ptr()
+    a.sink, a.out, a.ldo = wt.sink.data_ptr(), out.data_ptr(), out.stride(0)
+    _call("kca_latent_tiles", a, b.tiles.shape[0])
     return out
 
 
@@ -169,11 +247,19 @@ def head_mm(x, hx: int, w, y, row_of: torch.Tensor | None = None):
     assert x.stride(1) == 1 and (H - 1) * hx + K <= x.shape[1] and y.is_contiguous() and y.shape[1] == H * N
     assert row_of is None or row_of.dtype == torch.int32
     assert y.shape[0] == (x.shape[0] if row_of is None else row_of.shape[0])
-    fn = _lib.require().kca_head_mm
     P, LL, I = ctypes.c_void_p, ctypes.c_longlong, ctypes.c_int
-    fn.argtypes, fn.restype = [I, P, LL, I, P, P, LL, I, I, I, I, I, P, P], I
-    rc = fn(code, x.data_ptr(), x.stride(0), hx, w.data_ptr(), y.data_ptr(), y.stride(0), N, y.shape[0], H, N, K,
+    args = (x.data_ptr(), x.stride(0), hx, w.data_ptr(), y.data_ptr(), y.stride(0), N, y.shape[0], H, N, K,
             _lib.ptr(row_of), _lib.stream())
+    types = [P, LL, I, P, P, LL, I, I, I, I, I, P, P]
+    rc = 10
+    if code == 1:
+        fn = _lib.require().kca_head_mm_mfma
+        fn.argtypes, fn.restype = types, I
+        rc = fn(*args)
+    if rc == 10:
+        fn = _lib.require().kca_head_mm
+        fn.argtypes, fn.restype = [I] + types, I
+        rc = fn(code, *args)
     if rc != 0:
         raise RuntimeError(f"kca_head_mm returned status {rc} (unsupported shape/arguments)")
     _lib.LAUNCHES[0] += 1
@@ -193,4 +279,5 @@ def _reference(sp, wt, q, pages, table, pos, slots, out, rows):
     return out
 
 
-__all__ = ["LatentHeads", "LatentWeights", "latent_append", "attend_rows", "rows_plan", "head_mm", "rotate"]
+__all__ = ["LatentHeads", "LatentWeights", "Prompts", "latent_append", "attend_rows", "attend_prompts", "plan_prompts",
+           "tiles_ok", "rows_plan", "head_mm", "rotate"]

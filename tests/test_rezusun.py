@@ -412,8 +412,8 @@ class Latent:
             q = torch.nn.functional.linear(la.latent_append(sp, wt, x, pages, table, pos, slot), uq)
             a = (sp, wt, q, pages, table, pos, slot, out)
             if n > 1 and device == "cuda" and la.tiles_ok(sp, dtype, out.stride(0)):
-                pl = la.plan_prompts(ent, min_rows=2)
-                la.attend_prompts(*a, ukv, {k: i32(v) for k, v in pl.items()}, torch.nn.functional.linear)
+                arr, num = la.plan_prompts(ent, min_rows=2)
+                la.attend_prompts(*a, ukv, la.Prompts(**{k: i32(v) for k, v in arr.items()}, **num), torch.nn.functional.linear)
             else:
                 la.attend_rows(*a, at + n)
             outs.append(out[:n])
@@ -490,6 +490,18 @@ def test_sink_takes_its_share(device, dtype):
         got = d.run(cuts, device, dtype)
         for h in range(3):
             assert rel(got[:, 32 * h:32 * h + 32], want[:, 32 * h:32 * h + 32]) < (1e-5 if dtype == F32 else 2.5e-2), (cuts, h)
+
+
+@pytest.mark.gpu
+@pytest.mark.parametrize("dim,rot", [(8, 8), (40, 24), (64, 32), (96, 64), (128, 64), (192, 64)])
+@pytest.mark.parametrize("vdim", [24, 64, 128, 200])
+def test_prompt_tile_sizes(dim, rot, vdim):
+    """Every matrix-core instance (padded and exact head sizes), a second portion in mid-page."""
+    d = Latent(latent(2, dim, rot, vdim, 24, 40), 150, seed=90)
+    assert la.tiles_ok(d.sp, BF16, 2 * vdim + 16)
+    want = d.want(d.x)
+    assert rel(d.run([150], "cuda", BF16), want) < 2.5e-2
+    assert rel(d.run([37, 113], "cuda", BF16), want) < 2.5e-2
 
 
 @pytest.mark.gpu
