@@ -28,10 +28,11 @@ struct ChunkArgs {
   DeltaArgs d;
   const int* ck;         // [nchunk][4]: first row, rows, first row of the entry, position of the chunk's first row
   const int* en;         // [nent][6]: first row, rows, position, slot, first chunk, chunks
-  bf16_t* m;             // [nchunk][H][DK][DK]: M[c][c']
-  bf16_t* b;             // [nchunk][H][DV][DK]: B^T
-  bf16_t* q;             // [nchunk][H][64][DK]: Q'
-  bf16_t* oo;            // [nchunk][H][DV][64]: O'^T
+  // the maps lie as the run kernel's lanes read them, every fragment of a wave contiguous:
+  bf16_t* m;             // [nchunk][H][DK / 16][DK / 32][64 lanes][8]: M[c = lane & 15][c' = 8 (lane >> 4) ..]
+  bf16_t* b;             // [nchunk][H][DV / 16][DK / 16][64 lanes][4]: B[c = 4 (lane >> 4) ..][v = lane & 15]
+  bf16_t* q;             // [nchunk][H][4][DK / 32][64 lanes][8]: Q'[t = lane & 15][c' = 8 (lane >> 4) ..]
+  bf16_t* oo;            // [nchunk][H][DV / 16][4][64 lanes][4]: O'[t = 4 (lane >> 4) ..][v = lane & 15]
   float* e;              // [nchunk][H][DK]: decay of the whole chunk
 };
 
@@ -69,15 +70,23 @@ __device__ __forceinline__ f32x4 up4(s16x4 v) {
                __uint_as_float(u.y & 0xffff0000u)};
 }
 
+// CPL neighbouring channels as loaded
 template <int CPL>
-__device__ __forceinline__ void ldc(const bf16_t* p, bool ok, float (&v)[CPL]) {
-  if constexpr (CPL == 2) {
-    const uint32_t u = ok ? *reinterpret_cast<const uint32_t*>(p) : 0u;
-    v[0] = __uint_as_float(u << 16);
-    v[1] = __uint_as_float(u & 0xffff0000u);
-  } else {
-    v[0] = ok ? bf2f(*p) : 0.f;
-  }
+__device__ __forceinline__ uint32_t ldr(const bf16_t* p) {
+  if constexpr (CPL == 2) return *reinterpret_cast<const uint32_t*>(p);
+  else return *p;
+}
+template <int CPL>
+__device__ __forceinline__ void unr(uint32_t u, bool ok, float (&v)[CPL]) {
+  v[0] = ok ? __uint_as_float(u << 16) : 0.f;
+  if constexpr (CPL == 2) v[1] = ok ? __uint_as_float(u & 0xffff0000u) : 0.f;
+}
+// sum over the wave, the same scalar for every lane
+__device__ __forceinline__ float wave_total(float x) {
+  x = lanes_reduce<16>(x, [](float a, float b) { return a + b; });
+  x += __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(x), 0x142, 0xa, 0xf, true));  // rows 1, 3 += rows 0, 2
+  x += __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(x), 0x143, 0xc, 0xf, true));  // rows 2, 3 += row 1
+  return __int_as_float(__builtin_amdgcn_readlane(__float_as_int(x), 63));
 }
 template <int CPL>
 __device__ __forceinline__ void stc(bf16_t* p, const float (&v)[CPL]) {
@@ -87,12 +96,12 @@ __device__ __forceinline__ void stc(bf16_t* p, const float (&v)[CPL]) {
 
 template <int KIND, int DK, int DV>
 struct Lds {
-  static constexpr int LK = DK + 8, LV = DV + 8, LA = CT + 8, LN = CT + 4;
+  static constexpr int LK = DK + 8, LV = DV + 8, LA = CT + 8;
   bf16_t lq[CT * LK], lz[CT * LK], rk[CT * LK], rp[KIND == 0 ? CT * LK : 8];  // first the diagonal blocks' operands
   bf16_t v[CT * LV];
   bf16_t azk[CT * LA], aqk[CT * LA], aqp[KIND == 0 ? CT * LA : 8];
-  float n[CT * LN];
-  float ti[4][16][20];
+  bf16_t nb[KIND == 0 ? CT * LA : 8];  // N (KIND 1: -azk)
+  float nd[4][16][20], ti[4][16][20];  // its diagonal blocks, the inverses of I - those
   float tot[8][DK];    // log decay of every 8 tokens
   float et[4][DK];     // decay of every block of 16
   float pre[4][DK];    // decay from the chunk's start to the block's
@@ -117,107 +126,161 @@ __global__ void __launch_bounds__(512) delta_map_kernel(ChunkArgs p) {
   float q[8][CPL], u[8][CPL], pv[8][CPL], G[8][CPL], kn[8];
   {
     const bf16_t* x = reinterpret_cast<const bf16_t*>(a.x);
-    const bf16_t* dw = reinterpret_cast<const bf16_t*>(a.dw);
-    float w0[CPL], ab[CPL];
-    ldc<CPL>(reinterpret_cast<const bf16_t*>(a.w0) + h * a.dk + c0, inc, w0);
-    float A = 0.f;
+    const int t0 = 8 * w, cv = lane * CPV, cs = inc ? c0 : 0, vs = cv < a.dv ? cv : 0;
+    const bool inv = cv < a.dv;
     const int gq = h / (a.H / a.G), nqk = a.G * a.dk;
-    if constexpr (KIND == 0) ldc<CPL>(reinterpret_cast<const bf16_t*>(a.ab) + h * a.dk + c0, inc, ab);
-    else A = expf(bf2f(reinterpret_cast<const bf16_t*>(a.ab)[h]));
-    const int t0 = 8 * w, slot = a.slot[row0], C = 2 * nqk + a.H * a.dv;
-    // rows t0 - 3 .. t0 + 7 of a projection column block through the convolution and silu
-    auto conv = [&](int col, int ch, bool ok, auto cpl, auto&& put) {
-      constexpr int N = decltype(cpl)::value;
-      float in[11][N], tp[4][N];
+    // every load is issued before the first use, at addresses that exist: rows and channels past the end repeat
+    // others and are blanked afterwards
+    uint32_t rw[8], rb[8];
+    const bf16_t* dw = reinterpret_cast<const bf16_t*>(a.dw) + h * a.dk + cs;
+    const uint32_t rw0 = ldr<CPL>(reinterpret_cast<const bf16_t*>(a.w0) + h * a.dk + cs);
+    uint32_t rab = 0;
+    if constexpr (KIND == 0) rab = ldr<CPL>(reinterpret_cast<const bf16_t*>(a.ab) + h * a.dk + cs);
+    else rab = reinterpret_cast<const bf16_t*>(a.ab)[h];
 #pragma unroll
-      for (int i = 0; i < 11; ++i) {
-        const int t = t0 + i - 3, r = row0 + t;
-        if (r >= first) {
-          ldc<N>(x + (long long)r * a.ld + col, ok && t < n, in[i]);
-        } else {  // before this batch's part of the sequence: what its slot keeps
-          const int ps = pos0 + t;
-#pragma unroll
-          for (int e = 0; e < N; ++e)
-            in[i][e] = ok && ps >= 0 && 3 - i < a.taps ? a.ring[((long long)slot * a.taps + ps % a.taps) * C + ch + e] : 0.f;
-        }
-      }
-#pragma unroll
-      for (int i = 0; i < 4; ++i)  // tap i: the row i tokens back
-#pragma unroll
-        for (int e = 0; e < N; ++e)
-          tp[i][e] = ok && i < a.taps ? bf2f(reinterpret_cast<const bf16_t*>(a.conv)[(long long)(ch + e) * a.taps + a.taps - 1 - i]) : 0.f;
+    for (int i = 0; i < 8; ++i) {
+      const long long r = row0 + min(t0 + i, n - 1);
+      rw[i] = ldr<CPL>(dw + r * a.ldw);
+      if constexpr (KIND == 1) rb[i] = x[r * a.ld + a.o_a + h];
+    }
+    if constexpr (KIND == 0) {
+      uint32_t rq[8], rk[8], ra[8], rv[8];
 #pragma unroll
       for (int i = 0; i < 8; ++i) {
-        float y[N];
-#pragma unroll
-        for (int e = 0; e < N; ++e) {
-          float v = tp[0][e] * in[i + 3][e];
-#pragma unroll
-          for (int j = 1; j < 4; ++j) v = fmaf(tp[j][e], in[i + 3 - j][e], v);
-          y[e] = t0 + i < n ? v * __builtin_amdgcn_rcpf(1.f + __expf(-v)) : 0.f;
-        }
-        put(i, y);
+        const bf16_t* xr = x + (long long)(row0 + min(t0 + i, n - 1)) * a.ld + h * a.dk + cs;
+        rq[i] = ldr<CPL>(xr + a.o_q);
+        rk[i] = ldr<CPL>(xr + a.o_k);
+        ra[i] = ldr<CPL>(xr + a.o_a);
+        rv[i] = ldr<CPV>(xr + a.o_v);  // (dk = dv)
       }
-    };
-    if constexpr (KIND == 1) {
-      conv(a.o_q + gq * a.dk + c0, gq * a.dk + c0, inc, std::integral_constant<int, CPL>{},
-           [&](int i, const float (&y)[CPL]) {
-#pragma unroll
-             for (int e = 0; e < CPL; ++e) q[i][e] = y[e];
-           });
-      conv(a.o_k + gq * a.dk + c0, nqk + gq * a.dk + c0, inc, std::integral_constant<int, CPL>{},
-           [&](int i, const float (&y)[CPL]) {
-#pragma unroll
-             for (int e = 0; e < CPL; ++e) u[i][e] = y[e];
-           });
-      const int cv = lane * CPV;
-      conv(a.o_v + h * a.dv + cv, 2 * nqk + h * a.dv + cv, cv < a.dv, std::integral_constant<int, CPV>{},
-           [&](int i, const float (&y)[CPV]) { stc<CPV>(s.v + (t0 + i) * L::LV + cv, y); });
-    } else {
-      const int cv = lane * CPV;
 #pragma unroll
       for (int i = 0; i < 8; ++i) {
         const bool ok = t0 + i < n;
-        const bf16_t* xr = x + (long long)(row0 + t0 + i) * a.ld;
-        ldc<CPL>(xr + a.o_q + h * a.dk + c0, ok && inc, q[i]);
-        ldc<CPL>(xr + a.o_k + h * a.dk + c0, ok && inc, u[i]);
-        ldc<CPL>(xr + a.o_a + h * a.dk + c0, ok && inc, pv[i]);
         float v[CPV];
-        ldc<CPV>(xr + a.o_v + h * a.dv + cv, ok && cv < a.dv, v);
+        unr<CPL>(rq[i], ok && inc, q[i]);
+        unr<CPL>(rk[i], ok && inc, u[i]);
+        unr<CPL>(ra[i], ok && inc, pv[i]);
+        unr<CPV>(rv[i], ok && inv, v);
         stc<CPV>(s.v + (t0 + i) * L::LV + cv, v);
       }
+    } else {
+      // rows t0 - 3 .. t0 + 7 of the three column blocks, then the convolutions
+      uint32_t rq[11], rk[11], rv[11], tq[4], tk[4], tv[4], tq1[4], tk1[4], tv1[4];
+#pragma unroll
+      for (int i = 0; i < 11; ++i) {
+        const bf16_t* xr = x + (long long)min(max(row0 + t0 + i - 3, first), row0 + n - 1) * a.ld;
+        rq[i] = ldr<CPL>(xr + a.o_q + gq * a.dk + cs);
+        rk[i] = ldr<CPL>(xr + a.o_k + gq * a.dk + cs);
+        rv[i] = ldr<CPV>(xr + a.o_v + h * a.dv + vs);
+      }
+      const int chq = gq * a.dk + cs, chk = nqk + chq, chv = 2 * nqk + h * a.dv + vs;
+      const bf16_t* cw = reinterpret_cast<const bf16_t*>(a.conv);
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {  // tap i: the row i tokens back
+        const int o = max(a.taps - 1 - i, 0);
+        tq[i] = cw[chq * a.taps + o];
+        tk[i] = cw[chk * a.taps + o];
+        tv[i] = cw[chv * a.taps + o];
+        if (CPL == 2) tq1[i] = cw[(chq + 1) * a.taps + o], tk1[i] = cw[(chk + 1) * a.taps + o];
+        if (CPV == 2) tv1[i] = cw[(chv + 1) * a.taps + o];
+      }
+      float hq[3][CPL], hk[3][CPL], hv[3][CPV];  // the three rows before
+      if (w == 0 && row0 == first) {             // ... which the sequence's slot keeps
+        const int slot = a.slot[row0], C = 2 * nqk + a.H * a.dv;
+#pragma unroll
+        for (int i = 0; i < 3; ++i) {
+          const int ps = pos0 + i - 3;
+          const bool ok = ps >= 0 && 3 - i < a.taps;
+          const float* r = a.ring + ((long long)slot * a.taps + (ok ? ps % a.taps : 0)) * C;
+#pragma unroll
+          for (int e = 0; e < CPL; ++e) {
+            const float x0 = r[chq + e], x1 = r[chk + e];
+            hq[i][e] = ok ? x0 : 0.f;
+            hk[i][e] = ok ? x1 : 0.f;
+          }
+#pragma unroll
+          for (int e = 0; e < CPV; ++e) {
+            const float x2 = r[chv + e];
+            hv[i][e] = ok ? x2 : 0.f;
+          }
+        }
+      } else {
+#pragma unroll
+        for (int i = 0; i < 3; ++i) {
+          unr<CPL>(rq[i], true, hq[i]);
+          unr<CPL>(rk[i], true, hk[i]);
+          unr<CPV>(rv[i], true, hv[i]);
+        }
+      }
+      auto conv = [&](auto cpl, const auto& hist, const uint32_t(&raw)[11], const uint32_t(&ta)[4], const uint32_t(&tb)[4], bool okc,
+                      auto&& put) {
+        constexpr int N = decltype(cpl)::value;
+        float tp[4][N], p1[N], p2[N], p3[N];
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+          tp[i][0] = i < a.taps ? __uint_as_float(ta[i] << 16) : 0.f;
+          if constexpr (N == 2) tp[i][1] = i < a.taps ? __uint_as_float(tb[i] << 16) : 0.f;
+        }
+#pragma unroll
+        for (int e = 0; e < N; ++e) p3[e] = hist[0][e], p2[e] = hist[1][e], p1[e] = hist[2][e];
+#pragma unroll
+        for (int i = 0; i < 8; ++i) {
+          float z[N], y[N];
+          unr<N>(raw[i + 3], true, z);
+          const bool ok = okc && t0 + i < n;
+#pragma unroll
+          for (int e = 0; e < N; ++e) {
+            const float v = fmaf(tp[3][e], p3[e], fmaf(tp[2][e], p2[e], fmaf(tp[1][e], p1[e], tp[0][e] * z[e])));
+            y[e] = ok ? v * __builtin_amdgcn_rcpf(1.f + __expf(-v)) : 0.f;
+            p3[e] = p2[e];
+            p2[e] = p1[e];
+            p1[e] = z[e];
+          }
+          put(i, y);
+        }
+      };
+      conv(std::integral_constant<int, CPL>{}, hq, rq, tq, tq1, inc, [&](int i, const float (&y)[CPL]) {
+#pragma unroll
+        for (int e = 0; e < CPL; ++e) q[i][e] = y[e];
+      });
+      conv(std::integral_constant<int, CPL>{}, hk, rk, tk, tk1, inc, [&](int i, const float (&y)[CPL]) {
+#pragma unroll
+        for (int e = 0; e < CPL; ++e) u[i][e] = y[e];
+      });
+      conv(std::integral_constant<int, CPV>{}, hv, rv, tv, tv1, inv,
+           [&](int i, const float (&y)[CPV]) { stc<CPV>(s.v + (t0 + i) * L::LV + cv, y); });
     }
-    auto add = [](float x, float y) { return x + y; };
-    float run[CPL];
+    float w0[CPL], ab[CPL], run[CPL];
+    unr<CPL>(rw0, true, w0);
+    if constexpr (KIND == 0) unr<CPL>(rab, true, ab);
+    const float A = KIND == 1 ? __expf(__uint_as_float(rab << 16)) : 0.f;
 #pragma unroll
     for (int e = 0; e < CPL; ++e) run[e] = 0.f;
 #pragma unroll
     for (int i = 0; i < 8; ++i) {
-      const int t = t0 + i;
-      const bool ok = t < n;
+      const bool ok = t0 + i < n;
       float lw[CPL], sk = 0.f, sq = 0.f;
-      ldc<CPL>(dw + (long long)(row0 + t) * a.ldw + h * a.dk + c0, ok && inc, lw);
+      unr<CPL>(rw[i], true, lw);
 #pragma unroll
       for (int e = 0; e < CPL; ++e) {
         sk = fmaf(u[i][e], u[i][e], sk);
         sq = fmaf(q[i][e], q[i][e], sq);
       }
-      sk = lanes_reduce<64>(sk, add) + 1e-6f;
+      sk = wave_total(sk) + 1e-6f;
       const float ik = rsqrtf(sk);
-      float iq = 1.f, beta = 0.f;
+      float iq = 1.f;
+      kn[i] = sk * ik;  // k = u * kn
       if constexpr (KIND == 1) {
-        iq = a.qscale * rsqrtf(lanes_reduce<64>(sq, add) + 1e-6f);
-        beta = ok ? sigmoid(bf2f(x[(long long)(row0 + t) * a.ld + a.o_a + h])) : 0.f;
+        iq = a.qscale * rsqrtf(wave_total(sq) + 1e-6f);
+        kn[i] = ok ? __builtin_amdgcn_rcpf(1.f + __expf(-__uint_as_float(rb[i] << 16))) : 0.f;
       }
-      kn[i] = KIND == 0 ? sk * ik : beta;  // k = u * kn
 #pragma unroll
       for (int e = 0; e < CPL; ++e) {
-        float l = 0.f;
-        if (ok && inc) {
-          if constexpr (KIND == 0) l = -0.60653065971263342f * __builtin_amdgcn_rcpf(1.f + __expf(-(lw[e] + w0[e])));
-          else l = fmaxf(-A * (fmaxf(lw[e] + w0[e], 0.f) + log1pf(__expf(-fabsf(lw[e] + w0[e])))), kFloor);
-        }
-        run[e] += l;
+        const float z = lw[e] + w0[e];
+        float l;
+        if constexpr (KIND == 0) l = -0.60653065971263342f * __builtin_amdgcn_rcpf(1.f + __expf(-z));
+        else l = fmaxf(-A * (fmaxf(z, 0.f) + __logf(1.f + __expf(-fabsf(z)))), kFloor);
+        run[e] += ok && inc ? l : 0.f;
         G[i][e] = run[e];
         u[i][e] *= ik;
         q[i][e] *= iq;
@@ -326,18 +389,18 @@ __global__ void __launch_bounds__(512) delta_map_kernel(ChunkArgs p) {
       for (int r = 0; r < 4; ++r) {
         const int t = 16 * blk + 4 * g4 + r, j = 16 * J + l15;
         (half ? s.aqk : s.azk)[t * L::LA + j] = f2bf(ak[J][r]);
-        if (!half) s.n[t * L::LN + j] = KIND == 0 ? ap[J][r] : -ak[J][r];
-        else if constexpr (KIND == 0) s.aqp[t * L::LA + j] = f2bf(ap[J][r]);
+        if constexpr (KIND == 0) (half ? s.aqp : s.nb)[t * L::LA + j] = f2bf(ap[J][r]);
+        if (!half && J == blk) s.nd[blk][4 * g4 + r][l15] = KIND == 0 ? ap[J][r] : -ak[J][r];
       }
-  __syncthreads();
   // ------------------------------------------------- inverses of the diagonal blocks: a lane per column
+  wave_sync();
   if (!half && lane < 16) {
     float x[16];
 #pragma unroll
     for (int r = 0; r < 16; ++r) {
       float v = r == lane ? 1.f : 0.f;
 #pragma unroll
-      for (int k = 0; k < r; ++k) v = fmaf(s.n[(16 * blk + r) * L::LN + 16 * blk + k], x[k], v);
+      for (int k = 0; k < r; ++k) v = fmaf(s.nd[blk][r][k], x[k], v);
       x[r] = v;
       s.ti[blk][r][lane] = v;
     }
@@ -354,7 +417,7 @@ __global__ void __launch_bounds__(512) delta_map_kernel(ChunkArgs p) {
     const bool isw = ct < DK / 16;
     const int col = isw ? ct * 16 : ct * 16 - DK;
     f32x4 X[4];
-    s16x4 vb[4];
+    s16x4 vb[4], sb[4];
 #pragma unroll
     for (int I = 0; I < 4; ++I) {
       f32x4 y = {0.f, 0.f, 0.f, 0.f};
@@ -369,8 +432,9 @@ __global__ void __launch_bounds__(512) delta_map_kernel(ChunkArgs p) {
       }
 #pragma unroll
       for (int J = 0; J < I; ++J)
-        y = mm16f(*reinterpret_cast<const float4*>(s.n + (16 * I + l15) * L::LN + 16 * J + 4 * g4), X[J], y);
+        y = mm16(row4((KIND == 0 ? s.nb : s.azk) + (16 * I + l15) * L::LA + 16 * J + 4 * g4), sb[J], y);
       X[I] = mm16f(*reinterpret_cast<const float4*>(&s.ti[I][l15][4 * g4]), y, f32x4{0.f, 0.f, 0.f, 0.f});
+      sb[I] = KIND == 0 ? pk4(X[I]) : neg4(pk4(X[I]));
     }
     s16x4 xb[4];
 #pragma unroll
@@ -380,6 +444,7 @@ __global__ void __launch_bounds__(512) delta_map_kernel(ChunkArgs p) {
     }
     if (isw) {
       const int cw = col + 4 * g4;  // this lane's four columns c'
+      const int fo = ((col >> 5) * 64 + ((col >> 3 & 2) + (g4 >> 1)) * 16 + l15) * 8 + (g4 & 1) * 4;
 #pragma unroll
       for (int I = 0; I < 4; ++I) {
         const int t = 16 * I + l15;
@@ -389,9 +454,9 @@ __global__ void __launch_bounds__(512) delta_map_kernel(ChunkArgs p) {
 #pragma unroll
         for (int J = 0; J <= I; ++J)
           y = mm16(KIND == 0 ? xb[J] : neg4(xb[J]), row4((KIND == 0 ? s.aqp : s.aqk) + t * L::LA + 16 * J + 4 * g4), y);
-        *reinterpret_cast<s16x4*>(gq + t * DK + cw) = pk4(y);
+        *reinterpret_cast<s16x4*>(gq + I * KS * 512 + fo) = pk4(y);
       }
-#pragma unroll 2
+#pragma unroll 4
       for (int c = 0; c < DK; c += 16) {
         f32x4 y = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
@@ -400,10 +465,9 @@ __global__ void __launch_bounds__(512) delta_map_kernel(ChunkArgs p) {
           if (J) y *= f;
           y = mm16(KIND == 0 ? xb[J] : neg4(xb[J]), tok4<L::LK>(KIND == 0 ? s.rp : s.rk, 16 * J, c), y);
         }
-        *reinterpret_cast<s16x4*>(gm + (c + l15) * DK + cw) = pk4(y);
+        *reinterpret_cast<s16x4*>(gm + (c >> 4) * KS * 512 + fo) = pk4(y);
       }
     } else {
-      const int v = col + l15;
 #pragma unroll
       for (int I = 0; I < 4; ++I) {
         f32x4 y = {0.f, 0.f, 0.f, 0.f};
@@ -417,9 +481,9 @@ __global__ void __launch_bounds__(512) delta_map_kernel(ChunkArgs p) {
             y = mm16(row4(s.aqk + o), xb[J], y);
           }
         }
-        *reinterpret_cast<s16x4*>(go + v * CT + 16 * I + 4 * g4) = pk4(y);
+        *reinterpret_cast<s16x4*>(go + ((col >> 4) * 4 + I) * 256 + lane * 4) = pk4(y);
       }
-#pragma unroll 2
+#pragma unroll 4
       for (int c = 0; c < DK; c += 16) {
         f32x4 y = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
@@ -429,7 +493,7 @@ __global__ void __launch_bounds__(512) delta_map_kernel(ChunkArgs p) {
           if constexpr (KIND == 0) y = mm16(tok4<L::LK>(s.rp, 16 * J, c), xb[J], y);
           y = mm16(tok4<L::LK>(s.rk, 16 * J, c), KIND == 0 ? vb[J] : xb[J], y);
         }
-        *reinterpret_cast<s16x4*>(gb + v * DK + c + 4 * g4) = pk4(y);
+        *reinterpret_cast<s16x4*>(gb + ((col >> 4) * (DK / 16) + (c >> 4)) * 256 + lane * 4) = pk4(y);
       }
     }
   }
@@ -463,20 +527,20 @@ __global__ void __launch_bounds__(256) delta_run_kernel(ChunkArgs p) {
   };
   auto load = [&](int i, Frag& f) {
     const long long cb = (long long)(ch0 + i) * a.H + h;
-    const bf16_t* gm = p.m + cb * DK * DK + (w * (DK / 4) + l15) * DK + 8 * g4;
-    const bf16_t* gq = p.q + cb * CT * DK + (16 * w + l15) * DK + 8 * g4;
+    const bf16_t* gm = p.m + cb * DK * DK + w * MT * KS * 512 + lane * 8;
+    const bf16_t* gq = p.q + cb * CT * DK + w * KS * 512 + lane * 8;
 #pragma unroll
     for (int k = 0; k < KS; ++k) {
 #pragma unroll
-      for (int m = 0; m < MT; ++m) f.m[m][k] = *reinterpret_cast<const bf16x8*>(gm + m * 16 * DK + 32 * k);
-      f.q[k] = *reinterpret_cast<const bf16x8*>(gq + 32 * k);
+      for (int m = 0; m < MT; ++m) f.m[m][k] = *reinterpret_cast<const bf16x8*>(gm + (m * KS + k) * 512);
+      f.q[k] = *reinterpret_cast<const bf16x8*>(gq + k * 512);
     }
 #pragma unroll
     for (int m = 0; m < MT; ++m) {
-      f.b[m] = row4(p.b + cb * DV * DK + v * DK + r0 + 16 * m);
+      f.b[m] = row4(p.b + cb * DV * DK + (vt * (DK / 16) + w * MT + m) * 256 + lane * 4);
       f.e[m] = *reinterpret_cast<const float4*>(p.e + cb * DK + r0 + 16 * m);
     }
-    f.o = row4(p.oo + cb * DV * CT + v * CT + 16 * w + 4 * g4);
+    f.o = row4(p.oo + cb * DV * CT + (vt * 4 + w) * 256 + lane * 4);
   };
   auto chunk = [&](int i, const Frag& f) {
     bf16_t* im = img[i & 1];
@@ -499,23 +563,32 @@ __global__ void __launch_bounds__(256) delta_run_kernel(ChunkArgs p) {
       for (int m = 0; m < MT; ++m) st[m] = mm32(f.m[m][k], x, st[m]);
       o = mm32(f.q[k], x, o);
     }
-    if (v < a.dv)
+    float* op = a.o + ((long long)(row0 + i * CT + 16 * w + 4 * g4) * a.H + h) * a.dv + v;
+    const long long os = (long long)a.H * a.dv;
+    if (vt * 16 + 16 <= a.dv && i * CT + CT <= n) {
 #pragma unroll
-      for (int r = 0; r < 4; ++r) {
-        const int t = i * CT + 16 * w + 4 * g4 + r;
-        if (t < n) a.o[((long long)(row0 + t) * a.H + h) * a.dv + v] = o[r];
-      }
-  };
-  Frag f0, f1;
-  load(0, f0);
-  for (int i = 0; i < nc; i += 2) {  // the next chunk's maps are in flight under this one's products
-    if (i + 1 < nc) load(i + 1, f1);
-    chunk(i, f0);
-    if (i + 1 < nc) {
-      if (i + 2 < nc) load(i + 2, f0);
-      chunk(i + 1, f1);
+      for (int r = 0; r < 4; ++r) op[r * os] = o[r];
+    } else if (v < a.dv) {
+#pragma unroll
+      for (int r = 0; r < 4; ++r)
+        if (i * CT + 16 * w + 4 * g4 + r < n) op[r * os] = o[r];
     }
+  };
+  // two chunks ahead of the products, unconditionally (past the end: the last chunk again)
+  Frag f0, f1, f2;
+  load(0, f0);
+  load(min(1, nc - 1), f1);
+  int i = 0;
+  for (; i + 3 <= nc; i += 3) {
+    load(min(i + 2, nc - 1), f2);
+    chunk(i, f0);
+    load(min(i + 3, nc - 1), f0);
+    chunk(i + 1, f1);
+    load(min(i + 4, nc - 1), f1);
+    chunk(i + 2, f2);
   }
+  if (i < nc) chunk(i, f0);
+  if (i + 1 < nc) chunk(i + 1, f1);
 #pragma unroll
   for (int m = 0; m < MT; ++m)
 #pragma unroll

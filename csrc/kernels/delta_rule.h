@@ -69,14 +69,26 @@ __device__ __forceinline__ float log_decay(float lw, float w0, float A) {
 // silu(convolution) of input column `col` (convolution channel ch) at row t
 template <typename E>
 __device__ __forceinline__ float conv_silu(const DeltaArgs& a, int t, int col, int ch) {
-  const int pos = a.pos[t], back = a.e0 ? t - a.e0[t] : 0, C = 2 * a.G * a.dk + a.H * a.dv;
+  const int pos = a.pos[t], C = 2 * a.G * a.dk + a.H * a.dv;
   const E* x = reinterpret_cast<const E*>(a.x) + (long long)t * a.ld + col;
   const E* w = reinterpret_cast<const E*>(a.conv) + (long long)ch * a.taps + a.taps - 1;
-  float y = 0.f;
-  for (int i = 0; i < a.taps && i <= pos; ++i) {
-    const float v = i <= back ? ld<E>(x - i * a.ld)
-                              : a.ring[((long long)a.slot[t] * a.taps + (pos - i) % a.taps) * C + ch];
-    y = fmaf(ld<E>(w - i), v, y);
+  const float* r = a.ring + (long long)a.slot[t] * a.taps * C + ch;
+  float y = ld<E>(w) * ld<E>(x);
+  if (!a.e0 && a.taps <= 4) {  // one token an entry: the loads of all taps fly together
+    float v[3], c[3];
+#pragma unroll
+    for (int i = 1; i < 4; ++i) {
+      const bool ok = i < a.taps && i <= pos;
+      v[i - 1] = r[(ok ? (pos - i) % a.taps : 0) * C];
+      c[i - 1] = ld<E>(w - (i < a.taps ? i : 0));
+      if (!ok) c[i - 1] = 0.f, v[i - 1] = 0.f;
+    }
+#pragma unroll
+    for (int i = 0; i < 3; ++i) y = fmaf(c[i], v[i], y);
+  } else {
+    const int back = a.e0 ? t - a.e0[t] : 0;
+    for (int i = 1; i < a.taps && i <= pos; ++i)
+      y = fmaf(ld<E>(w - i), i <= back ? ld<E>(x - i * a.ld) : r[((pos - i) % a.taps) * C], y);
   }
   return y / (1.f + expf(-y));
 }
@@ -96,7 +108,7 @@ __device__ __forceinline__ void ring_store(const DeltaArgs& a, int t, int h, int
 }
 
 // LDS of one head: floats
-__host__ __device__ __forceinline__ int prep_floats(int dk, int dv, int rw, int rg) { return 5 * dk + 2 * dv + rw + rg + 32; }
+__host__ __device__ __forceinline__ int prep_floats(int dk, int dv, int rw, int rg) { return 5 * dk + 2 * dv + rw + rg + 64; }
 
 struct Head {
   float *w, *z, *p, *k, *q, *v, *gate, *tw, *tg, *red;
@@ -123,70 +135,117 @@ __device__ __forceinline__ float dot4(const E* row, const float* v, int n, int s
   return lanes_reduce<4>(s, [](float x, float y) { return x + y; });
 }
 
-// vectors of (token row t, head h) in LDS, by the whole workgroup of NT threads
+// sums of two values over the workgroup; `red` holds 2 floats a wave
+__device__ __forceinline__ void block_sum2(float& x, float& y, float* red) {
+  x = wave_sum(x);
+  y = wave_sum(y);
+  if ((threadIdx.x & 63) == 0) red[2 * (threadIdx.x >> 6)] = x, red[2 * (threadIdx.x >> 6) + 1] = y;
+  __syncthreads();
+  x = y = 0.f;
+  for (int i = 0; i < (int)(blockDim.x >> 6); ++i) x += red[2 * i], y += red[2 * i + 1];
+}
+
+// vectors of (token row t, head h) in LDS, by a workgroup of at least max(256, dk) threads
 template <typename E, int KIND>
 __device__ __forceinline__ void prep_head(const DeltaArgs& a, int t, int h, Head& s) {
   const int tid = threadIdx.x, NT = blockDim.x, dk = a.dk, dv = a.dv, sub = tid & 3;
   const E* x = reinterpret_cast<const E*>(a.x) + (long long)t * a.ld;
   const int g = h / (a.H / a.G), nqk = a.G * dk;
-  if (!a.dw)
-    for (int i = tid; i < a.rank_w; i += NT) {
-      const float v = ld<E>(x + a.o_w + i);
-      s.tw[i] = KIND == 0 ? tanh_t<E>(v) : v;
-    }
-  if (KIND == 1 && !a.dg)
-    for (int i = tid; i < a.rank_g; i += NT) s.tg[i] = ld<E>(x + a.o_g + i);
+  // loads whose results are needed late
+  const int cs = tid < dk ? tid : 0;
+  const float w0 = ld<E>(reinterpret_cast<const E*>(a.w0) + h * dk + cs);
+  float al = 0.f, ab = 0.f;
+  if constexpr (KIND == 0) {
+    al = ld<E>(x + a.o_a + h * dk + cs);
+    ab = ld<E>(reinterpret_cast<const E*>(a.ab) + h * dk + cs);
+  } else {
+    al = ld<E>(x + a.o_a + h);
+    ab = ld<E>(reinterpret_cast<const E*>(a.ab) + h);
+  }
+  const int ndot = a.dw ? 0 : dk, ng = (KIND == 1 && !a.dg) ? dv : 0, rw = a.rank_w, rg = a.rank_g;
+  auto dot_row = [&](int i) {
+    return i < ndot ? reinterpret_cast<const E*>(a.lo_w) + (long long)(h * dk + i) * rw
+                    : reinterpret_cast<const E*>(a.lo_g) + (long long)(h * dv + i - ndot) * rg;
+  };
+  // the first turn's low-rank rows
+  U16x8 pre[4];
+  const int i0 = tid / 4, n0 = i0 < ndot ? rw : rg;
+  const bool fast = sizeof(E) == 2 && i0 < ndot + ng && n0 % 8 == 0 && n0 <= 128 &&
+                    ((uintptr_t)a.lo_w & 15) == 0 && ((uintptr_t)a.lo_g & 15) == 0;
+  if (fast) {
+    const E* row = dot_row(i0);
+#pragma unroll
+    for (int j = 0; j < 4; ++j) pre[j] = *reinterpret_cast<const U16x8*>(row + (8 * sub + 32 * j < n0 ? 8 * sub + 32 * j : 0));
+  }
   float sk = 0.f, sq = 0.f;
-  for (int c = tid; c < dk; c += NT) {
-    float q, k;
-    if constexpr (KIND == 0) {
-      q = ld<E>(x + a.o_q + h * dk + c);
-      k = ld<E>(x + a.o_k + h * dk + c);
+  const int items = 2 * dk + dv + (a.dw ? 0 : rw) + (KIND == 1 && !a.dg ? rg : 0);
+  for (int i = tid; i < items; i += NT) {
+    if (i < 2 * dk) {
+      const bool key = i >= dk;
+      const int c = key ? i - dk : i;
+      float v;
+      if constexpr (KIND == 0) v = ld<E>(x + (key ? a.o_k : a.o_q) + h * dk + c);
+      else v = conv_silu<E>(a, t, (key ? a.o_k : a.o_q) + g * dk + c, (key ? nqk : 0) + g * dk + c);
+      (key ? s.k : s.q)[c] = v;
+      if (key) sk = fmaf(v, v, sk);
+      else sq = fmaf(v, v, sq);
+    } else if (i < 2 * dk + dv) {
+      const int c = i - 2 * dk;
+      if constexpr (KIND == 0) {
+        s.v[c] = ld<E>(x + a.o_v + h * dv + c);
+        s.gate[c] = sigmoid(ld<E>(x + a.o_g + h * dv + c));
+      } else {
+        s.v[c] = conv_silu<E>(a, t, a.o_v + h * dv + c, 2 * nqk + h * dv + c);
+        if (a.dg) s.gate[c] = sigmoid(ld<E>(reinterpret_cast<const E*>(a.dg) + (long long)t * a.ldg + h * dv + c));
+      }
     } else {
-      q = conv_silu<E>(a, t, a.o_q + g * dk + c, g * dk + c);
-      k = conv_silu<E>(a, t, a.o_k + g * dk + c, nqk + g * dk + c);
+      const int c = i - 2 * dk - dv;
+      if (!a.dw && c < rw) {
+        const float v = ld<E>(x + a.o_w + c);
+        s.tw[c] = KIND == 0 ? tanh_t<E>(v) : v;
+      } else {
+        s.tg[c - (a.dw ? 0 : rw)] = ld<E>(x + a.o_g + c - (a.dw ? 0 : rw));
+      }
     }
-    s.q[c] = q;
-    s.k[c] = k;
-    sk = fmaf(k, k, sk);
-    sq = fmaf(q, q, sq);
   }
-  for (int c = tid; c < dv; c += NT) {
-    if constexpr (KIND == 0) s.v[c] = ld<E>(x + a.o_v + h * dv + c);
-    else s.v[c] = conv_silu<E>(a, t, a.o_v + h * dv + c, 2 * nqk + h * dv + c);
-  }
-  const float ik = 1.f / sqrtf(block_sum(sk, s.red) + 1e-6f);  // (its barriers also publish tw, tg)
-  const float iq = KIND == 1 ? a.qscale / sqrtf(block_sum(sq, s.red + 16) + 1e-6f) : 1.f;
-  float A = 0.f, beta = 0.f;
-  if constexpr (KIND == 1) {
-    A = ld<E>(reinterpret_cast<const E*>(a.ab) + h);
-    beta = sigmoid(ld<E>(x + a.o_a + h));
-  }
+  block_sum2(sk, sq, s.red);  // (its barrier also publishes the vectors so far)
+  const float ik = 1.f / sqrtf(sk + 1e-6f), iq = KIND == 1 ? a.qscale / sqrtf(sq + 1e-6f) : 1.f;
   // decays (and, channel, gates): four lanes a dot
-  const int ndot = a.dw ? 0 : dk, ng = (KIND == 1 && !a.dg) ? dv : 0;
-  for (int i0 = 0; i0 < ndot + ng; i0 += NT / 4) {
-    const int i = i0 + tid / 4;
-    if (i < ndot) {
-      const float d = dot4<E>(reinterpret_cast<const E*>(a.lo_w) + (long long)(h * dk + i) * a.rank_w, s.tw, a.rank_w, sub);
-      if (sub == 0) s.w[i] = d;
-    } else if (i < ndot + ng) {
-      const int c = i - ndot;
-      const float d = dot4<E>(reinterpret_cast<const E*>(a.lo_g) + (long long)(h * dv + c) * a.rank_g, s.tg, a.rank_g, sub);
-      if (sub == 0) s.gate[c] = sigmoid(d);
+  for (int i = i0; i < ndot + ng; i += NT / 4) {
+    const bool dec = i < ndot;
+    const int n = dec ? rw : rg;
+    const float* v = dec ? s.tw : s.tg;
+    float d = 0.f;
+    if (fast && i == i0) {
+#pragma unroll
+      for (int j = 0; j < 4; ++j) {
+        const int o = 8 * sub + 32 * j;
+        if (o < n)
+#pragma unroll
+          for (int e = 0; e < 8; ++e) d = fmaf(bf2f(pre[j].v[e]), v[o + e], d);
+      }
+      d = lanes_reduce<4>(d, [](float p, float q) { return p + q; });
+    } else {
+      d = dot4<E>(dot_row(i), v, n, sub);
+    }
+    if (sub == 0) {
+      if (dec) s.w[i] = d;
+      else s.gate[i - ndot] = sigmoid(d);
     }
   }
   __syncthreads();
   float qp = 0.f, qk = 0.f;
-  for (int c = tid; c < dk; c += NT) {
+  if (tid < dk) {
+    const int c = tid;
     const float lw = a.dw ? ld<E>(reinterpret_cast<const E*>(a.dw) + (long long)t * a.ldw + h * dk + c) : s.w[c];
-    const float w = expf(log_decay<KIND>(lw, ld<E>(reinterpret_cast<const E*>(a.w0) + h * dk + c), A));
+    const float w = expf(log_decay<KIND>(lw, w0, ab));
     const float k = s.k[c], u = k * ik, q = s.q[c] * iq;
     float p, kw = k;
     if constexpr (KIND == 0) {
-      p = -u * sigmoid(ld<E>(x + a.o_a + h * dk + c) + ld<E>(reinterpret_cast<const E*>(a.ab) + h * dk + c));
+      p = -u * sigmoid(al + ab);
       s.z[c] = u;
     } else {
-      kw = beta * u;
+      kw = sigmoid(al) * u;
       p = -kw;
       s.z[c] = w * u;
     }
@@ -194,15 +253,12 @@ __device__ __forceinline__ void prep_head(const DeltaArgs& a, int t, int h, Head
     s.p[c] = p;
     s.k[c] = kw;
     s.q[c] = q;
-    qp = fmaf(q, p, qp);
-    qk = fmaf(q, kw, qk);
+    qp = q * p;
+    qk = q * kw;
   }
-  for (int c = tid; c < dv; c += NT) {
-    if constexpr (KIND == 0) s.gate[c] = sigmoid(ld<E>(x + a.o_g + h * dv + c));
-    else if (a.dg) s.gate[c] = sigmoid(ld<E>(reinterpret_cast<const E*>(a.dg) + (long long)t * a.ldg + h * dv + c));
-  }
-  s.qp = block_sum(qp, s.red);
-  s.qk = block_sum(qk, s.red + 16);  // (and the vectors are visible to the workgroup)
+  block_sum2(qp, qk, s.red + 32);  // (and the vectors are visible to the workgroup)
+  s.qp = qp;
+  s.qk = qk;
 }
 
 }  // namespace delta

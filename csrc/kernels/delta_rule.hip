@@ -80,7 +80,7 @@ __device__ __forceinline__ void rows_of(const float* src, int dk, int rg, float 
 }
 
 template <typename E, int KIND, int R, int CW>
-__global__ void __launch_bounds__(1024) delta_step_kernel(DeltaArgs a) {
+__global__ void __launch_bounds__(R > 8 ? 512 : 1024) delta_step_kernel(DeltaArgs a) {
   extern __shared__ float smem[];
   const int b = blockIdx.x, h = blockIdx.y, tid = threadIdx.x, wv = tid >> 6, lane = tid & 63, nw = blockDim.x >> 6;
   const int dk = a.dk, dv = a.dv, rg = lane & 15, cg = lane >> 4;
@@ -115,20 +115,22 @@ __global__ void __launch_bounds__(1024) delta_step_kernel(DeltaArgs a) {
           ss = fmaf(o[e], o[e], ss);
         }
   }
-  const float n = 1.f / sqrtf(block_sum(ss, hd.red) / (float)dv + a.eps);
+  float none = 0.f;
+  block_sum2(ss, none, hd.red);
+  const float n = 1.f / sqrtf(ss / (float)dv + a.eps);
   E* out = reinterpret_cast<E*>(a.out) + (long long)b * a.ldo + h * dv;
   const E* gain = reinterpret_cast<const E*>(a.gain) + (KIND == 0 ? h * dv : 0);
   for (int c = tid; c < dv; c += blockDim.x) delta::st<E>(out + c, hd.v[c] * n * delta::ld<E>(gain + c) * hd.gate[c]);
 }
 
 template <typename E, int KIND>
-__global__ void __launch_bounds__(128) delta_prep_kernel(DeltaArgs a) {
+__global__ void __launch_bounds__(256) delta_prep_kernel(DeltaArgs a) {
   extern __shared__ float smem[];
   const int t = a.rows ? a.rows[blockIdx.x] : (int)blockIdx.x, h = blockIdx.y, tid = threadIdx.x, dk = a.dk, dv = a.dv;
   Head hd(smem, dk, dv, a.rank_w, a.rank_g);
   prep_head<E, KIND>(a, t, h, hd);
   float* pk = a.pk + ((long long)blockIdx.x * a.H + h) * pk_stride(dk, dv);
-  for (int c = tid; c < 5 * dk + dv; c += 128) pk[c] = smem[c];  // w z p k q v lie in this order
+  for (int c = tid; c < 5 * dk + dv; c += 256) pk[c] = smem[c];  // w z p k q v lie in this order
   if (tid == 0) {
     pk[5 * dk + dv] = hd.qp;
     pk[5 * dk + dv + 1] = hd.qk;
@@ -182,23 +184,56 @@ __global__ void __launch_bounds__(256) delta_scan_kernel(DeltaArgs a) {
   st.store(S, dk, dv, rg, col);
 }
 
-// a wave per (token, head)
-template <typename E, int KIND>
+// NL lanes per (token, head), V channels each and turn (V = 4: rows aligned to 4 elements)
+template <typename E, int KIND, int NL, int V>
 __global__ void __launch_bounds__(256) delta_gate_kernel(DeltaArgs a, int T) {
-  const long long i = (long long)blockIdx.x * 4 + (threadIdx.x >> 6);
+  struct alignas(sizeof(E) * V) PackE { E v[V]; };
+  struct alignas(4 * V) PackF { float v[V]; };
+  const long long i = ((long long)blockIdx.x * 256 + threadIdx.x) / NL;
   if (i >= (long long)T * a.H) return;
-  const int t = (int)(i / a.H), h = (int)(i - (long long)t * a.H), lane = threadIdx.x & 63, dv = a.dv;
+  const int t = (int)(i / a.H), h = (int)(i - (long long)t * a.H), lane = threadIdx.x % NL, dv = a.dv;
   const float* o = a.o + ((long long)t * a.H + h) * dv;
-  float ss = 0.f;
-  for (int c = lane; c < dv; c += 64) ss = fmaf(o[c], o[c], ss);
-  const float n = 1.f / sqrtf(wave_sum(ss) / (float)dv + a.eps);
   const E* gain = reinterpret_cast<const E*>(a.gain) + (KIND == 0 ? h * dv : 0);
   const E* gt = KIND == 0 ? reinterpret_cast<const E*>(a.x) + (long long)t * a.ld + a.o_g + h * dv
                           : reinterpret_cast<const E*>(a.dg) + (long long)t * a.ldg + h * dv;
   E* out = reinterpret_cast<E*>(a.out) + (long long)t * a.ldo + h * dv;
-  for (int c = lane; c < dv; c += 64) delta::st<E>(out + c, o[c] * n * delta::ld<E>(gain + c) * sigmoid(delta::ld<E>(gt + c)));
+  const int c0 = lane * V;
+  PackF y;
+  PackE g, gn;  // the first turn's operands (the only one for usual head sizes)
+#pragma unroll
+  for (int e = 0; e < V; ++e) y.v[e] = 0.f;
+  if (c0 < dv) {
+    y = *reinterpret_cast<const PackF*>(o + c0);
+    g = *reinterpret_cast<const PackE*>(gt + c0);
+    gn = *reinterpret_cast<const PackE*>(gain + c0);
+  }
+  float ss = 0.f;
+#pragma unroll
+  for (int e = 0; e < V; ++e) ss = fmaf(y.v[e], y.v[e], ss);
+  for (int c = c0 + NL * V; c < dv; c += NL * V) {
+    const PackF x = *reinterpret_cast<const PackF*>(o + c);
+#pragma unroll
+    for (int e = 0; e < V; ++e) ss = fmaf(x.v[e], x.v[e], ss);
+  }
+  ss = lanes_reduce<NL>(ss, [](float p, float q) { return p + q; });
+  const float n = 1.f / sqrtf(ss / (float)dv + a.eps);
+  for (int c = c0; c < dv; c += NL * V) {
+    if (c != c0) {
+      y = *reinterpret_cast<const PackF*>(o + c);
+      g = *reinterpret_cast<const PackE*>(gt + c);
+      gn = *reinterpret_cast<const PackE*>(gain + c);
+    }
+    PackE r;
+#pragma unroll
+    for (int e = 0; e < V; ++e) {
+      const float z = delta::ld<E>(g.v + e);
+      const float sg = sizeof(E) == 4 ? sigmoid(z) : __builtin_amdgcn_rcpf(1.f + __expf(-z));
+      delta::st<E>(r.v + e, y.v[e] * n * delta::ld<E>(gn.v + e) * sg);
+    }
+    *reinterpret_cast<PackE*>(out + c) = r;
+  }
   if constexpr (KIND == 1)
-    if (a.e1[t] - t <= a.taps) ring_store<E>(a, t, h, lane, 64);
+    if (a.e1[t] - t <= a.taps) ring_store<E>(a, t, h, lane, NL);
 }
 
 int rows_r(int dk) {  // rows a lane holds: 16 row groups
@@ -223,7 +258,8 @@ bool wide(const DeltaArgs& a) { return a.dv % 4 == 0 && (uintptr_t)a.state % 16 
 template <typename E, int KIND, int R, int CW>
 int step_go(const DeltaArgs& a, int B, hipStream_t s) {
   int nw = (a.dv + 4 * CW - 1) / (4 * CW);
-  nw = nw < 4 ? 4 : nw > 16 ? 16 : nw;
+  const int most = R > 8 ? 8 : 16;  // (the kernel's launch bound)
+  nw = nw < 4 ? 4 : nw > most ? most : nw;
   const size_t lds = (size_t)prep_floats(a.dk, a.dv, a.rank_w, a.rank_g) * 4;
   if (lds > 64 * 1024) return 10;
   hipLaunchKernelGGL((delta_step_kernel<E, KIND, R, CW>), dim3(B, a.H), dim3(64 * nw), lds, s, a);
@@ -252,12 +288,22 @@ template <typename E, int KIND>
 int prep_go(const DeltaArgs& a, int T, hipStream_t s) {
   const size_t lds = (size_t)prep_floats(a.dk, a.dv, a.rank_w, a.rank_g) * 4;
   if (lds > 64 * 1024) return 10;
-  hipLaunchKernelGGL((delta_prep_kernel<E, KIND>), dim3(T, a.H), dim3(128), lds, s, a);
+  hipLaunchKernelGGL((delta_prep_kernel<E, KIND>), dim3(T, a.H), dim3(256), lds, s, a);
   return hipGetLastError() == hipSuccess ? 0 : 4;
 }
 template <typename E, int KIND>
 int gate_go(const DeltaArgs& a, int T, hipStream_t s) {
-  hipLaunchKernelGGL((delta_gate_kernel<E, KIND>), dim3((unsigned)(((long long)T * a.H + 3) / 4)), dim3(256), 0, s, a, T);
+  const int al = sizeof(E) * 4;
+  const bool v4 = a.dv % 4 == 0 && a.ldo % 4 == 0 && (KIND == 0 ? a.ld % 4 == 0 && a.o_g % 4 == 0 : a.ldg % 4 == 0) &&
+                  (uintptr_t)a.out % al == 0 && (uintptr_t)(KIND == 0 ? a.x : a.dg) % al == 0 && (uintptr_t)a.gain % al == 0 &&
+                  (uintptr_t)a.o % 16 == 0;
+  const long long n = (long long)T * a.H;
+#define GO(NL, V) hipLaunchKernelGGL((delta_gate_kernel<E, KIND, NL, V>), dim3((unsigned)((n * NL + 255) / 256)), dim3(256), 0, s, a, T)
+  if (!v4) GO(64, 1);
+  else if (a.dv <= 64) GO(16, 4);
+  else if (a.dv <= 128) GO(32, 4);
+  else GO(64, 4);
+#undef GO
   return hipGetLastError() == hipSuccess ? 0 : 4;
 }
 

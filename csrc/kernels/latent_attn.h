@@ -24,7 +24,7 @@ struct LatentArgs {
   const void* q;            // [T][H][D + R]
   const void* qa;           // [T][H][C] absorbed queries W_uk^T q
   const void* sink;         // [H]
-  float* part;              // partial softmaxes [rows][H][nsplit][C + 2]: m, l, sum of weighted latents
+  float* part;              // partial softmaxes [rows][H][nsplit][C + 4]: m, l, -, -, sum of weighted latents
   int nsplit, chunk;        // keys per split
   const int* row_of;        // rows kernel: token row of block b (nullable: b)
   const void* wuv;          // [H][E][C]

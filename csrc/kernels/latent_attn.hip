@@ -14,6 +14,35 @@ template <typename E> __device__ __forceinline__ float ex(float x);
 template <> __device__ __forceinline__ float ex<float>(float x) { return expf(x); }
 template <> __device__ __forceinline__ float ex<bf16_t>(float x) { return __expf(x); }
 
+// bf16 rows in multiples of 8 (at most 2048 of either latent): a thread keeps its elements between the passes
+__global__ void __launch_bounds__(256) latent_prep_vec_kernel(LatentArgs a) {
+  __shared__ float red[8];
+  const int t = blockIdx.x, tid = threadIdx.x, pos = a.pos[t], c = tid * 8;
+  const bf16_t* xq = reinterpret_cast<const bf16_t*>(a.x) + (long long)t * a.ld + a.o_q;
+  const bf16_t* xk = reinterpret_cast<const bf16_t*>(a.x) + (long long)t * a.ld + a.o_kv;
+  const long long pg = a.table[(long long)a.slot[t] * a.tstride + (pos >> a.shift)];
+  float q[8], k[8], gq[8], gk[8], sq = 0.f, sk = 0.f;
+  const int tq = c < a.Q ? c : 0, tk = c < a.C ? c : 0;
+  load8(xq + tq, q);
+  load8(xk + tk, k);
+  load8(reinterpret_cast<const bf16_t*>(a.gq) + tq, gq);
+  load8(reinterpret_cast<const bf16_t*>(a.gk) + tk, gk);
+#pragma unroll
+  for (int e = 0; e < 8; ++e) sq = fmaf(q[e], q[e], sq), sk = fmaf(k[e], k[e], sk);
+  sq = wave_sum(c < a.Q ? sq : 0.f);
+  sk = wave_sum(c < a.C ? sk : 0.f);
+  if ((tid & 63) == 0) red[tid >> 6] = sq, red[4 + (tid >> 6)] = sk;
+  bf16_t* row = reinterpret_cast<bf16_t*>(a.kc) + pg * a.k_sp + (long long)(pos & ((1 << a.shift) - 1)) * (a.C + a.R);
+  for (int i = tid - 192; i >= 0 && i < a.R; i += 64) latent::st<bf16_t>(row + a.C + i, rot<bf16_t>(xk + a.C, i, pos, a.freq, a.nr));
+  __syncthreads();
+  const float nq = 1.f / sqrtf((red[0] + red[1] + red[2] + red[3]) / (float)a.Q + a.eps);
+  const float nk = 1.f / sqrtf((red[4] + red[5] + red[6] + red[7]) / (float)a.C + a.eps);
+#pragma unroll
+  for (int e = 0; e < 8; ++e) q[e] *= nq * gq[e], k[e] *= nk * gk[e];
+  if (c < a.Q) store8(reinterpret_cast<bf16_t*>(a.cq) + (long long)t * a.Q + c, q);
+  if (c < a.C) store8(row + c, k);
+}
+
 template <typename E>
 __global__ void __launch_bounds__(256) latent_prep_kernel(LatentArgs a) {
   __shared__ float red[2][4];
@@ -104,11 +133,11 @@ __global__ void __launch_bounds__(256) latent_rows_kernel(LatentArgs a) {
     }
     __syncthreads();
   }
-  float* part = a.part + (((long long)b * a.H + h) * a.nsplit + sp) * (a.C + 2);
+  float* part = a.part + (((long long)b * a.H + h) * a.nsplit + sp) * (a.C + 4);
   if (tid == 0) part[0] = m, part[1] = l;
 #pragma unroll
   for (int i = 0; i < NC; ++i)
-    if (tid + 256 * i < a.C) part[2 + tid + 256 * i] = acc[i];
+    if (tid + 256 * i < a.C) part[4 + tid + 256 * i] = acc[i];
 }
 
 template <typename E>
@@ -117,7 +146,7 @@ __global__ void __launch_bounds__(256) latent_merge_kernel(LatentArgs a) {
   const int b = blockIdx.x, h = blockIdx.y, tid = threadIdx.x, lane = tid & 63, wv = tid >> 6;
   const int row = a.row_of ? a.row_of[b] : b, used = (a.pos[row] + a.chunk) / a.chunk;
   const float sink = ld<E>(reinterpret_cast<const E*>(a.sink) + h);
-  const int st = a.C + 2;
+  const int st = a.C + 4;
   const float* part = a.part + ((long long)b * a.H + h) * a.nsplit * st;
   float M = sink;
   for (int z = 0; z < used; ++z) M = fmaxf(M, part[(long long)z * st]);
@@ -125,7 +154,7 @@ __global__ void __launch_bounds__(256) latent_merge_kernel(LatentArgs a) {
   for (int z = 0; z < used; ++z) L += part[(long long)z * st + 1] * ex<E>(part[(long long)z * st] - M);
   for (int c = tid; c < a.C; c += 256) {
     float v = 0.f;
-    for (int z = 0; z < used; ++z) v = fmaf(ex<E>(part[(long long)z * st] - M), part[(long long)z * st + 2 + c], v);
+    for (int z = 0; z < used; ++z) v = fmaf(ex<E>(part[(long long)z * st] - M), part[(long long)z * st + 4 + c], v);
     o[c] = v / L;
   }
   __syncthreads();
@@ -160,8 +189,12 @@ KCA_API int kca_latent_prep(const LatentArgs* in, int dtype, int T, hipStream_t 
   const LatentArgs& a = *in;
   if (!latent_args_ok(a) || T < 1 || !a.x || !a.cq || !a.gq || !a.gk) return 1;
   if (dtype == 0) hipLaunchKernelGGL((latent_prep_kernel<float>), dim3(T), dim3(256), 0, s, a);
-  else if (dtype == 1) hipLaunchKernelGGL((latent_prep_kernel<bf16_t>), dim3(T), dim3(256), 0, s, a);
-  else return 3;
+  else if (dtype == 1) {
+    const uintptr_t al = (uintptr_t)a.x | (uintptr_t)a.cq | (uintptr_t)a.kc | (uintptr_t)a.gq | (uintptr_t)a.gk;
+    if ((a.Q | a.C | a.R | a.o_q | a.o_kv) % 8 == 0 && a.ld % 8 == 0 && a.k_sp % 8 == 0 && al % 16 == 0 && a.Q <= 2048 && a.C <= 2048)
+      hipLaunchKernelGGL(latent_prep_vec_kernel, dim3(T), dim3(256), 0, s, a);
+    else hipLaunchKernelGGL((latent_prep_kernel<bf16_t>), dim3(T), dim3(256), 0, s, a);
+  } else return 3;
   return hipGetLastError() == hipSuccess ? 0 : 4;
 }
 

@@ -43,17 +43,18 @@ __global__ void __launch_bounds__(256) head_mm_mfma_kernel(const bf16_t* x, long
     if (n0 + 4 * g4 + r < N) yr[r] = f2bf(acc[r]);
 }
 
-// NHG groups of 16 heads; NB 16-column tiles of the latent per wave; NPF 16-B chunks of a tile per thread
+// NHG groups of 16 heads; NB 16-column tiles of the latent per wave; NPF 16-B chunks of a tile per thread.
+// 2 NHG waves, a (32-key tile's half, head group) of the scores each; two workgroups share a CU.
 template <int NHG, int NB, int NPF>
-__global__ void __launch_bounds__(512) latent_rows_mfma_kernel(LatentArgs a) {
-  constexpr int HB = 16 * NHG, BK = 64;
+__global__ void __launch_bounds__(128 * NHG, NHG == 2 ? 2 : 1) latent_rows_mfma_kernel(LatentArgs a) {
+  constexpr int HB = 16 * NHG, BK = 32, NW = 2 * NHG, NT = 64 * NW, LP = BK + 8;
   extern __shared__ __attribute__((aligned(16))) char smem[];
-  const int KL = a.C + a.R, KP = (KL + 31) / 32 * 32, LS = KP + 8, LP = BK + 8;
-  bf16_t* sq = reinterpret_cast<bf16_t*>(smem);       // [HB][LS]
-  bf16_t* sk = sq + HB * LS;                          // [BK][LS]
-  bf16_t* sp = sk + BK * LS;                          // [HB][LP] weights
-  float* smax = reinterpret_cast<float*>(sp + HB * LP);  // [4][HB]
-  float* sl = smax + 4 * HB;                          // [4][HB]
+  const int KL = a.C + a.R, KP = (KL + 31) / 32 * 32, LS = KP + 8;
+  bf16_t* sq = reinterpret_cast<bf16_t*>(smem);          // [HB][LS]
+  bf16_t* sk = sq + HB * LS;                             // [BK][LS]
+  bf16_t* sp = sk + BK * LS;                             // [HB][LP] weights
+  float* smax = reinterpret_cast<float*>(sp + HB * LP);  // [2][HB]
+  float* sl = smax + 2 * HB;                             // [2][HB]
   const int tid = threadIdx.x, lane = tid & 63, w = tid >> 6, l15 = lane & 15, g4 = lane >> 4;
   const int b = blockIdx.x, h0 = blockIdx.y * HB, spl = blockIdx.z;
   const int row = a.row_of ? a.row_of[b] : b, pos = a.pos[row], kv = pos + 1;
@@ -64,46 +65,60 @@ __global__ void __launch_bounds__(512) latent_rows_mfma_kernel(LatentArgs a) {
   const int pmask = (1 << a.shift) - 1, CH = KL / 8, total = BK * CH;
   const bf16_t* kc = reinterpret_cast<const bf16_t*>(a.kc);
 
+  // this thread's chunks of a tile: row in the tile, place in the row's image
+  int tr[NPF], to[NPF];
+#pragma unroll
+  for (int i = 0; i < NPF; ++i) {
+    const int c = min(tid + NT * i, total - 1);
+    tr[i] = c / CH;
+    to[i] = (c - tr[i] * CH) * 8;
+  }
   auto load = [&](int k0, u32x4 (&st)[NPF]) {
 #pragma unroll
     for (int i = 0; i < NPF; ++i) {
-      const int c = tid + 512 * i, r = c / CH, key = k0 + r;
-      st[i] = u32x4{0u, 0u, 0u, 0u};
-      if (c < total && key < hi)
-        st[i] = *reinterpret_cast<const u32x4*>(kc + (long long)tbl[key >> a.shift] * a.k_sp + (long long)(key & pmask) * KL +
-                                                (c - r * CH) * 8);
+      const int key = min(k0 + tr[i], hi - 1);  // (past the end: a repeated row, whose weight is zero)
+      st[i] = *reinterpret_cast<const u32x4*>(kc + (long long)tbl[key >> a.shift] * a.k_sp + (key & pmask) * KL + to[i]);
     }
   };
   auto store = [&](const u32x4 (&st)[NPF]) {
 #pragma unroll
-    for (int i = 0; i < NPF; ++i) {
-      const int c = tid + 512 * i, r = c / CH;
-      if (c < total) *reinterpret_cast<u32x4*>(sk + r * LS + (c - r * CH) * 8) = st[i];
-    }
+    for (int i = 0; i < NPF; ++i)
+      if (tid + NT * i < total) *reinterpret_cast<u32x4*>(sk + tr[i] * LS + to[i]) = st[i];
   };
   u32x4 st[NPF];
   load(lo, st);
   {  // queries: absorbed part, rotated part, zero padding
     const bf16_t* qa = reinterpret_cast<const bf16_t*>(a.qa) + ((long long)b * a.H + h0) * a.C;
     const bf16_t* qr = reinterpret_cast<const bf16_t*>(a.q) + ((long long)row * a.H + h0) * (a.D + a.R) + a.D;
-    for (int i = tid; i < HB * (a.C / 8); i += 512) {
-      const int hh = i / (a.C / 8), c = (i - hh * (a.C / 8)) * 8;
+    const int cc = a.C / 8, rest = KP - a.C, pr = rest / 2;
+    for (int i = tid; i < HB * cc; i += NT) {
+      const int hh = i / cc, c = (i - hh * cc) * 8;
       u32x4 v = {0u, 0u, 0u, 0u};
       if (hh < nh) v = *reinterpret_cast<const u32x4*>(qa + (long long)hh * a.C + c);
       *reinterpret_cast<u32x4*>(sq + hh * LS + c) = v;
     }
-    const int rest = KP - a.C;
-    for (int i = tid; i < HB * rest; i += 512) {
-      const int hh = i / rest, c = i - hh * rest;
-      float v = 0.f;
-      if (hh < nh && c < a.R) v = latent::rot<bf16_t>(qr + (long long)hh * (a.D + a.R), c, pos, a.freq, a.nr);
-      sq[hh * LS + a.C + c] = f2bf(v);
+    for (int i = tid; i < HB * pr; i += NT) {  // pairs
+      const int hh = i / pr, c = (i - hh * pr) * 2;
+      float x = 0.f, y = 0.f;
+      if (hh < nh && c < a.R) {
+        const uint32_t u = *reinterpret_cast<const uint32_t*>(qr + (long long)hh * (a.D + a.R) + c);
+        x = __uint_as_float(u << 16);
+        y = __uint_as_float(u & 0xffff0000u);
+        if (c < a.nr) {
+          float sn, cs;
+          sincosf((float)pos * a.freq[c >> 1], &sn, &cs);
+          const float z = x * cs - y * sn;
+          y = y * cs + x * sn;
+          x = z;
+        }
+      }
+      *reinterpret_cast<uint32_t*>(sq + hh * LS + a.C + c) = pk_bf16(x, y);
     }
     const int pad = KP - KL;
-    for (int i = tid; i < BK * pad; i += 512) sk[(i / pad) * LS + KL + i % pad] = 0;
+    for (int i = tid; i < BK * pad; i += NT) sk[(i / pad) * LS + KL + i % pad] = 0;
   }
   const float sl2 = a.scale * kLog2e;
-  const int kt = w & 3, hg = w >> 2;
+  const int kt = w & 1, hg = w >> 1;
   float m[NHG][4], l[4];
   f32x4 acc[NHG][NB];
 #pragma unroll
@@ -116,83 +131,85 @@ __global__ void __launch_bounds__(512) latent_rows_mfma_kernel(LatentArgs a) {
   for (int g = 0; g < NHG; ++g)
 #pragma unroll
     for (int n = 0; n < NB; ++n) acc[g][n] = f32x4{0.f, 0.f, 0.f, 0.f};
+  const bf16_t* qp = sq + (16 * hg + l15) * LS + 8 * g4;
+  const bf16_t* kp = sk + (16 * kt + l15) * LS + 8 * g4;
   for (int k0 = lo; k0 < hi; k0 += BK) {
     __syncthreads();  // the tile before is read
     store(st);
     __syncthreads();
-    if (k0 + BK < hi) load(k0 + BK, st);
-    f32x4 s = {0.f, 0.f, 0.f, 0.f};
-    if (hg < NHG) {
-      const bf16_t* qp = sq + (16 * hg + l15) * LS + 8 * g4;
-      const bf16_t* kp = sk + (16 * kt + l15) * LS + 8 * g4;
-      f32x4 s2 = {0.f, 0.f, 0.f, 0.f};
-      int k = 0;
-      for (; k + 32 < KP; k += 64) {
-        s = mm32(*reinterpret_cast<const bf16x8*>(qp + k), *reinterpret_cast<const bf16x8*>(kp + k), s);
-        s2 = mm32(*reinterpret_cast<const bf16x8*>(qp + k + 32), *reinterpret_cast<const bf16x8*>(kp + k + 32), s2);
-      }
-      if (k < KP) s = mm32(*reinterpret_cast<const bf16x8*>(qp + k), *reinterpret_cast<const bf16x8*>(kp + k), s);
-      const bool in = k0 + 16 * kt + l15 < hi;
+    load(min(k0 + BK, hi - 1), st);  // (past the end: not used)
+    f32x4 s = {0.f, 0.f, 0.f, 0.f}, s2 = s;
+    int k = 0;
+    for (; k + 128 <= KP; k += 128) {
+      bf16x8 fq[4], fk[4];
 #pragma unroll
-      for (int r = 0; r < 4; ++r) {
-        s[r] = in ? (s[r] + s2[r]) * sl2 : -INFINITY;
-        const float mx = lanes_reduce<16>(s[r], [](float x, float y) { return fmaxf(x, y); });
-        if (l15 == 0) smax[kt * HB + 16 * hg + 4 * g4 + r] = mx;
+      for (int i = 0; i < 4; ++i) {
+        fq[i] = *reinterpret_cast<const bf16x8*>(qp + k + 32 * i);
+        fk[i] = *reinterpret_cast<const bf16x8*>(kp + k + 32 * i);
       }
+      s = mm32(fq[0], fk[0], s);
+      s2 = mm32(fq[1], fk[1], s2);
+      s = mm32(fq[2], fk[2], s);
+      s2 = mm32(fq[3], fk[3], s2);
+    }
+    for (; k < KP; k += 32) s = mm32(*reinterpret_cast<const bf16x8*>(qp + k), *reinterpret_cast<const bf16x8*>(kp + k), s);
+    const bool in = k0 + 16 * kt + l15 < hi;
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      s[r] = in ? (s[r] + s2[r]) * sl2 : -INFINITY;
+      const float mx = lanes_reduce<16>(s[r], [](float x, float y) { return fmaxf(x, y); });
+      if (l15 == 0) smax[kt * HB + 16 * hg + 4 * g4 + r] = mx;
     }
     __syncthreads();
     float al[NHG][4];
+    bool same = true;
 #pragma unroll
     for (int g = 0; g < NHG; ++g)
 #pragma unroll
       for (int r = 0; r < 4; ++r) {
         const float* q = smax + 16 * g + 4 * g4 + r;
-        const float mn = fmaxf(fmaxf(fmaxf(q[0], q[HB]), fmaxf(q[2 * HB], q[3 * HB])), m[g][r]);
+        const float mn = fmaxf(fmaxf(q[0], q[HB]), m[g][r]);
+        same = same && mn == m[g][r];
         al[g][r] = __builtin_amdgcn_exp2f(m[g][r] - mn);
         m[g][r] = mn;
       }
-    if (hg < NHG) {
 #pragma unroll
-      for (int r = 0; r < 4; ++r) {
-        const float mn = NHG == 1 || hg == 0 ? m[0][r] : m[NHG - 1][r];
-        const float am = NHG == 1 || hg == 0 ? al[0][r] : al[NHG - 1][r];
-        const float e = __builtin_amdgcn_exp2f(s[r] - mn);
-        l[r] = fmaf(l[r], am, e);
-        sp[(16 * hg + 4 * g4 + r) * LP + 16 * kt + l15] = f2bf(e);
-      }
+    for (int r = 0; r < 4; ++r) {
+      const float mn = NHG == 1 || hg == 0 ? m[0][r] : m[NHG - 1][r];
+      const float am = NHG == 1 || hg == 0 ? al[0][r] : al[NHG - 1][r];
+      const float e = __builtin_amdgcn_exp2f(s[r] - mn);
+      l[r] = fmaf(l[r], am, e);
+      sp[(16 * hg + 4 * g4 + r) * LP + 16 * kt + l15] = f2bf(e);
     }
-    __syncthreads();
-    bf16x8 pf[NHG][2];
-#pragma unroll
-    for (int g = 0; g < NHG; ++g)
-#pragma unroll
-      for (int k = 0; k < 2; ++k) pf[g][k] = *reinterpret_cast<const bf16x8*>(sp + (16 * g + l15) * LP + 32 * k + 8 * g4);
-#pragma unroll
-    for (int n = 0; n < NB; ++n) {
-      const int c = (w + 8 * n) * 16;
+    if (!__all(same))
 #pragma unroll
       for (int g = 0; g < NHG; ++g)
 #pragma unroll
-        for (int r = 0; r < 4; ++r) acc[g][n][r] *= al[g][r];
+        for (int n = 0; n < NB; ++n)
+#pragma unroll
+          for (int r = 0; r < 4; ++r) acc[g][n][r] *= al[g][r];
+    __syncthreads();
+    bf16x8 pf[NHG];
+#pragma unroll
+    for (int g = 0; g < NHG; ++g) pf[g] = *reinterpret_cast<const bf16x8*>(sp + (16 * g + l15) * LP + 8 * g4);
+#pragma unroll
+    for (int n = 0; n < NB; ++n) {
+      const int c = (w + NW * n) * 16;
       if (c >= a.C) continue;
+      const bf16_t* p0 = sk + (8 * g4 + (l15 >> 2)) * LS + c + 4 * (l15 & 3);
+      const bf16x8 vf = cat8(lds_tr4(reinterpret_cast<const char*>(p0), 0), lds_tr4(reinterpret_cast<const char*>(p0 + 4 * LS), 0));
 #pragma unroll
-      for (int k = 0; k < 2; ++k) {
-        const bf16_t* p0 = sk + (32 * k + 8 * g4 + (l15 >> 2)) * LS + c + 4 * (l15 & 3);
-        const bf16x8 vf = cat8(lds_tr4(reinterpret_cast<const char*>(p0), 0), lds_tr4(reinterpret_cast<const char*>(p0 + 4 * LS), 0));
-#pragma unroll
-        for (int g = 0; g < NHG; ++g) acc[g][n] = mm32(pf[g][k], vf, acc[g][n]);
-      }
+      for (int g = 0; g < NHG; ++g) acc[g][n] = mm32(pf[g], vf, acc[g][n]);
     }
   }
-  // sums of the four key tiles
-  if (hg < NHG)
+  // sums of the two key halves
 #pragma unroll
-    for (int r = 0; r < 4; ++r) {
-      const float t = lanes_reduce<16>(l[r], [](float x, float y) { return x + y; });
-      if (l15 == 0) sl[kt * HB + 16 * hg + 4 * g4 + r] = t;
-    }
+  for (int r = 0; r < 4; ++r) {
+    const float t = lanes_reduce<16>(l[r], [](float x, float y) { return x + y; });
+    if (l15 == 0) sl[kt * HB + 16 * hg + 4 * g4 + r] = t;
+  }
   __syncthreads();
-  const int stp = a.C + 2;
+  const int stp = a.C + 4;
 #pragma unroll
   for (int g = 0; g < NHG; ++g)
 #pragma unroll
@@ -202,77 +219,89 @@ __global__ void __launch_bounds__(512) latent_rows_mfma_kernel(LatentArgs a) {
       float* part = a.part + (((long long)b * a.H + h0 + hh) * a.nsplit + spl) * stp;
       if (w == 0 && l15 == 0) {
         part[0] = m[g][r] * kLn2;
-        part[1] = sl[hh] + sl[HB + hh] + sl[2 * HB + hh] + sl[3 * HB + hh];
+        part[1] = sl[hh] + sl[HB + hh];
       }
 #pragma unroll
       for (int n = 0; n < NB; ++n) {
-        const int c = (w + 8 * n) * 16 + l15;
-        if (c < a.C) part[2 + c] = acc[g][n][r];
+        const int c = (w + NW * n) * 16 + l15;
+        if (c < a.C) part[4 + c] = acc[g][n][r];
       }
     }
 }
 
 constexpr int MSPL = 256;  // splits the merge kernel takes
 
-__global__ void __launch_bounds__(256) latent_merge_mfma_kernel(LatentArgs a, int rows) {
+// MR tokens of a head (a row of the products is a token; rows past MR are zero); 8 waves
+template <int MR>
+__global__ void __launch_bounds__(512) latent_merge_mfma_kernel(LatentArgs a, int rows) {
   extern __shared__ __attribute__((aligned(16))) char smem[];
   const int CP = (a.C + 31) / 32 * 32, LS = CP + 8;
   bf16_t* ob = reinterpret_cast<bf16_t*>(smem);            // [16][LS]
-  float* wz = reinterpret_cast<float*>(ob + 16 * LS);      // [16][nsplit]
+  float* wz = reinterpret_cast<float*>(ob + 16 * LS);      // [MR][nsplit]
   const int tid = threadIdx.x, lane = tid & 63, w = tid >> 6, l15 = lane & 15, g4 = lane >> 4;
-  const int h = blockIdx.y, b0 = blockIdx.x * 16, nb = min(16, rows - b0), st = a.C + 2;
+  const int h = blockIdx.y, b0 = blockIdx.x * MR, nb = min(MR, rows - b0), st = a.C + 4;
   const float sink = bf2f(reinterpret_cast<const bf16_t*>(a.sink)[h]);
-  for (int i = w; i < nb; i += 4) {
+  const bf16x8 zero = {};
+  // W_uv fragments of this wave's first 16 outputs
+  bf16x8 fw[4];
+  const bf16_t* wr = reinterpret_cast<const bf16_t*>(a.wuv) + ((long long)h * a.E + min(w * 16 + l15, a.E - 1)) * a.C;
+#pragma unroll
+  for (int i = 0; i < 4; ++i) fw[i] = 32 * i + 8 * g4 < a.C ? *reinterpret_cast<const bf16x8*>(wr + 32 * i + 8 * g4) : zero;
+  for (int i = w; i < nb; i += 8) {
     const int row = a.row_of ? a.row_of[b0 + i] : b0 + i, used = (a.pos[row] + a.chunk) / a.chunk;
     const float* part = a.part + ((long long)(b0 + i) * a.H + h) * a.nsplit * st;
-    float M = sink;
+    float M = sink, L = 0.f;
     for (int z = lane; z < used; z += 64) M = fmaxf(M, part[(long long)z * st]);
     M = wave_max(M);
-    float L = 0.f;
     for (int z = lane; z < used; z += 64) L += part[(long long)z * st + 1] * __expf(part[(long long)z * st] - M);
     L = 1.f / (wave_sum(L) + __expf(sink - M));
     for (int z = lane; z < used; z += 64) wz[i * a.nsplit + z] = __expf(part[(long long)z * st] - M) * L;
   }
   __syncthreads();
-  const int cb = (CP + 63) / 64;
-  for (int u = w; u < 16 * cb; u += 4) {
-    const int i = u / cb, c = (u - i * cb) * 64 + lane;
-    if (c >= CP) continue;
-    float v = 0.f;
+  // four columns a thread, eight splits' loads in flight
+  const int cq = CP / 4;
+  for (int u = tid; u < 16 * cq; u += 512) {
+    const int i = u / cq, c = (u - i * cq) * 4;
+    float4 v = make_float4(0.f, 0.f, 0.f, 0.f);
     if (i < nb && c < a.C) {
       const int row = a.row_of ? a.row_of[b0 + i] : b0 + i, used = (a.pos[row] + a.chunk) / a.chunk;
-      const float* part = a.part + ((long long)(b0 + i) * a.H + h) * a.nsplit * st + 2 + c;
+      const float* part = a.part + ((long long)(b0 + i) * a.H + h) * a.nsplit * st + 4 + c;
       for (int z0 = 0; z0 < used; z0 += 8) {
-        float x[8];
+        float4 x[8];
 #pragma unroll
-        for (int j = 0; j < 8; ++j) x[j] = part[(long long)min(z0 + j, used - 1) * st];
+        for (int j = 0; j < 8; ++j) x[j] = *reinterpret_cast<const float4*>(part + (long long)min(z0 + j, used - 1) * st);
 #pragma unroll
-        for (int j = 0; j < 8; ++j)
-          if (z0 + j < used) v = fmaf(wz[i * a.nsplit + z0 + j], x[j], v);
+        for (int j = 0; j < 8; ++j) {
+          const float f = z0 + j < used ? wz[i * a.nsplit + z0 + j] : 0.f;
+          v.x = fmaf(f, x[j].x, v.x);
+          v.y = fmaf(f, x[j].y, v.y);
+          v.z = fmaf(f, x[j].z, v.z);
+          v.w = fmaf(f, x[j].w, v.w);
+        }
       }
     }
-    ob[i * LS + c] = f2bf(v);
+    *reinterpret_cast<uint2*>(ob + i * LS + c) = make_uint2(pack_bf16x2(v.x, v.y), pack_bf16x2(v.z, v.w));
   }
   __syncthreads();
   const int b = b0 + l15;
-  const int row = b < rows ? (a.row_of ? a.row_of[b] : b) : 0;
+  const bool live = l15 < nb;
+  const int row = live ? (a.row_of ? a.row_of[b] : b) : 0;
   bf16_t* out = reinterpret_cast<bf16_t*>(a.out) + row * a.ldo + (long long)h * a.E;
-  const bf16x8 zero = {};
-  for (int e0 = w * 16; e0 < a.E; e0 += 64) {
-    const bf16_t* wr = reinterpret_cast<const bf16_t*>(a.wuv) + ((long long)h * a.E + min(e0 + l15, a.E - 1)) * a.C;
+  for (int e0 = w * 16; e0 < a.E; e0 += 128) {
+    const bf16_t* wp = reinterpret_cast<const bf16_t*>(a.wuv) + ((long long)h * a.E + min(e0 + l15, a.E - 1)) * a.C;
     f32x4 acc = {0.f, 0.f, 0.f, 0.f};
     for (int k0 = 0; k0 < CP; k0 += 128) {
       bf16x8 fa[4];
 #pragma unroll
       for (int i = 0; i < 4; ++i) {
         const int k = k0 + 32 * i + 8 * g4;
-        fa[i] = k < a.C ? *reinterpret_cast<const bf16x8*>(wr + k) : zero;
+        fa[i] = k0 == 0 && e0 == w * 16 ? fw[i] : k < a.C ? *reinterpret_cast<const bf16x8*>(wp + k) : zero;
       }
 #pragma unroll
       for (int i = 0; i < 4; ++i)
         if (k0 + 32 * i < CP) acc = mm32(fa[i], *reinterpret_cast<const bf16x8*>(ob + l15 * LS + k0 + 32 * i + 8 * g4), acc);
     }
-    if (b < rows)
+    if (live)
 #pragma unroll
       for (int r = 0; r < 4; ++r)
         if (e0 + 4 * g4 + r < a.E) out[e0 + 4 * g4 + r] = f2bf(acc[r]);
@@ -482,20 +511,23 @@ __global__ void __launch_bounds__(256, DV > 128 ? 1 : 2) latent_tile_kernel(Late
 template <int NHG, int NB, int NPF>
 int rows_go(const LatentArgs& a, int rows, hipStream_t s) {
   const int KP = (a.C + a.R + 31) / 32 * 32, HB = 16 * NHG;
-  const size_t lds = (size_t)(HB + 64) * (KP + 8) * 2 + (size_t)HB * 72 * 2 + (size_t)8 * HB * 4;
-  if (lds > 160 * 1024 || (a.C + a.R) > 64 * NPF) return 10;
+  const size_t lds = (size_t)(HB + 32) * (KP + 8) * 2 + (size_t)HB * 40 * 2 + (size_t)4 * HB * 4;
+  if (lds > 160 * 1024 || 32 * ((a.C + a.R) / 8) > 128 * NHG * NPF || a.C > 32 * NHG * NB) return 10;
   auto kern = latent_rows_mfma_kernel<NHG, NB, NPF>;
   if (hipFuncSetAttribute((const void*)kern, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds) != hipSuccess) return 5;
-  hipLaunchKernelGGL(kern, dim3(rows, (a.H + HB - 1) / HB, a.nsplit), dim3(512), lds, s, a);
+  hipLaunchKernelGGL(kern, dim3(rows, (a.H + HB - 1) / HB, a.nsplit), dim3(128 * NHG), lds, s, a);
   return hipGetLastError() == hipSuccess ? 0 : 4;
 }
-template <int NHG>
-int rows_nb(const LatentArgs& a, int rows, hipStream_t s) {
+int rows_heads(const LatentArgs& a, int rows, hipStream_t s) {
   const int KL = a.C + a.R;
-  if (a.C <= 128) return KL <= 256 ? rows_go<NHG, 1, 4>(a, rows, s) : 10;
-  if (a.C <= 256) return KL <= 256 ? rows_go<NHG, 2, 4>(a, rows, s) : rows_go<NHG, 2, 9>(a, rows, s);
-  if (a.C <= 512) return rows_go<NHG, 4, 9>(a, rows, s);
-  return 10;
+  if (a.H > 16) {
+    if (a.C <= 128 && KL <= 256) return rows_go<2, 2, 4>(a, rows, s);
+    if (a.C <= 256 && KL <= 384) return rows_go<2, 4, 6>(a, rows, s);
+    return rows_go<2, 8, 9>(a, rows, s);
+  }
+  if (a.C <= 128 && KL <= 256) return rows_go<1, 4, 8>(a, rows, s);
+  if (a.C <= 256 && KL <= 384) return rows_go<1, 8, 12>(a, rows, s);
+  return rows_go<1, 16, 18>(a, rows, s);
 }
 
 template <int DK, int DV>
@@ -533,15 +565,19 @@ KCA_API int kca_latent_rows_mfma(const LatentArgs* in, int rows, int max_kv, hip
   if (!latent_args_ok(a) || rows < 1 || !a.q || !a.qa || !a.part || a.nsplit < 1 || a.nsplit > 65535 || a.chunk < 1) return 1;
   if ((long long)a.nsplit * a.chunk < max_kv) return 2;
   if (a.C % 8 || a.R % 8 || a.k_sp % 8 || !al16(a.kc) || !al16(a.qa)) return 10;
-  return a.H > 16 ? rows_nb<2>(a, rows, s) : rows_nb<1>(a, rows, s);
+  return rows_heads(a, rows, s);
 }
 
 KCA_API int kca_latent_merge_mfma(const LatentArgs* in, int rows, hipStream_t s) {
   const LatentArgs& a = *in;
   if (!latent_args_ok(a) || rows < 1 || !a.part || !a.out || !a.wuv || !a.sink || a.chunk < 1 || a.H > 65535) return 1;
   if (a.C % 8 || !al16(a.wuv) || a.nsplit > MSPL || a.C > 1024) return 10;
-  const size_t lds = (size_t)16 * ((a.C + 31) / 32 * 32 + 8) * 2 + (size_t)16 * a.nsplit * 4;
-  hipLaunchKernelGGL(latent_merge_mfma_kernel, dim3((rows + 15) / 16, a.H), dim3(256), lds, s, a, rows);
+  // few tokens: a workgroup each, so that the partials stream on more of them
+  const int mr = rows <= 32 ? 4 : 16;
+  const size_t lds = (size_t)16 * ((a.C + 31) / 32 * 32 + 8) * 2 + (size_t)mr * a.nsplit * 4;
+  const dim3 g((rows + mr - 1) / mr, a.H);
+  if (mr == 4) hipLaunchKernelGGL(latent_merge_mfma_kernel<4>, g, dim3(512), lds, s, a, rows);
+  else hipLaunchKernelGGL(latent_merge_mfma_kernel<16>, g, dim3(512), lds, s, a, rows);
   return hipGetLastError() == hipSuccess ? 0 : 4;
 }
 

@@ -147,7 +147,7 @@ def rows_plan(sp: LatentHeads, rows: int, max_kv: int) -> tuple[int, int, int]:
     chunk = -(-(max_kv if rows * sp.heads >= 4096 else decode_chunk(rows, max(1, sp.heads // 16), max_kv)) // 64) * 64
     chunk = max(chunk, -(-max_kv // (64 * MAX_SPLITS)) * 64)
     n = -(-max_kv // chunk)
-    return n, chunk, rows * sp.heads * n * (sp.kv_rank + 2)
+    return n, chunk, rows * sp.heads * n * (sp.kv_rank + 4)
 
 
 def attend_rows(sp: LatentHeads, wt: LatentWeights, q, pages, table, pos, slots, out, max_kv: int, *,
