@@ -36,7 +36,6 @@ struct ChunkArgs {
   float* e;              // [nchunk][H][DK]: decay of the whole chunk
 };
 
-__device__ __forceinline__ f32x4 mm16(s16x4 a, s16x4 b, f32x4 c) { return __builtin_amdgcn_mfma_f32_16x16x16bf16_1k(a, b, c, 0, 0, 0); }
 __device__ __forceinline__ f32x4 mm32(bf16x8 a, bf16x8 b, f32x4 c) { return __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, b, c, 0, 0, 0); }
 // 16 x 16 x 16 in fp32: a = four consecutive elements of row lane & 15 from column 4 (lane >> 4), b in the
 // accumulators' layout (rows 4 (lane >> 4) + r of column lane & 15)
@@ -46,10 +45,23 @@ __device__ __forceinline__ f32x4 mm16f(float4 a, f32x4 b, f32x4 c) {
   c = __builtin_amdgcn_mfma_f32_16x16x4f32(a.z, b[2], c, 0, 0, 0);
   return __builtin_amdgcn_mfma_f32_16x16x4f32(a.w, b[3], c, 0, 0, 0);
 }
+typedef float f32x2 __attribute__((ext_vector_type(2)));
+typedef __bf16 bf16x2v __attribute__((ext_vector_type(2)));
+__device__ __forceinline__ uint32_t pk2(float lo, float hi) {  // one v_cvt_pk
+  return __builtin_bit_cast(uint32_t, __builtin_convertvector(f32x2{lo, hi}, bf16x2v));
+}
 __device__ __forceinline__ s16x4 pk4(f32x4 v) {
-  const uint2 u = make_uint2(pack_bf16x2(v[0], v[1]), pack_bf16x2(v[2], v[3]));
+  const uint2 u = make_uint2(pk2(v[0], v[1]), pk2(v[2], v[3]));
   return __builtin_bit_cast(s16x4, u);
 }
+// operands of two token blocks side by side: the matrix instruction's 8 slots of a lane group hold its four
+// tokens of either block, on both sides alike
+__device__ __forceinline__ bf16x8 two(s16x4 a, s16x4 b) {
+  return __builtin_bit_cast(bf16x8, __builtin_shufflevector(a, b, 0, 1, 2, 3, 4, 5, 6, 7));
+}
+// one block: the other half of the slots zero. (Not the 16-deep instruction: a sum that passes from one bf16 matrix
+// instruction to another kind of them, into other registers, came out wrong; one kind throughout does not.)
+__device__ __forceinline__ f32x4 mm16(s16x4 a, s16x4 b, f32x4 c) { return mm32(two(a, s16x4{0, 0, 0, 0}), two(b, s16x4{0, 0, 0, 0}), c); }
 __device__ __forceinline__ s16x4 neg4(s16x4 v) {
   uint2 u = __builtin_bit_cast(uint2, v);
   u.x ^= 0x80008000u;
@@ -90,7 +102,7 @@ __device__ __forceinline__ float wave_total(float x) {
 }
 template <int CPL>
 __device__ __forceinline__ void stc(bf16_t* p, const float (&v)[CPL]) {
-  if constexpr (CPL == 2) *reinterpret_cast<uint32_t*>(p) = pack_bf16x2(v[0], v[1]);
+  if constexpr (CPL == 2) *reinterpret_cast<uint32_t*>(p) = pk2(v[0], v[1]);
   else *p = f2bf(v[0]);
 }
 
@@ -98,95 +110,104 @@ template <int KIND, int DK, int DV>
 struct Lds {
   static constexpr int LK = DK + 8, LV = DV + 8, LA = CT + 8;
   bf16_t lq[CT * LK], lz[CT * LK], rk[CT * LK], rp[KIND == 0 ? CT * LK : 8];  // first the diagonal blocks' operands
+  bf16_t lq3[16 * LK], lz3[16 * LK];                        // block 3's rows relative to block 2's start
+  bf16_t rk0[16 * LK], rp0[KIND == 0 ? 16 * LK : 8];        // block 0's columns relative to block 1's end
   bf16_t v[CT * LV];
   bf16_t azk[CT * LA], aqk[CT * LA], aqp[KIND == 0 ? CT * LA : 8];
   bf16_t nb[KIND == 0 ? CT * LA : 8];  // N (KIND 1: -azk)
   float nd[4][16][20], ti[4][16][20];  // its diagonal blocks, the inverses of I - those
   float tot[8][DK];    // log decay of every 8 tokens
-  float et[4][DK];     // decay of every block of 16
   float pre[4][DK];    // decay from the chunk's start to the block's
 };
 
+// One wave's operands of an item as loaded: its 8 tokens (KIND 1: and the 3 rows before) of each column block
+template <int KIND>
+struct Raw {
+  static constexpr int NR = KIND == 0 ? 8 : 11;
+  uint32_t q[NR], k[NR], v[NR], a[8], w[8], w0, ab;
+  uint32_t tq[KIND ? 4 : 1], tk[KIND ? 4 : 1], tv[KIND ? 4 : 1];  // taps of two channels
+};
+
+// A workgroup walks (chunk, head) items; an item's loads are issued while the one before is solved.
 template <int KIND, int DK, int DV>
-__global__ void __launch_bounds__(512) delta_map_kernel(ChunkArgs p) {
+__global__ void __launch_bounds__(512) delta_map_kernel(ChunkArgs p, int items) {
   using L = Lds<KIND, DK, DV>;
   constexpr int CPL = DK / 64, CPV = DV / 64, KS = DK / 32;
   extern __shared__ __attribute__((aligned(16))) char smem[];
   L& s = *reinterpret_cast<L*>(smem);
   const DeltaArgs& a = p.d;
   const int tid = threadIdx.x, lane = tid & 63, w = __builtin_amdgcn_readfirstlane(tid >> 6);
-  const int lid = blockIdx.x, ci = lid / a.H, h = lid - ci * a.H;
-  const int* ck = p.ck + ci * 4;
-  const int row0 = ck[0], n = ck[1], first = ck[2], pos0 = ck[3];
   const int l15 = lane & 15, g4 = lane >> 4, blk = w >> 1, half = w & 1;
+  const int c0 = lane * CPL, cv = lane * CPV, t0 = 8 * w;
+  const bool inc = c0 < a.dk, inv = cv < a.dv;
+  const int cs = inc ? c0 : 0, vs = inv ? cv : 0;  // channels that exist
+  const int nqk = a.G * a.dk, per = a.H / a.G;
 
-  // ------------------------------------------------------- vectors of 8 tokens, CPL channels a lane
-  const int c0 = lane * CPL;
-  const bool inc = c0 < a.dk;
-  float q[8][CPL], u[8][CPL], pv[8][CPL], G[8][CPL], kn[8];
-  {
+  // at addresses that exist: rows past the end repeat others and are blanked at their use
+  auto fetch = [&](int item, Raw<KIND>& r) {
+    const int ci = item / a.H, h = item - ci * a.H;
+    const int* ck = p.ck + ci * 4;
+    const int row0 = ck[0], n = ck[1], first = ck[2];
     const bf16_t* x = reinterpret_cast<const bf16_t*>(a.x);
-    const int t0 = 8 * w, cv = lane * CPV, cs = inc ? c0 : 0, vs = cv < a.dv ? cv : 0;
-    const bool inv = cv < a.dv;
-    const int gq = h / (a.H / a.G), nqk = a.G * a.dk;
-    // every load is issued before the first use, at addresses that exist: rows and channels past the end repeat
-    // others and are blanked afterwards
-    uint32_t rw[8], rb[8];
     const bf16_t* dw = reinterpret_cast<const bf16_t*>(a.dw) + h * a.dk + cs;
-    const uint32_t rw0 = ldr<CPL>(reinterpret_cast<const bf16_t*>(a.w0) + h * a.dk + cs);
-    uint32_t rab = 0;
-    if constexpr (KIND == 0) rab = ldr<CPL>(reinterpret_cast<const bf16_t*>(a.ab) + h * a.dk + cs);
-    else rab = reinterpret_cast<const bf16_t*>(a.ab)[h];
+    r.w0 = ldr<CPL>(reinterpret_cast<const bf16_t*>(a.w0) + h * a.dk + cs);
+    if constexpr (KIND == 0) r.ab = ldr<CPL>(reinterpret_cast<const bf16_t*>(a.ab) + h * a.dk + cs);
+    else r.ab = reinterpret_cast<const bf16_t*>(a.ab)[h];
+    const int gq = KIND == 0 ? h : h / per;
+#pragma unroll
+    for (int i = 0; i < Raw<KIND>::NR; ++i) {
+      const int t = KIND == 0 ? t0 + i : t0 + i - 3;
+      const bf16_t* xr = x + (long long)min(KIND == 0 ? row0 + t : max(row0 + t, first), row0 + n - 1) * a.ld;
+      r.q[i] = ldr<CPL>(xr + a.o_q + gq * a.dk + cs);
+      r.k[i] = ldr<CPL>(xr + a.o_k + gq * a.dk + cs);
+      r.v[i] = ldr<CPV>(xr + a.o_v + h * a.dv + vs);
+    }
 #pragma unroll
     for (int i = 0; i < 8; ++i) {
-      const long long r = row0 + min(t0 + i, n - 1);
-      rw[i] = ldr<CPL>(dw + r * a.ldw);
-      if constexpr (KIND == 1) rb[i] = x[r * a.ld + a.o_a + h];
+      const long long t = row0 + min(t0 + i, n - 1);
+      r.w[i] = ldr<CPL>(dw + t * a.ldw);
+      if constexpr (KIND == 0) r.a[i] = ldr<CPL>(x + t * a.ld + a.o_a + h * a.dk + cs);
+      else r.a[i] = x[t * a.ld + a.o_a + h];
     }
-    if constexpr (KIND == 0) {
-      uint32_t rq[8], rk[8], ra[8], rv[8];
+    if constexpr (KIND == 1) {
+      const bf16_t* cw = reinterpret_cast<const bf16_t*>(a.conv);
+      const int chq = gq * a.dk + cs, chk = nqk + chq, chv = 2 * nqk + h * a.dv + vs;
 #pragma unroll
-      for (int i = 0; i < 8; ++i) {
-        const bf16_t* xr = x + (long long)(row0 + min(t0 + i, n - 1)) * a.ld + h * a.dk + cs;
-        rq[i] = ldr<CPL>(xr + a.o_q);
-        rk[i] = ldr<CPL>(xr + a.o_k);
-        ra[i] = ldr<CPL>(xr + a.o_a);
-        rv[i] = ldr<CPV>(xr + a.o_v);  // (dk = dv)
+      for (int i = 0; i < 4; ++i) {  // tap i: the row i tokens back
+        const int o = max(a.taps - 1 - i, 0);
+        r.tq[i] = cw[chq * a.taps + o] | (uint32_t)cw[(chq + CPL - 1) * a.taps + o] << 16;
+        r.tk[i] = cw[chk * a.taps + o] | (uint32_t)cw[(chk + CPL - 1) * a.taps + o] << 16;
+        r.tv[i] = cw[chv * a.taps + o] | (uint32_t)cw[(chv + CPV - 1) * a.taps + o] << 16;
       }
+    }
+  };
+  Raw<KIND> raw;
+  fetch(blockIdx.x, raw);
+#pragma unroll 1
+  for (int item = blockIdx.x; item < items; item += gridDim.x) {
+  const int ci = item / a.H, h = item - ci * a.H;
+  const int* ck = p.ck + ci * 4;
+  const int row0 = ck[0], n = ck[1], first = ck[2], pos0 = ck[3];
+
+  // ------------------------------------------------------- vectors of 8 tokens, CPL channels a lane
+  float q[8][CPL], u[8][CPL], pv[8][CPL], G[8][CPL], kn[8];
+  {
+    if constexpr (KIND == 0) {
 #pragma unroll
       for (int i = 0; i < 8; ++i) {
         const bool ok = t0 + i < n;
         float v[CPV];
-        unr<CPL>(rq[i], ok && inc, q[i]);
-        unr<CPL>(rk[i], ok && inc, u[i]);
-        unr<CPL>(ra[i], ok && inc, pv[i]);
-        unr<CPV>(rv[i], ok && inv, v);
+        unr<CPL>(raw.q[i], ok && inc, q[i]);
+        unr<CPL>(raw.k[i], ok && inc, u[i]);
+        unr<CPL>(raw.a[i], ok && inc, pv[i]);
+        unr<CPV>(raw.v[i], ok && inv, v);
         stc<CPV>(s.v + (t0 + i) * L::LV + cv, v);
       }
     } else {
-      // rows t0 - 3 .. t0 + 7 of the three column blocks, then the convolutions
-      uint32_t rq[11], rk[11], rv[11], tq[4], tk[4], tv[4], tq1[4], tk1[4], tv1[4];
-#pragma unroll
-      for (int i = 0; i < 11; ++i) {
-        const bf16_t* xr = x + (long long)min(max(row0 + t0 + i - 3, first), row0 + n - 1) * a.ld;
-        rq[i] = ldr<CPL>(xr + a.o_q + gq * a.dk + cs);
-        rk[i] = ldr<CPL>(xr + a.o_k + gq * a.dk + cs);
-        rv[i] = ldr<CPV>(xr + a.o_v + h * a.dv + vs);
-      }
-      const int chq = gq * a.dk + cs, chk = nqk + chq, chv = 2 * nqk + h * a.dv + vs;
-      const bf16_t* cw = reinterpret_cast<const bf16_t*>(a.conv);
-#pragma unroll
-      for (int i = 0; i < 4; ++i) {  // tap i: the row i tokens back
-        const int o = max(a.taps - 1 - i, 0);
-        tq[i] = cw[chq * a.taps + o];
-        tk[i] = cw[chk * a.taps + o];
-        tv[i] = cw[chv * a.taps + o];
-        if (CPL == 2) tq1[i] = cw[(chq + 1) * a.taps + o], tk1[i] = cw[(chk + 1) * a.taps + o];
-        if (CPV == 2) tv1[i] = cw[(chv + 1) * a.taps + o];
-      }
       float hq[3][CPL], hk[3][CPL], hv[3][CPV];  // the three rows before
       if (w == 0 && row0 == first) {             // ... which the sequence's slot keeps
         const int slot = a.slot[row0], C = 2 * nqk + a.H * a.dv;
+        const int chq = h / per * a.dk + cs, chk = nqk + chq, chv = 2 * nqk + h * a.dv + vs;
 #pragma unroll
         for (int i = 0; i < 3; ++i) {
           const int ps = pos0 + i - 3;
@@ -207,26 +228,22 @@ __global__ void __launch_bounds__(512) delta_map_kernel(ChunkArgs p) {
       } else {
 #pragma unroll
         for (int i = 0; i < 3; ++i) {
-          unr<CPL>(rq[i], true, hq[i]);
-          unr<CPL>(rk[i], true, hk[i]);
-          unr<CPV>(rv[i], true, hv[i]);
+          unr<CPL>(raw.q[i], true, hq[i]);
+          unr<CPL>(raw.k[i], true, hk[i]);
+          unr<CPV>(raw.v[i], true, hv[i]);
         }
       }
-      auto conv = [&](auto cpl, const auto& hist, const uint32_t(&raw)[11], const uint32_t(&ta)[4], const uint32_t(&tb)[4], bool okc,
-                      auto&& put) {
+      auto conv = [&](auto cpl, const auto& hist, const auto& rw, const auto& tap, bool okc, auto&& put) {
         constexpr int N = decltype(cpl)::value;
         float tp[4][N], p1[N], p2[N], p3[N];
 #pragma unroll
-        for (int i = 0; i < 4; ++i) {
-          tp[i][0] = i < a.taps ? __uint_as_float(ta[i] << 16) : 0.f;
-          if constexpr (N == 2) tp[i][1] = i < a.taps ? __uint_as_float(tb[i] << 16) : 0.f;
-        }
+        for (int i = 0; i < 4; ++i) unr<N>(tap[i], i < a.taps, tp[i]);
 #pragma unroll
         for (int e = 0; e < N; ++e) p3[e] = hist[0][e], p2[e] = hist[1][e], p1[e] = hist[2][e];
 #pragma unroll
         for (int i = 0; i < 8; ++i) {
           float z[N], y[N];
-          unr<N>(raw[i + 3], true, z);
+          unr<N>(rw[i + 3], true, z);
           const bool ok = okc && t0 + i < n;
 #pragma unroll
           for (int e = 0; e < N; ++e) {
@@ -239,28 +256,28 @@ __global__ void __launch_bounds__(512) delta_map_kernel(ChunkArgs p) {
           put(i, y);
         }
       };
-      conv(std::integral_constant<int, CPL>{}, hq, rq, tq, tq1, inc, [&](int i, const float (&y)[CPL]) {
+      conv(std::integral_constant<int, CPL>{}, hq, raw.q, raw.tq, inc, [&](int i, const float (&y)[CPL]) {
 #pragma unroll
         for (int e = 0; e < CPL; ++e) q[i][e] = y[e];
       });
-      conv(std::integral_constant<int, CPL>{}, hk, rk, tk, tk1, inc, [&](int i, const float (&y)[CPL]) {
+      conv(std::integral_constant<int, CPL>{}, hk, raw.k, raw.tk, inc, [&](int i, const float (&y)[CPL]) {
 #pragma unroll
         for (int e = 0; e < CPL; ++e) u[i][e] = y[e];
       });
-      conv(std::integral_constant<int, CPV>{}, hv, rv, tv, tv1, inv,
+      conv(std::integral_constant<int, CPV>{}, hv, raw.v, raw.tv, inv,
            [&](int i, const float (&y)[CPV]) { stc<CPV>(s.v + (t0 + i) * L::LV + cv, y); });
     }
     float w0[CPL], ab[CPL], run[CPL];
-    unr<CPL>(rw0, true, w0);
-    if constexpr (KIND == 0) unr<CPL>(rab, true, ab);
-    const float A = KIND == 1 ? __expf(__uint_as_float(rab << 16)) : 0.f;
+    unr<CPL>(raw.w0, true, w0);
+    if constexpr (KIND == 0) unr<CPL>(raw.ab, true, ab);
+    const float A = KIND == 1 ? __expf(__uint_as_float(raw.ab << 16)) : 0.f;
 #pragma unroll
     for (int e = 0; e < CPL; ++e) run[e] = 0.f;
 #pragma unroll
     for (int i = 0; i < 8; ++i) {
       const bool ok = t0 + i < n;
       float lw[CPL], sk = 0.f, sq = 0.f;
-      unr<CPL>(rw[i], true, lw);
+      unr<CPL>(raw.w[i], true, lw);
 #pragma unroll
       for (int e = 0; e < CPL; ++e) {
         sk = fmaf(u[i][e], u[i][e], sk);
@@ -272,7 +289,7 @@ __global__ void __launch_bounds__(512) delta_map_kernel(ChunkArgs p) {
       kn[i] = sk * ik;  // k = u * kn
       if constexpr (KIND == 1) {
         iq = a.qscale * rsqrtf(wave_total(sq) + 1e-6f);
-        kn[i] = ok ? __builtin_amdgcn_rcpf(1.f + __expf(-__uint_as_float(rb[i] << 16))) : 0.f;
+        kn[i] = ok ? __builtin_amdgcn_rcpf(1.f + __expf(-__uint_as_float(raw.a[i] << 16))) : 0.f;
       }
 #pragma unroll
       for (int e = 0; e < CPL; ++e) {
@@ -291,96 +308,129 @@ __global__ void __launch_bounds__(512) delta_map_kernel(ChunkArgs p) {
     for (int e = 0; e < CPL; ++e) s.tot[w][c0 + e] = run[e];
   }
   __syncthreads();
-  // decays of the blocks, and of what lies before them
+  // decays of what lies before the blocks
   if (tid < DK) {
     float acc = 0.f;
 #pragma unroll
     for (int b = 0; b < 4; ++b) {
       const float t = s.tot[2 * b][tid] + s.tot[2 * b + 1][tid];
-      s.et[b][tid] = __expf(t);
       s.pre[b][tid] = __expf(acc);
       acc += t;
     }
     p.e[((long long)ci * a.H + h) * DK + tid] = __expf(acc);
   }
-  float mid[CPL], tot[CPL];
+  // decays of the tokens relative to their block's middle: f = e^(G - mid); b0: of the token before the first
+  float f[8][CPL], fi[8][CPL], b0[CPL], em[CPL], er[CPL];
 #pragma unroll
   for (int e = 0; e < CPL; ++e) {
-    mid[e] = s.tot[w & ~1][c0 + e];
-    tot[e] = mid[e] + s.tot[w | 1][c0 + e];
-    if (half)
-#pragma unroll
-      for (int i = 0; i < 8; ++i) G[i][e] += mid[e];
-  }
-  // the four operand images relative to `ref` on both sides (diagonal blocks) or to the block's start and end
-  auto image = [&](bool diag) {
+    const float mid = s.tot[w & ~1][c0 + e], late = s.tot[w | 1][c0 + e];
+    em[e] = __expf(mid);   // from the block's start to its middle
+    er[e] = __expf(late);  // ... from there to its end
+    b0[e] = half ? 1.f : __expf(-mid);
 #pragma unroll
     for (int i = 0; i < 8; ++i) {
-      const int o = (8 * w + i) * L::LK + c0;
+      f[i][e] = __expf(half ? G[i][e] : G[i][e] - mid);
+      fi[i][e] = __builtin_amdgcn_rcpf(f[i][e]);
+    }
+  }
+  // The four operand images. PASS 0: relative to the block's middle on both sides (diagonal blocks); 1: to its
+  // start and end, with block 3's rows and block 0's columns also a block further; 2: the columns alone, decayed
+  // to the chunk's end
+  auto image = [&](auto pass) {
+    constexpr int PASS = decltype(pass)::value;
+    float fx[CPL], fe[CPL];
+#pragma unroll
+    for (int e = 0; e < CPL; ++e) {
+      fx[e] = 1.f;
+      fe[e] = PASS ? er[e] : 1.f;
+      if (PASS == 1 && (blk == 3 || blk == 0)) {
+        const int o = blk == 3 ? 4 : 2;
+        fx[e] = __expf(s.tot[o][c0 + e] + s.tot[o + 1][c0 + e]);
+      }
+      if (PASS == 2) {
+        float z = 0.f;
+        for (int o = 2 * blk + 2; o < 8; ++o) z += s.tot[o][c0 + e];
+        fe[e] *= __expf(z);
+      }
+    }
+#pragma unroll
+    for (int i = 0; i < 8; ++i) {
+      const int o = (8 * w + i) * L::LK + c0, o1 = (8 * half + i) * L::LK + c0;
       float yq[CPL], yz[CPL], yk[CPL], yp[CPL];
 #pragma unroll
       for (int e = 0; e < CPL; ++e) {
-        const float before = i ? G[i ? i - 1 : 0][e] : (half ? mid[e] : 0.f);
-        const float lref = diag ? mid[e] : 0.f, rref = diag ? mid[e] : tot[e];
-        const float fl = __expf(G[i][e] - lref), fr = __expf(rref - G[i][e]);
-        yq[e] = q[i][e] * fl;
-        yz[e] = u[i][e] * (KIND == 0 ? __expf(before - lref) : fl);
+        const float fr = fi[i][e] * fe[e];
         yk[e] = u[i][e] * kn[i] * fr;
         if constexpr (KIND == 0) yp[e] = pv[i][e] * fr;
+        if constexpr (PASS < 2) {
+          const float before = i ? f[i ? i - 1 : 0][e] : b0[e];
+          yq[e] = q[i][e] * f[i][e];
+          yz[e] = u[i][e] * (KIND == 0 ? before : f[i][e]);
+          if (PASS == 1) yq[e] *= em[e], yz[e] *= em[e];
+        }
       }
-      stc<CPL>(s.lq + o, yq);
-      stc<CPL>(s.lz + o, yz);
       stc<CPL>(s.rk + o, yk);
       if constexpr (KIND == 0) stc<CPL>(s.rp + o, yp);
+      if constexpr (PASS < 2) {
+        stc<CPL>(s.lq + o, yq);
+        stc<CPL>(s.lz + o, yz);
+      }
+      if constexpr (PASS == 1) {
+        if (blk == 3) {
+#pragma unroll
+          for (int e = 0; e < CPL; ++e) yq[e] *= fx[e], yz[e] *= fx[e];
+          stc<CPL>(s.lq3 + o1, yq);
+          stc<CPL>(s.lz3 + o1, yz);
+        } else if (blk == 0) {
+#pragma unroll
+          for (int e = 0; e < CPL; ++e) {
+            yk[e] *= fx[e];
+            if constexpr (KIND == 0) yp[e] *= fx[e];
+          }
+          stc<CPL>(s.rk0 + o1, yk);
+          if constexpr (KIND == 0) stc<CPL>(s.rp0 + o1, yp);
+        }
+      }
     }
   };
-  image(true);
+  image(std::integral_constant<int, 0>{});
   __syncthreads();
   // ---------------------------------------------- decayed products: rows of block `blk`, z (half 0) or q (half 1)
-  const bf16_t* left = half ? s.lq : s.lz;
   f32x4 ak[4], ap[4];
-  auto block = [&](int J, bool scaled, int s0, int s1) {
+  auto block = [&](int J, const bf16_t* left, const bf16_t* rk, const bf16_t* rp) {
     f32x4 x = {0.f, 0.f, 0.f, 0.f}, y = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
     for (int k = 0; k < KS; ++k) {
-      const int o = k * 32 + 8 * g4;
-      bf16x8 fa = *reinterpret_cast<const bf16x8*>(left + (16 * blk + l15) * L::LK + o);
-      if (scaled) {
-        const U16x8 r = __builtin_bit_cast(U16x8, fa);
-        float v[8], f[8], f2[8];
-        load8f(&s.et[s0][o], f);
-        load8f(&s.et[s1][o], f2);
-        U16x8 z;
-#pragma unroll
-        for (int e = 0; e < 8; ++e) {
-          v[e] = bf2f(r.v[e]) * f[e] * (s1 != s0 ? f2[e] : 1.f);
-          z.v[e] = f2bf(v[e]);
-        }
-        fa = __builtin_bit_cast(bf16x8, z);
-      }
-      x = mm32(fa, *reinterpret_cast<const bf16x8*>(s.rk + (16 * J + l15) * L::LK + o), x);
-      if constexpr (KIND == 0) y = mm32(fa, *reinterpret_cast<const bf16x8*>(s.rp + (16 * J + l15) * L::LK + o), y);
+      const int o = l15 * L::LK + k * 32 + 8 * g4;
+      const bf16x8 fa = *reinterpret_cast<const bf16x8*>(left + o);
+      x = mm32(fa, *reinterpret_cast<const bf16x8*>(rk + o), x);
+      if constexpr (KIND == 0) y = mm32(fa, *reinterpret_cast<const bf16x8*>(rp + o), y);
     }
     ak[J] = x;
     ap[J] = y;
   };
+  constexpr int BR = 16 * L::LK;  // a block's rows
+  const bf16_t *left = (half ? s.lq : s.lz) + blk * BR, *left3 = half ? s.lq3 : s.lz3;
 #pragma unroll
   for (int J = 0; J < 4; ++J)
     if (J == blk) {
-      block(J, false, 0, 0);
+      block(J, left, s.rk + J * BR, s.rp + (KIND == 0 ? J * BR : 0));
 #pragma unroll
       for (int r = 0; r < 4; ++r)
         if (half ? l15 > 4 * g4 + r : l15 >= 4 * g4 + r) ak[J][r] = ap[J][r] = 0.f;
+      if (!half)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) s.nd[blk][4 * g4 + r][l15] = KIND == 0 ? ap[J][r] : -ak[J][r];
     }
   __syncthreads();
-  image(false);
+  image(std::integral_constant<int, 1>{});
   __syncthreads();
 #pragma unroll
   for (int J = 0; J < 3; ++J)
     if (J < blk) {
-      if (J == blk - 1) block(J, false, 0, 0);
-      else if (J == blk - 2) block(J, true, blk - 1, blk - 1);
-      else block(J, true, 1, 2);
+      const bool far = blk >= 2 && J < 2;  // rows from block 2's start, columns to block 1's end
+      block(J, far && blk == 3 ? left3 : left, far && J == 0 ? s.rk0 : s.rk + J * BR,
+            KIND == 1 ? s.rp : far && J == 0 ? s.rp0 : s.rp + J * BR);
     }
 #pragma unroll
   for (int J = 0; J < 4; ++J)
@@ -390,21 +440,22 @@ __global__ void __launch_bounds__(512) delta_map_kernel(ChunkArgs p) {
         const int t = 16 * blk + 4 * g4 + r, j = 16 * J + l15;
         (half ? s.aqk : s.azk)[t * L::LA + j] = f2bf(ak[J][r]);
         if constexpr (KIND == 0) (half ? s.aqp : s.nb)[t * L::LA + j] = f2bf(ap[J][r]);
-        if (!half && J == blk) s.nd[blk][4 * g4 + r][l15] = KIND == 0 ? ap[J][r] : -ak[J][r];
       }
-  // ------------------------------------------------- inverses of the diagonal blocks: a lane per column
-  wave_sync();
-  if (!half && lane < 16) {
+  // inverses of the four diagonal blocks, a lane per (block, column), by a wave without products of its own here
+  if (w == 0) {
     float x[16];
 #pragma unroll
     for (int r = 0; r < 16; ++r) {
-      float v = r == lane ? 1.f : 0.f;
+      float v = r == l15 ? 1.f : 0.f;
 #pragma unroll
-      for (int k = 0; k < r; ++k) v = fmaf(s.nd[blk][r][k], x[k], v);
+      for (int k = 0; k < r; ++k) v = fmaf(s.nd[g4][r][k], x[k], v);
       x[r] = v;
-      s.ti[blk][r][lane] = v;
+      s.ti[g4][r][l15] = v;
     }
   }
+  __syncthreads();
+  image(std::integral_constant<int, 2>{});
+  fetch(min(item + (int)gridDim.x, items - 1), raw);
   __syncthreads();
   // ----------------------------------------------- solve and maps, 16 columns of [W | U] a wave and turn
   const long long cb = (long long)ci * a.H + h;
@@ -412,90 +463,104 @@ __global__ void __launch_bounds__(512) delta_map_kernel(ChunkArgs p) {
   bf16_t* gb = p.b + cb * DV * DK;
   bf16_t* gq = p.q + cb * CT * DK;
   bf16_t* go = p.oo + cb * DV * CT;
-#pragma unroll 1
-  for (int ct = w; ct < (DK + DV) / 16; ct += 8) {
-    const bool isw = ct < DK / 16;
-    const int col = isw ? ct * 16 : ct * 16 - DK;
+  auto solve = [&](int I, f32x4 y, const f32x4* X, const s16x4* sb) {  // (I - N) X = Y, one block row
+    if (I == 1) y = mm16(row4((KIND == 0 ? s.nb : s.azk) + (16 + l15) * L::LA + 4 * g4), sb[0], y);
+    if (I >= 2) {
+      const bf16_t* nr = (KIND == 0 ? s.nb : s.azk) + (16 * I + l15) * L::LA + 4 * g4;
+      y = mm32(two(row4(nr), row4(nr + 16)), two(sb[0], sb[1]), y);
+      if (I == 3) y = mm16(row4(nr + 32), sb[2], y);
+    }
+    return mm16f(*reinterpret_cast<const float4*>(&s.ti[I][l15][4 * g4]), y, f32x4{0.f, 0.f, 0.f, 0.f});
+  };
+  // sum over the token blocks 0 .. I of rows (of A at `rows`) times operands x
+  auto low = [&](const bf16_t* rows, int I, const s16x4* x, f32x4 y, bool rows_first) {
+    const bf16_t* r = rows + (16 * I + l15) * L::LA + 4 * g4;
+    if (I == 0) return rows_first ? mm16(row4(r), x[0], y) : mm16(x[0], row4(r), y);
+    const bf16x8 ra = two(row4(r), row4(r + 16)), xa = two(x[0], x[1]);
+    y = rows_first ? mm32(ra, xa, y) : mm32(xa, ra, y);
+    if (I == 2) y = rows_first ? mm16(row4(r + 32), x[2], y) : mm16(x[2], row4(r + 32), y);
+    if (I == 3) {
+      const bf16x8 rb = two(row4(r + 32), row4(r + 48)), xc = two(x[2], x[3]);
+      y = rows_first ? mm32(rb, xc, y) : mm32(xc, rb, y);
+    }
+    return y;
+  };
+  auto wtile = [&](int col) {  // 16 columns of W -> M, Q'
     f32x4 X[4];
-    s16x4 vb[4], sb[4];
+    s16x4 xb[4], sb[4];
 #pragma unroll
     for (int I = 0; I < 4; ++I) {
-      f32x4 y = {0.f, 0.f, 0.f, 0.f};
-      if (isw) {
-        const float f = s.pre[I][col + l15];
+      f32x4 y;
+      const float fp = s.pre[I][col + l15];
 #pragma unroll
-        for (int r = 0; r < 4; ++r) y[r] = bf2f(s.lz[(16 * I + 4 * g4 + r) * L::LK + col + l15]) * f;
-      } else {
-        vb[I] = tok4<L::LV>(s.v, 16 * I, col);
-#pragma unroll
-        for (int J = 0; J <= I; ++J) y = mm16(row4(s.azk + (16 * I + l15) * L::LA + 16 * J + 4 * g4), vb[J], y);
-      }
-#pragma unroll
-      for (int J = 0; J < I; ++J)
-        y = mm16(row4((KIND == 0 ? s.nb : s.azk) + (16 * I + l15) * L::LA + 16 * J + 4 * g4), sb[J], y);
-      X[I] = mm16f(*reinterpret_cast<const float4*>(&s.ti[I][l15][4 * g4]), y, f32x4{0.f, 0.f, 0.f, 0.f});
-      sb[I] = KIND == 0 ? pk4(X[I]) : neg4(pk4(X[I]));
-    }
-    s16x4 xb[4];
-#pragma unroll
-    for (int I = 0; I < 4; ++I) {
-      if (KIND == 1 && !isw) X[I] = up4(vb[I]) - X[I];  // V - U
+      for (int r = 0; r < 4; ++r) y[r] = bf2f(s.lz[(16 * I + 4 * g4 + r) * L::LK + col + l15]) * fp;
+      X[I] = solve(I, y, X, sb);
       xb[I] = pk4(X[I]);
+      if (KIND == 1) xb[I] = neg4(xb[I]);  // N, P and A_qp carry a minus sign
+      sb[I] = xb[I];
     }
-    if (isw) {
-      const int cw = col + 4 * g4;  // this lane's four columns c'
-      const int fo = ((col >> 5) * 64 + ((col >> 3 & 2) + (g4 >> 1)) * 16 + l15) * 8 + (g4 & 1) * 4;
+    const int cw = col + 4 * g4;  // this lane's four columns c'
+    const int fo = ((col >> 5) * 64 + ((col >> 3 & 2) + (g4 >> 1)) * 16 + l15) * 8 + (g4 & 1) * 4;
 #pragma unroll
-      for (int I = 0; I < 4; ++I) {
-        const int t = 16 * I + l15;
-        f32x4 y = up4(row4(s.lq + t * L::LK + cw));
-        const float4 f = *reinterpret_cast<const float4*>(&s.pre[I][cw]);
-        y[0] *= f.x; y[1] *= f.y; y[2] *= f.z; y[3] *= f.w;
-#pragma unroll
-        for (int J = 0; J <= I; ++J)
-          y = mm16(KIND == 0 ? xb[J] : neg4(xb[J]), row4((KIND == 0 ? s.aqp : s.aqk) + t * L::LA + 16 * J + 4 * g4), y);
-        *reinterpret_cast<s16x4*>(gq + I * KS * 512 + fo) = pk4(y);
-      }
+    for (int I = 0; I < 4; ++I) {
+      f32x4 y = up4(row4(s.lq + (16 * I + l15) * L::LK + cw));
+      const float4 fp = *reinterpret_cast<const float4*>(&s.pre[I][cw]);
+      y[0] *= fp.x; y[1] *= fp.y; y[2] *= fp.z; y[3] *= fp.w;
+      *reinterpret_cast<s16x4*>(gq + I * KS * 512 + fo) = pk4(low(KIND == 0 ? s.aqp : s.aqk, I, xb, y, false));
+    }
+    const bf16x8 x01 = two(xb[0], xb[1]), x23 = two(xb[2], xb[3]);
+    const bf16_t* img = KIND == 0 ? s.rp : s.rk;
 #pragma unroll 4
-      for (int c = 0; c < DK; c += 16) {
-        f32x4 y = {0.f, 0.f, 0.f, 0.f};
+    for (int c = 0; c < DK; c += 16) {
+      f32x4 y = mm32(x01, two(tok4<L::LK>(img, 0, c), tok4<L::LK>(img, 16, c)), f32x4{0.f, 0.f, 0.f, 0.f});
+      y = mm32(x23, two(tok4<L::LK>(img, 32, c), tok4<L::LK>(img, 48, c)), y);
+      *reinterpret_cast<s16x4*>(gm + (c >> 4) * KS * 512 + fo) = pk4(y);
+    }
+  };
+  auto utile = [&](int col) {  // 16 columns of U -> B, O'
+    f32x4 X[4];
+    s16x4 vb[4], xb[4], sb[4];
 #pragma unroll
-        for (int J = 0; J < 4; ++J) {
-          const float f = s.et[J][c + l15];
-          if (J) y *= f;
-          y = mm16(KIND == 0 ? xb[J] : neg4(xb[J]), tok4<L::LK>(KIND == 0 ? s.rp : s.rk, 16 * J, c), y);
-        }
-        *reinterpret_cast<s16x4*>(gm + (c >> 4) * KS * 512 + fo) = pk4(y);
-      }
-    } else {
+    for (int I = 0; I < 4; ++I) vb[I] = tok4<L::LV>(s.v, 16 * I, col);
 #pragma unroll
-      for (int I = 0; I < 4; ++I) {
-        f32x4 y = {0.f, 0.f, 0.f, 0.f};
-#pragma unroll
-        for (int J = 0; J <= I; ++J) {
-          const int o = (16 * I + l15) * L::LA + 16 * J + 4 * g4;
-          if constexpr (KIND == 0) {
-            y = mm16(row4(s.aqp + o), xb[J], y);
-            y = mm16(row4(s.aqk + o), vb[J], y);
-          } else {
-            y = mm16(row4(s.aqk + o), xb[J], y);
-          }
-        }
-        *reinterpret_cast<s16x4*>(go + ((col >> 4) * 4 + I) * 256 + lane * 4) = pk4(y);
-      }
-#pragma unroll 4
-      for (int c = 0; c < DK; c += 16) {
-        f32x4 y = {0.f, 0.f, 0.f, 0.f};
-#pragma unroll
-        for (int J = 0; J < 4; ++J) {
-          const float4 f = *reinterpret_cast<const float4*>(&s.et[J][c + 4 * g4]);
-          if (J) y[0] *= f.x, y[1] *= f.y, y[2] *= f.z, y[3] *= f.w;
-          if constexpr (KIND == 0) y = mm16(tok4<L::LK>(s.rp, 16 * J, c), xb[J], y);
-          y = mm16(tok4<L::LK>(s.rk, 16 * J, c), KIND == 0 ? vb[J] : xb[J], y);
-        }
-        *reinterpret_cast<s16x4*>(gb + ((col >> 4) * (DK / 16) + (c >> 4)) * 256 + lane * 4) = pk4(y);
+    for (int I = 0; I < 4; ++I) {
+      X[I] = solve(I, low(s.azk, I, vb, f32x4{0.f, 0.f, 0.f, 0.f}, true), X, sb);
+      sb[I] = xb[I] = pk4(X[I]);
+      if (KIND == 1) {
+        sb[I] = neg4(sb[I]);
+        xb[I] = pk4(up4(vb[I]) - X[I]);  // V - U
       }
     }
+#pragma unroll
+    for (int I = 0; I < 4; ++I) {
+      f32x4 y = low(KIND == 0 ? s.aqp : s.aqk, I, xb, f32x4{0.f, 0.f, 0.f, 0.f}, true);
+      if constexpr (KIND == 0) y = low(s.aqk, I, vb, y, true);
+      *reinterpret_cast<s16x4*>(go + ((col >> 4) * 4 + I) * 256 + lane * 4) = pk4(y);
+    }
+    const bf16x8 x01 = two(xb[0], xb[1]), x23 = two(xb[2], xb[3]), v01 = two(vb[0], vb[1]), v23 = two(vb[2], vb[3]);
+    const bf16_t* img = KIND == 0 ? s.rp : s.rk;
+#pragma unroll 4
+    for (int c = 0; c < DK; c += 16) {
+      f32x4 y = mm32(two(tok4<L::LK>(img, 0, c), tok4<L::LK>(img, 16, c)), x01, f32x4{0.f, 0.f, 0.f, 0.f});
+      y = mm32(two(tok4<L::LK>(img, 32, c), tok4<L::LK>(img, 48, c)), x23, y);
+      if constexpr (KIND == 0) {
+        y = mm32(two(tok4<L::LK>(s.rk, 0, c), tok4<L::LK>(s.rk, 16, c)), v01, y);
+        y = mm32(two(tok4<L::LK>(s.rk, 32, c), tok4<L::LK>(s.rk, 48, c)), v23, y);
+      }
+      *reinterpret_cast<s16x4*>(gb + ((col >> 4) * (DK / 16) + (c >> 4)) * 256 + lane * 4) = pk4(y);
+    }
+  };
+  if constexpr (DK == 128 && DV == 128) {
+    wtile(16 * w);
+    utile(16 * w);
+  } else {
+#pragma unroll 1
+    for (int ct = w; ct < (DK + DV) / 16; ct += 8) {
+      if (ct < DK / 16) wtile(16 * ct);
+      else utile(16 * ct - DK);
+    }
+  }
+  __syncthreads();  // the next item reuses the LDS
   }
 }
 
@@ -563,15 +628,15 @@ __global__ void __launch_bounds__(256) delta_run_kernel(ChunkArgs p) {
       for (int m = 0; m < MT; ++m) st[m] = mm32(f.m[m][k], x, st[m]);
       o = mm32(f.q[k], x, o);
     }
-    float* op = a.o + ((long long)(row0 + i * CT + 16 * w + 4 * g4) * a.H + h) * a.dv + v;
+    bf16_t* op = reinterpret_cast<bf16_t*>(a.o) + ((long long)(row0 + i * CT + 16 * w + 4 * g4) * a.H + h) * a.dv + v;
     const long long os = (long long)a.H * a.dv;
     if (vt * 16 + 16 <= a.dv && i * CT + CT <= n) {
 #pragma unroll
-      for (int r = 0; r < 4; ++r) op[r * os] = o[r];
+      for (int r = 0; r < 4; ++r) op[r * os] = f2bf(o[r]);
     } else if (v < a.dv) {
 #pragma unroll
       for (int r = 0; r < 4; ++r)
-        if (i * CT + 16 * w + 4 * g4 + r < n) op[r * os] = o[r];
+        if (i * CT + 16 * w + 4 * g4 + r < n) op[r * os] = f2bf(o[r]);
     }
   };
   // two chunks ahead of the products, unconditionally (past the end: the last chunk again)
@@ -604,7 +669,8 @@ int map_go(const ChunkArgs& p, int nchunk, hipStream_t s) {
   constexpr int lds = sizeof(Lds<KIND, DK, DV>);
   static_assert(lds <= 160 * 1024, "LDS");
   if (hipFuncSetAttribute((const void*)kern, hipFuncAttributeMaxDynamicSharedMemorySize, lds) != hipSuccess) return 5;
-  hipLaunchKernelGGL(kern, dim3(nchunk * p.d.H), dim3(512), lds, s, p);
+  const int items = nchunk * p.d.H, per_cu = lds <= 80 * 1024 ? 2 : 1;
+  hipLaunchKernelGGL(kern, dim3(items < 256 * per_cu ? items : 256 * per_cu), dim3(512), lds, s, p, items);
   return hipGetLastError() == hipSuccess ? 0 : 4;
 }
 template <int DK, int DV>

@@ -37,7 +37,7 @@ struct DeltaArgs {
   long long ldo;
   const int* rows;          // prep kernel: token row of prepared row b (nullable: b)
   float* pk;                // prepared vectors [rows][H][pk_stride]: w z p k q [dk], v [dv], q.p, q.k
-  float* o;                 // read-outs [T][H dv]
+  void* o;                  // read-outs [T][H dv] in the compute type
   const int* ent;           // scan kernel: [n][5]: first row, rows, position of the first row, slot, first prepared row
 };
 

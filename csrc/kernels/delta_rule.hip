@@ -137,7 +137,7 @@ __global__ void __launch_bounds__(256) delta_prep_kernel(DeltaArgs a) {
   }
 }
 
-template <int R, int CW>
+template <typename E, int R, int CW>
 __global__ void __launch_bounds__(256) delta_scan_kernel(DeltaArgs a) {
   const int* en = a.ent + blockIdx.x * 5;
   const int row0 = en[0], n = en[1], pos0 = en[2], slot = en[3], pk0 = en[4], h = blockIdx.y;
@@ -148,7 +148,7 @@ __global__ void __launch_bounds__(256) delta_scan_kernel(DeltaArgs a) {
   const int ps = pk_stride(dk, dv);
   const long long step = (long long)a.H * ps;
   const float* pk = a.pk + ((long long)pk0 * a.H + h) * ps;
-  float* o = a.o + (long long)row0 * a.H * dv + h * dv + col;
+  E* o = reinterpret_cast<E*>(a.o) + (long long)row0 * a.H * dv + h * dv + col;
   Cols<R, CW> st;
   st.load(S, dk, dv, rg, col, pos0 > 0);
   float w[R], z[R], p[R], k[R], q[R], v[CW], qp, qk;
@@ -178,7 +178,7 @@ __global__ void __launch_bounds__(256) delta_scan_kernel(DeltaArgs a) {
     if (rg == 0)
 #pragma unroll
       for (int e = 0; e < CW; ++e)
-        if (col + e < dv) o[e] = y[e];
+        if (col + e < dv) delta::st<E>(o + e, y[e]);
     o += (long long)a.H * dv;
   }
   st.store(S, dk, dv, rg, col);
@@ -188,38 +188,36 @@ __global__ void __launch_bounds__(256) delta_scan_kernel(DeltaArgs a) {
 template <typename E, int KIND, int NL, int V>
 __global__ void __launch_bounds__(256) delta_gate_kernel(DeltaArgs a, int T) {
   struct alignas(sizeof(E) * V) PackE { E v[V]; };
-  struct alignas(4 * V) PackF { float v[V]; };
   const long long i = ((long long)blockIdx.x * 256 + threadIdx.x) / NL;
   if (i >= (long long)T * a.H) return;
   const int t = (int)(i / a.H), h = (int)(i - (long long)t * a.H), lane = threadIdx.x % NL, dv = a.dv;
-  const float* o = a.o + ((long long)t * a.H + h) * dv;
+  const E* o = reinterpret_cast<const E*>(a.o) + ((long long)t * a.H + h) * dv;
   const E* gain = reinterpret_cast<const E*>(a.gain) + (KIND == 0 ? h * dv : 0);
   const E* gt = KIND == 0 ? reinterpret_cast<const E*>(a.x) + (long long)t * a.ld + a.o_g + h * dv
                           : reinterpret_cast<const E*>(a.dg) + (long long)t * a.ldg + h * dv;
   E* out = reinterpret_cast<E*>(a.out) + (long long)t * a.ldo + h * dv;
   const int c0 = lane * V;
-  PackF y;
-  PackE g, gn;  // the first turn's operands (the only one for usual head sizes)
+  PackE y, g, gn;  // the first turn's operands (the only one for usual head sizes)
 #pragma unroll
-  for (int e = 0; e < V; ++e) y.v[e] = 0.f;
+  for (int e = 0; e < V; ++e) delta::st<E>(y.v + e, 0.f);
   if (c0 < dv) {
-    y = *reinterpret_cast<const PackF*>(o + c0);
+    y = *reinterpret_cast<const PackE*>(o + c0);
     g = *reinterpret_cast<const PackE*>(gt + c0);
     gn = *reinterpret_cast<const PackE*>(gain + c0);
   }
   float ss = 0.f;
 #pragma unroll
-  for (int e = 0; e < V; ++e) ss = fmaf(y.v[e], y.v[e], ss);
+  for (int e = 0; e < V; ++e) ss = fmaf(delta::ld<E>(y.v + e), delta::ld<E>(y.v + e), ss);
   for (int c = c0 + NL * V; c < dv; c += NL * V) {
-    const PackF x = *reinterpret_cast<const PackF*>(o + c);
+    const PackE x = *reinterpret_cast<const PackE*>(o + c);
 #pragma unroll
-    for (int e = 0; e < V; ++e) ss = fmaf(x.v[e], x.v[e], ss);
+    for (int e = 0; e < V; ++e) ss = fmaf(delta::ld<E>(x.v + e), delta::ld<E>(x.v + e), ss);
   }
   ss = lanes_reduce<NL>(ss, [](float p, float q) { return p + q; });
   const float n = 1.f / sqrtf(ss / (float)dv + a.eps);
   for (int c = c0; c < dv; c += NL * V) {
     if (c != c0) {
-      y = *reinterpret_cast<const PackF*>(o + c);
+      y = *reinterpret_cast<const PackE*>(o + c);
       g = *reinterpret_cast<const PackE*>(gt + c);
       gn = *reinterpret_cast<const PackE*>(gain + c);
     }
@@ -228,7 +226,7 @@ __global__ void __launch_bounds__(256) delta_gate_kernel(DeltaArgs a, int T) {
     for (int e = 0; e < V; ++e) {
       const float z = delta::ld<E>(g.v + e);
       const float sg = sizeof(E) == 4 ? sigmoid(z) : __builtin_amdgcn_rcpf(1.f + __expf(-z));
-      delta::st<E>(r.v + e, y.v[e] * n * delta::ld<E>(gn.v + e) * sg);
+      delta::st<E>(r.v + e, delta::ld<E>(y.v + e) * n * delta::ld<E>(gn.v + e) * sg);
     }
     *reinterpret_cast<PackE*>(out + c) = r;
   }
@@ -272,14 +270,15 @@ int step_r(const DeltaArgs& a, int B, hipStream_t s) {
 #undef F
 }
 
-template <int R, int CW>
+template <typename E, int R, int CW>
 int scan_go(const DeltaArgs& a, int nent, hipStream_t s) {
   const int nblk = (a.dv + 4 * CW - 1) / (4 * CW);
-  hipLaunchKernelGGL((delta_scan_kernel<R, CW>), dim3(nent, a.H, (nblk + 3) / 4), dim3(256), 0, s, a);
+  hipLaunchKernelGGL((delta_scan_kernel<E, R, CW>), dim3(nent, a.H, (nblk + 3) / 4), dim3(256), 0, s, a);
   return hipGetLastError() == hipSuccess ? 0 : 4;
 }
+template <typename E>
 int scan_r(const DeltaArgs& a, int nent, hipStream_t s) {
-#define F(R) (wide(a) ? scan_go<R, 4>(a, nent, s) : scan_go<R, 1>(a, nent, s))
+#define F(R) (wide(a) ? scan_go<E, R, 4>(a, nent, s) : scan_go<E, R, 1>(a, nent, s))
   DELTA_R(F)
 #undef F
 }
@@ -332,10 +331,12 @@ KCA_API int kca_delta_prep(const DeltaArgs* in, int dtype, int kind, int T, hipS
 }
 
 // a.o of nent entries from a.pk; the slots' states advance
-KCA_API int kca_delta_scan(const DeltaArgs* in, int nent, hipStream_t s) {
+KCA_API int kca_delta_scan(const DeltaArgs* in, int dtype, int nent, hipStream_t s) {
   const DeltaArgs& a = *in;
   if (nent < 1 || !a.pk || !a.o || !a.ent || !a.state || a.H < 1 || a.H > 65535 || a.dk < 1 || a.dk > 256 || a.dv < 1) return 1;
-  return scan_r(a, nent, s);
+  if (dtype == 0) return scan_r<float>(a, nent, s);
+  if (dtype == 1) return scan_r<bf16_t>(a, nent, s);
+  return 3;
 }
 
 // a.out of every (token, head) from a.o

@@ -199,7 +199,7 @@ def delta_portions(sp: DeltaHeads, wt: DeltaWeights, x, state, ring, b: Portions
     assert all(t.dtype == torch.int32 and t.is_contiguous() for t in (b.e0, b.e1, b.ent, b.short, b.rows, b.chunked, b.chunks))
     a.e0, a.e1 = b.e0.data_ptr(), b.e1.data_ptr()
     kind, dev, H = 0 if sp.general else 1, x.device, sp.heads
-    o = torch.empty(T, H * sp.vdim, device=dev, dtype=torch.float32)
+    o = torch.empty(T, H * sp.vdim, device=dev, dtype=x.dtype)
     a.o = o.data_ptr()
     chunked = chunks_ok(sp, x.dtype) and b.chunks.shape[0] > 0
     if chunked:
@@ -221,7 +221,7 @@ def delta_portions(sp: DeltaHeads, wt: DeltaWeights, x, state, ring, b: Portions
         pk = torch.empty(n * H * (-(-(5 * sp.dim + sp.vdim + 2) // 4) * 4), device=dev, dtype=torch.float32)
         a.pk, a.rows, a.ent = pk.data_ptr(), _lib.ptr(rows), ent.data_ptr()
         _call("kca_delta_prep", a, code, kind, n)
-        _call("kca_delta_scan", a, ent.shape[0])
+        _call("kca_delta_scan", a, code, ent.shape[0])
     _call("kca_delta_gate", a, code, kind, T)
     return out
 

@@ -17,7 +17,7 @@ import numpy as np
 import torch
 
 from . import _lib
-from .decode import decode_chunk, gather_kv
+from .decode import gather_kv
 from .rms_shift import native_dt
 
 
@@ -144,8 +144,9 @@ def latent_append(sp: LatentHeads, wt: LatentWeights, x, pages, table, pos, slot
 
 def rows_plan(sp: LatentHeads, rows: int, max_kv: int) -> tuple[int, int, int]:
     """(splits, keys per split, partial floats)."""
-    chunk = -(-(max_kv if rows * sp.heads >= 4096 else decode_chunk(rows, max(1, sp.heads // 16), max_kv)) // 64) * 64
-    chunk = max(chunk, -(-max_kv // (64 * MAX_SPLITS)) * 64)
+    want = -(-512 // (rows * -(-sp.heads // 32)))  # two workgroups a CU, 64 keys each at least
+    chunk = max_kv if rows * sp.heads >= 4096 else max(64, -(-max_kv // want))
+    chunk = -(-max(chunk, -(-max_kv // MAX_SPLITS)) // 64) * 64
     n = -(-max_kv // chunk)
     return n, chunk, rows * sp.heads * n * (sp.kv_rank + 4)
 
