@@ -43,7 +43,8 @@ the headline always prints):
                             the same requests without the HTTP layer.
 
 ``--megusun`` runs none of this: it prints one line with Megusun's prefill / decode throughput beside
-GPT-J of equal size and each kernel's distance from its roofline (bench/megusun_bench.py).
+GPT-J of equal size and each kernel's distance from its roofline (bench/megusun_bench.py). ``--rezusun`` does
+the same for Rezusun beside Megusun and GPT-J (bench/rezusun_bench.py).
 
 ``KCA_BENCH_SHARED_GPU=1`` (rehearsal only, parallel/shared_gpu.py): N ranks
 share cuda:0 with gloo collectives staged through the host, so the N > 1 paths
@@ -99,6 +100,8 @@ def main():
     ap.add_argument("--megusun", choices=["models", "kernels", "all"], default=None,
                     help="instead of the headline: Megusun prefill / decode throughput beside GPT-J of equal size "
                          "('models') and kernel rooflines ('kernels'), random weights, one GPU (bench/megusun_bench.py)")
+    ap.add_argument("--rezusun", choices=["models", "kernels", "all"], default=None,
+                    help="the same for Rezusun beside Megusun and GPT-J (bench/rezusun_bench.py)")
     # rehearsal shrink flags (tests/test_bench_shared_gpu.py): NOT the BASELINE config
     ap.add_argument("--layers", type=int, default=0)
     ap.add_argument("--hidden", type=int, default=0)
@@ -117,15 +120,17 @@ def main():
               + json.dumps({"world_size": int(os.environ.get("WORLD_SIZE", "1"))}), flush=True)
         return
 
-    if args.megusun:
-        mb = _load_bench("megusun_bench")
-        rec = {"bench": "megusun", "dtype": "bf16", "data": "synthetic"}
-        if args.megusun != "kernels":
-            rec["models"] = mb.run_models()
-        if args.megusun != "models":
-            rec["kernels"] = mb.run_kernels()
-        print(json.dumps(rec), flush=True)
-        return
+    for design in ("megusun", "rezusun"):
+        what = getattr(args, design)
+        if what:
+            mb = _load_bench(design + "_bench")
+            rec = {"bench": design, "dtype": "bf16", "data": "synthetic"}
+            if what != "kernels":
+                rec["models"] = mb.run_models()
+            if what != "models":
+                rec["kernels"] = mb.run_kernels()
+            print(json.dumps(rec), flush=True)
+            return
 
     import torch
     import torch.distributed as dist
