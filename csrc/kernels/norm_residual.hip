@@ -3,8 +3,10 @@
 //   h_t = N(x_t; g)
 // N(v; g) is a layer norm (v - mean) / sqrt(var + eps) * g or an RMS norm v / sqrt(mean v^2 + eps) * g.
 // a: the sublayer's output rows, b its bias (optional), ls a per-coordinate scale. The stream x is fp32 and
-// double buffered; statistics are two-pass fp32 over registers; h is rounded once.
+// double buffered; h is rounded once. Statistics are fp32 and two-pass within a wave; the waves of a row merge
+// theirs by counts (one barrier a norm). Few rows load gains and scales ahead of the statistics (AHEAD).
 #include "common.h"
+#include "lanes.h"
 
 namespace {
 
@@ -59,25 +61,18 @@ __device__ __forceinline__ void stv(bf16_t* p, const float (&v)[VEC]) {
     for (int i = 0; i < VEC; ++i) p[i] = f2bf(v[i]);
 }
 
-// sum over the NT threads of a row; `red` holds NT / 64 floats of this reduction alone (no barrier before
-// the writes is needed as every reduction of a row has its own)
-template <int NT>
-__device__ __forceinline__ float row_sum(float v, float* red) {
-  v = wave_sum(v);
-  if constexpr (NT == 64) return v;
-  if ((threadIdx.x & 63) == 0) red[threadIdx.x >> 6] = v;
-  __syncthreads();
-  float t = 0.f;
-#pragma unroll
-  for (int i = 0; i < NT / 64; ++i) t += red[i];
-  return t;
-}
+// a vector of parameters as loaded
+template <typename E, int VEC>
+struct alignas(VEC * sizeof(E)) Pack {
+  E v[VEC];
+  __device__ __forceinline__ float at(int i) const { return ldf<E>(v + i); }
+};
 
-template <typename E, int VEC, int NCH, int NT>
+template <typename E, int VEC, int NCH, int NT, bool AHEAD>
 __global__ void __launch_bounds__(256) norm_residual_kernel(NormArgs p) {
   constexpr int RPB = 256 / NT;  // rows of a workgroup (one wave each when NT == 64)
   static_assert(RPB == 1 || NT == 64, "a row is a wave or the workgroup");
-  __shared__ float red[4][NT / 64];
+  __shared__ float2 red[2][NT / 64];  // a norm each
   const int tid = threadIdx.x % NT, d = p.d;
   const int r = blockIdx.x * RPB + threadIdx.x / NT;
   if (r >= p.T) return;  // (whole waves; RPB == 1: never)
@@ -98,51 +93,91 @@ __global__ void __launch_bounds__(256) norm_residual_kernel(NormArgs p) {
       for (int e = 0; e < VEC; ++e) x[c][e] = 0.f;
     }
   }
-  auto stats = [&](float (&q)[NCH][VEC], float* r0, float* r1, float& mean, float& rstd) {
-    mean = 0.f;
+  using P = Pack<E, VEC>;
+  auto par = [&](const void* q, int c) { return *reinterpret_cast<const P*>(reinterpret_cast<const E*>(q) + min((c * NT + tid) * VEC, d - VEC)); };
+  P pgb[AHEAD ? NCH : 1], pls[AHEAD ? NCH : 1], pg[AHEAD ? NCH : 1];
+  if constexpr (AHEAD) {
+#pragma unroll
+    for (int c = 0; c < NCH; ++c) {
+      if (a) pgb[c] = par(p.gb, c);
+      if (a && p.ls) pls[c] = par(p.ls, c);
+      if (p.h) pg[c] = par(p.g, c);
+    }
+  }
+  auto get = [&](const P* ahead, const void* q, int c) {
+    if constexpr (AHEAD) return ahead[c];
+    else return par(q, c);
+  };
+  auto add = [](float u, float w) { return u + w; };
+  // mean and 1 / deviation of a row
+  auto stats = [&](float (&q)[NCH][VEC], float2* rd, float& mean, float& rstd) {
+    auto count = [&](int w) {  // elements of the row's wave w
+      int n = 0;
+#pragma unroll
+      for (int c = 0; c < NCH; ++c) n += min(max(d - (c * NT + 64 * w) * VEC, 0), 64 * VEC);
+      return (float)n;
+    };
+    const int wv = NT == 64 ? 0 : threadIdx.x >> 6;
+    float s = 0.f, ss = 0.f, mw = 0.f;
     if (p.layer) {
-      float s = 0.f;
 #pragma unroll
       for (int c = 0; c < NCH; ++c)
 #pragma unroll
         for (int e = 0; e < VEC; ++e) s += (c * NT + tid) * VEC < d ? q[c][e] : 0.f;
-      mean = row_sum<NT>(s, r0) * inv;
+      s = lanes_reduce<64>(s, add);
+      mw = s * __builtin_amdgcn_rcpf(fmaxf(count(wv), 1.f));
     }
-    float ss = 0.f;
 #pragma unroll
     for (int c = 0; c < NCH; ++c)
 #pragma unroll
       for (int e = 0; e < VEC; ++e) {
-        const float y = (c * NT + tid) * VEC < d ? q[c][e] - mean : 0.f;
+        const float y = (c * NT + tid) * VEC < d ? q[c][e] - mw : 0.f;
         ss = fmaf(y, y, ss);
       }
-    rstd = 1.f / sqrtf(row_sum<NT>(ss, r1) * inv + p.eps);
+    ss = lanes_reduce<64>(ss, add);
+    mean = mw;
+    if constexpr (NT > 64) {
+      if ((threadIdx.x & 63) == 0) rd[wv] = make_float2(s, ss);
+      __syncthreads();
+      float2 o[NT / 64];
+      s = ss = 0.f;
+#pragma unroll
+      for (int i = 0; i < NT / 64; ++i) {
+        o[i] = rd[i];
+        s += o[i].x;
+        ss += o[i].y;
+      }
+      mean = s * inv;  // (RMS norm: 0)
+      if (p.layer)
+#pragma unroll
+        for (int i = 0; i < NT / 64; ++i) {
+          const float n = count(i), off = o[i].x - n * mean;
+          ss = fmaf(off, off * __builtin_amdgcn_rcpf(fmaxf(n, 1.f)), ss);
+        }
+    }
+    rstd = 1.f / sqrtf(ss * inv + p.eps);
   };
   if (a) {
     if (p.bias) {
 #pragma unroll
       for (int c = 0; c < NCH; ++c) {
-        const int i = (c * NT + tid) * VEC;
-        if (i >= d) continue;
-        float b[VEC];
-        ldv<E, VEC>(reinterpret_cast<const E*>(p.bias) + i, b);
+        const P b = par(p.bias, c);
 #pragma unroll
-        for (int e = 0; e < VEC; ++e) v[c][e] += b[e];
+        for (int e = 0; e < VEC; ++e) v[c][e] += b.at(e);
       }
     }
     float mean, rstd;
-    stats(v, red[0], red[1], mean, rstd);
+    stats(v, red[0], mean, rstd);
 #pragma unroll
     for (int c = 0; c < NCH; ++c) {
-      const int i = (c * NT + tid) * VEC;
-      if (i >= d) continue;
-      float g[VEC], s[VEC];
-      ldv<E, VEC>(reinterpret_cast<const E*>(p.gb) + i, g);
-      if (p.ls) ldv<E, VEC>(reinterpret_cast<const E*>(p.ls) + i, s);
+      if ((c * NT + tid) * VEC >= d) continue;
+      const P g = get(pgb, p.gb, c);
+      P s;
+      if (p.ls) s = get(pls, p.ls, c);
 #pragma unroll
       for (int e = 0; e < VEC; ++e) {
-        const float n = (v[c][e] - mean) * rstd * g[e];
-        x[c][e] = p.ls ? fmaf(s[e], n, x[c][e]) : x[c][e] + n;
+        const float n = (v[c][e] - mean) * rstd * g.at(e);
+        x[c][e] = p.ls ? fmaf(s.at(e), n, x[c][e]) : x[c][e] + n;
       }
     }
   }
@@ -155,41 +190,43 @@ __global__ void __launch_bounds__(256) norm_residual_kernel(NormArgs p) {
   }
   if (!p.h) return;
   float mean, rstd;
-  stats(x, red[2], red[3], mean, rstd);
+  stats(x, red[1], mean, rstd);
 #pragma unroll
   for (int c = 0; c < NCH; ++c) {
     const int i = (c * NT + tid) * VEC;
     if (i >= d) continue;
-    float g[VEC];
-    ldv<E, VEC>(reinterpret_cast<const E*>(p.g) + i, g);
+    const P g = get(pg, p.g, c);
+    float y[VEC];
 #pragma unroll
-    for (int e = 0; e < VEC; ++e) g[e] = (x[c][e] - mean) * rstd * g[e];
-    stv<VEC>(reinterpret_cast<E*>(p.h) + (long long)r * d + i, g);
+    for (int e = 0; e < VEC; ++e) y[e] = (x[c][e] - mean) * rstd * g.at(e);
+    stv<VEC>(reinterpret_cast<E*>(p.h) + (long long)r * d + i, y);
   }
 }
 
 template <typename E>
 int launch(const NormArgs& a, hipStream_t s) {
   const bool v4 = a.d % 4 == 0 && a.lda % 4 == 0;
-#define GO(V, N, NT)                                                                                               \
-  hipLaunchKernelGGL((norm_residual_kernel<E, V, N, NT>), dim3((a.T + 256 / NT - 1) / (256 / NT)), dim3(256), 0, s, a)
+#define GO(V, N, NT, AHEAD)                                                                                          \
+  hipLaunchKernelGGL((norm_residual_kernel<E, V, N, NT, AHEAD>), dim3((a.T + 256 / NT - 1) / (256 / NT)), dim3(256), 0, s, a)
+  const bool few = a.T <= 256;
   if (v4 && a.T >= 512 && a.d <= 1024) {  // many short rows: a wave each, no barriers
-    if (a.d <= 256) GO(4, 1, 64);
-    else if (a.d <= 512) GO(4, 2, 64);
-    else GO(4, 4, 64);
+    if (a.d <= 256) GO(4, 1, 64, false);
+    else if (a.d <= 512) GO(4, 2, 64, false);
+    else GO(4, 4, 64, false);
   } else if (v4) {
     const int n = (a.d + 1023) / 1024;
-    if (n <= 1) GO(4, 1, 256);
-    else if (n <= 2) GO(4, 2, 256);
-    else if (n <= 4) GO(4, 4, 256);
-    else if (n <= 8) GO(4, 8, 256);
-    else if (n <= 16) GO(4, 16, 256);
+    if (n <= 1) GO(4, 1, 256, true);
+    else if (n <= 2) GO(4, 2, 256, true);
+    else if (n <= 4 && few) GO(4, 4, 256, true);
+    else if (n <= 4) GO(4, 4, 256, false);
+    else if (n <= 8) GO(4, 8, 256, false);
+    else if (n <= 16) GO(4, 16, 256, false);
     else return 10;
   } else {
     const int n = (a.d + 255) / 256;
-    if (n <= 1) GO(1, 1, 256);
-    else if (n <= 4) GO(1, 4, 256);
-    else if (n <= 16) GO(1, 16, 256);
+    if (n <= 1) GO(1, 1, 256, false);
+    else if (n <= 4) GO(1, 4, 256, false);
+    else if (n <= 16) GO(1, 16, 256, false);
     else return 10;
   }
 #undef GO
