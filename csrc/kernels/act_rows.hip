@@ -1,6 +1,7 @@
 // Activations over strided rows (the producer's and the consumer's buffers are column slices of wider ones).
 // MODE 0: y = gelu(x), exact (erf) form; 1: y = silu(g) * u * s with [g | u] side by side in a row and an
-// optional number s per row; 2: y = gelu_tanh(g) * u; 3: y = tanh(x). An optional bias per input column.
+// optional number s per row; 2: y = gelu_tanh(g) * u; 3: y = tanh(x); 4: y = max(x, 0)^2;
+// 5: y = cap tanh(x / cap). An optional bias per input column. x and y may be the same.
 #include "common.h"
 
 namespace {
@@ -23,7 +24,7 @@ __device__ __forceinline__ float tanh_t(float u) {
 
 template <typename E, int V, int MODE>
 __global__ void __launch_bounds__(256) act_rows_kernel(const E* x, long long ldx, const float* rs, const E* bias, E* y,
-                                                       long long ldy, int T, int F) {
+                                                       long long ldy, int T, int F, float cap) {
   constexpr bool GATED = MODE == 1 || MODE == 2;
   const int per = F / V;
   const long long n = (long long)T * per;
@@ -58,7 +59,9 @@ __global__ void __launch_bounds__(256) act_rows_kernel(const E* x, long long ldx
       else if constexpr (MODE == 1) v = g[e] / (1.f + (sizeof(E) == 4 ? expf(-g[e]) : __expf(-g[e]))) * u[e] * s;
       else if constexpr (MODE == 2)
         v = 0.5f * g[e] * (1.f + tanh_t<E>(0.7978845608028654f * (g[e] + 0.044715f * g[e] * g[e] * g[e]))) * u[e] * s;
-      else v = tanh_t<E>(g[e]);
+      else if constexpr (MODE == 3) v = tanh_t<E>(g[e]);
+      else if constexpr (MODE == 4) v = fmaxf(g[e], 0.f) * fmaxf(g[e], 0.f);
+      else v = cap * tanh_t<E>(g[e] / cap);
       o.v[e] = from_f<E>(v);
     }
     *reinterpret_cast<Pack<E, V>*>(y + t * ldy + c) = o;
@@ -67,15 +70,17 @@ __global__ void __launch_bounds__(256) act_rows_kernel(const E* x, long long ldx
 
 template <typename E, int V>
 void go(int mode, const void* x, long long ldx, const void* rs, const void* bias, void* y, long long ldy, int T, int F,
-        hipStream_t s) {
+        float cap, hipStream_t s) {
   const int g = kca_grid((long long)T * (F / V), 256);
 #define GO(M)                                                                                                          \
   hipLaunchKernelGGL((act_rows_kernel<E, V, M>), dim3(g), dim3(256), 0, s, (const E*)x, ldx, (const float*)rs,         \
-                     (const E*)bias, (E*)y, ldy, T, F)
+                     (const E*)bias, (E*)y, ldy, T, F, cap)
   if (mode == 0) GO(0);
   else if (mode == 1) GO(1);
   else if (mode == 2) GO(2);
-  else GO(3);
+  else if (mode == 3) GO(3);
+  else if (mode == 4) GO(4);
+  else GO(5);
 #undef GO
 }
 
@@ -83,16 +88,16 @@ void go(int mode, const void* x, long long ldx, const void* rs, const void* bias
 
 // dtype: 0 fp32, 1 bf16
 KCA_API int kca_act_rows(int dtype, int mode, const void* x, long long ldx, const void* rs, const void* bias, void* y,
-                         long long ldy, int T, int F, hipStream_t s) {
-  if (mode < 0 || mode > 3) return 1;
+                         long long ldy, int T, int F, float cap, hipStream_t s) {
+  if (mode < 0 || mode > 5 || (mode == 5 && !(cap > 0.f))) return 1;
   const bool gated = mode == 1 || mode == 2;
   if (T < 1 || F < 1 || !x || !y || ldx < (gated ? 2LL : 1LL) * F || ldy < F) return 1;
   const int V = dtype == 0 ? 4 : 8;
   const bool v = F % V == 0 && ldx % V == 0 && ldy % V == 0 && (uintptr_t)x % 16 == 0 && (uintptr_t)y % 16 == 0 &&
                  (uintptr_t)bias % 16 == 0;
-  if (dtype == 0) v ? go<float, 4>(mode, x, ldx, rs, bias, y, ldy, T, F, s) : go<float, 1>(mode, x, ldx, rs, bias, y, ldy, T, F, s);
+  if (dtype == 0) v ? go<float, 4>(mode, x, ldx, rs, bias, y, ldy, T, F, cap, s) : go<float, 1>(mode, x, ldx, rs, bias, y, ldy, T, F, cap, s);
   else if (dtype == 1)
-    v ? go<bf16_t, 8>(mode, x, ldx, rs, bias, y, ldy, T, F, s) : go<bf16_t, 1>(mode, x, ldx, rs, bias, y, ldy, T, F, s);
+    v ? go<bf16_t, 8>(mode, x, ldx, rs, bias, y, ldy, T, F, cap, s) : go<bf16_t, 1>(mode, x, ldx, rs, bias, y, ldy, T, F, cap, s);
   else return 3;
   return hipGetLastError() == hipSuccess ? 0 : 4;
 }

@@ -5,8 +5,13 @@
 // KIND 1 (channel): q, k, v pass a short causal convolution and silu; q (times qscale) and k become unit
 //   vectors, shared by the H / G heads of a group; w = exp(-exp(A) softplus(lw + dt)), z = w k,
 //   p = -beta k, k <- beta k.
-// The read-out is RMS-normed per head, times a gain, times sigmoid(gate).
+// KIND 2 (head): as 1, with one decay per head, exp(-exp(A) softplus(lw + dt)), lw a projection itself.
+// KIND 3 (state space): q, k, v are C, B, x after the convolution (with a bias) and silu; with dt = softplus(lw + bias)
+//   w = exp(-exp(A) dt), k <- dt k, p = z = 0, and the read-out adds D v.
+// KIND 0 - 2: the read-out is RMS-normed per head, times a gain, times sigmoid(gate) (2: silu). KIND 3: times
+// silu(gate), then RMS-normed in equal parts of all heads, times a gain.
 // Everything after the projections is fp32. `prep_head` derives one head's vectors of one token in LDS.
+// KIND 2 and 3 portions read convolution results that a kernel of their own made (`cx`).
 #pragma once
 #include "common.h"
 #include "lanes.h"
@@ -14,7 +19,7 @@
 struct DeltaArgs {
   const void* x;            // projection rows, row stride ld; column offsets below
   long long ld;
-  int o_q, o_k, o_v, o_a, o_g, o_w;  // a: removal logits | beta logits; g: gate logits | its inner; w: decay inner
+  int o_q, o_k, o_v, o_a, o_g, o_w;  // a: removal logits | beta logits; g: gate logits | its inner; w: decay inner | logits
   int H, G, dk, dv, taps, rank_w, rank_g;
   const void* lo_w;         // [H dk][rank_w] second step of the decay projection
   const void* lo_g;         // [H dv][rank_g] ... of the gate (KIND 1)
@@ -22,10 +27,10 @@ struct DeltaArgs {
   long long ldw;
   const void* dg;           // [T][H dv]
   long long ldg;
-  const void* w0;           // [H dk]: w0 | dt bias
+  const void* w0;           // [H dk]: w0 | dt bias (KIND 2, 3: [H])
   const void* ab;           // a's bias [H dk] | A [H]
   const void* conv;         // [2 G dk + H dv][taps], last column the current token's
-  const void* gain;         // [H dv] | [dv]
+  const void* gain;         // [H dv] (KIND 0, 3) | [dv]
   float eps, qscale;
   float* state;             // [slots][H][dk][dv]
   float* ring;              // [slots][taps][2 G dk + H dv]: convolution inputs, position p in row p % taps
@@ -39,6 +44,10 @@ struct DeltaArgs {
   float* pk;                // prepared vectors [rows][H][pk_stride]: w z p k q [dk], v [dv], q.p, q.k
   void* o;                  // read-outs [T][H dv] in the compute type
   const int* ent;           // scan kernel: [n][5]: first row, rows, position of the first row, slot, first prepared row
+  const void* cx;           // KIND 2, 3: rows [T][2 G dk + H dv] after convolution and silu (nullable: convolve here)
+  const void* convb;        // [2 G dk + H dv] its bias (nullable)
+  const void* skip;         // [H] D (nullable)
+  int norm_groups;          // KIND 3: equal parts of the closing norm
 };
 
 namespace delta {
@@ -56,6 +65,7 @@ __device__ __forceinline__ float tanh_t(float v) {
 }
 
 __device__ __forceinline__ float sigmoid(float v) { return 1.f / (1.f + expf(-v)); }
+__device__ __forceinline__ float silu(float v) { return v / (1.f + expf(-v)); }
 __device__ __forceinline__ float softplus(float v) { return fmaxf(v, 0.f) + log1pf(expf(-fabsf(v))); }
 __host__ __device__ __forceinline__ int pk_stride(int dk, int dv) { return (5 * dk + dv + 2 + 3) & ~3; }
 
@@ -74,6 +84,7 @@ __device__ __forceinline__ float conv_silu(const DeltaArgs& a, int t, int col, i
   const E* w = reinterpret_cast<const E*>(a.conv) + (long long)ch * a.taps + a.taps - 1;
   const float* r = a.ring + (long long)a.slot[t] * a.taps * C + ch;
   float y = ld<E>(w) * ld<E>(x);
+  if (a.convb) y += ld<E>(reinterpret_cast<const E*>(a.convb) + ch);
   if (!a.e0 && a.taps <= 4) {  // one token an entry: the loads of all taps fly together
     float v[3], c[3];
 #pragma unroll
@@ -153,16 +164,23 @@ __device__ __forceinline__ void prep_head(const DeltaArgs& a, int t, int h, Head
   const int g = h / (a.H / a.G), nqk = a.G * dk;
   // loads whose results are needed late
   const int cs = tid < dk ? tid : 0;
-  const float w0 = ld<E>(reinterpret_cast<const E*>(a.w0) + h * dk + cs);
-  float al = 0.f, ab = 0.f;
+  const float w0 = ld<E>(reinterpret_cast<const E*>(a.w0) + (KIND >= 2 ? h : h * dk + cs));
+  float al = 0.f, ab = 0.f, lh = 0.f;
   if constexpr (KIND == 0) {
     al = ld<E>(x + a.o_a + h * dk + cs);
     ab = ld<E>(reinterpret_cast<const E*>(a.ab) + h * dk + cs);
   } else {
-    al = ld<E>(x + a.o_a + h);
+    if constexpr (KIND < 3) al = ld<E>(x + a.o_a + h);
+    if constexpr (KIND >= 2) lh = ld<E>(x + a.o_w + h);
     ab = ld<E>(reinterpret_cast<const E*>(a.ab) + h);
   }
-  const int ndot = a.dw ? 0 : dk, ng = (KIND == 1 && !a.dg) ? dv : 0, rw = a.rank_w, rg = a.rank_g;
+  const bool low = KIND < 2 && !a.dw;  // second steps of the projections here
+  const int ndot = low ? dk : 0, ng = (KIND == 1 && !a.dg) ? dv : 0, rw = a.rank_w, rg = a.rank_g;
+  // a convolution channel: its column of x, its place among the channels
+  auto conv = [&](int col, int ch) {
+    if (KIND >= 2 && a.cx) return ld<E>(reinterpret_cast<const E*>(a.cx) + (long long)t * (2 * nqk + a.H * dv) + ch);
+    return conv_silu<E>(a, t, col, ch);
+  };
   auto dot_row = [&](int i) {
     return i < ndot ? reinterpret_cast<const E*>(a.lo_w) + (long long)(h * dk + i) * rw
                     : reinterpret_cast<const E*>(a.lo_g) + (long long)(h * dv + i - ndot) * rg;
@@ -178,14 +196,14 @@ __device__ __forceinline__ void prep_head(const DeltaArgs& a, int t, int h, Head
     for (int j = 0; j < 4; ++j) pre[j] = *reinterpret_cast<const U16x8*>(row + (8 * sub + 32 * j < n0 ? 8 * sub + 32 * j : 0));
   }
   float sk = 0.f, sq = 0.f;
-  const int items = 2 * dk + dv + (a.dw ? 0 : rw) + (KIND == 1 && !a.dg ? rg : 0);
+  const int items = 2 * dk + dv + (low ? rw : 0) + (KIND == 1 && !a.dg ? rg : 0);
   for (int i = tid; i < items; i += NT) {
     if (i < 2 * dk) {
       const bool key = i >= dk;
       const int c = key ? i - dk : i;
       float v;
       if constexpr (KIND == 0) v = ld<E>(x + (key ? a.o_k : a.o_q) + h * dk + c);
-      else v = conv_silu<E>(a, t, (key ? a.o_k : a.o_q) + g * dk + c, (key ? nqk : 0) + g * dk + c);
+      else v = conv((key ? a.o_k : a.o_q) + g * dk + c, (key ? nqk : 0) + g * dk + c);
       (key ? s.k : s.q)[c] = v;
       if (key) sk = fmaf(v, v, sk);
       else sq = fmaf(v, v, sq);
@@ -195,21 +213,23 @@ __device__ __forceinline__ void prep_head(const DeltaArgs& a, int t, int h, Head
         s.v[c] = ld<E>(x + a.o_v + h * dv + c);
         s.gate[c] = sigmoid(ld<E>(x + a.o_g + h * dv + c));
       } else {
-        s.v[c] = conv_silu<E>(a, t, a.o_v + h * dv + c, 2 * nqk + h * dv + c);
-        if (a.dg) s.gate[c] = sigmoid(ld<E>(reinterpret_cast<const E*>(a.dg) + (long long)t * a.ldg + h * dv + c));
+        s.v[c] = conv(a.o_v + h * dv + c, 2 * nqk + h * dv + c);
+        if constexpr (KIND == 2) s.gate[c] = silu(ld<E>(x + a.o_g + h * dv + c));
+        if (KIND == 1 && a.dg) s.gate[c] = sigmoid(ld<E>(reinterpret_cast<const E*>(a.dg) + (long long)t * a.ldg + h * dv + c));
       }
     } else {
       const int c = i - 2 * dk - dv;
-      if (!a.dw && c < rw) {
+      if (low && c < rw) {
         const float v = ld<E>(x + a.o_w + c);
         s.tw[c] = KIND == 0 ? tanh_t<E>(v) : v;
       } else {
-        s.tg[c - (a.dw ? 0 : rw)] = ld<E>(x + a.o_g + c - (a.dw ? 0 : rw));
+        s.tg[c - (low ? rw : 0)] = ld<E>(x + a.o_g + c - (low ? rw : 0));
       }
     }
   }
   block_sum2(sk, sq, s.red);  // (its barrier also publishes the vectors so far)
-  const float ik = 1.f / sqrtf(sk + 1e-6f), iq = KIND == 1 ? a.qscale / sqrtf(sq + 1e-6f) : 1.f;
+  const float ik = KIND == 3 ? 1.f : 1.f / sqrtf(sk + 1e-6f);
+  const float iq = KIND == 1 || KIND == 2 ? a.qscale / sqrtf(sq + 1e-6f) : 1.f;
   // decays (and, channel, gates): four lanes a dot
   for (int i = i0; i < ndot + ng; i += NT / 4) {
     const bool dec = i < ndot;
@@ -237,13 +257,16 @@ __device__ __forceinline__ void prep_head(const DeltaArgs& a, int t, int h, Head
   float qp = 0.f, qk = 0.f;
   if (tid < dk) {
     const int c = tid;
-    const float lw = a.dw ? ld<E>(reinterpret_cast<const E*>(a.dw) + (long long)t * a.ldw + h * dk + c) : s.w[c];
+    const float lw = KIND >= 2 ? lh : a.dw ? ld<E>(reinterpret_cast<const E*>(a.dw) + (long long)t * a.ldw + h * dk + c) : s.w[c];
     const float w = expf(log_decay<KIND>(lw, w0, ab));
     const float k = s.k[c], u = k * ik, q = s.q[c] * iq;
     float p, kw = k;
     if constexpr (KIND == 0) {
       p = -u * sigmoid(al + ab);
       s.z[c] = u;
+    } else if constexpr (KIND == 3) {
+      kw = k * softplus(lw + w0);
+      p = s.z[c] = 0.f;
     } else {
       kw = sigmoid(al) * u;
       p = -kw;
@@ -264,8 +287,11 @@ __device__ __forceinline__ void prep_head(const DeltaArgs& a, int t, int h, Head
 }  // namespace delta
 
 static inline bool delta_args_ok(const DeltaArgs& a, int kind) {
-  if ((kind != 0 && kind != 1) || a.H < 1 || a.G < 1 || a.H % a.G || a.dk < 1 || a.dv < 1 || a.dk > 256 || a.dv > 1024) return false;
+  if (kind < 0 || kind > 3 || a.H < 1 || a.G < 1 || a.H % a.G || a.dk < 1 || a.dv < 1 || a.dk > 256 || a.dv > 1024) return false;
   if (!a.x || !a.w0 || !a.ab || !a.gain || !a.state || !a.pos || !a.slot || !a.out) return false;
+  if (kind >= 2)
+    return a.conv && a.ring && a.taps >= 1 && a.rank_w == 0 && a.rank_g == 0 &&
+           (kind == 2 || (a.skip && a.norm_groups >= 1 && (a.H * a.dv) % a.norm_groups == 0));
   if (a.rank_w < 1 || (!a.dw && !a.lo_w)) return false;
   if (kind == 0) return a.G == a.H && a.dk == a.dv;
   return a.conv && a.ring && a.taps >= 1 && a.rank_g >= 1 && (a.dg || a.lo_g);

@@ -2,9 +2,12 @@
 // size or type (bf16 portions of usual head sizes run in chunks on the matrix cores: delta_chunk.hip).
 //
 //   step kernel   one token per row: projections -> vectors -> state update -> normed, gated output, one launch
+//                 (KIND 3: read-outs; the parts kernel norms them)
+//   conv kernel   KIND 2, 3: convolution and silu of every row of a batch of portions
 //   prep kernel   vectors of every (token, head) of a batch of portions
 //   scan kernel   an entry's tokens in order, state in registers; a wave owns 16 value columns of a head
 //   gate kernel   head norm, gain and gate of every (token, head); convolution inputs into the slots' rings
+//   parts kernel  KIND 3: gate and norm over equal parts of all heads; convolution inputs likewise
 //
 // The carried state of a sequence lives in its slot and counts as zero at position 0.
 #include "delta_rule.h"
@@ -45,6 +48,7 @@ struct Cols {
     }
   }
   // one token: the vectors at rows rg + 16 i (zero past dk), v at the lane's columns -> read-out
+  template <bool DELTA = true>
   __device__ __forceinline__ void token(const float (&w)[R], const float (&z)[R], const float (&p)[R], const float (&k)[R],
                                         const float (&q)[R], const float (&v)[CW], float qp, float qk, float (&o)[CW]) {
     float zs[CW], qs[CW];
@@ -55,21 +59,21 @@ struct Cols {
       const float qw = q[i] * w[i];
 #pragma unroll
       for (int e = 0; e < CW; ++e) {
-        zs[e] = fmaf(z[i], s[i][e], zs[e]);
+        if (DELTA) zs[e] = fmaf(z[i], s[i][e], zs[e]);
         qs[e] = fmaf(qw, s[i][e], qs[e]);
       }
     }
     auto add = [](float x, float y) { return x + y; };
 #pragma unroll
     for (int e = 0; e < CW; ++e) {
-      zs[e] = lanes_reduce<16>(zs[e], add);
+      if (DELTA) zs[e] = lanes_reduce<16>(zs[e], add);
       qs[e] = lanes_reduce<16>(qs[e], add);
       o[e] = qs[e] + qp * zs[e] + qk * v[e];  // q^T (w S + p s + k v)
     }
 #pragma unroll
     for (int i = 0; i < R; ++i)
 #pragma unroll
-      for (int e = 0; e < CW; ++e) s[i][e] = fmaf(w[i], s[i][e], fmaf(p[i], zs[e], k[i] * v[e]));
+      for (int e = 0; e < CW; ++e) s[i][e] = fmaf(w[i], s[i][e], DELTA ? fmaf(p[i], zs[e], k[i] * v[e]) : k[i] * v[e]);
   }
 };
 
@@ -91,7 +95,8 @@ __global__ void __launch_bounds__(R > 8 ? 512 : 1024) delta_step_kernel(DeltaArg
   st.load(S, dk, dv, rg, wv * 4 * CW + cg * CW, live);  // in flight while the vectors are made
   Head hd(smem, dk, dv, a.rank_w, a.rank_g);
   prep_head<E, KIND>(a, b, h, hd);
-  if constexpr (KIND == 1) ring_store<E>(a, b, h, tid, blockDim.x);
+  if constexpr (KIND >= 1) ring_store<E>(a, b, h, tid, blockDim.x);
+  const float skip = KIND == 3 ? delta::ld<E>(reinterpret_cast<const E*>(a.skip) + h) : 0.f;
   float w[R], z[R], p[R], k[R], q[R];
   rows_of<R>(hd.w, dk, rg, w);
   rows_of<R>(hd.z, dk, rg, z);
@@ -105,9 +110,15 @@ __global__ void __launch_bounds__(R > 8 ? 512 : 1024) delta_step_kernel(DeltaArg
     float v[CW], o[CW];
 #pragma unroll
     for (int e = 0; e < CW; ++e) v[e] = col + e < dv ? hd.v[col + e] : 0.f;
-    st.token(w, z, p, k, q, v, hd.qp, hd.qk, o);
+    st.template token<KIND != 3>(w, z, p, k, q, v, hd.qp, hd.qk, o);
     st.store(S, dk, dv, rg, col);
-    if (rg == 0)
+    if (KIND == 3 && rg == 0) {
+      E* out = reinterpret_cast<E*>(a.o) + ((long long)b * a.H + h) * dv + col;
+#pragma unroll
+      for (int e = 0; e < CW; ++e)
+        if (col + e < dv) delta::st<E>(out + e, fmaf(skip, v[e], o[e]));
+    }
+    if (KIND != 3 && rg == 0)
 #pragma unroll
       for (int e = 0; e < CW; ++e)
         if (col + e < dv) {  // (this wave alone reads and writes these columns of v)
@@ -115,6 +126,7 @@ __global__ void __launch_bounds__(R > 8 ? 512 : 1024) delta_step_kernel(DeltaArg
           ss = fmaf(o[e], o[e], ss);
         }
   }
+  if constexpr (KIND == 3) return;
   float none = 0.f;
   block_sum2(ss, none, hd.red);
   const float n = 1.f / sqrtf(ss / (float)dv + a.eps);
@@ -149,6 +161,7 @@ __global__ void __launch_bounds__(256) delta_scan_kernel(DeltaArgs a) {
   const long long step = (long long)a.H * ps;
   const float* pk = a.pk + ((long long)pk0 * a.H + h) * ps;
   E* o = reinterpret_cast<E*>(a.o) + (long long)row0 * a.H * dv + h * dv + col;
+  const float skip = a.skip ? delta::ld<E>(reinterpret_cast<const E*>(a.skip) + h) : 0.f;
   Cols<R, CW> st;
   st.load(S, dk, dv, rg, col, pos0 > 0);
   float w[R], z[R], p[R], k[R], q[R], v[CW], qp, qk;
@@ -178,7 +191,7 @@ __global__ void __launch_bounds__(256) delta_scan_kernel(DeltaArgs a) {
     if (rg == 0)
 #pragma unroll
       for (int e = 0; e < CW; ++e)
-        if (col + e < dv) delta::st<E>(o + e, y[e]);
+        if (col + e < dv) delta::st<E>(o + e, fmaf(skip, vn[e], y[e]));
     o += (long long)a.H * dv;
   }
   st.store(S, dk, dv, rg, col);
@@ -193,7 +206,7 @@ __global__ void __launch_bounds__(256) delta_gate_kernel(DeltaArgs a, int T) {
   const int t = (int)(i / a.H), h = (int)(i - (long long)t * a.H), lane = threadIdx.x % NL, dv = a.dv;
   const E* o = reinterpret_cast<const E*>(a.o) + ((long long)t * a.H + h) * dv;
   const E* gain = reinterpret_cast<const E*>(a.gain) + (KIND == 0 ? h * dv : 0);
-  const E* gt = KIND == 0 ? reinterpret_cast<const E*>(a.x) + (long long)t * a.ld + a.o_g + h * dv
+  const E* gt = KIND != 1 ? reinterpret_cast<const E*>(a.x) + (long long)t * a.ld + a.o_g + h * dv
                           : reinterpret_cast<const E*>(a.dg) + (long long)t * a.ldg + h * dv;
   E* out = reinterpret_cast<E*>(a.out) + (long long)t * a.ldo + h * dv;
   const int c0 = lane * V;
@@ -225,13 +238,140 @@ __global__ void __launch_bounds__(256) delta_gate_kernel(DeltaArgs a, int T) {
 #pragma unroll
     for (int e = 0; e < V; ++e) {
       const float z = delta::ld<E>(g.v + e);
-      const float sg = sizeof(E) == 4 ? sigmoid(z) : __builtin_amdgcn_rcpf(1.f + __expf(-z));
+      const float sg = (sizeof(E) == 4 ? sigmoid(z) : __builtin_amdgcn_rcpf(1.f + __expf(-z))) * (KIND == 2 ? z : 1.f);
       delta::st<E>(r.v + e, delta::ld<E>(y.v + e) * n * delta::ld<E>(gn.v + e) * sg);
     }
     *reinterpret_cast<PackE*>(out + c) = r;
   }
-  if constexpr (KIND == 1)
+  if constexpr (KIND >= 1)
     if (a.e1[t] - t <= a.taps) ring_store<E>(a, t, h, lane, NL);
+}
+
+// Rows of short convolutions: V channels and ROWS consecutive rows a thread. A row's earlier inputs are the rows
+// before it, back to its entry's first, then the slot's ring.
+constexpr int CONV_ROWS = 8;
+template <typename E, int V>
+__global__ void __launch_bounds__(256) delta_conv_kernel(DeltaArgs a, E* out, int T) {
+  struct alignas(sizeof(E) * V) PackE { E v[V]; };
+  const int nqk = a.G * a.dk, C = 2 * nqk + a.H * a.dv, per = C / V;
+  const long long i = (long long)blockIdx.x * 256 + threadIdx.x;
+  const int t0 = (int)(i / per) * CONV_ROWS, ch = (int)(i % per) * V;
+  if (t0 >= T) return;
+  const int col = ch < nqk ? a.o_q + ch : ch < 2 * nqk ? a.o_k + ch - nqk : a.o_v + ch - 2 * nqk;
+  const E* x = reinterpret_cast<const E*>(a.x) + col;
+  const E* w = reinterpret_cast<const E*>(a.conv) + (long long)ch * a.taps + a.taps - 1;
+  const int t1 = min(t0 + CONV_ROWS, T);
+  auto row = [&](int t, float (&v)[V]) {
+    const PackE u = *reinterpret_cast<const PackE*>(x + (long long)t * a.ld);
+#pragma unroll
+    for (int e = 0; e < V; ++e) v[e] = delta::ld<E>(u.v + e);
+  };
+  auto before = [&](int t, int n, float (&v)[V]) {  // the input n tokens before row t
+    if (t - n >= a.e0[t]) return row(t - n, v);
+    const int ps = a.pos[t] - n;
+    const float* r = a.ring + ((long long)a.slot[t] * a.taps + (ps >= 0 ? ps % a.taps : 0)) * C + ch;
+#pragma unroll
+    for (int e = 0; e < V; ++e) v[e] = ps >= 0 ? r[e] : 0.f;
+  };
+  auto put = [&](int t, const float (&y)[V]) {
+    PackE u;
+#pragma unroll
+    for (int e = 0; e < V; ++e) {
+      if constexpr (sizeof(E) == 4) delta::st<E>(u.v + e, silu(y[e]));
+      else delta::st<E>(u.v + e, y[e] * __builtin_amdgcn_rcpf(1.f + __expf(-y[e])));
+    }
+    *reinterpret_cast<PackE*>(out + (long long)t * C + ch) = u;
+  };
+  float bias[V];
+#pragma unroll
+  for (int e = 0; e < V; ++e) bias[e] = a.convb ? delta::ld<E>(reinterpret_cast<const E*>(a.convb) + ch + e) : 0.f;
+  if (a.taps > 4) {
+    for (int t = t0; t < t1; ++t) {
+      float y[V], v[V];
+#pragma unroll
+      for (int e = 0; e < V; ++e) y[e] = bias[e];
+      for (int n = 0; n < a.taps; ++n) {
+        before(t, n, v);
+#pragma unroll
+        for (int e = 0; e < V; ++e) y[e] = fmaf(delta::ld<E>(w + (long long)e * a.taps - n), v[e], y[e]);
+      }
+      put(t, y);
+    }
+    return;
+  }
+  float tap[4][V], h[4][V];  // h[n]: the input n tokens back
+#pragma unroll
+  for (int n = 0; n < 4; ++n)
+#pragma unroll
+    for (int e = 0; e < V; ++e) {
+      tap[n][e] = n < a.taps ? delta::ld<E>(w + (long long)e * a.taps - n) : 0.f;
+      h[n][e] = 0.f;
+    }
+  for (int t = t0; t < t1; ++t) {
+    if (t == t0 || a.e0[t] == t) {
+#pragma unroll
+      for (int n = 1; n < 4; ++n)
+        if (n < a.taps) before(t, n, h[n]);
+    }
+    row(t, h[0]);
+    float y[V];
+#pragma unroll
+    for (int e = 0; e < V; ++e)
+      y[e] = fmaf(tap[0][e], h[0][e], fmaf(tap[1][e], h[1][e], fmaf(tap[2][e], h[2][e], fmaf(tap[3][e], h[3][e], bias[e]))));
+    put(t, y);
+#pragma unroll
+    for (int n = 3; n > 0; --n)
+#pragma unroll
+      for (int e = 0; e < V; ++e) h[n][e] = h[n - 1][e];
+  }
+}
+
+// KIND 3: out = N(o * silu(z)) * gain of a row, N over norm_groups equal parts. WPP waves a part (WPP = all of them:
+// the workgroup takes the parts in turn). The gated row lies in LDS between its two uses, by the thread that made it.
+template <typename E, int V, int NW, bool ALL>
+__global__ void __launch_bounds__(64 * NW) delta_parts_kernel(DeltaArgs a) {
+  struct alignas(sizeof(E) * V) PackE { E v[V]; };
+  extern __shared__ __attribute__((aligned(16))) float u[];
+  __shared__ float red[NW];
+  const int t = blockIdx.x, tid = threadIdx.x, lane = tid & 63, wv = tid >> 6, n = a.H * a.dv, per = n / a.norm_groups;
+  const E* o = reinterpret_cast<const E*>(a.o) + (long long)t * n;
+  const E* z = reinterpret_cast<const E*>(a.x) + (long long)t * a.ld + a.o_g;
+  const E* gain = reinterpret_cast<const E*>(a.gain);
+  E* out = reinterpret_cast<E*>(a.out) + (long long)t * a.ldo;
+  const int step = (ALL ? 64 * NW : 64) * V, c0 = (ALL ? tid : lane) * V;
+  for (int g = ALL ? blockIdx.y : blockIdx.y * NW + wv; g < a.norm_groups; g += gridDim.y * (ALL ? 1 : NW)) {
+    float ss = 0.f;
+    float* up = u + (ALL ? 0 : wv * per);
+    for (int c = c0; c < per; c += step) {
+      const PackE y = *reinterpret_cast<const PackE*>(o + g * per + c), q = *reinterpret_cast<const PackE*>(z + g * per + c);
+#pragma unroll
+      for (int e = 0; e < V; ++e) {
+        const float x = delta::ld<E>(q.v + e);
+        const float v = delta::ld<E>(y.v + e) * (sizeof(E) == 4 ? silu(x) : x * __builtin_amdgcn_rcpf(1.f + __expf(-x)));
+        up[c + e] = v;
+        ss = fmaf(v, v, ss);
+      }
+    }
+    ss = wave_sum(ss);
+    if constexpr (ALL) {
+      if (lane == 0) red[wv] = ss;
+      __syncthreads();
+      ss = 0.f;
+#pragma unroll
+      for (int i = 0; i < NW; ++i) ss += red[i];
+      __syncthreads();
+    }
+    const float r = 1.f / sqrtf(ss / (float)per + a.eps);
+    for (int c = c0; c < per; c += step) {
+      const PackE w = *reinterpret_cast<const PackE*>(gain + g * per + c);
+      PackE y;
+#pragma unroll
+      for (int e = 0; e < V; ++e) delta::st<E>(y.v + e, up[c + e] * r * delta::ld<E>(w.v + e));
+      *reinterpret_cast<PackE*>(out + g * per + c) = y;
+    }
+  }
+  if (a.e1 && blockIdx.y == 0 && a.e1[t] - t <= a.taps)
+    for (int h = 0; h < a.H; ++h) ring_store<E>(a, t, h, tid, 64 * NW);
 }
 
 int rows_r(int dk) {  // rows a lane holds: 16 row groups
@@ -293,8 +433,8 @@ int prep_go(const DeltaArgs& a, int T, hipStream_t s) {
 template <typename E, int KIND>
 int gate_go(const DeltaArgs& a, int T, hipStream_t s) {
   const int al = sizeof(E) * 4;
-  const bool v4 = a.dv % 4 == 0 && a.ldo % 4 == 0 && (KIND == 0 ? a.ld % 4 == 0 && a.o_g % 4 == 0 : a.ldg % 4 == 0) &&
-                  (uintptr_t)a.out % al == 0 && (uintptr_t)(KIND == 0 ? a.x : a.dg) % al == 0 && (uintptr_t)a.gain % al == 0 &&
+  const bool v4 = a.dv % 4 == 0 && a.ldo % 4 == 0 && (KIND != 1 ? a.ld % 4 == 0 && a.o_g % 4 == 0 : a.ldg % 4 == 0) &&
+                  (uintptr_t)a.out % al == 0 && (uintptr_t)(KIND != 1 ? a.x : a.dg) % al == 0 && (uintptr_t)a.gain % al == 0 &&
                   (uintptr_t)a.o % 16 == 0;
   const long long n = (long long)T * a.H;
 #define GO(NL, V) hipLaunchKernelGGL((delta_gate_kernel<E, KIND, NL, V>), dim3((unsigned)((n * NL + 255) / 256)), dim3(256), 0, s, a, T)
@@ -306,20 +446,67 @@ int gate_go(const DeltaArgs& a, int T, hipStream_t s) {
   return hipGetLastError() == hipSuccess ? 0 : 4;
 }
 
+template <typename E>
+int conv_go(const DeltaArgs& a, void* out, int T, hipStream_t s) {
+  constexpr int W = sizeof(E) == 2 ? 8 : 4;
+  const int nqk = a.G * a.dk, C = 2 * nqk + a.H * a.dv;
+  const bool vec = nqk % W == 0 && C % W == 0 && a.ld % W == 0 && a.o_q % W == 0 && a.o_k % W == 0 && a.o_v % W == 0 &&
+                   (uintptr_t)a.x % 16 == 0 && (uintptr_t)out % 16 == 0;
+  const long long n = (long long)((T + CONV_ROWS - 1) / CONV_ROWS) * (C / (vec ? W : 1));
+  const dim3 g((unsigned)((n + 255) / 256));
+  if (vec) hipLaunchKernelGGL((delta_conv_kernel<E, W>), g, dim3(256), 0, s, a, (E*)out, T);
+  else hipLaunchKernelGGL((delta_conv_kernel<E, 1>), g, dim3(256), 0, s, a, (E*)out, T);
+  return hipGetLastError() == hipSuccess ? 0 : 4;
+}
+
+template <typename E, int V>
+int parts_v(const DeltaArgs& a, int T, hipStream_t s) {
+  const int n = a.H * a.dv, per = n / a.norm_groups;
+  const bool all = a.norm_groups < 4, few = T <= 64 && per > 2048;
+  const size_t lds = (size_t)per * 4 * (all ? 1 : 4);
+  if (lds > 128 * 1024) return 10;
+#define GO(NW, ALL)                                                                                                       \
+  {                                                                                                                       \
+    auto kern = delta_parts_kernel<E, V, NW, ALL>;                                                                        \
+    if (lds > 48 * 1024 && hipFuncSetAttribute((const void*)kern, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds) != hipSuccess) \
+      return 5;                                                                                                           \
+    hipLaunchKernelGGL(kern, dim3(T, ALL ? a.norm_groups : (a.norm_groups + NW - 1) / NW), dim3(64 * NW), lds, s, a);      \
+  }
+  if (!all) GO(4, false)
+  else if (few) GO(16, true)
+  else GO(4, true)
+#undef GO
+  return hipGetLastError() == hipSuccess ? 0 : 4;
+}
+template <typename E>
+int parts_go(const DeltaArgs& a, int T, hipStream_t s) {
+  constexpr int W = sizeof(E) == 2 ? 8 : 4;
+  const bool vec = (a.H * a.dv / a.norm_groups) % W == 0 && a.ld % W == 0 && a.ldo % W == 0 && a.o_g % W == 0 &&
+                   (uintptr_t)a.x % 16 == 0 && (uintptr_t)a.o % 16 == 0 && (uintptr_t)a.out % 16 == 0 && (uintptr_t)a.gain % 16 == 0;
+  return vec ? parts_v<E, W>(a, T, s) : parts_v<E, 1>(a, T, s);
+}
+
 }  // namespace
 
 // Mirrored by ops/delta_rule.py
 KCA_API int kca_delta_abi() { return (int)sizeof(DeltaArgs); }
 
-#define DELTA_DISPATCH(FN, N)                                                                 \
-  if (dtype == 0) return kind == 0 ? FN<float, 0>(a, N, s) : FN<float, 1>(a, N, s);           \
-  if (dtype == 1) return kind == 0 ? FN<bf16_t, 0>(a, N, s) : FN<bf16_t, 1>(a, N, s);         \
+#define DELTA_KINDS(FN, N, E)                              \
+  switch (kind) {                                          \
+    case 0: return FN<E, 0>(a, N, s);                      \
+    case 1: return FN<E, 1>(a, N, s);                      \
+    case 2: return FN<E, 2>(a, N, s);                      \
+    default: return FN<E, 3>(a, N, s);                     \
+  }
+#define DELTA_DISPATCH(FN, N)                              \
+  if (dtype == 0) DELTA_KINDS(FN, N, float)                \
+  if (dtype == 1) DELTA_KINDS(FN, N, bf16_t)               \
   return 3;
 
 // one token per row
 KCA_API int kca_delta_step(const DeltaArgs* in, int dtype, int kind, int B, hipStream_t s) {
   const DeltaArgs& a = *in;
-  if (!delta_args_ok(a, kind) || B < 1 || a.H > 65535 || a.e0) return 1;
+  if (!delta_args_ok(a, kind) || B < 1 || a.H > 65535 || a.e0 || a.cx || (kind == 3 && !a.o)) return 1;
   DELTA_DISPATCH(step_r, B)
 }
 
@@ -342,6 +529,26 @@ KCA_API int kca_delta_scan(const DeltaArgs* in, int dtype, int nent, hipStream_t
 // a.out of every (token, head) from a.o
 KCA_API int kca_delta_gate(const DeltaArgs* in, int dtype, int kind, int T, hipStream_t s) {
   const DeltaArgs& a = *in;
-  if (!delta_args_ok(a, kind) || T < 1 || !a.o || !a.e0 || !a.e1 || (kind == 1 && !a.dg)) return 1;
-  DELTA_DISPATCH(gate_go, T)
+  if (!delta_args_ok(a, kind) || T < 1 || !a.o || !a.e0 || !a.e1 || kind > 2 || (kind == 1 && !a.dg)) return 1;
+  if (dtype == 0) return kind == 0 ? gate_go<float, 0>(a, T, s) : kind == 1 ? gate_go<float, 1>(a, T, s) : gate_go<float, 2>(a, T, s);
+  if (dtype == 1) return kind == 0 ? gate_go<bf16_t, 0>(a, T, s) : kind == 1 ? gate_go<bf16_t, 1>(a, T, s) : gate_go<bf16_t, 2>(a, T, s);
+  return 3;
+}
+
+// kind 2, 3: convolution and silu of every row -> out [T][2 G dk + H dv]
+KCA_API int kca_delta_conv(const DeltaArgs* in, int dtype, int kind, int T, void* out, hipStream_t s) {
+  const DeltaArgs& a = *in;
+  if (!delta_args_ok(a, kind) || kind < 2 || T < 1 || !a.e0 || !out) return 1;
+  if (dtype == 0) return conv_go<float>(a, out, T, s);
+  if (dtype == 1) return conv_go<bf16_t>(a, out, T, s);
+  return 3;
+}
+
+// kind 3: a.out of every token from a.o; a.e1 set: the entries' last inputs go into the rings
+KCA_API int kca_delta_parts(const DeltaArgs* in, int dtype, int T, hipStream_t s) {
+  const DeltaArgs& a = *in;
+  if (!delta_args_ok(a, 3) || T < 1 || !a.o) return 1;
+  if (dtype == 0) return parts_go<float>(a, T, s);
+  if (dtype == 1) return parts_go<bf16_t>(a, T, s);
+  return 3;
 }

@@ -12,23 +12,12 @@
 //                      every shape or type the matrix-core kernel does not take
 //   tile kernel        bf16 prompt portions on the matrix cores: 128 queries of one (entry, head) per
 //                      workgroup, one wave per (32 queries, map)
+#include "attn_rows.h"
 #include "attn_tile.h"
 #include "decode_tail.h"
 #include "lanes.h"
 
 namespace {
-
-template <typename E> struct El;
-template <> struct El<bf16_t> {
-  static __device__ __forceinline__ float ld(const bf16_t* p) { return bf2f(*p); }
-  static __device__ __forceinline__ void st(bf16_t* p, float v) { *p = f2bf(v); }
-  static __device__ __forceinline__ float ex(float x) { return __expf(x); }
-};
-template <> struct El<float> {
-  static __device__ __forceinline__ float ld(const float* p) { return *p; }
-  static __device__ __forceinline__ void st(float* p, float v) { *p = v; }
-  static __device__ __forceinline__ float ex(float x) { return expf(x); }
-};
 
 struct DiffArgs {
   const void* qkv;          // rows of the projection, row stride ld
@@ -83,25 +72,6 @@ __global__ void __launch_bounds__(256) kv_append_kernel(DiffArgs p, int T) {
 // waves, then the splits, merge at the end.
 
 constexpr int MAX_SPLITS = 256;
-
-// eight elements as loaded (converted where they are used); `left` of them exist
-template <typename E>
-struct Raw8 {
-  E v[8];
-  __device__ __forceinline__ float f(int i) const { return El<E>::ld(v + i); }
-};
-template <typename E, bool VEC>
-__device__ __forceinline__ void ld8g(const E* p, int left, Raw8<E>& x) {
-  if constexpr (VEC) {
-    u32x4* d = reinterpret_cast<u32x4*>(x.v);
-#pragma unroll
-    for (int i = 0; i < (int)sizeof(E) / 2; ++i)
-      d[i] = left > 0 ? reinterpret_cast<const u32x4*>(p)[i] : u32x4{0u, 0u, 0u, 0u};
-  } else {
-#pragma unroll
-    for (int i = 0; i < 8; ++i) x.v[i] = i < left ? p[i] : (E)0;
-  }
-}
 
 template <typename E, int RB, int LPK, int LPV, bool VEC>
 __global__ void __launch_bounds__(256) diff_rows_kernel(DiffArgs p) {
@@ -598,12 +568,6 @@ int rows_go(const DiffArgs& p, int rows, hipStream_t s) {
     if (hipFuncSetAttribute((const void*)kern, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds) != hipSuccess) return 5;
   hipLaunchKernelGGL(kern, dim3(rows, p.G * nsub, p.nsplit), dim3(256), lds, s, p);
   return hipGetLastError() == hipSuccess ? 0 : 4;
-}
-
-int lanes_for(int n) {  // lanes of 8 elements, a power of two
-  int l = 8;
-  while (l * 8 < n) l *= 2;
-  return l;
 }
 
 int rb_for(int Hg, bool vec) { return vec && Hg > 1 ? 4 : 1; }

@@ -156,6 +156,7 @@ __global__ __launch_bounds__(256) void skinny_gemm_kernel(
         float v = acc[r][m] + b;
         if (act == 1) v = gelu_tanh(v);
         else if (act == 2) v = 0.5f * v * (1.f + erff(v * 0.70710678118654752f));
+        else if (act == 3) v = fmaxf(v, 0.f) * fmaxf(v, 0.f);
         y[m * ldy + n0 + r] = f2bf(v);
       }
     }
@@ -330,6 +331,7 @@ __global__ __launch_bounds__(256) void gemv1_kernel(const bf16_t* __restrict__ x
     v += bias ? e2f<DT>(bias[n0 + r]) : 0.f;
     if (act == 1) v = gelu_tanh(v);
     else if (act == 2) v = 0.5f * v * (1.f + erff(v * 0.70710678118654752f));
+    else if (act == 3) v = fmaxf(v, 0.f) * fmaxf(v, 0.f);
     y[m * ldy + n0 + r] = (bf16_t)f2e<DT>(v);
   }
 }

@@ -5,6 +5,11 @@
 // a: the sublayer's output rows, b its bias (optional), ls a per-coordinate scale. The stream x is fp32 and
 // double buffered; h is rounded once. Statistics are fp32 and two-pass within a wave; the waves of a row merge
 // theirs by counts (one barrier a norm). Few rows load gains and scales ahead of the statistics (AHEAD).
+//
+// Pre-norms (prenorm_kernel), RMS throughout:
+//   x_t = src_t + a_t     or   x_t = src_t + mul * (N(a_t; ga) + N(b_t; gb))
+//   h_t = x_t / sqrt(mean x_t^2 + eps) * (1 + g),   raw_t = x_t rounded (a column block of a wider buffer)
+// src: the stream, scaled embedding rows, or rows of a product plus one vector.
 #include "common.h"
 #include "lanes.h"
 
@@ -233,6 +238,180 @@ int launch(const NormArgs& a, hipStream_t s) {
   return hipGetLastError() == hipSuccess ? 0 : 4;
 }
 
+struct PreArgs {
+  const float* x_in;          // one source: the stream,
+  const void* embed;          // embedding rows (times escale),
+  const long long* tokens;
+  float escale;
+  const void* base;           // or rows (stride ldbase) plus vec
+  long long ldbase;
+  const void* vec;
+  const void* a;              // sublayer output (nullable)
+  long long lda;
+  const void* ga;             // gain of its norm (nullable: added as it is)
+  const void* b;              // a second one, normed too (nullable)
+  long long ldb;
+  const void* gb;
+  float mul;                  // of the normed outputs
+  const void* g;              // the next norm's gain minus one
+  float eps;
+  const int* rows;            // output row i reads token rows[i] (nullable)
+  float* x_out;               // nullable
+  void* raw;                  // nullable, row stride ldr
+  long long ldr;
+  void* h;                    // nullable
+  int T, d;
+};
+
+template <typename E, int VEC, int NCH, int NT, bool AHEAD>
+__global__ void __launch_bounds__(256) prenorm_kernel(PreArgs p) {
+  constexpr int RPB = 256 / NT;  // rows of a workgroup (one wave each when NT == 64)
+  static_assert(RPB == 1 || NT == 64, "a row is a wave or the workgroup");
+  __shared__ float2 red[2][NT / 64];
+  const int tid = threadIdx.x % NT, d = p.d;
+  const int r = blockIdx.x * RPB + threadIdx.x / NT;
+  if (r >= p.T) return;  // (whole waves; RPB == 1: never)
+  const int t = p.rows ? p.rows[r] : r;
+  const float inv = 1.f / (float)d;
+  using P = Pack<E, VEC>;
+  float x[NCH][VEC], u[NCH][VEC], v[NCH][VEC];
+  auto at = [&](int c) { return (c * NT + tid) * VEC; };
+  auto par = [&](const void* q, int c) { return *reinterpret_cast<const P*>(reinterpret_cast<const E*>(q) + min(at(c), d - VEC)); };
+  const long long tok = p.embed ? p.tokens[t] : 0;
+#pragma unroll
+  for (int c = 0; c < NCH; ++c) {
+    const int i = at(c);
+#pragma unroll
+    for (int e = 0; e < VEC; ++e) x[c][e] = u[c][e] = v[c][e] = 0.f;
+    if (i < d) {
+      if (p.x_in) ldv<float, VEC>(p.x_in + (long long)t * d + i, x[c]);
+      else if (p.embed) ldv<E, VEC>(reinterpret_cast<const E*>(p.embed) + tok * d + i, x[c]);
+      else ldv<E, VEC>(reinterpret_cast<const E*>(p.base) + (long long)t * p.ldbase + i, x[c]);
+      if (p.a) ldv<E, VEC>(reinterpret_cast<const E*>(p.a) + (long long)t * p.lda + i, u[c]);
+      if (p.b) ldv<E, VEC>(reinterpret_cast<const E*>(p.b) + (long long)t * p.ldb + i, v[c]);
+    }
+  }
+  P pa[AHEAD ? NCH : 1], pb[AHEAD ? NCH : 1], pg[AHEAD ? NCH : 1];
+  if constexpr (AHEAD) {
+#pragma unroll
+    for (int c = 0; c < NCH; ++c) {
+      if (p.ga) pa[c] = par(p.ga, c);
+      if (p.gb) pb[c] = par(p.gb, c);
+      if (p.h) pg[c] = par(p.g, c);
+    }
+  }
+  auto get = [&](const P* ahead, const void* q, int c) {
+    if constexpr (AHEAD) return ahead[c];
+    else return par(q, c);
+  };
+  auto add = [](float y, float z) { return y + z; };
+  // sums of squares of two rows (elements past d are zero)
+  auto sums = [&](const float (&y)[NCH][VEC], const float (&z)[NCH][VEC], bool both, float2* rd) {
+    float2 s = make_float2(0.f, 0.f);
+#pragma unroll
+    for (int c = 0; c < NCH; ++c)
+#pragma unroll
+      for (int e = 0; e < VEC; ++e) {
+        s.x = fmaf(y[c][e], y[c][e], s.x);
+        if (both) s.y = fmaf(z[c][e], z[c][e], s.y);
+      }
+    s.x = lanes_reduce<64>(s.x, add);
+    if (both) s.y = lanes_reduce<64>(s.y, add);
+    if constexpr (NT > 64) {
+      if ((threadIdx.x & 63) == 0) rd[threadIdx.x >> 6] = s;
+      __syncthreads();
+      s = make_float2(0.f, 0.f);
+#pragma unroll
+      for (int i = 0; i < NT / 64; ++i) s.x += rd[i].x, s.y += rd[i].y;
+    }
+    return s;
+  };
+  if (p.embed) {
+#pragma unroll
+    for (int c = 0; c < NCH; ++c)
+#pragma unroll
+      for (int e = 0; e < VEC; ++e) x[c][e] *= p.escale;
+  } else if (p.vec && !p.x_in) {
+#pragma unroll
+    for (int c = 0; c < NCH; ++c) {
+      if (at(c) >= d) continue;
+      const P w = par(p.vec, c);
+#pragma unroll
+      for (int e = 0; e < VEC; ++e) x[c][e] += w.at(e);
+    }
+  }
+  if (p.ga) {
+    const float2 s = sums(u, v, p.b != nullptr, red[0]);
+    const float na = p.mul / sqrtf(s.x * inv + p.eps), nb = p.mul / sqrtf(s.y * inv + p.eps);
+#pragma unroll
+    for (int c = 0; c < NCH; ++c) {
+      if (at(c) >= d) continue;
+      const P ga = get(pa, p.ga, c);
+#pragma unroll
+      for (int e = 0; e < VEC; ++e) u[c][e] *= na * ga.at(e);
+      if (p.b) {
+        const P gb = get(pb, p.gb, c);
+#pragma unroll
+        for (int e = 0; e < VEC; ++e) u[c][e] = fmaf(v[c][e], nb * gb.at(e), u[c][e]);
+      }
+    }
+  }
+#pragma unroll
+  for (int c = 0; c < NCH; ++c) {
+    const int i = at(c);
+    if (p.a)
+#pragma unroll
+      for (int e = 0; e < VEC; ++e) x[c][e] += u[c][e];
+    if (i < d) {
+      if (p.x_out) stv<VEC>(p.x_out + (long long)r * d + i, x[c]);
+      if (p.raw) stv<VEC>(reinterpret_cast<E*>(p.raw) + (long long)r * p.ldr + i, x[c]);
+    }
+  }
+  if (!p.h) return;
+  const float n = 1.f / sqrtf(sums(x, x, false, red[1]).x * inv + p.eps);
+#pragma unroll
+  for (int c = 0; c < NCH; ++c) {
+    const int i = at(c);
+    if (i >= d) continue;
+    const P g = get(pg, p.g, c);
+    float y[VEC];
+#pragma unroll
+    for (int e = 0; e < VEC; ++e) y[e] = x[c][e] * n * (1.f + g.at(e));
+    stv<VEC>(reinterpret_cast<E*>(p.h) + (long long)r * d + i, y);
+  }
+}
+
+template <typename E>
+int launch_pre(const PreArgs& a, hipStream_t s) {
+  const bool v4 = a.d % 4 == 0 && a.lda % 4 == 0 && a.ldb % 4 == 0 && a.ldbase % 4 == 0 && a.ldr % 4 == 0 &&
+                  (uintptr_t)a.raw % (4 * sizeof(E)) == 0;
+#define GO(V, N, NT, AHEAD)                                                                                          \
+  hipLaunchKernelGGL((prenorm_kernel<E, V, N, NT, AHEAD>), dim3((a.T + 256 / NT - 1) / (256 / NT)), dim3(256), 0, s, a)
+  const bool few = a.T <= 256;
+  if (v4 && a.T >= 512 && a.d <= 1024) {  // many short rows: a wave each, no barriers
+    if (a.d <= 256) GO(4, 1, 64, false);
+    else if (a.d <= 512) GO(4, 2, 64, false);
+    else GO(4, 4, 64, false);
+  } else if (v4) {
+    const int n = (a.d + 1023) / 1024;
+    if (n <= 1) GO(4, 1, 256, true);
+    else if (n <= 2) GO(4, 2, 256, true);
+    else if (n <= 4 && few) GO(4, 4, 256, true);
+    else if (n <= 4) GO(4, 4, 256, false);
+    else if (n <= 8) GO(4, 8, 256, false);
+    else if (n <= 16) GO(4, 16, 256, false);
+    else return 10;
+  } else {
+    const int n = (a.d + 255) / 256;
+    if (n <= 1) GO(1, 1, 256, false);
+    else if (n <= 4) GO(1, 4, 256, false);
+    else if (n <= 16) GO(1, 16, 256, false);
+    else return 10;
+  }
+#undef GO
+  return hipGetLastError() == hipSuccess ? 0 : 4;
+}
+
 }  // namespace
 
 // dtype: 0 fp32, 1 bf16 (of embed, a, bias, gains, ls, h)
@@ -246,5 +425,21 @@ KCA_API int kca_norm_residual(int dtype, const void* x_in, const void* embed, co
                    (float*)x_out, h, T, d, layer};
   if (dtype == 0) return launch<float>(p, s);
   if (dtype == 1) return launch<bf16_t>(p, s);
+  return 3;
+}
+
+// Mirrored by ops/norm_residual.py
+KCA_API int kca_prenorm_abi() { return (int)sizeof(PreArgs); }
+
+// dtype: 0 fp32, 1 bf16 (of every tensor but the stream)
+KCA_API int kca_prenorm(const PreArgs* in, int dtype, hipStream_t s) {
+  const PreArgs& p = *in;
+  const int src = (p.x_in != nullptr) + (p.embed != nullptr) + (p.base != nullptr);
+  if (p.T < 1 || p.d < 1 || src != 1 || (p.embed && !p.tokens) || (!p.a && (p.ga || p.b)) || (p.b && (!p.ga || !p.gb)) ||
+      (p.h && !p.g) || (!p.h && !p.x_out && !p.raw))
+    return 1;
+  if (p.x_in && p.x_in == p.x_out && p.rows) return 2;
+  if (dtype == 0) return launch_pre<float>(p, s);
+  if (dtype == 1) return launch_pre<bf16_t>(p, s);
   return 3;
 }

@@ -79,7 +79,7 @@ struct MmJob {
   int N;
   int tiles;              // workgroups of this job (set by the host entry point)
   const uint16_t* bias;   // [N] (nullable)
-  int act;                // 0 none, 1 GELU tanh, 2 GELU erf (not with res)
+  int act;                // 0 none, 1 GELU tanh, 2 GELU erf, 3 squared ReLU (not with res)
   uint16_t* y;            // [M, N] (row stride ldy)
   long long ldy;
   const uint16_t* res;    // [M, N] residual added after the bias (nullable; may alias y)
@@ -128,6 +128,9 @@ __device__ __forceinline__ void mm_store(const MmJob& J, int M, int n_base, int 
   } else if (J.act == 2) {
 #pragma unroll
     for (int i = 0; i < 4; ++i) o[i] = 0.5f * o[i] * (1.f + erff(o[i] * 0.70710678118654752f));
+  } else if (J.act == 3) {
+#pragma unroll
+    for (int i = 0; i < 4; ++i) o[i] = fmaxf(o[i], 0.f) * fmaxf(o[i], 0.f);
   }
   if (J.res && ok) {
     const uint2 r = *reinterpret_cast<const uint2*>(J.res + (long long)m * J.ldr + n);

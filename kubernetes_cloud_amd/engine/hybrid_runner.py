@@ -11,7 +11,7 @@ A layer's token mixer is an object of ``mixers`` (attention over the paged cache
 state); around it a parallel layer takes three or four launches beside the vendor (or skinny matrix-core)
 products -- residual + norm + token shift, the mixer's core, the feed-forward's activation or experts; mixer and
 feed-forward close in one product -- and a sandwich layer one norm launch per sublayer (output norm, layer scale,
-residual and the next norm together). Layers may run several times in a row (``cfg.runs``); every run has its own
+residual and the next norm together); a pre-norm layer is one norm launch per sublayer too. Layers may run several times in a row (``cfg.runs``); every run has its own
 cache or state.
 
 What a sequence owns besides its KV pages lives in ``SlotState``: the last normed row of every parallel layer
@@ -31,12 +31,13 @@ from ..ops import skinny_mm as smm
 from ..ops.delta_rule import Portions, plan_portions
 from ..ops.gemv import skinny_linear
 from ..ops.latent_attention import Prompts, plan_prompts
-from ..ops.norm_residual import NormedBranch, norm_residual
+from ..ops.norm_residual import Embedded, NormedBranch, NormedPair, Rows, norm_residual, prenorm
 from ..ops.rms_shift import Branch, rms_shift
 from .mixers import make_mixer
 from .runner import KVCache, SlotState, StepRunner
 
 SPLIT_CLOSE = (1024, 4096)  # rows between which the closing product runs as two (HybridRunner._close)
+ACTS = {2: "gelu", 3: "relu2"}  # activation codes of the streaming products
 SKINNY_M = 16   # rows up to which projections stream on the skinny matrix-core kernel
 
 
@@ -72,7 +73,8 @@ class HybridRunner(StepRunner):
             self.mixers.append(make_mixer(model.layers[i], cfg, r, self._linear, first.get(i)))
             first.setdefault(i, self.mixers[-1])
         shapes, widths = [], {"shift": (len(cfg.runs), d)} if cfg.block == "parallel" else {}
-        for mx in self.mixers:
+        members = [m for mx in self.mixers for m in mx.members()]
+        for mx in members:
             shape = mx.cache_shape()
             if shape is not None:
                 mx.index = len(shapes)
@@ -81,16 +83,17 @@ class HybridRunner(StepRunner):
         self.cache = KVCache(len(shapes), max_slots, 0, self.max_len, 0, self.device, self.dtype, page_size=page_size,
                              n_pages=kv_pages, layer_shapes=shapes)
         self.state = SlotState(max_slots, widths, self.device)
-        for mx in self.mixers:
+        for mx in members:
             mx.cache, mx.state = self.cache, self.state
-        self._forward_layers = {"parallel": self._parallel, "sandwich": self._sandwich}[cfg.block]
+        self._members = members
+        self._forward_layers = {"parallel": self._parallel, "sandwich": self._sandwich, "prenorm": self._prenorm}[cfg.block]
         if self.device.type == "cuda":
             from ..utils import tunable
             tunable.ensure(tunable.DECODE_FILE)
 
     # ---------------------------------------------------------------- linear
     def _linear(self, x, w, out=None, act: int = 0):
-        """x W^T (act 2: exact GELU). Few bf16 rows stream the weight on the GEMV / skinny matrix-core kernels."""
+        """x W^T (act 2: exact GELU, 3: squared ReLU). Few bf16 rows stream the weight on the GEMV / skinny matrix-core kernels."""
         T = x.shape[0]
         if (x.is_cuda and x.dtype == torch.bfloat16 and T <= SKINNY_M and w.shape[0] % 4 == 0 and smm.supported(x, w)
                 and (out is None or (out.data_ptr() % 16 == 0 and out.stride(0) % 8 == 0))):
@@ -101,7 +104,7 @@ class HybridRunner(StepRunner):
             return smm.mm(x, w, None, act, out=out, packed=self._packed_w(w))
         y = F.linear(x, w)
         if act:
-            return moe.act_rows(y, torch.empty_like(y) if out is None else out, gated=False)
+            return moe.act_rows(y, y if out is None else out, gated=False, act=ACTS[act])
         if out is not None:
             out.copy_(y)
             return out
@@ -144,7 +147,9 @@ class HybridRunner(StepRunner):
     def _forward(self, b: _Batch, want: torch.Tensor | None, layers_out: list | None = None) -> torch.Tensor:
         """Logits of the rows in ``want`` (None: every row). ``layers_out`` collects the residual stream after
         every layer run."""
-        return self._linear(self._forward_layers(b, want, layers_out), self.model.head)
+        logits = self._linear(self._forward_layers(b, want, layers_out), self.model.head_weight)
+        cap = self.cfg.logit_softcap
+        return moe.act_rows(logits, logits, False, act="softcap", cap=cap) if cap else logits
 
     def _parallel(self, b, want, layers_out):
         """One norm and token shift a layer feed mixer and feed-forward side by side."""
@@ -200,6 +205,46 @@ class HybridRunner(StepRunner):
         if layers_out is not None:
             layers_out.append(norm_residual(x, branch, None, eps, **src)[0])
         return norm_residual(x, branch, m.final_norm, eps, rows=want, keep_x=False, **src)[1]
+
+    def _prenorm(self, b, want, layers_out):
+        """Mixer and feed-forward in turn, each normed before. A loop's passes start from a product of the stream
+        beside the embedding output: both lie in one buffer, rounded, [x | x0]."""
+        m, cfg, eps, T, d = self.model, self.cfg, self.cfg.norm_eps, b.T, self.cfg.hidden
+        x, branch = Embedded(m.wte, b.tokens, cfg.embed_scale), None
+        entry = cfg.loop is not None and cfg.loop.entry and cfg.loop.start < cfg.loop.stop and cfg.loop.times > 0
+        xx0 = torch.empty(T, 2 * d, device=m.wte.device, dtype=m.wte.dtype) if entry else None
+        for r, (i, opens) in enumerate(zip(cfg.runs, cfg.opens)):
+            L = m.layers[i]
+            if entry and r == 0:
+                prenorm(x, None, None, eps, raw=xx0[:, d:], keep_x=False)
+            if entry and opens is not None:
+                out = prenorm(x, branch, None, eps, raw=xx0[:, :d], keep_x=layers_out is not None)[0]
+                if layers_out is not None and r:
+                    layers_out.append(out)
+                x, branch = Rows(self._linear(xx0, m.loop_in), m.loop_step[opens]), None
+                x, h = prenorm(x, None, L.norm, eps)
+            else:
+                x, h = prenorm(x, branch, L.norm, eps)
+                if layers_out is not None and r:
+                    layers_out.append(x.clone())
+            branch = self._mix(L, self.mixers[r], h, b)
+            if L.spec.mlp is not None:
+                x, h = prenorm(x, branch, L.norm2, eps)
+                y = self._linear(h, L.w_up, act=3 if L.spec.mlp.act == "relu2" else 2)
+                branch = self._linear(y, L.w_down)
+        if layers_out is not None:
+            layers_out.append(prenorm(x, branch, None, eps)[0])
+        return prenorm(x, branch, m.final_norm, eps, rows=want, keep_x=False)[1]
+
+    def _mix(self, L, mixer, h, b):
+        """A pre-norm layer's mixer -> what it adds to the stream."""
+        pair = getattr(mixer, "sides", None)
+        y = torch.empty(b.T, mixer.out_width if pair else L.spec.mixer.out_cols, device=h.device, dtype=h.dtype)
+        mixer(self._linear(h, L.w_in), y, b)
+        if not pair:
+            return self._linear(y, L.w_out)
+        ys = [self._linear(y[:, o], s.w_out) for o, s in zip(mixer.outs, (L.left, L.right))]
+        return NormedPair(ys[0], L.left.out_norm, ys[1], L.right.out_norm, L.spec.mixer.mul)
 
     # ------------------------------------------------------- portions + tokens
     def _plan(self, entries, want_rows) -> tuple[_Batch, torch.Tensor | None]:
@@ -295,7 +340,7 @@ class HybridRunner(StepRunner):
     # ---------------------------------------------------------------- decode
     def _step_buffers(self, Bb: int, Kb: int) -> dict:
         need = {"ws": (1, torch.float32), "cnt": (1, torch.int32)}
-        for mx in self.mixers:
+        for mx in self._members:
             for k, (n, dt) in mx.buffers(Bb, Kb, self.dtype).items():
                 need[k] = (max(n, need.get(k, (1, dt))[0]), dt)
         return {k: torch.zeros(n, device=self.device, dtype=dt) for k, (n, dt) in need.items()}

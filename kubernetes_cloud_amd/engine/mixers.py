@@ -8,8 +8,10 @@ from __future__ import annotations
 
 import torch
 
-from ..models.hybrid_config import (ChannelDeltaSpec, DiffAttentionSpec, GatedRecurrenceSpec, GeneralDeltaSpec,
-                                    LatentAttentionSpec)
+from ..models.hybrid_config import (BiasedAttentionSpec, ChannelDeltaSpec, DiffAttentionSpec, GatedRecurrenceSpec,
+                                    GeneralDeltaSpec, HeadDeltaSpec, LatentAttentionSpec, SideBySideSpec, SsdSpec,
+                                    aligned_parts)
+from ..ops import biased_attention as ba
 from ..ops import delta_rule as dr
 from ..ops import diff_attention as da
 from ..ops import gated_scan as gs
@@ -18,13 +20,17 @@ from ..ops import moe
 
 
 class Mixer:
-    """``run``: index of the layer run; ``linear``: the runner's projection; ``twin``: the mixer of an earlier
+    """``run``: the layer run (names its state); ``linear``: the runner's projection; ``twin``: the mixer of an earlier
     pass over the same layer (shares what is derived from the weights). ``cache`` / ``index`` (the layer's
     place in it) and ``state`` are set once the runner has made them."""
 
-    def __init__(self, layer, cfg, run: int, linear, twin: Mixer | None = None):
+    def __init__(self, layer, cfg, run: int | str, linear, twin: Mixer | None = None):
         self.layer, self.run, self.linear = layer, run, linear
         self.cache = self.index = self.state = None
+
+    def members(self) -> list:
+        """The mixers that keep something: itself, or the ones it is made of."""
+        return [self]
 
     def cache_shape(self):
         """(key heads, key size, value heads, value size) of the layer's pages, None without a cache."""
@@ -119,10 +125,18 @@ class DeltaRuleMixer(Mixer):
         super().__init__(layer, cfg, run, linear)
         mx, L = layer.spec.mixer, layer
         at = lambda *names: tuple(mx.parts[n][0] for n in names)  # noqa: E731
-        if mx.general:
+        if isinstance(mx, GeneralDeltaSpec):
             self.sp = dr.DeltaHeads(True, mx.heads, mx.heads, mx.dim, mx.dim, at("r", "k", "v", "a", "g", "w1"),
                                     mx.rank_w, cfg.norm_eps)
             self.wt = dr.DeltaWeights(L.w2, L.w0, L.a_bias, L.gain)
+        elif isinstance(mx, HeadDeltaSpec):
+            self.sp = dr.DeltaHeads(False, mx.heads, mx.kv_heads, mx.dim, mx.vdim, at("q", "k", "v", "b", "g", "a"), 0,
+                                    cfg.norm_eps, mx.taps, form="head")
+            self.wt = dr.DeltaWeights(None, L.dt_bias, L.a_log, L.gain, conv=L.conv)
+        elif isinstance(mx, SsdSpec):
+            self.sp = dr.DeltaHeads(False, mx.heads, mx.groups, mx.state, mx.vdim, at("C", "B", "x", "dt", "z", "dt"), 0,
+                                    cfg.norm_eps, mx.taps, form="ssd", norm_groups=mx.norm_groups)
+            self.wt = dr.DeltaWeights(None, L.dt_bias, L.a_log, L.gain, conv=L.conv, conv_b=L.conv_b, skip=L.skip)
         else:
             self.sp = dr.DeltaHeads(False, mx.heads, mx.kv_heads, mx.dim, mx.vdim, at("q", "k", "v", "b", "g1", "a1"),
                                     mx.rank_w, cfg.norm_eps, mx.taps, mx.rank_g)
@@ -141,17 +155,73 @@ class DeltaRuleMixer(Mixer):
         if b.single:
             dr.delta_step(sp, wt, x, S, ring, b.pos, b.slots, out)
             return
+        if sp.kind >= 2:
+            dr.delta_portions(sp, wt, x, S, ring, b.portions, out)
+            return
         tanh = lambda t: moe.act_rows(t, torch.empty_like(t, memory_format=torch.contiguous_format), False, act="tanh")  # noqa: E731
         inner, gate = dr.low_rank_inner(sp, x, tanh)
         dr.delta_portions(sp, wt, x, S, ring, b.portions, out, self.linear(inner, wt.lo_w),
                           None if gate is None else self.linear(gate, wt.lo_g))
 
 
+class BiasedAttentionMixer(Mixer):
+    def __init__(self, layer, cfg, run, linear, twin=None):
+        super().__init__(layer, cfg, run, linear)
+        mx, L = layer.spec.mixer, layer
+        self.sp = ba.BiasedHeads(mx.heads, mx.kv_heads, mx.dim, mx.vdim, mx.scale, cfg.norm_eps,
+                                 tuple(mx.parts[n][0] for n in "qkvg"))
+        self.wt = twin.wt if twin is not None else ba.BiasedWeights(L.q_norm, L.k_norm, ba.bias_by_distance(L.rel, mx.bias_max),
+                                                                    L.sink.float())
+
+    def cache_shape(self):
+        mx = self.layer.spec.mixer
+        return mx.kv_heads, mx.dim, mx.kv_heads, mx.vdim
+
+    def buffers(self, rows, max_kv, dtype):
+        _, _, w, c = ba.rows_plan(self.sp, rows, max_kv)
+        return {"ws": (w, torch.float32), "cnt": (c, torch.int32)}
+
+    def __call__(self, x, out, b):
+        a = (self.sp, self.wt, x, self.cache.k[self.index], self.cache.v[self.index], self.cache.table, b.pos, b.slots)
+        if b.single:
+            ba.attend_rows(*a, out, b.max_kv, fused_append=True, ws=b.bufs.get("ws"), cnt=b.bufs.get("cnt"))
+            return
+        ba.append(*a)
+        if out.is_cuda and ba.tiles_ok(self.sp, out.dtype, self.cache.page_size, x.stride(0), out.stride(0)):
+            if b.tiles is not None:
+                ba.attend_tiles(*a, out, b.tiles)
+            if b.row_of is not None:
+                ba.attend_rows(*a, out, b.row_kv, fused_append=False, row_of=b.row_of)
+        else:
+            ba.attend_rows(*a, out, b.max_kv, fused_append=False)
+
+
+class SideBySideMixer(Mixer):
+    """Two mixers over column blocks of the projection rows, into column blocks of the output rows."""
+
+    def __init__(self, layer, cfg, run, linear, twin=None):
+        super().__init__(layer, cfg, run, linear)
+        self.sides = [make_mixer(m, cfg, f"{run}.{k}", linear, twin and twin.sides[k]) for k, m in enumerate((layer.left, layer.right))]
+        mx = layer.spec.mixer
+        self.cols = (slice(0, mx.left.in_rows), slice(mx.in_rows - mx.right.in_rows, mx.in_rows))
+        parts, self.out_width = aligned_parts({"left": mx.left.out_cols, "right": mx.right.out_cols})
+        self.outs = tuple(slice(o, o + n) for o, n in parts.values())
+
+    def members(self):
+        return [m for s in self.sides for m in s.members()]
+
+    def __call__(self, x, out, b):
+        for m, c, o in zip(self.sides, self.cols, self.outs):
+            m(x[:, c], out[:, o], b)
+
+
 MIXERS = {DiffAttentionSpec: DiffAttentionMixer, GatedRecurrenceSpec: GatedRecurrenceMixer,
-          LatentAttentionSpec: LatentAttentionMixer, GeneralDeltaSpec: DeltaRuleMixer, ChannelDeltaSpec: DeltaRuleMixer}
+          LatentAttentionSpec: LatentAttentionMixer, GeneralDeltaSpec: DeltaRuleMixer, ChannelDeltaSpec: DeltaRuleMixer,
+          HeadDeltaSpec: DeltaRuleMixer, SsdSpec: DeltaRuleMixer, BiasedAttentionSpec: BiasedAttentionMixer,
+          SideBySideSpec: SideBySideMixer}
 
 
-def make_mixer(layer, cfg, run: int, linear, twin: Mixer | None = None) -> Mixer:
+def make_mixer(layer, cfg, run: int | str, linear, twin: Mixer | None = None) -> Mixer:
     return MIXERS[type(layer.spec.mixer)](layer, cfg, run, linear, twin)
 
 

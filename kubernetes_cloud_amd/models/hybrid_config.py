@@ -206,8 +206,157 @@ class ChannelDeltaSpec:
 
 
 @dataclasses.dataclass(frozen=True)
+class BiasedAttentionSpec:
+    """Attention without rotation: RMS-normed queries and keys, a learned bias by bucketed distance (``bias_rows``
+    buckets, spaced in ln(distance) up to ``bias_max`` beyond the near half), a learned sink per head, and a
+    sigmoid gate on the heads' outputs."""
+    heads: int
+    kv_heads: int
+    dim: int
+    vdim: int
+    scale: float
+    bias_max: float
+    bias_rows: int = 32
+
+    def __post_init__(self):
+        if self.heads % self.kv_heads:
+            raise ValueError(f"{self.heads} query heads over {self.kv_heads} key/value heads")
+
+    @property
+    def _sizes(self) -> dict:
+        return {"q": self.heads * self.dim, "k": self.kv_heads * self.dim, "v": self.kv_heads * self.vdim,
+                "g": self.heads * self.vdim}
+
+    @property
+    def parts(self) -> dict:
+        return aligned_parts(self._sizes)[0]
+
+    @property
+    def in_rows(self) -> int:
+        return aligned_parts(self._sizes)[1]
+
+    @property
+    def out_cols(self) -> int:
+        return self.heads * self.vdim
+
+    @property
+    def extra(self) -> dict:
+        return {"q_norm": (self.dim,), "k_norm": (self.dim,), "rel": (self.bias_rows, self.heads), "sink": (self.heads,)}
+
+
+@dataclasses.dataclass(frozen=True)
+class HeadDeltaSpec:
+    """Gated delta rule with one decay per head: q / k heads shared by groups of value heads, short causal
+    convolutions before unit keys and queries, a silu gate on the normed read-out."""
+    heads: int
+    kv_heads: int
+    dim: int
+    vdim: int
+    taps: int
+
+    def __post_init__(self):
+        if self.heads % self.kv_heads:
+            raise ValueError(f"{self.heads} heads over {self.kv_heads} query/key heads")
+
+    @property
+    def conv_channels(self) -> int:
+        return 2 * self.kv_heads * self.dim + self.heads * self.vdim
+
+    @property
+    def _sizes(self) -> dict:
+        n = self.kv_heads * self.dim
+        return {"q": n, "k": n, "v": self.heads * self.vdim, "g": self.heads * self.vdim, "b": self.heads, "a": self.heads}
+
+    @property
+    def parts(self) -> dict:
+        return aligned_parts(self._sizes)[0]
+
+    @property
+    def in_rows(self) -> int:
+        return aligned_parts(self._sizes)[1]
+
+    @property
+    def out_cols(self) -> int:
+        return self.heads * self.vdim
+
+    @property
+    def extra(self) -> dict:
+        H = self.heads
+        return {"conv": (self.conv_channels, self.taps), "dt_bias": (H,), "a_log": (H,), "gain": (self.vdim,)}
+
+
+@dataclasses.dataclass(frozen=True)
+class SsdSpec:
+    """Selective state space with one decay per head (state-space duality): ``groups`` of heads share B and C of
+    size ``state``; a short causal convolution with a bias; the gated output is normed in ``norm_groups`` parts."""
+    heads: int
+    groups: int
+    state: int
+    vdim: int
+    taps: int
+    norm_groups: int = 1
+
+    def __post_init__(self):
+        if self.heads % self.groups:
+            raise ValueError(f"{self.heads} heads over {self.groups} groups")
+        if self.heads * self.vdim % self.norm_groups:
+            raise ValueError(f"{self.heads * self.vdim} channels in {self.norm_groups} equal parts")
+
+    @property
+    def conv_channels(self) -> int:
+        return 2 * self.groups * self.state + self.heads * self.vdim
+
+    @property
+    def _sizes(self) -> dict:
+        n = self.groups * self.state
+        return {"C": n, "B": n, "x": self.heads * self.vdim, "z": self.heads * self.vdim, "dt": self.heads}
+
+    @property
+    def parts(self) -> dict:
+        return aligned_parts(self._sizes)[0]
+
+    @property
+    def in_rows(self) -> int:
+        return aligned_parts(self._sizes)[1]
+
+    @property
+    def out_cols(self) -> int:
+        return self.heads * self.vdim
+
+    @property
+    def extra(self) -> dict:
+        """``conv`` / ``conv_b``: channels in the order C, B, x."""
+        H = self.heads
+        return {"conv": (self.conv_channels, self.taps), "conv_b": (self.conv_channels,), "dt_bias": (H,), "a_log": (H,),
+                "skip": (H,), "gain": (self.out_cols,)}
+
+
+@dataclasses.dataclass(frozen=True)
+class SideBySideSpec:
+    """Two mixers of the same input, each with an output projection and an output norm of its own; the layer adds
+    ``mul`` times the sum of the normed outputs."""
+    left: BiasedAttentionSpec | HeadDeltaSpec | SsdSpec
+    right: BiasedAttentionSpec | HeadDeltaSpec | SsdSpec
+    mul: float = 0.5
+
+    @property
+    def in_rows(self) -> int:
+        return self.left.in_rows + self.right.in_rows
+
+    @property
+    def out_cols(self) -> int:
+        return self.left.out_cols + self.right.out_cols
+
+    @property
+    def extra(self) -> dict:
+        return {f"{s}.{k}": v for s in ("left", "right") for k, v in getattr(self, s).extra.items()}
+
+
+@dataclasses.dataclass(frozen=True)
 class DenseSpec:
+    """W_down act(W_up h); ``act``: "gelu" (exact) or "relu2" (squared ReLU)."""
     ff: int
+    act: str = "gelu"
 
 
 @dataclasses.dataclass(frozen=True)
@@ -231,17 +380,20 @@ class MoESpec:
 
 @dataclasses.dataclass(frozen=True)
 class LayerSpec:
-    mixer: (DiffAttentionSpec | GatedRecurrenceSpec | LatentAttentionSpec | GeneralDeltaSpec | ChannelDeltaSpec)
+    mixer: (DiffAttentionSpec | GatedRecurrenceSpec | LatentAttentionSpec | GeneralDeltaSpec | ChannelDeltaSpec |
+            BiasedAttentionSpec | HeadDeltaSpec | SsdSpec | SideBySideSpec)
     mlp: DenseSpec | GatedDenseSpec | MoESpec | None
 
 
 @dataclasses.dataclass(frozen=True)
 class LoopSpec:
     """Layers ``start`` .. ``stop - 1`` run ``times`` times in a row with the same weights; every pass has its
-    own cache or state."""
+    own cache or state. ``entry``: a pass starts from a projection of the stream beside the embedding output, plus
+    one vector per pass."""
     start: int
     stop: int
     times: int
+    entry: bool = False
 
 
 @dataclasses.dataclass
@@ -252,7 +404,12 @@ class HybridConfig:
     layers: tuple
     norm_eps: float = 1e-5
     residual_mult: float = 1.0
-    block: str = "parallel"      # one norm feeds mixer and feed-forward | "sandwich": in turn, normed before and after
+    # one norm feeds mixer and feed-forward | "sandwich": in turn, normed before and after | "prenorm": in turn,
+    # RMS-normed before, gains stored around zero
+    block: str = "parallel"
+    embed_scale: float = 1.0
+    tied: bool = False           # the embedding table is the output projection
+    logit_softcap: float = 0.0   # cap tanh(logits / cap); 0: none
     loop: LoopSpec | None = None
     max_pos: int = 8192          # serving default; the design itself sets no limit
     bos_token_id: int | None = None
@@ -274,6 +431,16 @@ class HybridConfig:
             raise ValueError(f"loop {lp} over {n} layers")
         return (*range(lp.start), *(tuple(range(lp.start, lp.stop)) * lp.times), *range(lp.stop, n))
 
+    @property
+    def opens(self) -> tuple:
+        """For every run, the loop pass it opens, or None."""
+        lp = self.loop
+        if lp is None or lp.start == lp.stop:
+            return (None,) * len(self.runs)
+        n = lp.stop - lp.start
+        return tuple((r - lp.start) // n if 0 <= r - lp.start < n * lp.times and (r - lp.start) % n == 0 else None
+                     for r in range(len(self.runs)))
+
     def to_hf(self) -> dict:
         return dict(self.hf)
 
@@ -284,13 +451,16 @@ class HybridConfig:
                 n *= x
             return n
 
-        d = self.hidden
-        n = 2 * self.vocab_size * d + (1 if self.block == "parallel" else d)
+        d, pre = self.hidden, self.block == "prenorm"
+        n = (1 if self.tied else 2) * self.vocab_size * d + (1 if self.block == "parallel" else d)
+        if self.loop is not None and self.loop.entry:
+            n += (2 * d + self.loop.times) * d
         for L in self.layers:
             n += (L.mixer.in_rows + L.mixer.out_cols) * d + sum(numel(s) for s in L.mixer.extra.values())
-            n += 1 + d if self.block == "parallel" else 3 * d
+            n += 2 * d if isinstance(L.mixer, SideBySideSpec) else 0
+            n += 1 + d if self.block == "parallel" else d if pre else 3 * d
             if isinstance(L.mlp, DenseSpec):
-                n += 2 * d * L.mlp.ff
+                n += 2 * d * L.mlp.ff + (d if pre else 0)
             elif isinstance(L.mlp, GatedDenseSpec):
                 n += 3 * d * L.mlp.ff + 2 * L.mlp.ff + 4 * d
             elif L.mlp is not None:
@@ -300,4 +470,5 @@ class HybridConfig:
 
 
 __all__ = ["HybridConfig", "LayerSpec", "LoopSpec", "DiffAttentionSpec", "GatedRecurrenceSpec", "LatentAttentionSpec",
-           "GeneralDeltaSpec", "ChannelDeltaSpec", "DenseSpec", "GatedDenseSpec", "MoESpec", "aligned_parts"]
+           "GeneralDeltaSpec", "ChannelDeltaSpec", "BiasedAttentionSpec", "HeadDeltaSpec", "SsdSpec", "SideBySideSpec",
+           "DenseSpec", "GatedDenseSpec", "MoESpec", "aligned_parts"]

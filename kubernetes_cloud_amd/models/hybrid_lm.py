@@ -1,5 +1,6 @@
-"""Decoders whose layers mix tokens differently (``HybridConfig``): differential or latent attention, a gated
-recurrence or a delta rule, beside a dense, gated, routed or no feed-forward, on an fp32 residual stream.
+"""Decoders whose layers mix tokens differently (``HybridConfig``): differential, latent or biased attention, a gated
+recurrence, a delta rule, a state space, or two of them side by side, beside a dense, gated, routed or no
+feed-forward, on an fp32 residual stream.
 
 ``block`` "parallel": with h the normed stream and hs its token-shifted copy,
 
@@ -9,6 +10,11 @@ recurrence or a delta rule, beside a dense, gated, routed or no feed-forward, on
 
     x <- x + scale * N(mixer(N(x))),   x <- x + scale2 * N(ff(N(x)))
 
+"prenorm": the same two sublayers, RMS-normed before only (gains stored minus one); two mixers side by side are
+normed after their own output projections and averaged,
+
+    x <- x + mixer(N(x))   |   x + mul (N(left(N(x))) + N(right(N(x)))),      x <- x + ff(N(x))
+
 The modules hold weights laid out for the kernels; the step itself (cache, state, batching) is
 ``engine.hybrid_runner``. Layout:
 
@@ -16,6 +22,7 @@ The modules hold weights laid out for the kernels; the step itself (cache, state
   blocks start at multiples of 8 rows)
 * ``w_out``  the mixer's output projection; parallel layers put the dense (or shared-expert) down projection
   beside it, [d, mixer + ff]: both branches close in one product, summed in fp32 before its rounding
+* two mixers side by side: one ``w_in`` for both; ``left`` / ``right`` hold the rest of each
 * ``w_up``   gate and up projections of a gated feed-forward, one above the other
 * experts stacked: gate-and-up [E, 2F, d], down [E, d, F]
 """
@@ -24,11 +31,22 @@ from __future__ import annotations
 import torch
 import torch.nn as nn
 
-from .hybrid_config import DenseSpec, GatedDenseSpec, HybridConfig, LayerSpec, MoESpec
+from .hybrid_config import DenseSpec, GatedDenseSpec, HybridConfig, LayerSpec, MoESpec, SideBySideSpec
 
 
 def _p(*shape):
     return nn.Parameter(torch.empty(*shape), requires_grad=False)
+
+
+class SideMixer(nn.Module):
+    """One of two mixers side by side: its parameters behind the layer's common input projection."""
+
+    def __init__(self, d: int, mixer):
+        super().__init__()
+        self.spec = LayerSpec(mixer, None)
+        for name, shape in mixer.extra.items():
+            setattr(self, name, _p(*shape))
+        self.w_out, self.out_norm = _p(d, mixer.out_cols), _p(d)
 
 
 class HybridLayer(nn.Module):
@@ -37,9 +55,23 @@ class HybridLayer(nn.Module):
         d, mx, mlp = cfg.hidden, spec.mixer, spec.mlp
         self.spec = spec
         self.w_in = _p(mx.in_rows, d)
-        for name, shape in mx.extra.items():
+        pair = isinstance(mx, SideBySideSpec)
+        if pair and cfg.block != "prenorm":
+            raise ValueError(f"mixers side by side belong to prenorm layers, not {cfg.block}")
+        for name, shape in ({} if pair else mx.extra).items():
             setattr(self, name, _p(*shape))
         self.moe = isinstance(mlp, MoESpec)
+        if cfg.block == "prenorm":
+            if mlp is not None and not isinstance(mlp, DenseSpec):
+                raise ValueError(f"prenorm layers take a dense feed-forward or none, not {type(mlp).__name__}")
+            self.norm = _p(d)
+            if pair:
+                self.left, self.right = SideMixer(d, mx.left), SideMixer(d, mx.right)
+            else:
+                self.w_out = _p(d, mx.out_cols)
+            if mlp is not None:
+                self.norm2, self.w_up, self.w_down = _p(d), _p(mlp.ff, d), _p(d, mlp.ff)
+            return
         if cfg.block == "sandwich":
             if mlp is not None and not isinstance(mlp, GatedDenseSpec):
                 raise ValueError(f"sandwich layers take a gated feed-forward or none, not {type(mlp).__name__}")
@@ -76,16 +108,27 @@ class HybridLM(nn.Module):
         self.cfg = cfg
         self.wte = _p(cfg.vocab_size, cfg.hidden)
         self.layers = nn.ModuleList([HybridLayer(cfg, s) for s in cfg.layers])
-        self.final_norm = _p(cfg.hidden) if cfg.block == "sandwich" else nn.Parameter(torch.empty(()), requires_grad=False)
-        self.head = _p(cfg.vocab_size, cfg.hidden)
+        self.final_norm = _p(cfg.hidden) if cfg.block != "parallel" else nn.Parameter(torch.empty(()), requires_grad=False)
+        self.head = None if cfg.tied else _p(cfg.vocab_size, cfg.hidden)
+        if cfg.loop is not None and cfg.loop.entry:
+            if cfg.block != "prenorm":
+                raise ValueError(f"projected loop entries belong to prenorm layers, not {cfg.block}")
+            self.loop_in, self.loop_step = _p(cfg.hidden, 2 * cfg.hidden), _p(cfg.loop.times, cfg.hidden)
+
+    @property
+    def head_weight(self) -> torch.Tensor:
+        return self.wte if self.head is None else self.head
 
     @torch.no_grad()
     def init_weights(self, std: float = 0.02, seed: int | None = None):
         g = torch.Generator(device=self.wte.device)
         if seed is not None:
             g.manual_seed(seed)
+        around_zero = ("norm", "norm2", "final_norm") if self.cfg.block == "prenorm" else ()
         for name, p in self.named_parameters():
-            if p.dim() >= 2:
+            if name.rsplit(".", 1)[-1] in around_zero:
+                p.zero_()
+            elif p.dim() >= 2:
                 p.normal_(0.0, std, generator=g)
             elif any(k in name for k in ("norm", "scale", "gain")):
                 p.fill_(1.0)

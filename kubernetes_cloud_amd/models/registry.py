@@ -48,6 +48,18 @@ def _rezusun() -> Family:
                   rezusun.with_shapes)
 
 
+def _begopel() -> Family:
+    from . import begopel
+    from .hybrid_lm import build_hybrid
+
+    def runner():
+        from ..engine.hybrid_runner import HybridRunner
+        return HybridRunner
+    return Family("begopel", begopel.read_config, build_hybrid, begopel.to_native, begopel.from_native, runner,
+                  ("norm_residual", "delta_rule", "delta_chunk", "biased_attn", "act_rows", "gemv", "skinny_mfma"),
+                  begopel.with_shapes)
+
+
 def _causal_lm() -> Family:
     from .causal_lm import build_causal_lm
     from .config import LMConfig
@@ -59,7 +71,7 @@ def _causal_lm() -> Family:
     return Family("causal_lm", LMConfig.read_hf, build_causal_lm, hf_to_native, native_to_hf, runner)
 
 
-FAMILIES = {"Megusun": _megusun, "Rezusun": _rezusun}   # config.json "architecture" -> family
+FAMILIES = {"Megusun": _megusun, "Rezusun": _rezusun, "Begopel": _begopel}   # config.json "architecture" -> family
 
 
 def family_of_dict(cfg: dict) -> Family:

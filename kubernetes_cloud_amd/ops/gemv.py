@@ -14,7 +14,7 @@ import torch.nn.functional as F
 
 from . import _lib
 
-ACT = {None: 0, "none": 0, "tanh": 1, "gelu_tanh": 1, "erf": 2, "none_erf": 2}
+ACT = {None: 0, "none": 0, "tanh": 1, "gelu_tanh": 1, "erf": 2, "none_erf": 2, "relu2": 3}
 
 
 def _act_ref(y, act):
@@ -22,6 +22,8 @@ def _act_ref(y, act):
         return F.gelu(y.float(), approximate="tanh").to(y.dtype)
     if act == 2:
         return F.gelu(y.float()).to(y.dtype)
+    if act == 3:
+        return (torch.relu(y.float()) ** 2).to(y.dtype)
     return y
 
 
@@ -92,6 +94,8 @@ def _linear_act(x, weight, bias, act):
     if not act:
         return F.linear(x, weight, bias)
     y = F.linear(x, weight, bias)
+    if act == 3:
+        return _act_ref(y, act)
     f16 = _lib.native_f16(y) and _lib.has("kca_gelu_fwd_f16")
     if (_lib.use_native(y) or f16) and y.is_contiguous() and y.numel() % 8 == 0 and y.data_ptr() % 16 == 0 \
             and y.dtype in (torch.bfloat16, torch.float16):

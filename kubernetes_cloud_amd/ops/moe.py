@@ -122,13 +122,14 @@ def experts(h: torch.Tensor, ids: torch.Tensor, weights: torch.Tensor, gate_up: 
     return y
 
 
-ACT_ROWS = {"gelu": 0, "silu_gated": 1, "gelu_tanh_gated": 2, "tanh": 3}
+ACT_ROWS = {"gelu": 0, "silu_gated": 1, "gelu_tanh_gated": 2, "tanh": 3, "relu2": 4, "softcap": 5}
 
 
 def act_rows(x: torch.Tensor, out: torch.Tensor, gated: bool, row_scale: torch.Tensor | None = None, *,
-             act: str | None = None, bias: torch.Tensor | None = None) -> torch.Tensor:
+             act: str | None = None, bias: torch.Tensor | None = None, cap: float = 0.0) -> torch.Tensor:
     """out = gelu(x) (exact), or silu(gate) * up * row_scale with x = [gate | up]; strided rows. ``act`` names
-    another form (``ACT_ROWS``); ``bias`` is added to x first."""
+    another form (``ACT_ROWS``; "softcap": cap tanh(x / cap)); ``bias`` is added to x first. Without a gate, out
+    may be x."""
     T, F = out.shape
     act = act or ("silu_gated" if gated else "gelu")
     gated = act.endswith("_gated")
@@ -143,10 +144,11 @@ def act_rows(x: torch.Tensor, out: torch.Tensor, gated: bool, row_scale: torch.T
                  0.5 * g * (1 + torch.tanh(math.sqrt(2 / math.pi) * (g + 0.044715 * g ** 3)))) * xf[:, F:]
             out.copy_(y if row_scale is None else y * row_scale[:, None])
         else:
-            out.copy_(torch.tanh(xf) if act == "tanh" else 0.5 * xf * (1 + torch.erf(xf / math.sqrt(2.0))))
+            out.copy_(torch.tanh(xf) if act == "tanh" else torch.relu(xf) ** 2 if act == "relu2" else
+                      cap * torch.tanh(xf / cap) if act == "softcap" else 0.5 * xf * (1 + torch.erf(xf / math.sqrt(2.0))))
         return out
     _lib.call("kca_act_rows", code, ACT_ROWS[act], x.data_ptr(), x.stride(0), _lib.ptr(row_scale), _lib.ptr(bias),
-              out.data_ptr(), out.stride(0), T, F, _lib.stream())
+              out.data_ptr(), out.stride(0), T, F, float(cap), _lib.stream())
     return out
 
 

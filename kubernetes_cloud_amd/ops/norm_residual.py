@@ -3,11 +3,16 @@
     x_t = x_in_t + ls * N(a_t + b; gb)        what a sublayer adds, normed and scaled
     h_t = N(x_t; g)                           what the next sublayer reads
 
-N: layer norm without a bias, or RMS norm. bf16 and fp32 GPU tensors run the kernel; CPU tensors run the
-reference below.
+N: layer norm without a bias, or RMS norm. Pre-norm layers (``prenorm``, RMS throughout) add a sublayer's output
+as it is, or the weighted sum of two normed ones, and norm with a gain stored around zero:
+
+    x_t = src_t + a_t   |   src_t + mul * (N(a_t; ga) + N(b_t; gb)),      h_t = N(x_t; 1 + g)
+
+bf16 and fp32 GPU tensors run the kernels; CPU tensors run the references below.
 """
 from __future__ import annotations
 
+import ctypes
 import dataclasses
 
 import torch
@@ -58,10 +63,100 @@ def norm_residual(x: torch.Tensor | None, branch: NormedBranch | None, gain: tor
     return x_out, h
 
 
+@dataclasses.dataclass
+class Embedded:
+    """A stream that starts at ``table[tokens] * scale``."""
+    table: torch.Tensor
+    tokens: torch.Tensor
+    scale: float = 1.0
+
+
+@dataclasses.dataclass
+class Rows:
+    """A stream that starts at a product's rows ``a`` [T, d] plus one vector."""
+    a: torch.Tensor
+    vec: torch.Tensor | None = None
+
+
+@dataclasses.dataclass
+class NormedPair:
+    """``mul * (N(a; gain_a) + N(b; gain_b))`` of two sublayers' outputs."""
+    a: torch.Tensor
+    gain_a: torch.Tensor
+    b: torch.Tensor
+    gain_b: torch.Tensor
+    mul: float = 0.5
+
+
+class _PreArgs(ctypes.Structure):
+    _P, _LL, _F, _I = ctypes.c_void_p, ctypes.c_longlong, ctypes.c_float, ctypes.c_int
+    _fields_ = [("x_in", _P), ("embed", _P), ("tokens", _P), ("escale", _F), ("base", _P), ("ldbase", _LL), ("vec", _P),
+                ("a", _P), ("lda", _LL), ("ga", _P), ("b", _P), ("ldb", _LL), ("gb", _P), ("mul", _F), ("g", _P),
+                ("eps", _F), ("rows", _P), ("x_out", _P), ("raw", _P), ("ldr", _LL), ("h", _P), ("T", _I), ("d", _I)]
+
+
+def prenorm(src: torch.Tensor | Embedded | Rows, branch: torch.Tensor | NormedPair | None, gain: torch.Tensor | None,
+            eps: float, *, raw: torch.Tensor | None = None, rows: torch.Tensor | None = None, keep_x: bool = True):
+    """-> (x_out fp32 | None, h | None). ``src``: the fp32 stream, or where it starts. ``branch``: what a sublayer
+    adds. ``gain``: the next norm's, minus one (None: no h). ``raw`` [T, d] (row stride free) receives x rounded to
+    its type. ``rows``: only these tokens."""
+    emb, prod = isinstance(src, Embedded), isinstance(src, Rows)
+    data = src.table if emb else src.a if prod else src
+    d = data.shape[1]
+    T = rows.shape[0] if rows is not None else (src.tokens if emb else data).shape[0]
+    pair = branch if isinstance(branch, NormedPair) else None
+    a = pair.a if pair else branch
+    ref = next(t for t in (gain, a, raw, data) if t is not None)
+    code = native_dt(ref, gain, a, raw, *((data,) if emb or prod else ()), src.vec if prod else None,
+                     *((pair.gain_a, pair.b, pair.gain_b) if pair else ()))
+    if code is None:
+        x = src.table[src.tokens].float() * src.scale if emb else src.a.float() if prod else src
+        if prod and src.vec is not None:
+            x = x + src.vec.float()
+        if pair:
+            x = x + pair.mul * (_norm(pair.a.float(), pair.gain_a, eps, False) + _norm(pair.b.float(), pair.gain_b, eps, False))
+        elif a is not None:
+            x = x + a.float()
+        if rows is not None:
+            x = x[rows.long()]
+        if raw is not None:
+            raw.copy_(x)
+        return (x if keep_x else None), (None if gain is None else _norm(x, 1 + gain.float(), eps, False).to(ref.dtype))
+    n_src = src.tokens.shape[0] if emb else data.shape[0]
+    assert data.stride(1) == 1 and (prod or data.is_contiguous()) and (emb or prod or data.dtype == torch.float32)
+    assert not emb or src.tokens.dtype == torch.int64
+    assert all(t is None or (t.stride(1) == 1 and t.shape == (n_src, d)) for t in (a, pair.b if pair else None))
+    vecs = (gain, src.vec if prod else None, *((pair.gain_a, pair.gain_b) if pair else ()))
+    assert all(t is None or (t.stride(-1) == 1 and t.numel() == d) for t in vecs)
+    assert raw is None or (raw.stride(1) == 1 and raw.shape == (T, d))
+    assert rows is None or rows.dtype == torch.int32
+    if _lib.require().kca_prenorm_abi() != ctypes.sizeof(_PreArgs):
+        raise RuntimeError("kca_prenorm descriptor: C and ctypes sizes differ")
+    x_out = torch.empty(T, d, device=ref.device, dtype=torch.float32) if keep_x else None
+    h = torch.empty(T, d, device=ref.device, dtype=ref.dtype) if gain is not None else None
+    p, k = _lib.ptr, _PreArgs()
+    if emb:
+        k.embed, k.tokens, k.escale = data.data_ptr(), src.tokens.data_ptr(), src.scale
+    elif prod:
+        k.base, k.ldbase, k.vec = data.data_ptr(), data.stride(0), p(src.vec)
+    else:
+        k.x_in = data.data_ptr()
+    if a is not None:
+        k.a, k.lda = a.data_ptr(), a.stride(0)
+    if pair:
+        k.ga, k.b, k.ldb, k.gb, k.mul = p(pair.gain_a), p(pair.b), pair.b.stride(0), p(pair.gain_b), pair.mul
+    k.g, k.eps, k.rows, k.x_out, k.raw, k.h, k.T, k.d = p(gain), eps, p(rows), p(x_out), p(raw), p(h), T, d
+    k.ldr = raw.stride(0) if raw is not None else 0
+    fn = _lib.require().kca_prenorm
+    fn.argtypes, fn.restype = [ctypes.c_void_p, ctypes.c_int, ctypes.c_void_p], ctypes.c_int
+    _lib.call("kca_prenorm", ctypes.addressof(k), code, _lib.stream())
+    return x_out, h
+
+
 def _norm(x, gain, eps, layer):
     if layer:
         x = x - x.mean(-1, keepdim=True)
     return x * torch.rsqrt((x * x).mean(-1, keepdim=True) + eps) * gain.float()
 
 
-__all__ = ["NormedBranch", "norm_residual"]
+__all__ = ["Embedded", "NormedBranch", "NormedPair", "Rows", "norm_residual", "prenorm"]

@@ -248,6 +248,8 @@ def _act_ref(y, act):
         return F.gelu(y, approximate="tanh")
     if act == 2:
         return F.gelu(y)
+    if act == 3:
+        return torch.relu(y) ** 2
     return y
 
 
