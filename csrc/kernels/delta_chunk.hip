@@ -14,14 +14,16 @@
 // Decayed products go through blocks of 16 tokens: rows relative to their block's start, columns to their
 // block's end, both at most 1; within a block both relative to its middle. There a log decay below -10 counts
 // as -10 (what it passes on, 5e-5 of the state, is far under the operands' rounding), which bounds the exponents.
-// KIND 1 has p = -k: N = -A_zk, A_qp = -A_qk, so half of the products fall together.
+// KIND 1 and 2 have p = -k: N = -A_zk, A_qp = -A_qk, so half of the products fall together.
+// KIND 2 has one decay per head: its products need no decayed images, the decays multiply the fp32 sums exactly
+// (head_map_kernel).
 #include "attn_tile.h"
+#include "chunk_ops.h"
 #include "delta_rule.h"
 
 namespace {
 using namespace delta;
 
-constexpr int CT = 64;   // tokens of a chunk
 constexpr float kFloor = -10.f;
 
 struct ChunkArgs {
@@ -35,52 +37,6 @@ struct ChunkArgs {
   bf16_t* oo;            // [nchunk][H][DV / 16][4][64 lanes][4]: O'[t = 4 (lane >> 4) ..][v = lane & 15]
   float* e;              // [nchunk][H][DK]: decay of the whole chunk
 };
-
-__device__ __forceinline__ f32x4 mm32(bf16x8 a, bf16x8 b, f32x4 c) { return __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, b, c, 0, 0, 0); }
-// 16 x 16 x 16 in fp32: a = four consecutive elements of row lane & 15 from column 4 (lane >> 4), b in the
-// accumulators' layout (rows 4 (lane >> 4) + r of column lane & 15)
-__device__ __forceinline__ f32x4 mm16f(float4 a, f32x4 b, f32x4 c) {
-  c = __builtin_amdgcn_mfma_f32_16x16x4f32(a.x, b[0], c, 0, 0, 0);
-  c = __builtin_amdgcn_mfma_f32_16x16x4f32(a.y, b[1], c, 0, 0, 0);
-  c = __builtin_amdgcn_mfma_f32_16x16x4f32(a.z, b[2], c, 0, 0, 0);
-  return __builtin_amdgcn_mfma_f32_16x16x4f32(a.w, b[3], c, 0, 0, 0);
-}
-typedef float f32x2 __attribute__((ext_vector_type(2)));
-typedef __bf16 bf16x2v __attribute__((ext_vector_type(2)));
-__device__ __forceinline__ uint32_t pk2(float lo, float hi) {  // one v_cvt_pk
-  return __builtin_bit_cast(uint32_t, __builtin_convertvector(f32x2{lo, hi}, bf16x2v));
-}
-__device__ __forceinline__ s16x4 pk4(f32x4 v) {
-  const uint2 u = make_uint2(pk2(v[0], v[1]), pk2(v[2], v[3]));
-  return __builtin_bit_cast(s16x4, u);
-}
-// operands of two token blocks side by side: the matrix instruction's 8 slots of a lane group hold its four
-// tokens of either block, on both sides alike
-__device__ __forceinline__ bf16x8 two(s16x4 a, s16x4 b) {
-  return __builtin_bit_cast(bf16x8, __builtin_shufflevector(a, b, 0, 1, 2, 3, 4, 5, 6, 7));
-}
-// one block: the other half of the slots zero. (Not the 16-deep instruction: a sum that passes from one bf16 matrix
-// instruction to another kind of them, into other registers, came out wrong; one kind throughout does not.)
-__device__ __forceinline__ f32x4 mm16(s16x4 a, s16x4 b, f32x4 c) { return mm32(two(a, s16x4{0, 0, 0, 0}), two(b, s16x4{0, 0, 0, 0}), c); }
-__device__ __forceinline__ s16x4 neg4(s16x4 v) {
-  uint2 u = __builtin_bit_cast(uint2, v);
-  u.x ^= 0x80008000u;
-  u.y ^= 0x80008000u;
-  return __builtin_bit_cast(s16x4, u);
-}
-// operand of four tokens (rows 4 (lane >> 4) of the block) at column lane & 15 of a row-major LDS image
-template <int LD>
-__device__ __forceinline__ s16x4 tok4(const bf16_t* img, int row, int col) {
-  const int lane = threadIdx.x & 63, gi = lane & 15;
-  const bf16_t* p = img + (row + 4 * (lane >> 4) + (gi >> 2)) * LD + col + 4 * (gi & 3);
-  return __builtin_bit_cast(s16x4, lds_tr4(reinterpret_cast<const char*>(p), 0));
-}
-__device__ __forceinline__ s16x4 row4(const bf16_t* p) { return *reinterpret_cast<const s16x4*>(p); }
-__device__ __forceinline__ f32x4 up4(s16x4 v) {
-  const uint2 u = __builtin_bit_cast(uint2, v);
-  return f32x4{__uint_as_float(u.x << 16), __uint_as_float(u.x & 0xffff0000u), __uint_as_float(u.y << 16),
-               __uint_as_float(u.y & 0xffff0000u)};
-}
 
 // CPL neighbouring channels as loaded
 template <int CPL>
@@ -109,16 +65,133 @@ __device__ __forceinline__ void stc(bf16_t* p, const float (&v)[CPL]) {
 template <int KIND, int DK, int DV>
 struct Lds {
   static constexpr int LK = DK + 8, LV = DV + 8, LA = CT + 8;
+  static constexpr int L3 = KIND == 2 ? 8 : 16 * LK;
   bf16_t lq[CT * LK], lz[CT * LK], rk[CT * LK], rp[KIND == 0 ? CT * LK : 8];  // first the diagonal blocks' operands
-  bf16_t lq3[16 * LK], lz3[16 * LK];                        // block 3's rows relative to block 2's start
-  bf16_t rk0[16 * LK], rp0[KIND == 0 ? 16 * LK : 8];        // block 0's columns relative to block 1's end
+  bf16_t lq3[L3], lz3[L3];                                  // block 3's rows relative to block 2's start
+  bf16_t rk0[L3], rp0[KIND == 0 ? 16 * LK : 8];             // block 0's columns relative to block 1's end
   bf16_t v[CT * LV];
   bf16_t azk[CT * LA], aqk[CT * LA], aqp[KIND == 0 ? CT * LA : 8];
-  bf16_t nb[KIND == 0 ? CT * LA : 8];  // N (KIND 1: -azk)
+  bf16_t nb[KIND == 0 ? CT * LA : 8];  // N (KIND 1, 2: -azk)
   float nd[4][16][20], ti[4][16][20];  // its diagonal blocks, the inverses of I - those
-  float tot[8][DK];    // log decay of every 8 tokens
-  float pre[4][DK];    // decay from the chunk's start to the block's
+  float tot[KIND == 2 ? 1 : 8][DK];  // log decay of every 8 tokens
+  float pre[KIND == 2 ? 1 : 4][DK];  // decay from the chunk's start to the block's
+  float fr[CT], lg[CT], beta[CT];    // KIND 2: decay from the chunk's start to the token, its log; write strengths
 };
+
+// Solve and maps of one (chunk, head) from its LDS images, 16 columns of [W | U] a wave and turn
+template <int KIND, int DK, int DV>
+__device__ __forceinline__ void chunk_maps(Lds<KIND, DK, DV>& s, const ChunkArgs& p, long long cb, int w) {
+  using L = Lds<KIND, DK, DV>;
+  constexpr int KS = DK / 32;
+  const int lane = threadIdx.x & 63, l15 = lane & 15, g4 = lane >> 4;
+  bf16_t* gm = p.m + cb * DK * DK;
+  bf16_t* gb = p.b + cb * DV * DK;
+  bf16_t* gq = p.q + cb * CT * DK;
+  bf16_t* go = p.oo + cb * DV * CT;
+  auto solve = [&](int I, f32x4 y, const f32x4* X, const s16x4* sb) {  // (I - N) X = Y, one block row
+    if (I == 1) y = mm16(row4((KIND == 0 ? s.nb : s.azk) + (16 + l15) * L::LA + 4 * g4), sb[0], y);
+    if (I >= 2) {
+      const bf16_t* nr = (KIND == 0 ? s.nb : s.azk) + (16 * I + l15) * L::LA + 4 * g4;
+      y = mm32(two(row4(nr), row4(nr + 16)), two(sb[0], sb[1]), y);
+      if (I == 3) y = mm16(row4(nr + 32), sb[2], y);
+    }
+    return mm16f(*reinterpret_cast<const float4*>(&s.ti[I][l15][4 * g4]), y, f32x4{0.f, 0.f, 0.f, 0.f});
+  };
+  // sum over the token blocks 0 .. I of rows (of A at `rows`) times operands x
+  auto low = [&](const bf16_t* rows, int I, const s16x4* x, f32x4 y, bool rows_first) {
+    const bf16_t* r = rows + (16 * I + l15) * L::LA + 4 * g4;
+    if (I == 0) return rows_first ? mm16(row4(r), x[0], y) : mm16(x[0], row4(r), y);
+    const bf16x8 ra = two(row4(r), row4(r + 16)), xa = two(x[0], x[1]);
+    y = rows_first ? mm32(ra, xa, y) : mm32(xa, ra, y);
+    if (I == 2) y = rows_first ? mm16(row4(r + 32), x[2], y) : mm16(x[2], row4(r + 32), y);
+    if (I == 3) {
+      const bf16x8 rb = two(row4(r + 32), row4(r + 48)), xc = two(x[2], x[3]);
+      y = rows_first ? mm32(rb, xc, y) : mm32(xc, rb, y);
+    }
+    return y;
+  };
+  auto wtile = [&](int col) {  // 16 columns of W -> M, Q'
+    f32x4 X[4];
+    s16x4 xb[4], sb[4];
+#pragma unroll
+    for (int I = 0; I < 4; ++I) {
+      f32x4 y;
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        const int t = 16 * I + 4 * g4 + r;
+        y[r] = bf2f(s.lz[t * L::LK + col + l15]) * (KIND == 2 ? s.fr[t] : s.pre[I][col + l15]);
+      }
+      X[I] = solve(I, y, X, sb);
+      xb[I] = pk4(X[I]);
+      if (KIND >= 1) xb[I] = neg4(xb[I]);  // N, P and A_qp carry a minus sign
+      sb[I] = xb[I];
+    }
+    const int cw = col + 4 * g4;  // this lane's four columns c'
+    const int fo = ((col >> 5) * 64 + ((col >> 3 & 2) + (g4 >> 1)) * 16 + l15) * 8 + (g4 & 1) * 4;
+#pragma unroll
+    for (int I = 0; I < 4; ++I) {
+      f32x4 y = up4(row4(s.lq + (16 * I + l15) * L::LK + cw));
+      if constexpr (KIND == 2) {
+        y *= s.fr[16 * I + l15];
+      } else {
+        const float4 fp = *reinterpret_cast<const float4*>(&s.pre[I][cw]);
+        y[0] *= fp.x; y[1] *= fp.y; y[2] *= fp.z; y[3] *= fp.w;
+      }
+      *reinterpret_cast<s16x4*>(gq + I * KS * 512 + fo) = pk4(low(KIND == 0 ? s.aqp : s.aqk, I, xb, y, false));
+    }
+    const bf16x8 x01 = two(xb[0], xb[1]), x23 = two(xb[2], xb[3]);
+    const bf16_t* img = KIND == 0 ? s.rp : s.rk;
+#pragma unroll 4
+    for (int c = 0; c < DK; c += 16) {
+      f32x4 y = mm32(x01, two(tok4<L::LK>(img, 0, c), tok4<L::LK>(img, 16, c)), f32x4{0.f, 0.f, 0.f, 0.f});
+      y = mm32(x23, two(tok4<L::LK>(img, 32, c), tok4<L::LK>(img, 48, c)), y);
+      *reinterpret_cast<s16x4*>(gm + (c >> 4) * KS * 512 + fo) = pk4(y);
+    }
+  };
+  auto utile = [&](int col) {  // 16 columns of U -> B, O'
+    f32x4 X[4];
+    s16x4 vb[4], xb[4], sb[4];
+#pragma unroll
+    for (int I = 0; I < 4; ++I) vb[I] = tok4<L::LV>(s.v, 16 * I, col);
+#pragma unroll
+    for (int I = 0; I < 4; ++I) {
+      X[I] = solve(I, low(s.azk, I, vb, f32x4{0.f, 0.f, 0.f, 0.f}, true), X, sb);
+      sb[I] = xb[I] = pk4(X[I]);
+      if (KIND >= 1) {
+        sb[I] = neg4(sb[I]);
+        xb[I] = pk4(up4(vb[I]) - X[I]);  // V - U
+      }
+    }
+#pragma unroll
+    for (int I = 0; I < 4; ++I) {
+      f32x4 y = low(KIND == 0 ? s.aqp : s.aqk, I, xb, f32x4{0.f, 0.f, 0.f, 0.f}, true);
+      if constexpr (KIND == 0) y = low(s.aqk, I, vb, y, true);
+      *reinterpret_cast<s16x4*>(go + ((col >> 4) * 4 + I) * 256 + lane * 4) = pk4(y);
+    }
+    const bf16x8 x01 = two(xb[0], xb[1]), x23 = two(xb[2], xb[3]), v01 = two(vb[0], vb[1]), v23 = two(vb[2], vb[3]);
+    const bf16_t* img = KIND == 0 ? s.rp : s.rk;
+#pragma unroll 4
+    for (int c = 0; c < DK; c += 16) {
+      f32x4 y = mm32(two(tok4<L::LK>(img, 0, c), tok4<L::LK>(img, 16, c)), x01, f32x4{0.f, 0.f, 0.f, 0.f});
+      y = mm32(two(tok4<L::LK>(img, 32, c), tok4<L::LK>(img, 48, c)), x23, y);
+      if constexpr (KIND == 0) {
+        y = mm32(two(tok4<L::LK>(s.rk, 0, c), tok4<L::LK>(s.rk, 16, c)), v01, y);
+        y = mm32(two(tok4<L::LK>(s.rk, 32, c), tok4<L::LK>(s.rk, 48, c)), v23, y);
+      }
+      *reinterpret_cast<s16x4*>(gb + ((col >> 4) * (DK / 16) + (c >> 4)) * 256 + lane * 4) = pk4(y);
+    }
+  };
+  if constexpr (DK == 128 && DV == 128) {
+    wtile(16 * w);
+    utile(16 * w);
+  } else {
+#pragma unroll 1
+    for (int ct = w; ct < (DK + DV) / 16; ct += 8) {
+      if (ct < DK / 16) wtile(16 * ct);
+      else utile(16 * ct - DK);
+    }
+  }
+}
 
 // One wave's operands of an item as loaded: its 8 tokens (KIND 1: and the 3 rows before) of each column block
 template <int KIND>
@@ -457,110 +530,141 @@ __global__ void __launch_bounds__(512) delta_map_kernel(ChunkArgs p, int items) 
   image(std::integral_constant<int, 2>{});
   fetch(min(item + (int)gridDim.x, items - 1), raw);
   __syncthreads();
-  // ----------------------------------------------- solve and maps, 16 columns of [W | U] a wave and turn
-  const long long cb = (long long)ci * a.H + h;
-  bf16_t* gm = p.m + cb * DK * DK;
-  bf16_t* gb = p.b + cb * DV * DK;
-  bf16_t* gq = p.q + cb * CT * DK;
-  bf16_t* go = p.oo + cb * DV * CT;
-  auto solve = [&](int I, f32x4 y, const f32x4* X, const s16x4* sb) {  // (I - N) X = Y, one block row
-    if (I == 1) y = mm16(row4((KIND == 0 ? s.nb : s.azk) + (16 + l15) * L::LA + 4 * g4), sb[0], y);
-    if (I >= 2) {
-      const bf16_t* nr = (KIND == 0 ? s.nb : s.azk) + (16 * I + l15) * L::LA + 4 * g4;
-      y = mm32(two(row4(nr), row4(nr + 16)), two(sb[0], sb[1]), y);
-      if (I == 3) y = mm16(row4(nr + 32), sb[2], y);
-    }
-    return mm16f(*reinterpret_cast<const float4*>(&s.ti[I][l15][4 * g4]), y, f32x4{0.f, 0.f, 0.f, 0.f});
-  };
-  // sum over the token blocks 0 .. I of rows (of A at `rows`) times operands x
-  auto low = [&](const bf16_t* rows, int I, const s16x4* x, f32x4 y, bool rows_first) {
-    const bf16_t* r = rows + (16 * I + l15) * L::LA + 4 * g4;
-    if (I == 0) return rows_first ? mm16(row4(r), x[0], y) : mm16(x[0], row4(r), y);
-    const bf16x8 ra = two(row4(r), row4(r + 16)), xa = two(x[0], x[1]);
-    y = rows_first ? mm32(ra, xa, y) : mm32(xa, ra, y);
-    if (I == 2) y = rows_first ? mm16(row4(r + 32), x[2], y) : mm16(x[2], row4(r + 32), y);
-    if (I == 3) {
-      const bf16x8 rb = two(row4(r + 32), row4(r + 48)), xc = two(x[2], x[3]);
-      y = rows_first ? mm32(rb, xc, y) : mm32(xc, rb, y);
-    }
-    return y;
-  };
-  auto wtile = [&](int col) {  // 16 columns of W -> M, Q'
-    f32x4 X[4];
-    s16x4 xb[4], sb[4];
-#pragma unroll
-    for (int I = 0; I < 4; ++I) {
-      f32x4 y;
-      const float fp = s.pre[I][col + l15];
-#pragma unroll
-      for (int r = 0; r < 4; ++r) y[r] = bf2f(s.lz[(16 * I + 4 * g4 + r) * L::LK + col + l15]) * fp;
-      X[I] = solve(I, y, X, sb);
-      xb[I] = pk4(X[I]);
-      if (KIND == 1) xb[I] = neg4(xb[I]);  // N, P and A_qp carry a minus sign
-      sb[I] = xb[I];
-    }
-    const int cw = col + 4 * g4;  // this lane's four columns c'
-    const int fo = ((col >> 5) * 64 + ((col >> 3 & 2) + (g4 >> 1)) * 16 + l15) * 8 + (g4 & 1) * 4;
-#pragma unroll
-    for (int I = 0; I < 4; ++I) {
-      f32x4 y = up4(row4(s.lq + (16 * I + l15) * L::LK + cw));
-      const float4 fp = *reinterpret_cast<const float4*>(&s.pre[I][cw]);
-      y[0] *= fp.x; y[1] *= fp.y; y[2] *= fp.z; y[3] *= fp.w;
-      *reinterpret_cast<s16x4*>(gq + I * KS * 512 + fo) = pk4(low(KIND == 0 ? s.aqp : s.aqk, I, xb, y, false));
-    }
-    const bf16x8 x01 = two(xb[0], xb[1]), x23 = two(xb[2], xb[3]);
-    const bf16_t* img = KIND == 0 ? s.rp : s.rk;
-#pragma unroll 4
-    for (int c = 0; c < DK; c += 16) {
-      f32x4 y = mm32(x01, two(tok4<L::LK>(img, 0, c), tok4<L::LK>(img, 16, c)), f32x4{0.f, 0.f, 0.f, 0.f});
-      y = mm32(x23, two(tok4<L::LK>(img, 32, c), tok4<L::LK>(img, 48, c)), y);
-      *reinterpret_cast<s16x4*>(gm + (c >> 4) * KS * 512 + fo) = pk4(y);
-    }
-  };
-  auto utile = [&](int col) {  // 16 columns of U -> B, O'
-    f32x4 X[4];
-    s16x4 vb[4], xb[4], sb[4];
-#pragma unroll
-    for (int I = 0; I < 4; ++I) vb[I] = tok4<L::LV>(s.v, 16 * I, col);
-#pragma unroll
-    for (int I = 0; I < 4; ++I) {
-      X[I] = solve(I, low(s.azk, I, vb, f32x4{0.f, 0.f, 0.f, 0.f}, true), X, sb);
-      sb[I] = xb[I] = pk4(X[I]);
-      if (KIND == 1) {
-        sb[I] = neg4(sb[I]);
-        xb[I] = pk4(up4(vb[I]) - X[I]);  // V - U
-      }
-    }
-#pragma unroll
-    for (int I = 0; I < 4; ++I) {
-      f32x4 y = low(KIND == 0 ? s.aqp : s.aqk, I, xb, f32x4{0.f, 0.f, 0.f, 0.f}, true);
-      if constexpr (KIND == 0) y = low(s.aqk, I, vb, y, true);
-      *reinterpret_cast<s16x4*>(go + ((col >> 4) * 4 + I) * 256 + lane * 4) = pk4(y);
-    }
-    const bf16x8 x01 = two(xb[0], xb[1]), x23 = two(xb[2], xb[3]), v01 = two(vb[0], vb[1]), v23 = two(vb[2], vb[3]);
-    const bf16_t* img = KIND == 0 ? s.rp : s.rk;
-#pragma unroll 4
-    for (int c = 0; c < DK; c += 16) {
-      f32x4 y = mm32(two(tok4<L::LK>(img, 0, c), tok4<L::LK>(img, 16, c)), x01, f32x4{0.f, 0.f, 0.f, 0.f});
-      y = mm32(two(tok4<L::LK>(img, 32, c), tok4<L::LK>(img, 48, c)), x23, y);
-      if constexpr (KIND == 0) {
-        y = mm32(two(tok4<L::LK>(s.rk, 0, c), tok4<L::LK>(s.rk, 16, c)), v01, y);
-        y = mm32(two(tok4<L::LK>(s.rk, 32, c), tok4<L::LK>(s.rk, 48, c)), v23, y);
-      }
-      *reinterpret_cast<s16x4*>(gb + ((col >> 4) * (DK / 16) + (c >> 4)) * 256 + lane * 4) = pk4(y);
-    }
-  };
-  if constexpr (DK == 128 && DV == 128) {
-    wtile(16 * w);
-    utile(16 * w);
-  } else {
-#pragma unroll 1
-    for (int ct = w; ct < (DK + DV) / 16; ct += 8) {
-      if (ct < DK / 16) wtile(16 * ct);
-      else utile(16 * ct - DK);
-    }
-  }
+  chunk_maps<KIND, DK, DV>(s, p, (long long)ci * a.H + h, w);
   __syncthreads();  // the next item reuses the LDS
+  }
+}
+
+// KIND 2 from convolution results: eight threads a token make the vectors, a lane a token the decays.
+template <int DK, int DV>
+__global__ void __launch_bounds__(512) head_map_kernel(ChunkArgs p, int items) {
+  using L = Lds<2, DK, DV>;
+  constexpr int NK = DK / 64, NV = DV / 64, KS = DK / 32;
+  extern __shared__ __attribute__((aligned(16))) char smem[];
+  L& s = *reinterpret_cast<L*>(smem);
+  const DeltaArgs& a = p.d;
+  const int tid = threadIdx.x, lane = tid & 63, w = __builtin_amdgcn_readfirstlane(tid >> 6);
+  const int l15 = lane & 15, g4 = lane >> 4, blk = w >> 1, half = w & 1, tok = tid >> 3, sub = tid & 7;
+  const int nqk = a.G * a.dk, C = 2 * nqk + a.H * a.dv, per = a.H / a.G;
+  struct Raw {
+    U16x8 q[NK], k[NK], v[NV];
+    bf16_t a, b, w0, al;
+  };
+  auto fetch = [&](int item, Raw& r) {  // at addresses that exist
+    const int ci = item / a.H, h = item - ci * a.H;
+    const int* ck = p.ck + ci * 4;
+    const long long row0 = ck[0];
+    const int n = ck[1];
+    const bf16_t* x = reinterpret_cast<const bf16_t*>(a.cx) + (row0 + min(tok, n - 1)) * C;
+#pragma unroll
+    for (int i = 0; i < NK; ++i) {
+      const int c = sub * 8 + 64 * i < a.dk ? sub * 8 + 64 * i : 0;
+      r.q[i] = *reinterpret_cast<const U16x8*>(x + h / per * a.dk + c);
+      r.k[i] = *reinterpret_cast<const U16x8*>(x + nqk + h / per * a.dk + c);
+    }
+#pragma unroll
+    for (int i = 0; i < NV; ++i)
+      r.v[i] = *reinterpret_cast<const U16x8*>(x + 2 * nqk + h * a.dv + (sub * 8 + 64 * i < a.dv ? sub * 8 + 64 * i : 0));
+    const bf16_t* y = reinterpret_cast<const bf16_t*>(a.x) + (row0 + min(lane, n - 1)) * a.ld;
+    r.a = y[a.o_w + h];
+    r.b = y[a.o_a + h];
+    r.w0 = reinterpret_cast<const bf16_t*>(a.w0)[h];
+    r.al = reinterpret_cast<const bf16_t*>(a.ab)[h];
+  };
+  Raw raw;
+  fetch(blockIdx.x, raw);
+#pragma unroll 1
+  for (int item = blockIdx.x; item < items; item += gridDim.x) {
+    const int ci = item / a.H, n = p.ck[ci * 4 + 1];
+    // a lane a token: running log decays and write strengths
+    float G = lane < n ? -expf(bf2f(raw.al)) * softplus(bf2f(raw.a) + bf2f(raw.w0)) : 0.f;
+#pragma unroll
+    for (int o = 1; o < 64; o <<= 1) {
+      const float u = __shfl_up(G, o, 64);
+      if (lane >= o) G += u;
+    }
+    const float end = __shfl(G, 63, 64), beta = lane < n ? sigmoid(bf2f(raw.b)) : 0.f;
+    if (w == 0) {
+      s.lg[lane] = G;
+      s.fr[lane] = __expf(G);
+      s.beta[lane] = beta;
+    }
+    const float late = __expf(end - __shfl(G, 8 * w + (lane >> 3), 64)) * __shfl(beta, 8 * w + (lane >> 3), 64);
+    p.e[(long long)item * DK + tid % DK] = __expf(end);
+    // eight threads a token: unit vectors
+    float q[NK][8], k[NK][8], sq = 0.f, sk = 0.f;
+#pragma unroll
+    for (int i = 0; i < NK; ++i) {
+      const bool ok = tok < n && sub * 8 + 64 * i < a.dk;
+#pragma unroll
+      for (int e = 0; e < 8; ++e) {
+        q[i][e] = ok ? bf2f(raw.q[i].v[e]) : 0.f;
+        k[i][e] = ok ? bf2f(raw.k[i].v[e]) : 0.f;
+        sq = fmaf(q[i][e], q[i][e], sq);
+        sk = fmaf(k[i][e], k[i][e], sk);
+      }
+    }
+    auto add = [](float x, float y) { return x + y; };
+    const float iq = a.qscale / sqrtf(lanes_reduce<8>(sq, add) + 1e-6f), ik = 1.f / sqrtf(lanes_reduce<8>(sk, add) + 1e-6f);
+#pragma unroll
+    for (int i = 0; i < NK; ++i) {
+      const int o = tok * L::LK + sub * 8 + 64 * i;
+      uint32_t zq[4], zk[4], zr[4];
+#pragma unroll
+      for (int e = 0; e < 4; ++e) {
+        const float k0 = k[i][2 * e] * ik, k1 = k[i][2 * e + 1] * ik;
+        zq[e] = pk2(q[i][2 * e] * iq, q[i][2 * e + 1] * iq);
+        zk[e] = pk2(k0, k1);
+        zr[e] = pk2(k0 * late, k1 * late);
+      }
+      *reinterpret_cast<u32x4*>(s.lq + o) = u32x4{zq[0], zq[1], zq[2], zq[3]};
+      *reinterpret_cast<u32x4*>(s.lz + o) = u32x4{zk[0], zk[1], zk[2], zk[3]};
+      *reinterpret_cast<u32x4*>(s.rk + o) = u32x4{zr[0], zr[1], zr[2], zr[3]};
+    }
+#pragma unroll
+    for (int i = 0; i < NV; ++i) {
+      const bool ok = tok < n && sub * 8 + 64 * i < a.dv;
+      *reinterpret_cast<u32x4*>(s.v + tok * L::LV + sub * 8 + 64 * i) =
+          ok ? __builtin_bit_cast(u32x4, raw.v[i]) : u32x4{0u, 0u, 0u, 0u};
+    }
+    __syncthreads();
+    // rows of block `blk`, keys (half 0) or queries (half 1), against the keys of the blocks up to it
+    const bf16_t* left = (half ? s.lq : s.lz) + 16 * blk * L::LK;
+#pragma unroll
+    for (int J = 0; J < 4; ++J)
+      if (J <= blk) {
+        f32x4 x = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+        for (int c = 0; c < KS; ++c) {
+          const int o = l15 * L::LK + c * 32 + 8 * g4;
+          x = mm32(*reinterpret_cast<const bf16x8*>(left + o), *reinterpret_cast<const bf16x8*>(s.lz + 16 * J * L::LK + o), x);
+        }
+        const int j = 16 * J + l15;
+        const float lj = s.lg[j], bj = s.beta[j];
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+          const int t = 16 * blk + 4 * g4 + r;
+          const float y = (half ? j <= t : j < t) ? x[r] * bj * __expf(s.lg[t] - lj) : 0.f;
+          (half ? s.aqk : s.azk)[t * L::LA + j] = f2bf(y);
+          if (J == blk && !half) s.nd[blk][4 * g4 + r][l15] = -y;
+        }
+      }
+    __syncthreads();
+    fetch(min(item + (int)gridDim.x, items - 1), raw);
+    if (w == 0) {  // inverses of the four diagonal blocks, a lane per (block, column)
+      float x[16];
+#pragma unroll
+      for (int r = 0; r < 16; ++r) {
+        float v = r == l15 ? 1.f : 0.f;
+#pragma unroll
+        for (int k = 0; k < r; ++k) v = fmaf(s.nd[g4][r][k], x[k], v);
+        x[r] = v;
+        s.ti[g4][r][l15] = v;
+      }
+    }
+    __syncthreads();
+    chunk_maps<2, DK, DV>(s, p, item, w);
+    __syncthreads();  // the next item reuses the LDS
   }
 }
 
@@ -665,7 +769,9 @@ __global__ void __launch_bounds__(256) delta_run_kernel(ChunkArgs p) {
 
 template <int KIND, int DK, int DV>
 int map_go(const ChunkArgs& p, int nchunk, hipStream_t s) {
-  auto kern = delta_map_kernel<KIND, DK, DV>;
+  void (*kern)(ChunkArgs, int);
+  if constexpr (KIND == 2) kern = head_map_kernel<DK, DV>;
+  else kern = delta_map_kernel<KIND, DK, DV>;
   constexpr int lds = sizeof(Lds<KIND, DK, DV>);
   static_assert(lds <= 160 * 1024, "LDS");
   if (hipFuncSetAttribute((const void*)kern, hipFuncAttributeMaxDynamicSharedMemorySize, lds) != hipSuccess) return 5;
@@ -681,7 +787,10 @@ int run_go(const ChunkArgs& p, int nent, hipStream_t s) {
 
 bool chunk_ok(const ChunkArgs& p, int kind) {
   const DeltaArgs& a = p.d;
-  return delta_args_ok(a, kind) && a.dk % 8 == 0 && a.dv % 8 == 0 && a.dk <= 128 && a.dv <= 128 && a.taps <= 4 && a.ld % 2 == 0 &&
+  if (kind == 2)
+    return delta_args_ok(a, kind) && a.dk % 8 == 0 && a.dv % 8 == 0 && a.dk <= 128 && a.dv <= 128 && (uintptr_t)a.cx % 16 == 0 &&
+           a.cx && a.o && p.ck && p.en && p.m && p.b && p.q && p.oo && p.e;
+  return kind < 2 && delta_args_ok(a, kind) && a.dk % 8 == 0 && a.dv % 8 == 0 && a.dk <= 128 && a.dv <= 128 && a.taps <= 4 && a.ld % 2 == 0 &&
          a.ldw % 2 == 0 && a.o_q % 2 == 0 && a.o_k % 2 == 0 && a.o_v % 2 == 0 && a.o_a % 2 == 0 && (uintptr_t)a.x % 4 == 0 &&
          (uintptr_t)a.dw % 4 == 0 && (uintptr_t)a.w0 % 4 == 0 && (uintptr_t)a.ab % 4 == 0 && a.dw && a.o && p.ck && p.en &&
          p.m && p.b && p.q && p.oo && p.e;
@@ -697,6 +806,10 @@ KCA_API int kca_delta_map(const ChunkArgs* in, int kind, int nchunk, hipStream_t
   if (nchunk < 1 || (long long)nchunk * p.d.H > 0x7fffffff) return 1;
   if (!chunk_ok(p, kind)) return 10;
   const bool k1 = p.d.dk > 64, v1 = p.d.dv > 64;
+  if (kind == 2) {
+    if (k1) return v1 ? map_go<2, 128, 128>(p, nchunk, s) : map_go<2, 128, 64>(p, nchunk, s);
+    return v1 ? map_go<2, 64, 128>(p, nchunk, s) : map_go<2, 64, 64>(p, nchunk, s);
+  }
   if (kind == 0) return k1 ? map_go<0, 128, 128>(p, nchunk, s) : map_go<0, 64, 64>(p, nchunk, s);
   if (k1) return v1 ? map_go<1, 128, 128>(p, nchunk, s) : map_go<1, 128, 64>(p, nchunk, s);
   return v1 ? map_go<1, 64, 128>(p, nchunk, s) : map_go<1, 64, 64>(p, nchunk, s);

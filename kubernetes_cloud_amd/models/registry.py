@@ -56,7 +56,7 @@ def _begopel() -> Family:
         from ..engine.hybrid_runner import HybridRunner
         return HybridRunner
     return Family("begopel", begopel.read_config, build_hybrid, begopel.to_native, begopel.from_native, runner,
-                  ("norm_residual", "delta_rule", "delta_chunk", "biased_attn", "act_rows", "gemv", "skinny_mfma"),
+                  ("norm_residual", "delta_rule", "delta_chunk", "ssd_chunk", "biased_attn", "act_rows", "gemv", "skinny_mfma"),
                   begopel.with_shapes)
 
 

@@ -51,6 +51,10 @@ class _ChunkArgs(ctypes.Structure):
     _fields_ = [("d", _Args), ("ck", _P), ("en", _P), ("m", _P), ("b", _P), ("q", _P), ("oo", _P), ("e", _P)]
 
 
+class _SsdArgs(ctypes.Structure):
+    _fields_ = [("d", _Args), ("ck", _P), ("en", _P), ("cb", _P), ("bt", _P), ("gd", _P)]
+
+
 FORMS = {"channel": 1, "head": 2, "ssd": 3}
 CHUNK = 64       # tokens of a matrix-core chunk
 CHUNK_MIN = 16   # shorter portions go token by token
@@ -139,9 +143,8 @@ def plan_portions(entries) -> dict:
 
 def chunks_ok(sp: DeltaHeads, dtype) -> bool:
     """Sizes the chunked matrix-core kernels take (others, and fp32, run token by token)."""
-    if sp.kind >= 2:
-        return False
-    return dtype == torch.bfloat16 and sp.dim % 8 == 0 and sp.vdim % 8 == 0 and max(sp.dim, sp.vdim) <= 128 and sp.taps <= 4
+    return (dtype == torch.bfloat16 and sp.dim % 8 == 0 and sp.vdim % 8 == 0 and sp.dim <= 128
+            and (sp.kind == 3 or sp.vdim <= 128) and (sp.kind != 1 or sp.taps <= 4))
 
 
 def _args(sp: DeltaHeads, wt: DeltaWeights, x, state, ring, pos, slots, out) -> tuple[_Args, int]:
@@ -243,7 +246,17 @@ def delta_portions(sp: DeltaHeads, wt: DeltaWeights, x, state, ring, b: Portions
     o = torch.empty(T, H * sp.vdim, device=dev, dtype=x.dtype)
     a.o = o.data_ptr()
     chunked = chunks_ok(sp, x.dtype) and b.chunks.shape[0] > 0
-    if chunked:
+    if chunked and kind == 3:
+        nc, G, DK = b.chunks.shape[0], sp.kv_heads, (64 if sp.dim <= 64 else 128)
+        cb, bt = (torch.empty(nc * G * n * CHUNK, device=dev, dtype=torch.bfloat16) for n in (CHUNK, DK))
+        gd = torch.empty(nc * H * 2 * CHUNK, device=dev, dtype=torch.float32)
+        if _lib.require().kca_ssd_chunk_abi() != ctypes.sizeof(_SsdArgs):
+            raise RuntimeError("kca_ssd_chunk descriptor: C and ctypes sizes differ")
+        c = _SsdArgs()
+        c.d, c.ck, c.en = a, b.chunks.data_ptr(), b.chunked.data_ptr()
+        c.cb, c.bt, c.gd = cb.data_ptr(), bt.data_ptr(), gd.data_ptr()
+        _call("kca_ssd_chunks", c, nc, b.chunked.shape[0])
+    elif chunked:
         nc, DK, DV = b.chunks.shape[0], (64 if sp.dim <= 64 else 128), (64 if sp.vdim <= 64 else 128)
         sizes = (DK * DK, DV * DK, CHUNK * DK, DV * CHUNK)
         ws = [torch.empty(nc * H * n, device=dev, dtype=torch.bfloat16) for n in sizes]

@@ -487,6 +487,20 @@ def test_recurrences(device, dtype, kind):
         assert float(S[3].sub(7).abs().max()) == 0 and float(S[0].sub(7).abs().max()) == 0  # other slots untouched
 
 
+@pytest.mark.gpu
+@pytest.mark.parametrize("state,vdim,heads", [(40, 32, 130), (104, 32, 128), (48, 64, 192), (128, 56, 200)])
+def test_many_state_space_heads(state, vdim, heads):
+    """Enough heads that a workgroup takes several column tiles."""
+    d = Recurrence("ssd", ssd(heads, 2, state, vdim, 4, 2)["mixer"], 80, seed=80)
+    wt = d.weights(lambda t: t.to("cuda", BF16))
+    S, ring = d.state(3, "cuda")
+    got = d.run([(d.x, 0, 1), (d.x[:70], 0, 2)], wt, S, ring, "cuda", BF16)
+    want = d.want(d.x)
+    assert rel(got[:80], want) < 2e-2 and rel(got[80:], want[:70]) < 2e-2
+    got = d.run([(d.x[70:], 70, 2)], wt, S, ring, "cuda", BF16)
+    assert rel(got, want[70:]) < 2e-2
+
+
 @pytest.mark.parametrize("device,dtype", WHERE)
 @pytest.mark.parametrize("kind", ["head", "head-128", "ssd", "ssd-128"])
 def test_long_recurrent_decoding(device, dtype, kind):
