@@ -348,7 +348,7 @@ __global__ void __launch_bounds__(256) biased_rows_kernel(BiasedArgs p) {
 // beside the head's bias row (BL; longer rows stay in global memory); S^T = K Q^T leaves a query per lane, and
 // P^T feeds O^T += V^T P^T from registers. Tiles beyond the last bucket's edge add one constant.
 template <int DK, int DV, bool BL>
-__global__ void __launch_bounds__(256, 2) biased_tile_kernel(BiasedArgs p) {
+__global__ void __launch_bounds__(256, DV > 128 ? 1 : 2) biased_tile_kernel(BiasedArgs p) {
   constexpr int BN = 32, TK = BN * DK * 2, TV = BN * DV * 2, BUF = TK + TV;
   constexpr int KS = DK / 16, NB = DV / 32;
   constexpr int CK = BN * (DK / 8), CV = BN * (DV / 8), NC = CK + CV;  // 16-B chunks per tile
@@ -356,8 +356,9 @@ __global__ void __launch_bounds__(256, 2) biased_tile_kernel(BiasedArgs p) {
   extern __shared__ __attribute__((aligned(16))) char smem[];  // [2][K | V], bias row
   const int tid = threadIdx.x, lane = tid & 63, qg = tid >> 6;
   const int l32 = lane & 31, hh = lane >> 5, gi = lane & 15;
-  const int lid = xcd_remap(blockIdx.x, gridDim.x);
-  const int ti = lid / p.H, h = lid % p.H, g = h / (p.H / p.G);
+  // tiles in their order (the longest first) on every XCD; one with an eighth of the heads shares their K / V in its L2
+  const int hx = p.H % 8 ? p.H : p.H / 8, j = p.H % 8 ? (int)blockIdx.x : (int)blockIdx.x >> 3;
+  const int ti = j / hx, h = j % hx + (p.H % 8 ? 0 : hx * (blockIdx.x & 7)), g = h / (p.H / p.G);
   const int* tl = p.tiles + ti * 4;
   const int row0 = tl[0], nrow = tl[1], pos0 = tl[2], slot = tl[3];
   const int qi = qg * 32 + l32;
@@ -373,34 +374,39 @@ __global__ void __launch_bounds__(256, 2) biased_tile_kernel(BiasedArgs p) {
   const bf16_t* vc = reinterpret_cast<const bf16_t*>(p.vc);
   const bf16_t* xr = reinterpret_cast<const bf16_t*>(p.x) + row * p.ld;
 
-  u32x4 st[CPT];
-  auto load = [&](int k0) {
-    const long long pg = tbl[k0 >> p.shift];
-    const int o0 = k0 & ((1 << p.shift) - 1);
+  // this thread's 16-B chunks of a tile: element offset from the tile's first row, LDS offset
+  int off[CPT], ldo[CPT], vrow[CPT];
+  bool on[CPT];
+#pragma unroll
+  for (int i = 0; i < CPT; ++i) {
+    const int c = tid + 256 * i, cv = c - CK;
+    const bool key = c < CK;
+    const int r = key ? c / (DK / 8) : cv / (DV / 8), ch = key ? c % (DK / 8) : cv % (DV / 8);
+    on[i] = c < NC && ch * 8 < (key ? D : Vd);
+    off[i] = on[i] ? r * (key ? D : Vd) + ch * 8 : 0;
+    ldo[i] = key ? img_off<DK>(r, ch) : TK + img_off<DV>(r, ch);
+    vrow[i] = key ? -1 : r;
+  }
+  auto page = [&](int t) { return tbl[min(t, ntiles - 1) * BN >> p.shift]; };
+  auto load = [&](int t, int pg, u32x4 (&st)[CPT]) {  // tile t of page pg (tiles past the end: the last again)
+    const int k0 = min(t, ntiles - 1) * BN;
+    const long long o0 = ((long long)g << p.shift) + (k0 & ((1 << p.shift) - 1));
+    const bf16_t *kb = kc + pg * p.k_sp + o0 * D, *vb = vc + pg * p.v_sp + o0 * Vd;
 #pragma unroll
     for (int i = 0; i < CPT; ++i) {
-      const int c = tid + 256 * i;
-      st[i] = u32x4{0u, 0u, 0u, 0u};
-      if (c < CK) {
-        const int r = c / (DK / 8), ch = c % (DK / 8);
-        if (ch * 8 < D)
-          st[i] = *reinterpret_cast<const u32x4*>(kc + pg * p.k_sp + (((long long)g << p.shift) + o0 + r) * D + ch * 8);
-      } else if (c < NC) {
-        const int cv = c - CK, r = cv / (DV / 8), ch = cv % (DV / 8);
-        if (ch * 8 < Vd && k0 + r < kv_hi)
-          st[i] = *reinterpret_cast<const u32x4*>(vc + pg * p.v_sp + (((long long)g << p.shift) + o0 + r) * Vd + ch * 8);
-      }
+      const bool key = 256 * i + 255 < CK || (256 * i < CK && tid + 256 * i < CK);
+      const u32x4 v = *reinterpret_cast<const u32x4*>((key ? kb : vb) + off[i]);
+      st[i] = on[i] && k0 + vrow[i] < kv_hi ? v : u32x4{0u, 0u, 0u, 0u};  // (a value past the last key may be anything)
     }
   };
-  auto store = [&](char* buf) {
+  auto store = [&](const u32x4 (&st)[CPT], char* buf) {
 #pragma unroll
-    for (int i = 0; i < CPT; ++i) {
-      const int c = tid + 256 * i;
-      if (c < CK) *reinterpret_cast<u32x4*>(buf + img_off<DK>(c / (DK / 8), c % (DK / 8))) = st[i];
-      else if (c < NC) *reinterpret_cast<u32x4*>(buf + TK + img_off<DV>((c - CK) / (DV / 8), (c - CK) % (DV / 8))) = st[i];
-    }
+    for (int i = 0; i < CPT; ++i)
+      if (256 * i + 255 < NC || tid + 256 * i < NC) *reinterpret_cast<u32x4*>(buf + ldo[i]) = st[i];
   };
-  load(0);
+  u32x4 st0[CPT], st1[CPT];
+  load(0, page(0), st0);
+  int pg = page(1);
   // the bias row in units of log2
   const float* gb = p.bias ? p.bias + (long long)h * p.nb : nullptr;
   float* lb = reinterpret_cast<float*>(smem + 2 * BUF);
@@ -454,13 +460,16 @@ __global__ void __launch_bounds__(256, 2) biased_tile_kernel(BiasedArgs p) {
     for (int r = 0; r < 16; ++r) o[b][r] = 0.f;
   float mref = -INFINITY, ls = 0.f;
 
-  store(smem);
+  store(st0, smem);
+  load(1, pg, st0);
+  pg = page(2);
   __syncthreads();
-  for (int t = 0; t < ntiles; ++t) {
+  // tile t; its successor lies in `next`, the one after that is loaded into `far2` meanwhile
+  auto step = [&](int t, const u32x4 (&next)[CPT], u32x4 (&far2)[CPT]) {
     const char* buf = smem + (t & 1) * BUF;
     const int k0 = t * BN;
-    const bool more = t + 1 < ntiles;
-    if (more) load(k0 + BN);
+    load(t + 2, pg, far2);
+    pg = page(t + 3);
     if (busy && k0 < wave_hi) {  // (tiles past the wave's last query: staging only)
       f32x16 s;
 #pragma unroll
@@ -549,8 +558,12 @@ __global__ void __launch_bounds__(256, 2) biased_tile_kernel(BiasedArgs p) {
         __builtin_amdgcn_sched_group_barrier(0x8, 2, 0);
       }
     }
-    if (more) store(smem + ((t + 1) & 1) * BUF);
+    store(next, smem + ((t + 1) & 1) * BUF);
     __syncthreads();
+  };
+  for (int t = 0; t < ntiles; t += 2) {
+    step(t, st0, st1);
+    if (t + 1 < ntiles) step(t + 1, st1, st0);
   }
   if (!live) return;
   float l = ls + __shfl_xor(ls, 32, 64);

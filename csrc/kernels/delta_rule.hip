@@ -259,15 +259,15 @@ __global__ void __launch_bounds__(256) delta_conv_kernel(DeltaArgs a, E* out, in
   if (t0 >= T) return;
   const int col = ch < nqk ? a.o_q + ch : ch < 2 * nqk ? a.o_k + ch - nqk : a.o_v + ch - 2 * nqk;
   const E* x = reinterpret_cast<const E*>(a.x) + col;
-  const E* w = reinterpret_cast<const E*>(a.conv) + (long long)ch * a.taps + a.taps - 1;
-  const int t1 = min(t0 + CONV_ROWS, T);
-  auto row = [&](int t, float (&v)[V]) {
-    const PackE u = *reinterpret_cast<const PackE*>(x + (long long)t * a.ld);
+  const E* w = reinterpret_cast<const E*>(a.conv) + (long long)ch * a.taps;
+  const int t1 = min(t0 + CONV_ROWS, T), first = a.e0[t0];
+  auto conv = [&](const PackE& u, float (&v)[V]) {
 #pragma unroll
     for (int e = 0; e < V; ++e) v[e] = delta::ld<E>(u.v + e);
   };
+  auto load = [&](int t) { return *reinterpret_cast<const PackE*>(x + (long long)t * a.ld); };
   auto before = [&](int t, int n, float (&v)[V]) {  // the input n tokens before row t
-    if (t - n >= a.e0[t]) return row(t - n, v);
+    if (t - n >= a.e0[t]) return conv(load(t - n), v);
     const int ps = a.pos[t] - n;
     const float* r = a.ring + ((long long)a.slot[t] * a.taps + (ps >= 0 ? ps % a.taps : 0)) * C + ch;
 #pragma unroll
@@ -293,27 +293,29 @@ __global__ void __launch_bounds__(256) delta_conv_kernel(DeltaArgs a, E* out, in
       for (int n = 0; n < a.taps; ++n) {
         before(t, n, v);
 #pragma unroll
-        for (int e = 0; e < V; ++e) y[e] = fmaf(delta::ld<E>(w + (long long)e * a.taps - n), v[e], y[e]);
+        for (int e = 0; e < V; ++e) y[e] = fmaf(delta::ld<E>(w + (long long)e * a.taps + a.taps - 1 - n), v[e], y[e]);
       }
       put(t, y);
     }
     return;
   }
   float tap[4][V], h[4][V];  // h[n]: the input n tokens back
+  auto taps = [&]() {
+    if (V > 1 && a.taps == 4 && (uintptr_t)a.conv % (sizeof(E) * V) == 0) {  // channel by channel, V values a load
 #pragma unroll
-  for (int n = 0; n < 4; ++n)
+      for (int j = 0; j < 4; ++j) {
+        const PackE u = *reinterpret_cast<const PackE*>(w + j * V);
 #pragma unroll
-    for (int e = 0; e < V; ++e) {
-      tap[n][e] = n < a.taps ? delta::ld<E>(w + (long long)e * a.taps - n) : 0.f;
-      h[n][e] = 0.f;
+        for (int e = 0; e < V; ++e) tap[3 - (j * V + e) % 4][(j * V + e) / 4] = delta::ld<E>(u.v + e);
+      }
+      return;
     }
-  for (int t = t0; t < t1; ++t) {
-    if (t == t0 || a.e0[t] == t) {
 #pragma unroll
-      for (int n = 1; n < 4; ++n)
-        if (n < a.taps) before(t, n, h[n]);
-    }
-    row(t, h[0]);
+    for (int n = 0; n < 4; ++n)
+#pragma unroll
+      for (int e = 0; e < V; ++e) tap[n][e] = n < a.taps ? delta::ld<E>(w + (long long)e * a.taps + a.taps - 1 - n) : 0.f;
+  };
+  auto row = [&](int t) {
     float y[V];
 #pragma unroll
     for (int e = 0; e < V; ++e)
@@ -323,15 +325,42 @@ __global__ void __launch_bounds__(256) delta_conv_kernel(DeltaArgs a, E* out, in
     for (int n = 3; n > 0; --n)
 #pragma unroll
       for (int e = 0; e < V; ++e) h[n][e] = h[n - 1][e];
+  };
+  if (t0 - 3 >= first && t0 + CONV_ROWS <= T && a.e0[t1 - 1] == first) {  // all inputs are rows of the entry
+    PackE u[CONV_ROWS + 3];
+#pragma unroll
+    for (int n = 0; n < CONV_ROWS + 3; ++n) u[n] = load(t0 - 3 + n);
+    taps();
+#pragma unroll
+    for (int n = 1; n < 4; ++n) conv(u[3 - n], h[n]);
+#pragma unroll
+    for (int n = 0; n < CONV_ROWS; ++n) {
+      conv(u[n + 3], h[0]);
+      row(t0 + n);
+    }
+    return;
+  }
+  taps();
+#pragma unroll
+  for (int n = 0; n < 4; ++n)
+#pragma unroll
+    for (int e = 0; e < V; ++e) h[n][e] = 0.f;
+  for (int t = t0; t < t1; ++t) {
+    if (t == t0 || a.e0[t] == t) {
+#pragma unroll
+      for (int n = 1; n < 4; ++n)
+        if (n < a.taps) before(t, n, h[n]);
+    }
+    conv(load(t), h[0]);
+    row(t);
   }
 }
 
-// KIND 3: out = N(o * silu(z)) * gain of a row, N over norm_groups equal parts. WPP waves a part (WPP = all of them:
-// the workgroup takes the parts in turn). The gated row lies in LDS between its two uses, by the thread that made it.
-template <typename E, int V, int NW, bool ALL>
+// KIND 3: out = N(o * silu(z)) * gain of a row, N over norm_groups equal parts. A part belongs to the workgroup (ALL)
+// or to a wave, NCH packs of V channels a thread (0: any size, the gated row read twice).
+template <typename E, int V, int NW, bool ALL, int NCH>
 __global__ void __launch_bounds__(64 * NW) delta_parts_kernel(DeltaArgs a) {
   struct alignas(sizeof(E) * V) PackE { E v[V]; };
-  extern __shared__ __attribute__((aligned(16))) float u[];
   __shared__ float red[NW];
   const int t = blockIdx.x, tid = threadIdx.x, lane = tid & 63, wv = tid >> 6, n = a.H * a.dv, per = n / a.norm_groups;
   const E* o = reinterpret_cast<const E*>(a.o) + (long long)t * n;
@@ -339,17 +368,43 @@ __global__ void __launch_bounds__(64 * NW) delta_parts_kernel(DeltaArgs a) {
   const E* gain = reinterpret_cast<const E*>(a.gain);
   E* out = reinterpret_cast<E*>(a.out) + (long long)t * a.ldo;
   const int step = (ALL ? 64 * NW : 64) * V, c0 = (ALL ? tid : lane) * V;
-  for (int g = ALL ? blockIdx.y : blockIdx.y * NW + wv; g < a.norm_groups; g += gridDim.y * (ALL ? 1 : NW)) {
-    float ss = 0.f;
-    float* up = u + (ALL ? 0 : wv * per);
-    for (int c = c0; c < per; c += step) {
-      const PackE y = *reinterpret_cast<const PackE*>(o + g * per + c), q = *reinterpret_cast<const PackE*>(z + g * per + c);
+  const int g = ALL ? blockIdx.y : blockIdx.y * NW + wv;
+  if (g < a.norm_groups) {  // (whole waves; ALL: always)
+    o += g * per;
+    z += g * per;
+    gain += g * per;
+    out += g * per;
+    auto gated = [&](const PackE& y, const PackE& q, float (&v)[V]) {
 #pragma unroll
       for (int e = 0; e < V; ++e) {
         const float x = delta::ld<E>(q.v + e);
-        const float v = delta::ld<E>(y.v + e) * (sizeof(E) == 4 ? silu(x) : x * __builtin_amdgcn_rcpf(1.f + __expf(-x)));
-        up[c + e] = v;
-        ss = fmaf(v, v, ss);
+        v[e] = delta::ld<E>(y.v + e) * (sizeof(E) == 4 ? silu(x) : x * __builtin_amdgcn_rcpf(1.f + __expf(-x)));
+      }
+    };
+    auto pack = [&](const E* p, int c) { return *reinterpret_cast<const PackE*>(p + c); };
+    constexpr int M = NCH ? NCH : 1;
+    PackE y[M], q[M], w[M];
+    float ss = 0.f, v[V], u[M][V];
+    if constexpr (NCH > 0) {
+#pragma unroll
+      for (int j = 0; j < NCH; ++j) {
+        const int c = min(c0 + j * step, per - V);
+        y[j] = pack(o, c);
+        q[j] = pack(z, c);
+        w[j] = pack(gain, c);
+      }
+#pragma unroll
+      for (int j = 0; j < NCH; ++j) {
+        gated(y[j], q[j], u[j]);
+        if (c0 + j * step < per)
+#pragma unroll
+          for (int e = 0; e < V; ++e) ss = fmaf(u[j][e], u[j][e], ss);
+      }
+    } else {
+      for (int c = c0; c < per; c += step) {
+        gated(pack(o, c), pack(z, c), v);
+#pragma unroll
+        for (int e = 0; e < V; ++e) ss = fmaf(v[e], v[e], ss);
       }
     }
     ss = wave_sum(ss);
@@ -359,19 +414,41 @@ __global__ void __launch_bounds__(64 * NW) delta_parts_kernel(DeltaArgs a) {
       ss = 0.f;
 #pragma unroll
       for (int i = 0; i < NW; ++i) ss += red[i];
-      __syncthreads();
     }
     const float r = 1.f / sqrtf(ss / (float)per + a.eps);
-    for (int c = c0; c < per; c += step) {
-      const PackE w = *reinterpret_cast<const PackE*>(gain + g * per + c);
-      PackE y;
+    auto put = [&](int c, const float (&x)[V], const PackE& gn) {
+      PackE s;
 #pragma unroll
-      for (int e = 0; e < V; ++e) delta::st<E>(y.v + e, up[c + e] * r * delta::ld<E>(w.v + e));
-      *reinterpret_cast<PackE*>(out + g * per + c) = y;
+      for (int e = 0; e < V; ++e) delta::st<E>(s.v + e, x[e] * r * delta::ld<E>(gn.v + e));
+      *reinterpret_cast<PackE*>(out + c) = s;
+    };
+    if constexpr (NCH > 0) {
+#pragma unroll
+      for (int j = 0; j < NCH; ++j)
+        if (c0 + j * step < per) put(c0 + j * step, u[j], w[j]);
+    } else {
+      for (int c = c0; c < per; c += step) {
+        gated(pack(o, c), pack(z, c), v);
+        put(c, v, pack(gain, c));
+      }
     }
   }
-  if (a.e1 && blockIdx.y == 0 && a.e1[t] - t <= a.taps)
-    for (int h = 0; h < a.H; ++h) ring_store<E>(a, t, h, tid, 64 * NW);
+  if (a.e1 && a.e1[t] - t <= a.taps) {  // all channels of an entry's last inputs, several loads in flight
+    const int nqk = a.G * a.dk, C = 2 * nqk + n, NT = 64 * NW * gridDim.y;
+    float* r = a.ring + ((long long)a.slot[t] * a.taps + a.pos[t] % a.taps) * C;
+    const E* x = reinterpret_cast<const E*>(a.x) + (long long)t * a.ld;
+    for (int c0 = blockIdx.y * 64 * NW + tid; c0 < C; c0 += 8 * NT) {
+      float v[8];
+#pragma unroll
+      for (int i = 0; i < 8; ++i) {
+        const int c = min(c0 + i * NT, C - 1);
+        v[i] = delta::ld<E>(x + (c < nqk ? a.o_q + c : c < 2 * nqk ? a.o_k + c - nqk : a.o_v + c - 2 * nqk));
+      }
+#pragma unroll
+      for (int i = 0; i < 8; ++i)
+        if (c0 + i * NT < C) r[c0 + i * NT] = v[i];
+    }
+  }
 }
 
 int rows_r(int dk) {  // rows a lane holds: 16 row groups
@@ -462,19 +539,22 @@ int conv_go(const DeltaArgs& a, void* out, int T, hipStream_t s) {
 template <typename E, int V>
 int parts_v(const DeltaArgs& a, int T, hipStream_t s) {
   const int n = a.H * a.dv, per = n / a.norm_groups;
-  const bool all = a.norm_groups < 4, few = T <= 64 && per > 2048;
-  const size_t lds = (size_t)per * 4 * (all ? 1 : 4);
-  if (lds > 128 * 1024) return 10;
-#define GO(NW, ALL)                                                                                                       \
-  {                                                                                                                       \
-    auto kern = delta_parts_kernel<E, V, NW, ALL>;                                                                        \
-    if (lds > 48 * 1024 && hipFuncSetAttribute((const void*)kern, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds) != hipSuccess) \
-      return 5;                                                                                                           \
-    hipLaunchKernelGGL(kern, dim3(T, ALL ? a.norm_groups : (a.norm_groups + NW - 1) / NW), dim3(64 * NW), lds, s, a);      \
+  const int packs = (per + V - 1) / V;
+#define GO(NW, ALL, NCH)                                                                                              \
+  hipLaunchKernelGGL((delta_parts_kernel<E, V, NW, ALL, NCH>), dim3(T, ALL ? a.norm_groups : (a.norm_groups + NW - 1) / NW), \
+                     dim3(64 * NW), 0, s, a)
+  if (a.norm_groups >= 4) {
+    if (packs <= 64) GO(4, false, 1);
+    else if (packs <= 128) GO(4, false, 2);
+    else if (packs <= 256) GO(4, false, 4);
+    else GO(4, false, 0);
+  } else {
+    if (packs <= 256) GO(4, true, 1);
+    else if (T <= 64 && packs <= 1024) GO(16, true, 1);
+    else if (packs <= 512) GO(4, true, 2);
+    else if (packs <= 1024) GO(4, true, 4);
+    else GO(4, true, 0);
   }
-  if (!all) GO(4, false)
-  else if (few) GO(16, true)
-  else GO(4, true)
 #undef GO
   return hipGetLastError() == hipSuccess ? 0 : 4;
 }
