@@ -66,20 +66,26 @@ template <int KIND, int DK, int DV>
 struct Lds {
   static constexpr int LK = DK + 8, LV = DV + 8, LA = CT + 8;
   static constexpr int L3 = KIND == 2 ? 8 : 16 * LK;
-  bf16_t lq[CT * LK], lz[CT * LK], rk[CT * LK], rp[KIND == 0 ? CT * LK : 8];  // first the diagonal blocks' operands
+  bf16_t lq[CT * LK], lz[CT * LK], rk[KIND == 2 ? 8 : CT * LK], rp[KIND == 0 ? CT * LK : 8];  // first the diagonal blocks' operands
   bf16_t lq3[L3], lz3[L3];                                  // block 3's rows relative to block 2's start
   bf16_t rk0[L3], rp0[KIND == 0 ? 16 * LK : 8];             // block 0's columns relative to block 1's end
   bf16_t v[CT * LV];
   bf16_t azk[CT * LA], aqk[CT * LA], aqp[KIND == 0 ? CT * LA : 8];
   bf16_t nb[KIND == 0 ? CT * LA : 8];  // N (KIND 1, 2: -azk)
-  float nd[4][16][20], ti[4][16][20];  // its diagonal blocks, the inverses of I - those
+  // its diagonal blocks, the inverses of I - those (KIND 2: in their place)
+  float nd[4][16][20], ti_[KIND == 2 ? 1 : 4][16][20];
+  __device__ __forceinline__ float (&ti())[4][16][20] {
+    if constexpr (KIND == 2) return nd;
+    else return ti_;
+  }
   float tot[KIND == 2 ? 1 : 8][DK];  // log decay of every 8 tokens
   float pre[KIND == 2 ? 1 : 4][DK];  // decay from the chunk's start to the block's
-  float fr[CT], lg[CT], beta[CT];    // KIND 2: decay from the chunk's start to the token, its log; write strengths
+  // KIND 2: decay from the chunk's start to the token, its log; write strengths, also decayed to the chunk's end
+  float fr[CT], lg[CT], beta[CT], late[CT];
 };
 
 // Solve and maps of one (chunk, head) from its LDS images, 16 columns of [W | U] a wave and turn
-template <int KIND, int DK, int DV>
+template <int KIND, int DK, int DV, int NW = 8>
 __device__ __forceinline__ void chunk_maps(Lds<KIND, DK, DV>& s, const ChunkArgs& p, long long cb, int w) {
   using L = Lds<KIND, DK, DV>;
   constexpr int KS = DK / 32;
@@ -95,7 +101,7 @@ __device__ __forceinline__ void chunk_maps(Lds<KIND, DK, DV>& s, const ChunkArgs
       y = mm32(two(row4(nr), row4(nr + 16)), two(sb[0], sb[1]), y);
       if (I == 3) y = mm16(row4(nr + 32), sb[2], y);
     }
-    return mm16f(*reinterpret_cast<const float4*>(&s.ti[I][l15][4 * g4]), y, f32x4{0.f, 0.f, 0.f, 0.f});
+    return mm16f(*reinterpret_cast<const float4*>(&s.ti()[I][l15][4 * g4]), y, f32x4{0.f, 0.f, 0.f, 0.f});
   };
   // sum over the token blocks 0 .. I of rows (of A at `rows`) times operands x
   auto low = [&](const bf16_t* rows, int I, const s16x4* x, f32x4 y, bool rows_first) {
@@ -109,6 +115,14 @@ __device__ __forceinline__ void chunk_maps(Lds<KIND, DK, DV>& s, const ChunkArgs
       y = rows_first ? mm32(rb, xc, y) : mm32(xc, rb, y);
     }
     return y;
+  };
+  // KIND 2: rows of X decayed to the chunk's end, for the plain key image
+  auto to_end = [&](const f32x4 (&X)[4], s16x4 (&xb)[4], float sign) {
+#pragma unroll
+    for (int I = 0; I < 4; ++I) {
+      const float4 l = *reinterpret_cast<const float4*>(&s.late[16 * I + 4 * g4]);
+      xb[I] = pk4(f32x4{X[I][0] * l.x, X[I][1] * l.y, X[I][2] * l.z, X[I][3] * l.w} * sign);
+    }
   };
   auto wtile = [&](int col) {  // 16 columns of W -> M, Q'
     f32x4 X[4];
@@ -139,8 +153,9 @@ __device__ __forceinline__ void chunk_maps(Lds<KIND, DK, DV>& s, const ChunkArgs
       }
       *reinterpret_cast<s16x4*>(gq + I * KS * 512 + fo) = pk4(low(KIND == 0 ? s.aqp : s.aqk, I, xb, y, false));
     }
+    if constexpr (KIND == 2) to_end(X, xb, -1.f);
     const bf16x8 x01 = two(xb[0], xb[1]), x23 = two(xb[2], xb[3]);
-    const bf16_t* img = KIND == 0 ? s.rp : s.rk;
+    const bf16_t* img = KIND == 0 ? s.rp : KIND == 1 ? s.rk : s.lz;
 #pragma unroll 4
     for (int c = 0; c < DK; c += 16) {
       f32x4 y = mm32(x01, two(tok4<L::LK>(img, 0, c), tok4<L::LK>(img, 16, c)), f32x4{0.f, 0.f, 0.f, 0.f});
@@ -159,7 +174,9 @@ __device__ __forceinline__ void chunk_maps(Lds<KIND, DK, DV>& s, const ChunkArgs
       sb[I] = xb[I] = pk4(X[I]);
       if (KIND >= 1) {
         sb[I] = neg4(sb[I]);
-        xb[I] = pk4(up4(vb[I]) - X[I]);  // V - U
+        const f32x4 d = up4(vb[I]) - X[I];  // V - U
+        xb[I] = pk4(d);
+        if (KIND == 2) X[I] = d;
       }
     }
 #pragma unroll
@@ -168,8 +185,9 @@ __device__ __forceinline__ void chunk_maps(Lds<KIND, DK, DV>& s, const ChunkArgs
       if constexpr (KIND == 0) y = low(s.aqk, I, vb, y, true);
       *reinterpret_cast<s16x4*>(go + ((col >> 4) * 4 + I) * 256 + lane * 4) = pk4(y);
     }
+    if constexpr (KIND == 2) to_end(X, xb, 1.f);  // (X: V - U by now)
     const bf16x8 x01 = two(xb[0], xb[1]), x23 = two(xb[2], xb[3]), v01 = two(vb[0], vb[1]), v23 = two(vb[2], vb[3]);
-    const bf16_t* img = KIND == 0 ? s.rp : s.rk;
+    const bf16_t* img = KIND == 0 ? s.rp : KIND == 1 ? s.rk : s.lz;
 #pragma unroll 4
     for (int c = 0; c < DK; c += 16) {
       f32x4 y = mm32(two(tok4<L::LK>(img, 0, c), tok4<L::LK>(img, 16, c)), x01, f32x4{0.f, 0.f, 0.f, 0.f});
@@ -181,12 +199,12 @@ __device__ __forceinline__ void chunk_maps(Lds<KIND, DK, DV>& s, const ChunkArgs
       *reinterpret_cast<s16x4*>(gb + ((col >> 4) * (DK / 16) + (c >> 4)) * 256 + lane * 4) = pk4(y);
     }
   };
-  if constexpr (DK == 128 && DV == 128) {
+  if constexpr (DK == 128 && DV == 128 && NW == 8) {
     wtile(16 * w);
     utile(16 * w);
   } else {
 #pragma unroll 1
-    for (int ct = w; ct < (DK + DV) / 16; ct += 8) {
+    for (int ct = w; ct < (DK + DV) / 16; ct += NW) {
       if (ct < DK / 16) wtile(16 * ct);
       else utile(16 * ct - DK);
     }
@@ -523,7 +541,7 @@ __global__ void __launch_bounds__(512) delta_map_kernel(ChunkArgs p, int items) 
 #pragma unroll
       for (int k = 0; k < r; ++k) v = fmaf(s.nd[g4][r][k], x[k], v);
       x[r] = v;
-      s.ti[g4][r][l15] = v;
+      s.ti()[g4][r][l15] = v;
     }
   }
   __syncthreads();
@@ -535,16 +553,17 @@ __global__ void __launch_bounds__(512) delta_map_kernel(ChunkArgs p, int items) 
   }
 }
 
-// KIND 2 from convolution results: eight threads a token make the vectors, a lane a token the decays.
+// KIND 2 from convolution results: four threads a token make the vectors, a lane a token the decays. Two workgroups
+// a CU, so that one solves while the other loads and stores.
 template <int DK, int DV>
-__global__ void __launch_bounds__(512) head_map_kernel(ChunkArgs p, int items) {
+__global__ void __launch_bounds__(256, 2) head_map_kernel(ChunkArgs p, int items) {
   using L = Lds<2, DK, DV>;
-  constexpr int NK = DK / 64, NV = DV / 64, KS = DK / 32;
+  constexpr int NK = DK / 32, NV = DV / 32, KS = DK / 32;
   extern __shared__ __attribute__((aligned(16))) char smem[];
   L& s = *reinterpret_cast<L*>(smem);
   const DeltaArgs& a = p.d;
   const int tid = threadIdx.x, lane = tid & 63, w = __builtin_amdgcn_readfirstlane(tid >> 6);
-  const int l15 = lane & 15, g4 = lane >> 4, blk = w >> 1, half = w & 1, tok = tid >> 3, sub = tid & 7;
+  const int l15 = lane & 15, g4 = lane >> 4, tok = tid >> 2, sub = tid & 3;
   const int nqk = a.G * a.dk, C = 2 * nqk + a.H * a.dv, per = a.H / a.G;
   struct Raw {
     U16x8 q[NK], k[NK], v[NV];
@@ -558,13 +577,13 @@ __global__ void __launch_bounds__(512) head_map_kernel(ChunkArgs p, int items) {
     const bf16_t* x = reinterpret_cast<const bf16_t*>(a.cx) + (row0 + min(tok, n - 1)) * C;
 #pragma unroll
     for (int i = 0; i < NK; ++i) {
-      const int c = sub * 8 + 64 * i < a.dk ? sub * 8 + 64 * i : 0;
+      const int c = sub * 8 + 32 * i < a.dk ? sub * 8 + 32 * i : 0;
       r.q[i] = *reinterpret_cast<const U16x8*>(x + h / per * a.dk + c);
       r.k[i] = *reinterpret_cast<const U16x8*>(x + nqk + h / per * a.dk + c);
     }
 #pragma unroll
     for (int i = 0; i < NV; ++i)
-      r.v[i] = *reinterpret_cast<const U16x8*>(x + 2 * nqk + h * a.dv + (sub * 8 + 64 * i < a.dv ? sub * 8 + 64 * i : 0));
+      r.v[i] = *reinterpret_cast<const U16x8*>(x + 2 * nqk + h * a.dv + (sub * 8 + 32 * i < a.dv ? sub * 8 + 32 * i : 0));
     const bf16_t* y = reinterpret_cast<const bf16_t*>(a.x) + (row0 + min(lane, n - 1)) * a.ld;
     r.a = y[a.o_w + h];
     r.b = y[a.o_a + h];
@@ -588,14 +607,14 @@ __global__ void __launch_bounds__(512) head_map_kernel(ChunkArgs p, int items) {
       s.lg[lane] = G;
       s.fr[lane] = __expf(G);
       s.beta[lane] = beta;
+      s.late[lane] = __expf(end - G) * beta;
     }
-    const float late = __expf(end - __shfl(G, 8 * w + (lane >> 3), 64)) * __shfl(beta, 8 * w + (lane >> 3), 64);
-    p.e[(long long)item * DK + tid % DK] = __expf(end);
-    // eight threads a token: unit vectors
+    if (tid < DK) p.e[(long long)item * DK + tid] = __expf(end);
+    // four threads a token: unit vectors
     float q[NK][8], k[NK][8], sq = 0.f, sk = 0.f;
 #pragma unroll
     for (int i = 0; i < NK; ++i) {
-      const bool ok = tok < n && sub * 8 + 64 * i < a.dk;
+      const bool ok = tok < n && sub * 8 + 32 * i < a.dk;
 #pragma unroll
       for (int e = 0; e < 8; ++e) {
         q[i][e] = ok ? bf2f(raw.q[i].v[e]) : 0.f;
@@ -605,48 +624,47 @@ __global__ void __launch_bounds__(512) head_map_kernel(ChunkArgs p, int items) {
       }
     }
     auto add = [](float x, float y) { return x + y; };
-    const float iq = a.qscale / sqrtf(lanes_reduce<8>(sq, add) + 1e-6f), ik = 1.f / sqrtf(lanes_reduce<8>(sk, add) + 1e-6f);
+    const float iq = a.qscale / sqrtf(lanes_reduce<4>(sq, add) + 1e-6f), ik = 1.f / sqrtf(lanes_reduce<4>(sk, add) + 1e-6f);
 #pragma unroll
     for (int i = 0; i < NK; ++i) {
-      const int o = tok * L::LK + sub * 8 + 64 * i;
-      uint32_t zq[4], zk[4], zr[4];
+      const int o = tok * L::LK + sub * 8 + 32 * i;
+      uint32_t zq[4], zk[4];
 #pragma unroll
       for (int e = 0; e < 4; ++e) {
-        const float k0 = k[i][2 * e] * ik, k1 = k[i][2 * e + 1] * ik;
         zq[e] = pk2(q[i][2 * e] * iq, q[i][2 * e + 1] * iq);
-        zk[e] = pk2(k0, k1);
-        zr[e] = pk2(k0 * late, k1 * late);
+        zk[e] = pk2(k[i][2 * e] * ik, k[i][2 * e + 1] * ik);
       }
       *reinterpret_cast<u32x4*>(s.lq + o) = u32x4{zq[0], zq[1], zq[2], zq[3]};
       *reinterpret_cast<u32x4*>(s.lz + o) = u32x4{zk[0], zk[1], zk[2], zk[3]};
-      *reinterpret_cast<u32x4*>(s.rk + o) = u32x4{zr[0], zr[1], zr[2], zr[3]};
     }
 #pragma unroll
     for (int i = 0; i < NV; ++i) {
-      const bool ok = tok < n && sub * 8 + 64 * i < a.dv;
-      *reinterpret_cast<u32x4*>(s.v + tok * L::LV + sub * 8 + 64 * i) =
+      const bool ok = tok < n && sub * 8 + 32 * i < a.dv;
+      *reinterpret_cast<u32x4*>(s.v + tok * L::LV + sub * 8 + 32 * i) =
           ok ? __builtin_bit_cast(u32x4, raw.v[i]) : u32x4{0u, 0u, 0u, 0u};
     }
     __syncthreads();
-    // rows of block `blk`, keys (half 0) or queries (half 1), against the keys of the blocks up to it
-    const bf16_t* left = (half ? s.lq : s.lz) + 16 * blk * L::LK;
+    // rows of block w, keys and queries, against the keys of the blocks up to it
 #pragma unroll
     for (int J = 0; J < 4; ++J)
-      if (J <= blk) {
-        f32x4 x = {0.f, 0.f, 0.f, 0.f};
+      if (J <= w) {
+        f32x4 xz = {0.f, 0.f, 0.f, 0.f}, xq = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
         for (int c = 0; c < KS; ++c) {
           const int o = l15 * L::LK + c * 32 + 8 * g4;
-          x = mm32(*reinterpret_cast<const bf16x8*>(left + o), *reinterpret_cast<const bf16x8*>(s.lz + 16 * J * L::LK + o), x);
+          const bf16x8 kj = *reinterpret_cast<const bf16x8*>(s.lz + 16 * J * L::LK + o);
+          xz = mm32(*reinterpret_cast<const bf16x8*>(s.lz + 16 * w * L::LK + o), kj, xz);
+          xq = mm32(*reinterpret_cast<const bf16x8*>(s.lq + 16 * w * L::LK + o), kj, xq);
         }
         const int j = 16 * J + l15;
         const float lj = s.lg[j], bj = s.beta[j];
 #pragma unroll
         for (int r = 0; r < 4; ++r) {
-          const int t = 16 * blk + 4 * g4 + r;
-          const float y = (half ? j <= t : j < t) ? x[r] * bj * __expf(s.lg[t] - lj) : 0.f;
-          (half ? s.aqk : s.azk)[t * L::LA + j] = f2bf(y);
-          if (J == blk && !half) s.nd[blk][4 * g4 + r][l15] = -y;
+          const int t = 16 * w + 4 * g4 + r;
+          const float d = bj * __expf(s.lg[t] - lj), z = j < t ? xz[r] * d : 0.f;
+          s.azk[t * L::LA + j] = f2bf(z);
+          s.aqk[t * L::LA + j] = f2bf(j <= t ? xq[r] * d : 0.f);
+          if (J == w) s.nd[w][4 * g4 + r][l15] = -z;
         }
       }
     __syncthreads();
@@ -659,11 +677,11 @@ __global__ void __launch_bounds__(512) head_map_kernel(ChunkArgs p, int items) {
 #pragma unroll
         for (int k = 0; k < r; ++k) v = fmaf(s.nd[g4][r][k], x[k], v);
         x[r] = v;
-        s.ti[g4][r][l15] = v;
+        s.ti()[g4][r][l15] = v;
       }
     }
     __syncthreads();
-    chunk_maps<2, DK, DV>(s, p, item, w);
+    chunk_maps<2, DK, DV, 4>(s, p, item, w);
     __syncthreads();  // the next item reuses the LDS
   }
 }
@@ -776,7 +794,7 @@ int map_go(const ChunkArgs& p, int nchunk, hipStream_t s) {
   static_assert(lds <= 160 * 1024, "LDS");
   if (hipFuncSetAttribute((const void*)kern, hipFuncAttributeMaxDynamicSharedMemorySize, lds) != hipSuccess) return 5;
   const int items = nchunk * p.d.H, per_cu = lds <= 80 * 1024 ? 2 : 1;
-  hipLaunchKernelGGL(kern, dim3(items < 256 * per_cu ? items : 256 * per_cu), dim3(512), lds, s, p, items);
+  hipLaunchKernelGGL(kern, dim3(items < 256 * per_cu ? items : 256 * per_cu), dim3(KIND == 2 ? 256 : 512), lds, s, p, items);
   return hipGetLastError() == hipSuccess ? 0 : 4;
 }
 template <int DK, int DV>

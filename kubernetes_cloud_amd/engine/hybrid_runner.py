@@ -243,8 +243,16 @@ class HybridRunner(StepRunner):
         mixer(self._linear(h, L.w_in), y, b)
         if not pair:
             return self._linear(y, L.w_out)
-        ys = [self._linear(y[:, o], s.w_out) for o, s in zip(mixer.outs, (L.left, L.right))]
-        return NormedPair(ys[0], L.left.out_norm, ys[1], L.right.out_norm, L.spec.mixer.mul)
+        ys, sides = [y[:, o] for o in mixer.outs], (L.left, L.right)
+        d = self.cfg.hidden
+        if h.is_cuda and h.dtype == torch.bfloat16 and 2 <= b.T <= SKINNY_M and d % 4 == 0 and \
+                all(smm.supported(x, s.w_out) for x, s in zip(ys, sides)):  # one launch for both
+            outs = [torch.empty(b.T, d, device=h.device, dtype=h.dtype) for _ in ys]
+            smm.launch([smm.job([smm.part(x, s.w_out, packed=self._packed_w(s.w_out))], d, o)
+                        for x, s, o in zip(ys, sides, outs)], b.T, h.dtype)
+        else:
+            outs = [self._linear(x, s.w_out) for x, s in zip(ys, sides)]
+        return NormedPair(outs[0], L.left.out_norm, outs[1], L.right.out_norm, L.spec.mixer.mul)
 
     # ------------------------------------------------------- portions + tokens
     def _plan(self, entries, want_rows) -> tuple[_Batch, torch.Tensor | None]:
