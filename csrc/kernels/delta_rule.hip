@@ -11,77 +11,10 @@
 //
 // The carried state of a sequence lives in its slot and counts as zero at position 0.
 #include "delta_rule.h"
+#include "state_cols.h"
 
 namespace {
 using namespace delta;
-
-// A wave's part of the state: CW columns from 4 column groups (lane >> 4), rows lane & 15 + 16 i.
-template <int R, int CW>
-struct Cols {
-  float s[R][CW];
-  __device__ __forceinline__ void load(const float* S, int dk, int dv, int rg, int col, bool live) {
-#pragma unroll
-    for (int i = 0; i < R; ++i) {
-      const int r = rg + 16 * i;
-#pragma unroll
-      for (int e = 0; e < CW; ++e) s[i][e] = 0.f;
-      if (live && r < dk && col < dv) {
-        const float* q = S + (long long)r * dv + col;
-        if constexpr (CW == 4) {
-          const float4 v = *reinterpret_cast<const float4*>(q);
-          s[i][0] = v.x; s[i][1] = v.y; s[i][2] = v.z; s[i][3] = v.w;
-        } else {
-          s[i][0] = *q;
-        }
-      }
-    }
-  }
-  __device__ __forceinline__ void store(float* S, int dk, int dv, int rg, int col) const {
-#pragma unroll
-    for (int i = 0; i < R; ++i) {
-      const int r = rg + 16 * i;
-      if (r < dk && col < dv) {
-        float* q = S + (long long)r * dv + col;
-        if constexpr (CW == 4) *reinterpret_cast<float4*>(q) = make_float4(s[i][0], s[i][1], s[i][2], s[i][3]);
-        else *q = s[i][0];
-      }
-    }
-  }
-  // one token: the vectors at rows rg + 16 i (zero past dk), v at the lane's columns -> read-out
-  template <bool DELTA = true>
-  __device__ __forceinline__ void token(const float (&w)[R], const float (&z)[R], const float (&p)[R], const float (&k)[R],
-                                        const float (&q)[R], const float (&v)[CW], float qp, float qk, float (&o)[CW]) {
-    float zs[CW], qs[CW];
-#pragma unroll
-    for (int e = 0; e < CW; ++e) zs[e] = qs[e] = 0.f;
-#pragma unroll
-    for (int i = 0; i < R; ++i) {
-      const float qw = q[i] * w[i];
-#pragma unroll
-      for (int e = 0; e < CW; ++e) {
-        if (DELTA) zs[e] = fmaf(z[i], s[i][e], zs[e]);
-        qs[e] = fmaf(qw, s[i][e], qs[e]);
-      }
-    }
-    auto add = [](float x, float y) { return x + y; };
-#pragma unroll
-    for (int e = 0; e < CW; ++e) {
-      if (DELTA) zs[e] = lanes_reduce<16>(zs[e], add);
-      qs[e] = lanes_reduce<16>(qs[e], add);
-      o[e] = qs[e] + qp * zs[e] + qk * v[e];  // q^T (w S + p s + k v)
-    }
-#pragma unroll
-    for (int i = 0; i < R; ++i)
-#pragma unroll
-      for (int e = 0; e < CW; ++e) s[i][e] = fmaf(w[i], s[i][e], DELTA ? fmaf(p[i], zs[e], k[i] * v[e]) : k[i] * v[e]);
-  }
-};
-
-template <int R>
-__device__ __forceinline__ void rows_of(const float* src, int dk, int rg, float (&x)[R]) {
-#pragma unroll
-  for (int i = 0; i < R; ++i) x[i] = rg + 16 * i < dk ? src[rg + 16 * i] : 0.f;
-}
 
 template <typename E, int KIND, int R, int CW>
 __global__ void __launch_bounds__(R > 8 ? 512 : 1024) delta_step_kernel(DeltaArgs a) {
@@ -451,23 +384,6 @@ __global__ void __launch_bounds__(64 * NW) delta_parts_kernel(DeltaArgs a) {
   }
 }
 
-int rows_r(int dk) {  // rows a lane holds: 16 row groups
-  const int n = (dk + 15) / 16;
-  return n <= 1 ? 1 : n <= 2 ? 2 : n <= 3 ? 3 : n <= 4 ? 4 : n <= 6 ? 6 : n <= 8 ? 8 : n <= 12 ? 12 : 16;
-}
-
-#define DELTA_R(F)                  \
-  switch (rows_r(a.dk)) {           \
-    case 1: return F(1);            \
-    case 2: return F(2);            \
-    case 3: return F(3);            \
-    case 4: return F(4);            \
-    case 6: return F(6);            \
-    case 8: return F(8);            \
-    case 12: return F(12);          \
-    default: return F(16);          \
-  }
-
 bool wide(const DeltaArgs& a) { return a.dv % 4 == 0 && (uintptr_t)a.state % 16 == 0; }
 
 template <typename E, int KIND, int R, int CW>
@@ -483,7 +399,7 @@ int step_go(const DeltaArgs& a, int B, hipStream_t s) {
 template <typename E, int KIND>
 int step_r(const DeltaArgs& a, int B, hipStream_t s) {
 #define F(R) (wide(a) ? step_go<E, KIND, R, 4>(a, B, s) : step_go<E, KIND, R, 1>(a, B, s))
-  DELTA_R(F)
+  KCA_STATE_ROWS(a.dk, F)
 #undef F
 }
 
@@ -496,7 +412,7 @@ int scan_go(const DeltaArgs& a, int nent, hipStream_t s) {
 template <typename E>
 int scan_r(const DeltaArgs& a, int nent, hipStream_t s) {
 #define F(R) (wide(a) ? scan_go<E, R, 4>(a, nent, s) : scan_go<E, R, 1>(a, nent, s))
-  DELTA_R(F)
+  KCA_STATE_ROWS(a.dk, F)
 #undef F
 }
 

@@ -1,6 +1,9 @@
-// Mixture of gated experts: sigmoid router, grouping, expert products.
+// Mixture of gated experts: router, grouping, expert products.
 //
-//   s = sigmoid(W_router h); the `top` experts with the largest scores take the token, with weight s
+//   s = sigmoid(W_router h); the `top` experts with the largest scores take the token, with weight s;  or
+//   s = softmax(W_router h); the `top` experts with the largest s + correction, out of the `keep` of `groups` equal groups
+//   of neighbours whose largest such score is largest, with weight s / (their sum + 1e-20). The last `identity` of the
+//   outputs have no weights: they pass the token on (norm_residual.hip adds it), and no expert row is made for them.
 //   expert(x) = W_down (silu(W_gate x) * (W_up x))
 // A weight scales the expert's input -- both first products are linear, so it multiplies their fp32 sums
 // before the activation -- or its output (`scale_in` 0). The router (and the shared expert's gate, one
@@ -38,39 +41,99 @@ struct RouteArgs {
   int* ids;            // [T][top]
   float* wts;          // [T][top]
   float* sg;           // [T]
-  int T, d, E, top;
+  int T, d, E, top;    // E: router outputs, identity experts included
+  int softmax, groups, keep;
+  const float* fix;    // [E] correction of the choice (softmax; nullable)
 };
 
-// One wave: the top experts of one token from its logits z[E] (LDS); ties go to the lower index.
-__device__ __forceinline__ void pick(const RouteArgs& p, float* z, int t, int lane, int* ids_lds = nullptr) {
-  for (int k = 0; k < p.top; ++k) {
-    float best = -INFINITY;
-    int bi = 0x7fffffff;
-    for (int e = lane; e < p.E; e += 64)
-      if (z[e] > best) best = z[e], bi = e;
+__device__ __forceinline__ void lds_order() {  // one wave's LDS writes before its later reads
+  __builtin_amdgcn_fence(__ATOMIC_RELEASE, "wavefront");
+  __builtin_amdgcn_wave_barrier();
+  __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "wavefront");
+}
+
+// largest of z[0 .. n) over the wave; ties go to the lower index
+__device__ __forceinline__ void wave_argmax(const float* z, int n, int lane, float& best, int& bi) {
+  best = -INFINITY;
+  bi = 0x7fffffff;
+  for (int e = lane; e < n; e += 64)
+    if (z[e] > best) best = z[e], bi = e;
 #pragma unroll
-    for (int o = 32; o > 0; o >>= 1) {
-      const float ob = __shfl_xor(best, o, 64);
-      const int oi = __shfl_xor(bi, o, 64);
-      if (ob > best || (ob == best && oi < bi)) best = ob, bi = oi;
+  for (int o = 32; o > 0; o >>= 1) {
+    const float ob = __shfl_xor(best, o, 64);
+    const int oi = __shfl_xor(bi, o, 64);
+    if (ob > best || (ob == best && oi < bi)) best = ob, bi = oi;
+  }
+  if (bi >= n) bi = 0;  // (no finite score left)
+}
+
+// One wave: softmax scores, corrected choice within the best groups. z: logits, c, w: E floats each (LDS).
+__device__ __forceinline__ void pick_softmax(const RouteArgs& p, float* z, float* c, float* w, int t, int lane, int* ids_lds) {
+  float mx = -INFINITY, sum = 0.f;
+  for (int e = lane; e < p.E; e += 64) mx = fmaxf(mx, z[e]);
+  mx = wave_max(mx);
+  for (int e = lane; e < p.E; e += 64) sum += expf(z[e] - mx);
+  sum = 1.f / wave_sum(sum);
+  for (int e = lane; e < p.E; e += 64) {
+    const float s = expf(z[e] - mx) * sum;
+    z[e] = s;
+    c[e] = s + (p.fix ? p.fix[e] : 0.f);
+  }
+  lds_order();
+  if (p.keep < p.groups) {
+    const int size = p.E / p.groups;
+    for (int g = lane; g < p.groups; g += 64) {
+      float best = -INFINITY;
+      for (int e = g * size; e < (g + 1) * size; ++e) best = fmaxf(best, c[e]);
+      w[g] = best;
     }
-    if (bi >= p.E) bi = 0;  // (no finite score left)
+    lds_order();
+    for (int g = lane; g < p.groups; g += 64) {
+      int ahead = 0;  // groups before this one
+      for (int j = 0; j < p.groups; ++j) ahead += w[j] > w[g] || (w[j] == w[g] && j < g);
+      if (ahead >= p.keep)
+        for (int e = g * size; e < (g + 1) * size; ++e) c[e] = -INFINITY;
+    }
+    lds_order();
+  }
+  float total = 0.f;
+  for (int k = 0; k < p.top; ++k) {
+    float best;
+    int bi;
+    wave_argmax(c, p.E, lane, best, bi);
+    total += z[bi];
+    if (lane == 0) {
+      p.ids[(long long)t * p.top + k] = bi;
+      if (ids_lds) ids_lds[t * p.top + k] = bi;
+      w[k] = z[bi];
+      c[bi] = -INFINITY;
+    }
+    lds_order();
+  }
+  for (int k = lane; k < p.top; k += 64) p.wts[(long long)t * p.top + k] = w[k] / (total + 1e-20f);
+}
+
+// One wave: the top experts of one token from its logits z[E] (LDS; softmax: E floats each at c and w).
+__device__ __forceinline__ void pick(const RouteArgs& p, float* z, float* c, float* w, int t, int lane, int* ids_lds = nullptr) {
+  if (p.softmax) return pick_softmax(p, z, c, w, t, lane, ids_lds);
+  for (int k = 0; k < p.top; ++k) {
+    float best;
+    int bi;
+    wave_argmax(z, p.E, lane, best, bi);
     if (lane == 0) {
       p.ids[(long long)t * p.top + k] = bi;
       if (ids_lds) ids_lds[t * p.top + k] = bi;
       p.wts[(long long)t * p.top + k] = sigmoid(best);
       z[bi] = -INFINITY;
     }
-    __builtin_amdgcn_fence(__ATOMIC_RELEASE, "wavefront");
-    __builtin_amdgcn_wave_barrier();
-    __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "wavefront");
+    lds_order();
   }
 }
 
 // any dims and type: one token per workgroup, a wave per expert row
 template <typename E>
 __global__ void __launch_bounds__(256) route_rows_kernel(RouteArgs p) {
-  extern __shared__ float z[];  // [E + 1]
+  extern __shared__ float z[];  // [E + 1], softmax: [2][E] more
   const int lane = threadIdx.x & 63, wv = threadIdx.x >> 6, t = blockIdx.x;
   const E* h = reinterpret_cast<const E*>(p.h) + (long long)t * p.d;
   const int n = p.E + (p.wsg ? 1 : 0);
@@ -82,12 +145,12 @@ __global__ void __launch_bounds__(256) route_rows_kernel(RouteArgs p) {
     if (lane == 0) z[e] = s;
   }
   __syncthreads();
-  if (wv == 0) pick(p, z, t, lane);
+  if (wv == 0) pick(p, z, z + n, z + n + p.E, t, lane);
   if (threadIdx.x == 64 && p.wsg) p.sg[t] = sigmoid(z[p.E]);
 }
 
 struct GroupArgs {
-  const int* ids;      // [n]
+  const int* ids;      // [n]; E and beyond: no expert row (inv -1)
   int n, E, mt;
   int *perm, *inv, *tiles, *ntiles;
 };
@@ -102,7 +165,8 @@ __device__ __forceinline__ void group_rows(const GroupArgs& p, int* sh) {
   int *cnt = sh, *off = sh + E, *toff = off + E + 1;
   for (int e = tid; e < E; e += NT) cnt[e] = 0;
   __syncthreads();
-  for (int i = tid; i < n; i += NT) atomicAdd(&cnt[p.ids[i]], 1);
+  for (int i = tid; i < n; i += NT)
+    if (p.ids[i] < E) atomicAdd(&cnt[p.ids[i]], 1);
   __syncthreads();
   if (tid < 64) {  // exclusive sums over the experts, 64 at a time
     int co = 0, to = 0;
@@ -135,8 +199,8 @@ __device__ __forceinline__ void group_rows(const GroupArgs& p, int* sh) {
   }
   __syncthreads();
   for (int i = tid; i < n; i += NT) {  // (the order within an expert does not matter: rows are independent)
-    const int pos = atomicAdd(&cnt[p.ids[i]], 1);
-    p.perm[pos] = i;
+    const int e = p.ids[i], pos = e < E ? atomicAdd(&cnt[e], 1) : -1;
+    if (pos >= 0) p.perm[pos] = i;
     p.inv[i] = pos;
   }
 }
@@ -150,9 +214,10 @@ __global__ void __launch_bounds__(1024) group_kernel(GroupArgs p) {
 // one workgroup, which also groups its assignments (the decode step)
 template <int NW, bool GROUP>
 __global__ void __launch_bounds__(NW * 64) route_mfma_kernel(RouteArgs p, GroupArgs gr) {
-  extern __shared__ __attribute__((aligned(16))) float lds[];  // z[16][zs], part[NW][16][64] (then group_rows'), ids
-  const int n = p.E + (p.wsg ? 1 : 0), zs = (n + 63) / 64 * 64;
-  float *z = lds, *part = lds + 16 * zs;
+  // z[16][zs], softmax: two more of them; part[NW][16][64] (then group_rows'), ids
+  extern __shared__ __attribute__((aligned(16))) float lds[];
+  const int n = p.E + (p.wsg ? 1 : 0), zs = (n + 63) / 64 * 64, zr = 16 * zs;
+  float *z = lds, *part = lds + (p.softmax ? 3 : 1) * zr;
   int* sids = reinterpret_cast<int*>(part + NW * 1024);  // GROUP: [T * top]
   const int tid = threadIdx.x, lane = tid & 63, wv = tid >> 6, r16 = lane & 15, g = lane >> 4;
   const int t0 = blockIdx.x * 16, d = p.d;
@@ -206,7 +271,7 @@ __global__ void __launch_bounds__(NW * 64) route_mfma_kernel(RouteArgs p, GroupA
   for (int r = wv; r < 16; r += NW) {
     if (t0 + r >= p.T) break;
     if (p.wsg && lane == 0) p.sg[t0 + r] = sigmoid(z[r * zs + p.E]);
-    pick(p, z + r * zs, t0 + r, lane, GROUP ? sids : nullptr);
+    pick(p, z + r * zs, z + zr + r * zs, z + 2 * zr + r * zs, t0 + r, lane, GROUP ? sids : nullptr);
   }
   if constexpr (GROUP) {
     __syncthreads();
@@ -493,8 +558,21 @@ int gemv_go(const ExpertArgs& a, int mt, int max_tiles, hipStream_t s) {
 bool al16(const void* p) { return (uintptr_t)p % 16 == 0; }
 
 template <int NW, bool GROUP>
+int route_lds(const RouteArgs& a) {
+  const int zs = (a.E + (a.wsg ? 1 : 0) + 63) / 64 * 64;
+  return ((a.softmax ? 3 : 1) * 16 * zs + NW * 1024 + (GROUP ? a.T * a.top : 0)) * 4;
+}
+constexpr int MAX_LDS = 160 * 1024;
+
+// softmax routers: equal groups, enough experts in the kept ones
+bool route_ok(const RouteArgs& a) {
+  return a.T >= 1 && a.d >= 1 && a.E >= 1 && a.E <= 1024 && a.top >= 1 && a.top <= a.E && a.h && a.wr && a.ids && a.wts && (!a.wsg || a.sg) &&
+         (!a.softmax || (a.groups >= 1 && a.E % a.groups == 0 && a.keep >= 1 && a.keep <= a.groups && a.top <= a.E / a.groups * a.keep));
+}
+
+template <int NW, bool GROUP>
 int route_go(const RouteArgs& a, const GroupArgs& g, hipStream_t s) {
-  const int zs = (a.E + (a.wsg ? 1 : 0) + 63) / 64 * 64, lds = (16 * zs + NW * 1024 + (GROUP ? a.T * a.top : 0)) * 4;
+  const int lds = route_lds<NW, GROUP>(a);
   auto kern = route_mfma_kernel<NW, GROUP>;
   if (lds > 48 * 1024 && hipFuncSetAttribute((const void*)kern, hipFuncAttributeMaxDynamicSharedMemorySize, lds) != hipSuccess)
     return 5;
@@ -506,12 +584,14 @@ int route_go(const RouteArgs& a, const GroupArgs& g, hipStream_t s) {
 
 // dtype: 0 fp32, 1 bf16
 KCA_API int kca_moe_route(int dtype, const void* h, const void* wr, const void* wsg, void* ids, void* wts, void* sg,
-                          int T, int d, int E, int top, hipStream_t s) {
-  if (T < 1 || d < 1 || E < 1 || E > 1024 || top < 1 || top > E || !h || !wr || !ids || !wts || (wsg && !sg)) return 1;
-  const RouteArgs a{h, wr, wsg, (int*)ids, (float*)wts, (float*)sg, T, d, E, top};
-  if (dtype == 1 && d % 8 == 0 && al16(h) && al16(wr) && al16(wsg)) return route_go<8, false>(a, GroupArgs{}, s);
-  if (dtype == 1) hipLaunchKernelGGL(route_rows_kernel<bf16_t>, dim3(T), dim3(256), (E + 1) * 4, s, a);
-  else if (dtype == 0) hipLaunchKernelGGL(route_rows_kernel<float>, dim3(T), dim3(256), (E + 1) * 4, s, a);
+                          int T, int d, int E, int top, int softmax, const void* fix, int groups, int keep, hipStream_t s) {
+  const RouteArgs a{h, wr, wsg, (int*)ids, (float*)wts, (float*)sg, T, d, E, top, softmax, groups, keep, (const float*)fix};
+  if (!route_ok(a)) return 1;
+  if (dtype == 1 && d % 8 == 0 && al16(h) && al16(wr) && al16(wsg) && route_lds<8, false>(a) <= MAX_LDS)
+    return route_go<8, false>(a, GroupArgs{}, s);
+  const int lds = ((softmax ? 3 : 1) * E + 1) * 4;
+  if (dtype == 1) hipLaunchKernelGGL(route_rows_kernel<bf16_t>, dim3(T), dim3(256), lds, s, a);
+  else if (dtype == 0) hipLaunchKernelGGL(route_rows_kernel<float>, dim3(T), dim3(256), lds, s, a);
   else return 3;
   return hipGetLastError() == hipSuccess ? 0 : 4;
 }
@@ -530,14 +610,14 @@ KCA_API int kca_moe_group(const void* ids, int n, int E, int mt, void* perm, voi
   return hipGetLastError() == hipSuccess ? 0 : 4;
 }
 
-// Both in one launch: bf16, at most 16 tokens (10: shape outside it)
+// Both in one launch: bf16, at most 16 tokens (10: shape outside it). E: router outputs, the first `real` with weights
 KCA_API int kca_moe_route_group(const void* h, const void* wr, const void* wsg, void* ids, void* wts, void* sg, int T,
-                                int d, int E, int top, int mt, void* perm, void* inv, void* tiles, int max_tiles,
-                                void* ntiles, hipStream_t s) {
-  if (T < 1 || d < 1 || E < 1 || E > 1024 || top < 1 || top > E || !h || !wr || !ids || !wts || (wsg && !sg)) return 1;
-  if (T > 16 || top > 64 || d % 8 || !al16(h) || !al16(wr) || !al16(wsg)) return 10;
-  const RouteArgs a{h, wr, wsg, (int*)ids, (float*)wts, (float*)sg, T, d, E, top};
-  const GroupArgs g{(const int*)ids, T * top, E, mt, (int*)perm, (int*)inv, (int*)tiles, (int*)ntiles};
+                                int d, int E, int real, int top, int softmax, const void* fix, int groups, int keep, int mt, void* perm,
+                                void* inv, void* tiles, int max_tiles, void* ntiles, hipStream_t s) {
+  const RouteArgs a{h, wr, wsg, (int*)ids, (float*)wts, (float*)sg, T, d, E, top, softmax, groups, keep, (const float*)fix};
+  if (!route_ok(a) || real < 1 || real > E) return 1;
+  if (T > 16 || top > 64 || d % 8 || !al16(h) || !al16(wr) || !al16(wsg) || route_lds<16, true>(a) > MAX_LDS) return 10;
+  const GroupArgs g{(const int*)ids, T * top, real, mt, (int*)perm, (int*)inv, (int*)tiles, (int*)ntiles};
   if (!group_ok(g, max_tiles)) return 1;
   return route_go<16, true>(a, g, s);
 }

@@ -10,6 +10,11 @@
 //   x_t = src_t + a_t     or   x_t = src_t + mul * (N(a_t; ga) + N(b_t; gb))
 //   h_t = x_t / sqrt(mean x_t^2 + eps) * (1 + g),   raw_t = x_t rounded (a column block of a wider buffer)
 // src: the stream, scaled embedding rows, or rows of a product plus one vector.
+//
+// Post-norms (postnorm_kernel): RMS norms of what a sublayer adds, gains of one number
+//   u_t = a_t + sum_k y[inv[t][k]] + (sum of wts[t][k] with inv -1) src_t      routed rows (moe.hip), identity experts
+//   x_t = src_t + ga u_t / sqrt(mean u_t^2 + eps)
+//   h_t = x_t rounded, or hmul g x_t / sqrt(mean x_t^2 + eps)
 #include "common.h"
 #include "lanes.h"
 
@@ -381,6 +386,154 @@ __global__ void __launch_bounds__(256) prenorm_kernel(PreArgs p) {
   }
 }
 
+struct PostArgs {
+  const float* x_in;          // one source: the stream,
+  const void* embed;          // embedding rows (times escale)
+  const long long* tokens;
+  float escale;
+  const void* a;              // sublayer output (nullable)
+  long long lda;
+  const void* y;              // routed rows (nullable), row stride d
+  const int* inv;             // [T][top] row of y; -1: the source itself, times
+  const float* wts;           // [T][top]
+  int top;
+  const void* ga;             // gain of their norm (nullable: nothing is added)
+  const void* g;              // gain of the closing norm (nullable: none)
+  float hmul, eps;
+  const int* rows;            // output row i reads token rows[i] (nullable)
+  float* x_out;               // nullable
+  void* h;                    // nullable
+  int T, d;
+};
+
+template <typename E, int VEC, int NCH, int NT>
+__global__ void __launch_bounds__(256) postnorm_kernel(PostArgs p) {
+  constexpr int RPB = 256 / NT;  // rows of a workgroup (one wave each when NT == 64)
+  static_assert(RPB == 1 || NT == 64, "a row is a wave or the workgroup");
+  __shared__ float red[2][NT / 64];
+  const int tid = threadIdx.x % NT, d = p.d;
+  const int r = blockIdx.x * RPB + threadIdx.x / NT;
+  if (r >= p.T) return;  // (whole waves; RPB == 1: never)
+  const int t = p.rows ? p.rows[r] : r;
+  const float inv = 1.f / (float)d;
+  float x[NCH][VEC], u[NCH][VEC];
+  auto at = [&](int c) { return (c * NT + tid) * VEC; };
+  const long long tok = p.embed ? p.tokens[t] : 0;
+  const float ga = p.ga ? ldf<E>(reinterpret_cast<const E*>(p.ga)) : 0.f, g = p.g ? ldf<E>(reinterpret_cast<const E*>(p.g)) : 0.f;
+#pragma unroll
+  for (int c = 0; c < NCH; ++c) {
+    const int i = at(c);
+#pragma unroll
+    for (int e = 0; e < VEC; ++e) x[c][e] = u[c][e] = 0.f;
+    if (i < d) {
+      if (p.x_in) ldv<float, VEC>(p.x_in + (long long)t * d + i, x[c]);
+      else ldv<E, VEC>(reinterpret_cast<const E*>(p.embed) + tok * d + i, x[c]);
+      if (p.a) ldv<E, VEC>(reinterpret_cast<const E*>(p.a) + (long long)t * p.lda + i, u[c]);
+    }
+  }
+  if (p.embed)
+#pragma unroll
+    for (int c = 0; c < NCH; ++c)
+#pragma unroll
+      for (int e = 0; e < VEC; ++e) x[c][e] *= p.escale;
+  if (p.y) {
+    const int* iv = p.inv + (long long)t * p.top;
+    const float* wt = p.wts + (long long)t * p.top;
+    float pass = 0.f;
+    for (int k0 = 0; k0 < p.top; k0 += 4) {  // four rows' loads together; past the end and identity experts: row 0 times zero
+      float v[4][NCH][VEC], on[4];
+#pragma unroll
+      for (int k = 0; k < 4; ++k) {
+        const bool in = k0 + k < p.top;
+        const int row = in ? iv[k0 + k] : 0;
+        on[k] = in && row >= 0 ? 1.f : 0.f;
+        if (in && row < 0) pass += wt[k0 + k];
+#pragma unroll
+        for (int c = 0; c < NCH; ++c) {
+#pragma unroll
+          for (int e = 0; e < VEC; ++e) v[k][c][e] = 0.f;
+          if (at(c) < d && on[k] != 0.f) ldv<E, VEC>(reinterpret_cast<const E*>(p.y) + (long long)row * d + at(c), v[k][c]);
+        }
+      }
+#pragma unroll
+      for (int k = 0; k < 4; ++k)
+#pragma unroll
+        for (int c = 0; c < NCH; ++c)
+#pragma unroll
+          for (int e = 0; e < VEC; ++e) u[c][e] += v[k][c][e];
+    }
+#pragma unroll
+    for (int c = 0; c < NCH; ++c)
+#pragma unroll
+      for (int e = 0; e < VEC; ++e) u[c][e] = fmaf(pass, x[c][e], u[c][e]);
+  }
+  auto rstd = [&](const float (&y)[NCH][VEC], float* rd) {  // (elements past d are zero)
+    float s = 0.f;
+#pragma unroll
+    for (int c = 0; c < NCH; ++c)
+#pragma unroll
+      for (int e = 0; e < VEC; ++e) s = fmaf(y[c][e], y[c][e], s);
+    s = lanes_reduce<64>(s, [](float a, float b) { return a + b; });
+    if constexpr (NT > 64) {
+      if ((threadIdx.x & 63) == 0) rd[threadIdx.x >> 6] = s;
+      __syncthreads();
+      s = 0.f;
+#pragma unroll
+      for (int i = 0; i < NT / 64; ++i) s += rd[i];
+    }
+    return 1.f / sqrtf(s * inv + p.eps);
+  };
+  if (p.ga) {
+    const float n = ga * rstd(u, red[0]);
+#pragma unroll
+    for (int c = 0; c < NCH; ++c)
+#pragma unroll
+      for (int e = 0; e < VEC; ++e) x[c][e] = fmaf(n, u[c][e], x[c][e]);
+  }
+  if (p.x_out) {
+#pragma unroll
+    for (int c = 0; c < NCH; ++c)
+      if (at(c) < d) stv<VEC>(p.x_out + (long long)r * d + at(c), x[c]);
+  }
+  if (!p.h) return;
+  const float n = p.g ? p.hmul * g * rstd(x, red[1]) : 1.f;
+#pragma unroll
+  for (int c = 0; c < NCH; ++c) {
+    float y[VEC];
+#pragma unroll
+    for (int e = 0; e < VEC; ++e) y[e] = x[c][e] * n;
+    if (at(c) < d) stv<VEC>(reinterpret_cast<E*>(p.h) + (long long)r * d + at(c), y);
+  }
+}
+
+template <typename E>
+int launch_post(const PostArgs& a, hipStream_t s) {
+  const bool v4 = a.d % 4 == 0 && a.lda % 4 == 0;
+#define GO(V, N, NT) \
+  hipLaunchKernelGGL((postnorm_kernel<E, V, N, NT>), dim3((a.T + 256 / NT - 1) / (256 / NT)), dim3(256), 0, s, a)
+  if (v4 && a.T >= 512 && a.d <= 1024) {  // many short rows: a wave each, no barriers
+    if (a.d <= 256) GO(4, 1, 64);
+    else if (a.d <= 512) GO(4, 2, 64);
+    else GO(4, 4, 64);
+  } else if (v4) {
+    const int n = (a.d + 1023) / 1024;
+    if (n <= 1) GO(4, 1, 256);
+    else if (n <= 2) GO(4, 2, 256);
+    else if (n <= 4) GO(4, 4, 256);
+    else if (n <= 8) GO(4, 8, 256);
+    else if (n <= 16) GO(4, 16, 256);
+    else return 10;
+  } else {
+    const int n = (a.d + 255) / 256;
+    if (n <= 1) GO(1, 1, 256);
+    else if (n <= 4) GO(1, 4, 256);
+    else if (n <= 16) GO(1, 16, 256);
+    else return 10;
+  }
+#undef GO
+  return hipGetLastError() == hipSuccess ? 0 : 4;
+}
+
 template <typename E>
 int launch_pre(const PreArgs& a, hipStream_t s) {
   const bool v4 = a.d % 4 == 0 && a.lda % 4 == 0 && a.ldb % 4 == 0 && a.ldbase % 4 == 0 && a.ldr % 4 == 0 &&
@@ -441,5 +594,19 @@ KCA_API int kca_prenorm(const PreArgs* in, int dtype, hipStream_t s) {
   if (p.x_in && p.x_in == p.x_out && p.rows) return 2;
   if (dtype == 0) return launch_pre<float>(p, s);
   if (dtype == 1) return launch_pre<bf16_t>(p, s);
+  return 3;
+}
+
+KCA_API int kca_postnorm_abi() { return (int)sizeof(PostArgs); }
+
+// dtype: 0 fp32, 1 bf16 (of every tensor but the stream and the router's weights)
+KCA_API int kca_postnorm(const PostArgs* in, int dtype, hipStream_t s) {
+  const PostArgs& p = *in;
+  if (p.T < 1 || p.d < 1 || (p.x_in != nullptr) == (p.embed != nullptr) || (p.embed && !p.tokens) || (p.ga && !p.a && !p.y) ||
+      (!p.ga && (p.a || p.y)) || (p.y && (!p.inv || !p.wts || p.top < 1)) || (!p.h && (!p.x_out || p.g)))
+    return 1;
+  if (p.x_in && p.x_in == p.x_out && p.rows) return 2;
+  if (dtype == 0) return launch_post<float>(p, s);
+  if (dtype == 1) return launch_post<bf16_t>(p, s);
   return 3;
 }

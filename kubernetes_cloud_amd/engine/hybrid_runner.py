@@ -11,8 +11,8 @@ A layer's token mixer is an object of ``mixers`` (attention over the paged cache
 state); around it a parallel layer takes three or four launches beside the vendor (or skinny matrix-core)
 products -- residual + norm + token shift, the mixer's core, the feed-forward's activation or experts; mixer and
 feed-forward close in one product -- and a sandwich layer one norm launch per sublayer (output norm, layer scale,
-residual and the next norm together); a pre-norm layer is one norm launch per sublayer too. Layers may run several times in a row (``cfg.runs``); every run has its own
-cache or state.
+residual and the next norm together); a pre-norm or post-norm layer is one norm launch per sublayer too. Layers may run
+several times in a row (``cfg.runs``); every run has its own cache or state.
 
 What a sequence owns besides its KV pages lives in ``SlotState``: the last normed row of every parallel layer
 (token shift) and the recurrent states. A batch with multi-token portions reads carried rows from a copy taken at
@@ -31,8 +31,9 @@ from ..ops import skinny_mm as smm
 from ..ops.delta_rule import Portions, plan_portions
 from ..ops.gemv import skinny_linear
 from ..ops.latent_attention import Prompts, plan_prompts
-from ..ops.norm_residual import Embedded, NormedBranch, NormedPair, Rows, norm_residual, prenorm
+from ..ops.norm_residual import Embedded, NormedBranch, NormedPair, NormedSum, Rows, norm_residual, postnorm, prenorm
 from ..ops.rms_shift import Branch, rms_shift
+from ..models.hybrid_config import MoESpec, SumSpec
 from .mixers import make_mixer
 from .runner import KVCache, SlotState, StepRunner
 
@@ -75,10 +76,8 @@ class HybridRunner(StepRunner):
         shapes, widths = [], {"shift": (len(cfg.runs), d)} if cfg.block == "parallel" else {}
         members = [m for mx in self.mixers for m in mx.members()]
         for mx in members:
-            shape = mx.cache_shape()
-            if shape is not None:
-                mx.index = len(shapes)
-                shapes.append(shape)
+            mx.index = len(shapes)
+            shapes += mx.cache_shapes(page_size)
             widths.update(mx.state_widths())
         self.cache = KVCache(len(shapes), max_slots, 0, self.max_len, 0, self.device, self.dtype, page_size=page_size,
                              n_pages=kv_pages, layer_shapes=shapes)
@@ -86,23 +85,27 @@ class HybridRunner(StepRunner):
         for mx in members:
             mx.cache, mx.state = self.cache, self.state
         self._members = members
-        self._forward_layers = {"parallel": self._parallel, "sandwich": self._sandwich, "prenorm": self._prenorm}[cfg.block]
+        self._forward_layers = {"parallel": self._parallel, "sandwich": self._sandwich, "prenorm": self._prenorm,
+                                "postnorm": self._postnorm}[cfg.block]
+        self._rules = [None if not isinstance(L.spec.mlp, MoESpec) else moe.Router(
+            L.spec.mlp.score == "softmax", L.correction.float() if L.spec.mlp.correction else None, L.spec.mlp.groups,
+            L.spec.mlp.keep, L.spec.mlp.identity) for L in model.layers]
         if self.device.type == "cuda":
             from ..utils import tunable
             tunable.ensure(tunable.DECODE_FILE)
 
     # ---------------------------------------------------------------- linear
-    def _linear(self, x, w, out=None, act: int = 0):
-        """x W^T (act 2: exact GELU, 3: squared ReLU). Few bf16 rows stream the weight on the GEMV / skinny matrix-core kernels."""
+    def _linear(self, x, w, out=None, act: int = 0, bias=None):
+        """x W^T + bias (act 2: exact GELU, 3: squared ReLU). Few bf16 rows stream the weight on the GEMV / skinny matrix-core kernels."""
         T = x.shape[0]
         if (x.is_cuda and x.dtype == torch.bfloat16 and T <= SKINNY_M and w.shape[0] % 4 == 0 and smm.supported(x, w)
                 and (out is None or (out.data_ptr() % 16 == 0 and out.stride(0) % 8 == 0))):
             if out is None:
                 out = torch.empty(T, w.shape[0], device=x.device, dtype=x.dtype)
             if T == 1:
-                return skinny_linear(x, w, None, act, out=out)
-            return smm.mm(x, w, None, act, out=out, packed=self._packed_w(w))
-        y = F.linear(x, w)
+                return skinny_linear(x, w, bias, act, out=out)
+            return smm.mm(x, w, bias, act, out=out, packed=self._packed_w(w))
+        y = F.linear(x, w, bias)
         if act:
             return moe.act_rows(y, y if out is None else out, gated=False, act=ACTS[act])
         if out is not None:
@@ -235,6 +238,39 @@ class HybridRunner(StepRunner):
         if layers_out is not None:
             layers_out.append(prenorm(x, branch, None, eps)[0])
         return prenorm(x, branch, m.final_norm, eps, rows=want, keep_x=False)[1]
+
+    def _postnorm(self, b, want, layers_out):
+        """Mixer and feed-forward in turn on the stream itself; what they add is normed."""
+        m, cfg, eps, dt = self.model, self.cfg, self.cfg.norm_eps, self.dtype
+        x, branch = Embedded(m.wte, b.tokens, cfg.embed_scale), None
+        for r, i in enumerate(cfg.runs):
+            L = m.layers[i]
+            x, h = postnorm(x, branch, eps, dt)
+            if layers_out is not None and r:
+                layers_out.append(x.clone())
+            cols = L.spec.mixer.out_cols
+            gaps = cols > L.spec.mixer.left.out_cols + L.spec.mixer.right.out_cols if isinstance(L.spec.mixer, SumSpec) else False
+            y = (torch.zeros if gaps else torch.empty)(b.T, cols, device=h.device, dtype=dt)
+            self.mixers[r](self._linear(h, L.w_in, bias=L.b_in), y, b)
+            branch = NormedSum(L.norm, self._linear(y, L.w_out))
+            if L.spec.mlp is not None:
+                x, h = postnorm(x, branch, eps, dt)
+                branch = self._routed(L, h, self._rules[i])
+        if layers_out is not None:
+            layers_out.append(postnorm(x, branch, eps, dt)[0])
+        return postnorm(x, branch, eps, dt, gain=m.final_norm, mul=cfg.logit_scale, rows=want, keep_x=False)[1]
+
+    def _routed(self, L, h, rule):
+        """A post-norm layer's routed experts (and the shared one)."""
+        mlp, T = L.spec.mlp, h.shape[0]
+        ids, wts, _, g = moe.route_group(h, L.router, mlp.top, None,
+                                         moe.tile_rows(T, mlp.top, mlp.outputs, h.shape[1], mlp.ff, h.dtype), rule)
+        y = moe.experts(h, ids, wts, L.gate_up, L.down, g, mlp.scale_in)
+        a = None
+        if mlp.shared_ff:
+            act = torch.empty(T, mlp.shared_ff, device=h.device, dtype=h.dtype)
+            a = self._linear(moe.act_rows(self._linear(h, L.w_up), act, gated=True), L.w_down)
+        return NormedSum(L.norm2, a, y, g.inv, wts)
 
     def _mix(self, L, mixer, h, b):
         """A pre-norm layer's mixer -> what it adds to the stream."""

@@ -6,23 +6,27 @@ batch (``hybrid_runner._Batch``) into the rows that the output projection reads.
 """
 from __future__ import annotations
 
+import dataclasses
+
 import torch
 
 from ..models.hybrid_config import (BiasedAttentionSpec, ChannelDeltaSpec, DiffAttentionSpec, GatedRecurrenceSpec,
-                                    GeneralDeltaSpec, HeadDeltaSpec, LatentAttentionSpec, SideBySideSpec, SsdSpec,
-                                    aligned_parts)
+                                    GeneralDeltaSpec, HeadDeltaSpec, LatentAttentionSpec, MatrixMemorySpec,
+                                    PooledAttentionSpec, SideBySideSpec, SsdSpec, SumSpec, aligned_parts)
 from ..ops import biased_attention as ba
 from ..ops import delta_rule as dr
 from ..ops import diff_attention as da
 from ..ops import gated_scan as gs
 from ..ops import latent_attention as la
+from ..ops import matrix_memory as mm
 from ..ops import moe
+from ..ops import pooled_attention as pa
 
 
 class Mixer:
     """``run``: the layer run (names its state); ``linear``: the runner's projection; ``twin``: the mixer of an earlier
-    pass over the same layer (shares what is derived from the weights). ``cache`` / ``index`` (the layer's
-    place in it) and ``state`` are set once the runner has made them."""
+    pass over the same layer (shares what is derived from the weights). ``cache`` / ``index`` (the layer's first
+    place in it) and ``state`` are set once the runner has made them. Mixers that a sum takes have ``weigh(mul)``."""
 
     def __init__(self, layer, cfg, run: int | str, linear, twin: Mixer | None = None):
         self.layer, self.run, self.linear = layer, run, linear
@@ -35,6 +39,11 @@ class Mixer:
     def cache_shape(self):
         """(key heads, key size, value heads, value size) of the layer's pages, None without a cache."""
         return None
+
+    def cache_shapes(self, page_size: int) -> list:
+        """All pages of the layer, in the form of ``KVCache``'s ``layer_shapes``."""
+        shape = self.cache_shape()
+        return [] if shape is None else [shape]
 
     def state_widths(self) -> dict:
         return {}
@@ -196,6 +205,71 @@ class BiasedAttentionMixer(Mixer):
             ba.attend_rows(*a, out, b.max_kv, fused_append=False)
 
 
+class PooledAttentionMixer(Mixer):
+    """The block means lie beside the tokens' keys and values in the same pages: a second entry of the cache."""
+
+    def __init__(self, layer, cfg, run, linear, twin=None):
+        super().__init__(layer, cfg, run, linear)
+        mx, L = layer.spec.mixer, layer
+        self.sp = pa.PooledHeads(mx.heads, mx.kv_heads, mx.dim, mx.vdim, mx.scale, cfg.norm_eps,
+                                 tuple(mx.parts[n][0] for n in "qkv"), mx.window, mx.pool, mx.rot_dims)
+        self.wt = twin.wt if twin is not None else pa.PooledWeights(
+            L.q_norm, L.k_norm, L.sink.float(), pa.rotary_frequencies(mx.rot_dims, mx.rot_base, mx.rot_scaling).to(L.sink.device))
+
+    def weigh(self, mul: float):
+        self.sp = dataclasses.replace(self.sp, mul=mul)
+
+    def cache_shape(self):
+        mx = self.layer.spec.mixer
+        return mx.kv_heads, mx.dim, mx.kv_heads, mx.vdim
+
+    def cache_shapes(self, page_size):
+        shape = self.cache_shape()
+        return [shape, (*shape, pa.block_rows(page_size, self.sp.pool))]
+
+    def buffers(self, rows, max_kv, dtype):
+        _, _, w, c = pa.rows_plan(self.sp, rows, self.sp.visible(max_kv))
+        return {"ws": (w, torch.float32), "cnt": (c, torch.int32)}
+
+    def __call__(self, x, out, b):
+        c, i = self.cache, self.index
+        pages = pa.PooledCache(c.k[i], c.v[i], c.k[i + 1], c.v[i + 1], c.table)
+        a = (self.sp, self.wt, x, pages, b.pos, b.slots)
+        if b.single:
+            pa.attend_rows(*a, out, b.max_kv, fused=True, ws=b.bufs.get("ws"), cnt=b.bufs.get("cnt"))
+            return
+        pa.prepare(*a)
+        if out.is_cuda and pa.tiles_ok(self.sp, out.dtype, c.page_size, x.stride(0), out.stride(0)):
+            if b.tiles is not None:
+                pa.attend_tiles(*a, out, b.tiles)
+            if b.row_of is not None:
+                pa.attend_rows(*a, out, b.row_kv, fused=False, row_of=b.row_of)
+        else:
+            pa.attend_rows(*a, out, b.max_kv, fused=False)
+
+
+class MatrixMemoryMixer(Mixer):
+    def __init__(self, layer, cfg, run, linear, twin=None):
+        super().__init__(layer, cfg, run, linear)
+        mx, L = layer.spec.mixer, layer
+        self.sp = mm.MemoryHeads(mx.heads, mx.dim, mx.vdim, tuple(mx.parts[n][0] for n in "qkvgif"), mx.gate_cap, cfg.norm_eps)
+        self.wt = mm.MemoryWeights(L.i_bias, L.f_bias, L.gain)
+
+    def weigh(self, mul: float):
+        self.sp = dataclasses.replace(self.sp, mul=mul)
+
+    def state_widths(self):
+        sp, r = self.sp, self.run
+        return {f"mem{r}": (1, sp.heads * sp.dim * sp.vdim), f"memn{r}": (1, sp.heads * sp.dim), f"memm{r}": (1, sp.heads)}
+
+    def __call__(self, x, out, b):
+        st = mm.MemoryState(*(self.state[f"{k}{self.run}"][0] for k in ("mem", "memn", "memm")))
+        if b.single:
+            mm.memory_step(self.sp, self.wt, x, st, b.pos, b.slots, out)
+        else:
+            mm.memory_portions(self.sp, self.wt, x, st, b.portions, out)
+
+
 class SideBySideMixer(Mixer):
     """Two mixers over column blocks of the projection rows, into column blocks of the output rows."""
 
@@ -215,10 +289,21 @@ class SideBySideMixer(Mixer):
             m(x[:, c], out[:, o], b)
 
 
+class SumMixer(SideBySideMixer):
+    """... whose rows carry the sides' weights, so that one output projection sums them."""
+
+    def __init__(self, layer, cfg, run, linear, twin=None):
+        super().__init__(layer, cfg, run, linear, twin)
+        mx = layer.spec.mixer
+        for m, mul in zip(self.sides, (mx.left_mul, mx.right_mul)):
+            m.weigh(mul)
+
+
 MIXERS = {DiffAttentionSpec: DiffAttentionMixer, GatedRecurrenceSpec: GatedRecurrenceMixer,
           LatentAttentionSpec: LatentAttentionMixer, GeneralDeltaSpec: DeltaRuleMixer, ChannelDeltaSpec: DeltaRuleMixer,
           HeadDeltaSpec: DeltaRuleMixer, SsdSpec: DeltaRuleMixer, BiasedAttentionSpec: BiasedAttentionMixer,
-          SideBySideSpec: SideBySideMixer}
+          SideBySideSpec: SideBySideMixer, PooledAttentionSpec: PooledAttentionMixer, MatrixMemorySpec: MatrixMemoryMixer,
+          SumSpec: SumMixer}
 
 
 def make_mixer(layer, cfg, run: int | str, linear, twin: Mixer | None = None) -> Mixer:

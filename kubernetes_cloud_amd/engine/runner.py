@@ -76,7 +76,8 @@ class KVCache:
                  device, dtype=torch.bfloat16, page_size: int = 0, n_pages: int | None = None,
                  layer_devices: list | None = None, layer_shapes: list | None = None):
         """``layer_shapes``: per layer (key heads, key size, value heads, value size) where they differ from
-        ``kv_heads`` x ``head_dim`` for both."""
+        ``kv_heads`` x ``head_dim`` for both, and as a fifth number the rows of a page where they are not its
+        positions (what a page keeps beside its tokens)."""
         if layer_shapes is None:
             layer_shapes = [(kv_heads, head_dim, kv_heads, head_dim)] * n_layers
         self.slots, self.max_len, self.scratch = slots, max_len, slots
@@ -106,10 +107,10 @@ class KVCache:
             self.n_pages = 0
             rows, per = slots + 1, max_len
             self.tables = {}
-        self.k = [torch.zeros((rows, kh, per, kd), device=d, dtype=dtype)
-                  for d, (kh, kd, _, _) in zip(self.layer_devices, layer_shapes)]
-        self.v = [torch.zeros((rows, vh, per, vd), device=d, dtype=dtype)
-                  for d, (_, _, vh, vd) in zip(self.layer_devices, layer_shapes)]
+        self.k = [torch.zeros((rows, kh, n[0] if n else per, kd), device=d, dtype=dtype)
+                  for d, (kh, kd, _, _, *n) in zip(self.layer_devices, layer_shapes)]
+        self.v = [torch.zeros((rows, vh, n[0] if n else per, vd), device=d, dtype=dtype)
+                  for d, (_, _, vh, vd, *n) in zip(self.layer_devices, layer_shapes)]
 
     def nbytes(self) -> int:
         return sum(t.numel() * t.element_size() for t in self.k + self.v)

@@ -16,7 +16,7 @@ import os
 
 
 SUPPORTED_MODEL_TYPES = ("gpt2", "gpt_neo", "gptj", "gpt_neox", "bloom", "xglm")
-SUPPORTED_ARCHITECTURES = ("Megusun", "Rezusun", "Begopel")  # native designs (models.registry), config.json "architecture"
+SUPPORTED_ARCHITECTURES = ("Megusun", "Rezusun", "Begopel", "Gibipel")  # native designs (models.registry), config.json "architecture"
 
 
 class UnsupportedModel(ValueError):

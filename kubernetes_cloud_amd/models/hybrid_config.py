@@ -353,6 +353,108 @@ class SideBySideSpec:
 
 
 @dataclasses.dataclass(frozen=True)
+class PooledAttentionSpec:
+    """Rotated sliding-window attention that sees the whole blocks of ``pool`` tokens before its ``window`` as their
+    means: biased projections, queries and keys RMS-normed over all heads at once, a learned sink per head.
+    ``rot_scaling``: (factor, low, high, original) of the three-band frequency scaling, or None."""
+    heads: int
+    kv_heads: int
+    dim: int
+    vdim: int
+    scale: float
+    window: int
+    pool: int
+    rot_base: float
+    rot_dims: int               # leading dims of a head that rotate, in pairs half of them apart
+    rot_scaling: tuple | None = None
+
+    def __post_init__(self):
+        if self.heads % self.kv_heads:
+            raise ValueError(f"{self.heads} query heads over {self.kv_heads} key/value heads")
+        if self.rot_dims % 2 or not 0 <= self.rot_dims <= self.dim:
+            raise ValueError(f"{self.rot_dims} of {self.dim} dimensions rotate in pairs")
+        if self.window < 1 or self.pool < 1:
+            raise ValueError(f"a window of {self.window} tokens, blocks of {self.pool}")
+
+    @property
+    def _sizes(self) -> dict:
+        return {"q": self.heads * self.dim, "k": self.kv_heads * self.dim, "v": self.kv_heads * self.vdim}
+
+    @property
+    def parts(self) -> dict:
+        return aligned_parts(self._sizes)[0]
+
+    @property
+    def in_rows(self) -> int:
+        return aligned_parts(self._sizes)[1]
+
+    @property
+    def out_cols(self) -> int:
+        return self.heads * self.vdim
+
+    @property
+    def extra(self) -> dict:
+        return {"q_norm": (self.heads * self.dim,), "k_norm": (self.kv_heads * self.dim,), "sink": (self.heads,)}
+
+
+@dataclasses.dataclass(frozen=True)
+class MatrixMemorySpec:
+    """Matrix memory with exponential gates (mLSTM): soft-capped log gates, a normaliser and a running maximum beside the
+    state, read-outs normed per head and gated."""
+    heads: int
+    dim: int
+    vdim: int
+    gate_cap: float
+
+    @property
+    def _sizes(self) -> dict:
+        n, e = self.heads * self.dim, self.heads * self.vdim
+        return {"q": n, "k": n, "v": e, "g": e, "i": self.heads, "f": self.heads}
+
+    @property
+    def parts(self) -> dict:
+        return aligned_parts(self._sizes)[0]
+
+    @property
+    def in_rows(self) -> int:
+        return aligned_parts(self._sizes)[1]
+
+    @property
+    def out_cols(self) -> int:
+        return self.heads * self.vdim
+
+    @property
+    def extra(self) -> dict:
+        return {"i_bias": (self.heads,), "f_bias": (self.heads,), "gain": (self.heads * self.vdim,)}
+
+
+@dataclasses.dataclass(frozen=True)
+class SumSpec:
+    """Two mixers of the same input behind one input and one output projection: each side's rows are weighted, then
+    both close in one product."""
+    left: PooledAttentionSpec | MatrixMemorySpec
+    right: PooledAttentionSpec | MatrixMemorySpec
+    left_mul: float = 1.0
+    right_mul: float = 1.0
+
+    @property
+    def in_rows(self) -> int:
+        return self.left.in_rows + self.right.in_rows
+
+    @property
+    def out_parts(self) -> dict:
+        return aligned_parts({"left": self.left.out_cols, "right": self.right.out_cols})[0]
+
+    @property
+    def out_cols(self) -> int:
+        return aligned_parts({"left": self.left.out_cols, "right": self.right.out_cols})[1]
+
+    @property
+    def extra(self) -> dict:
+        return {f"{s}.{k}": v for s in ("left", "right") for k, v in getattr(self, s).extra.items()}
+
+
+@dataclasses.dataclass(frozen=True)
 class DenseSpec:
     """W_down act(W_up h); ``act``: "gelu" (exact) or "relu2" (squared ReLU)."""
     ff: int
@@ -367,21 +469,40 @@ class GatedDenseSpec:
 
 @dataclasses.dataclass(frozen=True)
 class MoESpec:
+    """Routed gated experts. ``score`` "sigmoid": the largest scores are the weights; "softmax": the largest scores plus
+    ``correction`` within the ``keep`` best of ``groups`` equal groups, weighted by the scores over their sum.
+    ``identity``: router outputs behind the experts' whose choice passes the token on."""
     experts: int
     top: int
     ff: int
-    shared_ff: int = 0          # always-on expert behind a per-token gate (0: none)
+    shared_ff: int = 0          # always-on expert (0: none)
     scale_in: bool = True       # the router weight scales the expert's input (False: its output)
+    shared_gate: bool = True    # ... behind a per-token gate
+    score: str = "sigmoid"
+    identity: int = 0
+    groups: int = 1
+    keep: int = 1
+    correction: bool = False
 
     def __post_init__(self):
-        if not 1 <= self.top <= self.experts:
-            raise ValueError(f"top {self.top} of {self.experts} experts")
+        n = self.outputs
+        if n % self.groups or not 1 <= self.keep <= self.groups:
+            raise ValueError(f"{self.keep} of {self.groups} groups of {n} router outputs")
+        if not 1 <= self.top <= n // self.groups * self.keep:
+            raise ValueError(f"top {self.top} of {n // self.groups * self.keep} experts")
+        if self.score == "sigmoid" and (self.identity or self.groups > 1 or self.correction):
+            raise ValueError("identity experts, groups and corrections belong to softmax routers")
+
+    @property
+    def outputs(self) -> int:
+        """Rows of the router."""
+        return self.experts + self.identity
 
 
 @dataclasses.dataclass(frozen=True)
 class LayerSpec:
     mixer: (DiffAttentionSpec | GatedRecurrenceSpec | LatentAttentionSpec | GeneralDeltaSpec | ChannelDeltaSpec |
-            BiasedAttentionSpec | HeadDeltaSpec | SsdSpec | SideBySideSpec)
+            BiasedAttentionSpec | HeadDeltaSpec | SsdSpec | SideBySideSpec | PooledAttentionSpec | MatrixMemorySpec | SumSpec)
     mlp: DenseSpec | GatedDenseSpec | MoESpec | None
 
 
@@ -405,9 +526,10 @@ class HybridConfig:
     norm_eps: float = 1e-5
     residual_mult: float = 1.0
     # one norm feeds mixer and feed-forward | "sandwich": in turn, normed before and after | "prenorm": in turn,
-    # RMS-normed before, gains stored around zero
+    # RMS-normed before, gains stored around zero | "postnorm": in turn, RMS-normed after, gains of one number
     block: str = "parallel"
     embed_scale: float = 1.0
+    logit_scale: float = 1.0
     tied: bool = False           # the embedding table is the output projection
     logit_softcap: float = 0.0   # cap tanh(logits / cap); 0: none
     loop: LoopSpec | None = None
@@ -451,24 +573,28 @@ class HybridConfig:
                 n *= x
             return n
 
-        d, pre = self.hidden, self.block == "prenorm"
-        n = (1 if self.tied else 2) * self.vocab_size * d + (1 if self.block == "parallel" else d)
+        d, pre, post = self.hidden, self.block == "prenorm", self.block == "postnorm"
+        scalar = self.block in ("parallel", "postnorm")  # norms with one number
+        n = (1 if self.tied else 2) * self.vocab_size * d + (1 if scalar else d)
         if self.loop is not None and self.loop.entry:
             n += (2 * d + self.loop.times) * d
         for L in self.layers:
             n += (L.mixer.in_rows + L.mixer.out_cols) * d + sum(numel(s) for s in L.mixer.extra.values())
             n += 2 * d if isinstance(L.mixer, SideBySideSpec) else 0
-            n += 1 + d if self.block == "parallel" else d if pre else 3 * d
+            n += 1 + L.mixer.in_rows if post else 1 + d if scalar else d if pre else 3 * d
             if isinstance(L.mlp, DenseSpec):
                 n += 2 * d * L.mlp.ff + (d if pre else 0)
             elif isinstance(L.mlp, GatedDenseSpec):
                 n += 3 * d * L.mlp.ff + 2 * L.mlp.ff + 4 * d
             elif L.mlp is not None:
-                n += d * (L.mlp.experts + 3 * L.mlp.experts * L.mlp.ff)
-                n += d * (3 * L.mlp.shared_ff + 1) if L.mlp.shared_ff else 0
+                m = L.mlp
+                n += d * (m.outputs + 3 * m.experts * m.ff + 3 * m.shared_ff) + (m.outputs if m.correction else 0)
+                n += d if m.shared_ff and m.shared_gate else 0
+                n += 1 if post else 0
         return n
 
 
 __all__ = ["HybridConfig", "LayerSpec", "LoopSpec", "DiffAttentionSpec", "GatedRecurrenceSpec", "LatentAttentionSpec",
            "GeneralDeltaSpec", "ChannelDeltaSpec", "BiasedAttentionSpec", "HeadDeltaSpec", "SsdSpec", "SideBySideSpec",
+           "PooledAttentionSpec", "MatrixMemorySpec", "SumSpec",
            "DenseSpec", "GatedDenseSpec", "MoESpec", "aligned_parts"]

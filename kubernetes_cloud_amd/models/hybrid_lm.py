@@ -1,6 +1,6 @@
 """Decoders whose layers mix tokens differently (``HybridConfig``): differential, latent or biased attention, a gated
-recurrence, a delta rule, a state space, or two of them side by side, beside a dense, gated, routed or no
-feed-forward, on an fp32 residual stream.
+recurrence, a delta rule, a state space, windowed attention over block means, a matrix memory, or two of them side by
+side, beside a dense, gated, routed or no feed-forward, on an fp32 residual stream.
 
 ``block`` "parallel": with h the normed stream and hs its token-shifted copy,
 
@@ -15,6 +15,10 @@ normed after their own output projections and averaged,
 
     x <- x + mixer(N(x))   |   x + mul (N(left(N(x))) + N(right(N(x)))),      x <- x + ff(N(x))
 
+"postnorm": the same two sublayers on the stream itself, what they add RMS-normed with a gain of one number,
+
+    x <- x + N(mixer(x)),   x <- x + N(ff(x))
+
 The modules hold weights laid out for the kernels; the step itself (cache, state, batching) is
 ``engine.hybrid_runner``. Layout:
 
@@ -22,7 +26,9 @@ The modules hold weights laid out for the kernels; the step itself (cache, state
   blocks start at multiples of 8 rows)
 * ``w_out``  the mixer's output projection; parallel layers put the dense (or shared-expert) down projection
   beside it, [d, mixer + ff]: both branches close in one product, summed in fp32 before its rounding
-* two mixers side by side: one ``w_in`` for both; ``left`` / ``right`` hold the rest of each
+* two mixers side by side: one ``w_in`` for both; ``left`` / ``right`` hold the rest of each. Summed ones share
+  ``w_out`` too, [d, left | right]
+* ``b_in``   biases of the input projections (zero rows where there is none)
 * ``w_up``   gate and up projections of a gated feed-forward, one above the other
 * experts stacked: gate-and-up [E, 2F, d], down [E, d, F]
 """
@@ -31,22 +37,24 @@ from __future__ import annotations
 import torch
 import torch.nn as nn
 
-from .hybrid_config import DenseSpec, GatedDenseSpec, HybridConfig, LayerSpec, MoESpec, SideBySideSpec
+from .hybrid_config import DenseSpec, GatedDenseSpec, HybridConfig, LayerSpec, MoESpec, SideBySideSpec, SumSpec
 
 
 def _p(*shape):
-    return nn.Parameter(torch.empty(*shape), requires_grad=False)
+    return nn.Parameter(torch.empty(shape), requires_grad=False)
 
 
 class SideMixer(nn.Module):
-    """One of two mixers side by side: its parameters behind the layer's common input projection."""
+    """One of two mixers side by side: its parameters behind the layer's common input projection (``closes``: with an
+    output projection and norm of its own)."""
 
-    def __init__(self, d: int, mixer):
+    def __init__(self, d: int, mixer, closes: bool = True):
         super().__init__()
         self.spec = LayerSpec(mixer, None)
         for name, shape in mixer.extra.items():
             setattr(self, name, _p(*shape))
-        self.w_out, self.out_norm = _p(d, mixer.out_cols), _p(d)
+        if closes:
+            self.w_out, self.out_norm = _p(d, mixer.out_cols), _p(d)
 
 
 class HybridLayer(nn.Module):
@@ -58,9 +66,26 @@ class HybridLayer(nn.Module):
         pair = isinstance(mx, SideBySideSpec)
         if pair and cfg.block != "prenorm":
             raise ValueError(f"mixers side by side belong to prenorm layers, not {cfg.block}")
-        for name, shape in ({} if pair else mx.extra).items():
+        summed = isinstance(mx, SumSpec)
+        if summed and cfg.block != "postnorm":
+            raise ValueError(f"summed mixers belong to postnorm layers, not {cfg.block}")
+        for name, shape in ({} if pair or summed else mx.extra).items():
             setattr(self, name, _p(*shape))
+        if summed:
+            self.left, self.right = SideMixer(d, mx.left, False), SideMixer(d, mx.right, False)
         self.moe = isinstance(mlp, MoESpec)
+        if cfg.block == "postnorm":
+            if mlp is not None and (not self.moe or (mlp.shared_ff and mlp.shared_gate)):
+                raise ValueError("postnorm layers take routed experts, without a gate on the shared one, or no feed-forward")
+            self.b_in, self.norm = _p(mx.in_rows), _p()
+            self.w_out = _p(d, mx.out_cols)
+            if mlp is not None:
+                self.norm2, self.router = _p(), _p(mlp.outputs, d)
+                self.correction = _p(mlp.outputs) if mlp.correction else None
+                self.gate_up, self.down = _p(mlp.experts, 2 * mlp.ff, d), _p(mlp.experts, d, mlp.ff)
+                if mlp.shared_ff:
+                    self.w_up, self.w_down = _p(2 * mlp.shared_ff, d), _p(d, mlp.shared_ff)
+            return
         if cfg.block == "prenorm":
             if mlp is not None and not isinstance(mlp, DenseSpec):
                 raise ValueError(f"prenorm layers take a dense feed-forward or none, not {type(mlp).__name__}")
@@ -82,9 +107,11 @@ class HybridLayer(nn.Module):
                 self.w_up, self.b_up = _p(2 * mlp.ff, d), _p(2 * mlp.ff)
                 self.w_down, self.b_down = _p(d, mlp.ff), _p(d)
             return
+        if self.moe and (mlp.score != "sigmoid" or (mlp.shared_ff and not mlp.shared_gate)):
+            raise ValueError("parallel layers take sigmoid routers and a gated shared expert")
         if isinstance(mlp, GatedDenseSpec):
             raise ValueError("parallel layers take a dense or routed feed-forward, not a gated one")
-        self.norm = nn.Parameter(torch.empty(()), requires_grad=False)
+        self.norm = _p()
         self.shift = _p(d)
         self.ff_cols = mlp.ff if isinstance(mlp, DenseSpec) else mlp.shared_ff if self.moe else 0
         self.w_up = _p((2 if self.moe else 1) * self.ff_cols, d) if self.ff_cols else None
@@ -108,7 +135,7 @@ class HybridLM(nn.Module):
         self.cfg = cfg
         self.wte = _p(cfg.vocab_size, cfg.hidden)
         self.layers = nn.ModuleList([HybridLayer(cfg, s) for s in cfg.layers])
-        self.final_norm = _p(cfg.hidden) if cfg.block != "parallel" else nn.Parameter(torch.empty(()), requires_grad=False)
+        self.final_norm = _p() if cfg.block in ("parallel", "postnorm") else _p(cfg.hidden)
         self.head = None if cfg.tied else _p(cfg.vocab_size, cfg.hidden)
         if cfg.loop is not None and cfg.loop.entry:
             if cfg.block != "prenorm":

@@ -60,6 +60,17 @@ def _begopel() -> Family:
                   begopel.with_shapes)
 
 
+def _gibipel() -> Family:
+    from . import gibipel
+    from .hybrid_lm import build_hybrid
+
+    def runner():
+        from ..engine.hybrid_runner import HybridRunner
+        return HybridRunner
+    return Family("gibipel", gibipel.read_config, build_hybrid, gibipel.to_native, gibipel.from_native, runner,
+                  ("norm_residual", "pooled_attn", "matrix_memory", "moe", "act_rows", "gemv", "skinny_mfma"))
+
+
 def _causal_lm() -> Family:
     from .causal_lm import build_causal_lm
     from .config import LMConfig
@@ -71,7 +82,7 @@ def _causal_lm() -> Family:
     return Family("causal_lm", LMConfig.read_hf, build_causal_lm, hf_to_native, native_to_hf, runner)
 
 
-FAMILIES = {"Megusun": _megusun, "Rezusun": _rezusun, "Begopel": _begopel}   # config.json "architecture" -> family
+FAMILIES = {"Megusun": _megusun, "Rezusun": _rezusun, "Begopel": _begopel, "Gibipel": _gibipel}   # config.json "architecture" -> family
 
 
 def family_of_dict(cfg: dict) -> Family:

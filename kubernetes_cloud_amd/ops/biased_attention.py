@@ -28,7 +28,10 @@ class _Args(ctypes.Structure):
                 ("k_sp", _LL), ("v_sp", _LL), ("table", _P), ("tstride", _I), ("shift", _I), ("pos", _P), ("slot", _P),
                 ("out", _P), ("ldo", _LL), ("H", _I), ("G", _I), ("dim", _I), ("vdim", _I), ("scale", _F), ("eps", _F),
                 ("qn", _P), ("kn", _P), ("bias", _P), ("nb", _I), ("sink", _P), ("append", _I), ("nsplit", _I),
-                ("chunk", _I), ("ws", _P), ("cnt", _P), ("tiles", _P), ("row_of", _P)]
+                ("chunk", _I), ("ws", _P), ("cnt", _P), ("tiles", _P), ("row_of", _P),
+                # windowed attention over block means (ops/pooled_attention.py)
+                ("window", _I), ("pool", _I), ("per", _I), ("pool_mul", ctypes.c_uint), ("kb", _P), ("vb", _P),
+                ("kb_sp", _LL), ("vb_sp", _LL), ("freq", _P), ("rot", _I), ("mul", _F)]
 
 
 @dataclasses.dataclass(frozen=True)
@@ -114,7 +117,7 @@ def _args(sp: BiasedHeads, wt: BiasedWeights, x, k_pages, v_pages, table, pos, s
 
 def _call(name, a, *args):
     fn = getattr(_lib.require(), name)
-    kinds = [ctypes.c_longlong if i in (2, 3) and name == "kca_biased_rows" else ctypes.c_int for i in range(len(args))]
+    kinds = [ctypes.c_longlong if i in (2, 3) and name.endswith("_rows") else ctypes.c_int for i in range(len(args))]
     fn.argtypes, fn.restype = [ctypes.c_void_p, *kinds, ctypes.c_void_p], ctypes.c_int
     _lib.call(name, ctypes.addressof(a), *args, _lib.stream())
 

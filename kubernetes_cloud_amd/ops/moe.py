@@ -1,5 +1,5 @@
-"""Mixture of gated experts (``csrc/kernels/moe.hip``): sigmoid top-k router, grouping by expert, expert
-products with the router weight on the expert's input (or output), and the strided feed-forward
+"""Mixture of gated experts (``csrc/kernels/moe.hip``): top-k router (sigmoid scores, or softmax scores with a correction
+of the choice, expert groups and identity experts), grouping by expert, expert products with the router weight on the expert's input (or output), and the strided feed-forward
 activations (``csrc/kernels/act_rows.hip``).
 
 Expert weights are stacked: gate-and-up [E, 2F, d] (gate rows first), down [E, d, F].
@@ -17,30 +17,62 @@ from .rms_shift import native_dt
 GEMM_ROWS = 128
 
 
-def route(h: torch.Tensor, router: torch.Tensor, top: int, shared_gate: torch.Tensor | None = None):
+@dataclasses.dataclass(frozen=True)
+class Router:
+    """How scores become choices. sigmoid: the ``top`` largest scores, which are the weights. softmax: the largest
+    scores + ``correction`` (fp32 [outputs]) within the ``keep`` of ``groups`` equal groups of neighbours whose best one is
+    largest; the weights are the scores over their sum. The last ``identity`` router outputs have no expert: they
+    pass the token on."""
+    softmax: bool = False
+    correction: torch.Tensor | None = None
+    groups: int = 1
+    keep: int = 1
+    identity: int = 0
+
+
+SIGMOID = Router()
+
+
+def route(h: torch.Tensor, router: torch.Tensor, top: int, shared_gate: torch.Tensor | None = None,
+          rule: Router = SIGMOID):
     """h [T, d] -> (ids int32 [T, top], weights fp32 [T, top], sigmoid of the shared expert's gate [T] | None)."""
     code = native_dt(h, router, shared_gate)
     T, d = h.shape
     E = router.shape[0]
     if code is None:
-        s = torch.sigmoid(h.float() @ router.float().t())
-        w, ids = s.topk(top, dim=-1)
+        z = h.float() @ router.float().t()
         sg = torch.sigmoid(h.float() @ shared_gate.float().reshape(-1)) if shared_gate is not None else None
+        if rule.softmax:
+            s = torch.softmax(z, -1)
+            c = s if rule.correction is None else s + rule.correction
+            best = c.view(T, rule.groups, -1).amax(-1)
+            kept = torch.zeros_like(best, dtype=torch.bool).scatter_(1, best.topk(rule.keep, dim=-1).indices, True)
+            ids = c.masked_fill(~kept.repeat_interleave(E // rule.groups, 1), -torch.inf).topk(top, dim=-1).indices
+            w = s.gather(1, ids)
+            w = w / (w.sum(-1, keepdim=True) + 1e-20)
+        else:
+            w, ids = torch.sigmoid(z).topk(top, dim=-1)
         return ids.to(torch.int32), w, sg
     assert h.is_contiguous() and router.is_contiguous() and router.shape[1] == d
     ids = torch.empty(T, top, device=h.device, dtype=torch.int32)
     w = torch.empty(T, top, device=h.device, dtype=torch.float32)
     sg = torch.empty(T, device=h.device, dtype=torch.float32) if shared_gate is not None else None
     _lib.call("kca_moe_route", code, h.data_ptr(), router.data_ptr(), _lib.ptr(shared_gate), ids.data_ptr(),
-              w.data_ptr(), _lib.ptr(sg), T, d, E, top, _lib.stream())
+              w.data_ptr(), _lib.ptr(sg), T, d, E, top, *_rule_args(rule, E), _lib.stream())
     return ids, w, sg
+
+
+def _rule_args(rule: Router, E: int) -> tuple:
+    c = rule.correction
+    assert c is None or (c.is_contiguous() and c.dtype == torch.float32 and c.numel() == E and rule.softmax)
+    return int(rule.softmax), _lib.ptr(c), rule.groups, rule.keep
 
 
 @dataclasses.dataclass
 class Groups:
     """Assignments sorted by expert, in tiles of at most ``mt`` rows of one expert."""
     perm: torch.Tensor
-    inv: torch.Tensor     # [T, top]
+    inv: torch.Tensor     # [T, top]; -1: an identity expert
     tiles: torch.Tensor
     ntiles: torch.Tensor
     mt: int
@@ -62,33 +94,39 @@ def _groups(T: int, top: int, E: int, mt: int, device) -> Groups:
                   torch.empty(1, **z), mt)
 
 
-def route_group(h: torch.Tensor, router: torch.Tensor, top: int, shared_gate: torch.Tensor | None, mt: int):
+def route_group(h: torch.Tensor, router: torch.Tensor, top: int, shared_gate: torch.Tensor | None, mt: int,
+                rule: Router = SIGMOID):
     """``route`` and ``group`` -> (ids, weights, shared gate, groups); one launch for up to 16 bf16 tokens."""
     T, d = h.shape
     E = router.shape[0]
-    if native_dt(h, router, shared_gate) == 1 and T <= 16 and top <= 64 and d % 8 == 0:
-        g = _groups(T, top, E, mt, h.device)
+    real = E - rule.identity
+    if native_dt(h, router, shared_gate) == 1 and T <= 16 and top <= 64 and d % 8 == 0 and (not rule.softmax or E <= 384):
+        g = _groups(T, top, real, mt, h.device)
         ids = torch.empty(T, top, device=h.device, dtype=torch.int32)
         w = torch.empty(T, top, device=h.device, dtype=torch.float32)
         sg = torch.empty(T, device=h.device, dtype=torch.float32) if shared_gate is not None else None
         assert h.is_contiguous() and router.is_contiguous() and router.shape[1] == d
         _lib.call("kca_moe_route_group", h.data_ptr(), router.data_ptr(), _lib.ptr(shared_gate), ids.data_ptr(),
-                  w.data_ptr(), _lib.ptr(sg), T, d, E, top, mt, g.perm.data_ptr(), g.inv.data_ptr(),
+                  w.data_ptr(), _lib.ptr(sg), T, d, E, real, top, *_rule_args(rule, E), mt, g.perm.data_ptr(), g.inv.data_ptr(),
                   g.tiles.data_ptr(), g.tiles.shape[0], g.ntiles.data_ptr(), _lib.stream())
         return ids, w, sg, g
-    ids, w, sg = route(h, router, top, shared_gate)
-    return ids, w, sg, group(ids, E, mt)
+    ids, w, sg = route(h, router, top, shared_gate, rule)
+    return ids, w, sg, group(ids, real, mt)
 
 
 def group(ids: torch.Tensor, E: int, mt: int) -> Groups:
+    """Ids of ``E`` and beyond (identity experts) take no row."""
     T, top = ids.shape
     n = T * top
     g = _groups(T, top, E, mt, ids.device)
     mx = g.tiles.shape[0]
     if not ids.is_cuda:
-        order = torch.argsort(ids.reshape(-1), stable=True)
+        flat = ids.reshape(-1)
+        real = int((flat < E).sum())
+        order = torch.argsort(flat, stable=True)
         g.perm.copy_(order)
-        g.inv.view(-1)[order] = torch.arange(n, dtype=torch.int32)
+        g.inv.view(-1)[order] = torch.where(torch.arange(n) < real, torch.arange(n), -1).to(torch.int32)
+        g.perm[real:] = -1
         return g
     _lib.call("kca_moe_group", ids.data_ptr(), n, E, mt, g.perm.data_ptr(), g.inv.data_ptr(), g.tiles.data_ptr(), mx,
               g.ntiles.data_ptr(), _lib.stream())
@@ -105,6 +143,8 @@ def experts(h: torch.Tensor, ids: torch.Tensor, weights: torch.Tensor, gate_up: 
         flat, wt = ids.reshape(-1).long(), weights.reshape(-1)
         y = torch.empty(n, d, dtype=h.dtype)
         for pos, a in enumerate(g.perm.tolist()):
+            if a < 0:
+                break
             x, e = h[a // top].float(), int(flat[a])
             s_in, s_out = (float(wt[a]), 1.0) if scale_in else (1.0, float(wt[a]))
             u = gate_up[e].float() @ (x * s_in)
@@ -152,4 +192,4 @@ def act_rows(x: torch.Tensor, out: torch.Tensor, gated: bool, row_scale: torch.T
     return out
 
 
-__all__ = ["route", "group", "route_group", "experts", "act_rows", "tile_rows", "Groups"]
+__all__ = ["Router", "SIGMOID", "route", "group", "route_group", "experts", "act_rows", "tile_rows", "Groups"]

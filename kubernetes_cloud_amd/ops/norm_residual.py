@@ -8,6 +8,11 @@ as it is, or the weighted sum of two normed ones, and norm with a gain stored ar
 
     x_t = src_t + a_t   |   src_t + mul * (N(a_t; ga) + N(b_t; gb)),      h_t = N(x_t; 1 + g)
 
+Post-norm layers (``postnorm``, RMS, gains of one number) norm what a sublayer adds -- the sum of its rows, of routed
+experts' rows and of the stream itself where an identity expert was chosen -- and hand the stream on as it is:
+
+    x_t = src_t + ga N(a_t + sum_k y[inv[t, k]] + (sum of the weights of identity experts) src_t),      h_t = x_t
+
 bf16 and fp32 GPU tensors run the kernels; CPU tensors run the references below.
 """
 from __future__ import annotations
@@ -18,7 +23,7 @@ import dataclasses
 import torch
 
 from . import _lib
-from .rms_shift import native_dt
+from .rms_shift import DT, native_dt
 
 
 @dataclasses.dataclass
@@ -153,10 +158,78 @@ def prenorm(src: torch.Tensor | Embedded | Rows, branch: torch.Tensor | NormedPa
     return x_out, h
 
 
+@dataclasses.dataclass
+class NormedSum:
+    """What a sublayer adds before its norm: ``a`` [T, d] and / or routed rows ``y`` [n, d] through ``inv`` [T, top]
+    (-1: the stream itself, times its weight in ``wts``)."""
+    gain: torch.Tensor
+    a: torch.Tensor | None = None
+    y: torch.Tensor | None = None
+    inv: torch.Tensor | None = None
+    wts: torch.Tensor | None = None
+
+
+class _PostArgs(ctypes.Structure):
+    _P, _LL, _F, _I = ctypes.c_void_p, ctypes.c_longlong, ctypes.c_float, ctypes.c_int
+    _fields_ = [("x_in", _P), ("embed", _P), ("tokens", _P), ("escale", _F), ("a", _P), ("lda", _LL), ("y", _P), ("inv", _P),
+                ("wts", _P), ("top", _I), ("ga", _P), ("g", _P), ("hmul", _F), ("eps", _F), ("rows", _P), ("x_out", _P),
+                ("h", _P), ("T", _I), ("d", _I)]
+
+
+def postnorm(src: torch.Tensor | Embedded, branch: NormedSum | None, eps: float, dtype, *, gain: torch.Tensor | None = None,
+             mul: float = 1.0, rows: torch.Tensor | None = None, keep_x: bool = True):
+    """-> (x_out fp32 | None, h of ``dtype``). ``src``: the fp32 stream, or where it starts. h: the stream rounded, or with
+    ``gain`` (one number) its RMS norm times ``mul``. ``rows``: only these tokens."""
+    emb = isinstance(src, Embedded)
+    data = src.table if emb else src
+    n_src, d = (src.tokens if emb else data).shape[0], data.shape[1]
+    T = rows.shape[0] if rows is not None else n_src
+    br = branch or NormedSum(None)
+    assert all(t is None or t.dtype == dtype for t in (br.gain, gain, br.a, br.y, data if emb else None))
+    if not data.is_cuda:
+        x = src.table[src.tokens].float() * src.scale if emb else src
+        if branch is not None:
+            u = torch.zeros_like(x) if br.a is None else br.a.float()
+            if br.y is not None:
+                inv = br.inv.long()
+                u = u + br.y[inv.clamp(min=0)].float().masked_fill((inv < 0)[..., None], 0.0).sum(1)
+                u = u + (br.wts * (inv < 0)).sum(1, keepdim=True) * x
+            x = x + _norm(u, br.gain, eps, False)
+        if rows is not None:
+            x = x[rows.long()]
+        return (x if keep_x else None), (x if gain is None else _norm(x, gain, eps, False) * mul).to(dtype)
+    assert data.is_contiguous() and (data.dtype == torch.float32 or emb) and (not emb or src.tokens.dtype == torch.int64)
+    assert all(t is None or t.numel() == 1 for t in (br.gain, gain))
+    assert br.a is None or (br.a.stride(1) == 1 and br.a.shape == (n_src, d))
+    assert br.y is None or (br.y.is_contiguous() and br.y.shape[1] == d and br.inv.is_contiguous() and br.wts.is_contiguous()
+                            and br.inv.shape == br.wts.shape and br.inv.shape[0] == n_src and br.inv.dtype == torch.int32
+                            and br.wts.dtype == torch.float32)
+    assert rows is None or rows.dtype == torch.int32
+    if _lib.require().kca_postnorm_abi() != ctypes.sizeof(_PostArgs):
+        raise RuntimeError("kca_postnorm descriptor: C and ctypes sizes differ")
+    same = dtype == torch.float32 and gain is None  # the stream is already what the next product reads
+    x_out = torch.empty(T, d, device=data.device, dtype=torch.float32) if keep_x or same else None
+    h = None if same else torch.empty(T, d, device=data.device, dtype=dtype)
+    p, k = _lib.ptr, _PostArgs()
+    if emb:
+        k.embed, k.tokens, k.escale = data.data_ptr(), src.tokens.data_ptr(), src.scale
+    else:
+        k.x_in = data.data_ptr()
+    if br.a is not None:
+        k.a, k.lda = br.a.data_ptr(), br.a.stride(0)
+    if br.y is not None:
+        k.y, k.inv, k.wts, k.top = br.y.data_ptr(), br.inv.data_ptr(), br.wts.data_ptr(), br.inv.shape[1]
+    k.ga, k.g, k.hmul, k.eps, k.rows, k.x_out, k.h, k.T, k.d = (p(br.gain), p(gain), mul, eps, p(rows), p(x_out), p(h), T, d)
+    fn = _lib.require().kca_postnorm
+    fn.argtypes, fn.restype = [ctypes.c_void_p, ctypes.c_int, ctypes.c_void_p], ctypes.c_int
+    _lib.call("kca_postnorm", ctypes.addressof(k), DT[dtype], _lib.stream())
+    return x_out, (x_out if same else h)
+
+
 def _norm(x, gain, eps, layer):
     if layer:
         x = x - x.mean(-1, keepdim=True)
     return x * torch.rsqrt((x * x).mean(-1, keepdim=True) + eps) * gain.float()
 
 
-__all__ = ["Embedded", "NormedBranch", "NormedPair", "Rows", "norm_residual", "prenorm"]
+__all__ = ["Embedded", "NormedBranch", "NormedPair", "NormedSum", "Rows", "norm_residual", "postnorm", "prenorm"]
