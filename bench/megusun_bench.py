@@ -118,8 +118,13 @@ def _time(fns, reps=5):
     for f in fns:  # (on the stream that filled the operands)
         f()
     torch.cuda.synchronize()
+    s = torch.cuda.Stream()
+    with torch.cuda.stream(s):  # what the ops keep per stream
+        for f in fns:
+            f()
+    torch.cuda.synchronize()
     g = torch.cuda.CUDAGraph()
-    with torch.cuda.graph(g):
+    with torch.cuda.graph(g, stream=s):
         for f in fns:
             f()
     g.replay()

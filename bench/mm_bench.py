@@ -36,7 +36,7 @@ def _time_graph(fn, reps=20, iters=10):
             fn(i)
     torch.cuda.current_stream().wait_stream(s)
     g = torch.cuda.CUDAGraph()
-    with torch.cuda.graph(g):
+    with torch.cuda.graph(g, stream=s):
         for i in range(reps):
             fn(i)
     g.replay()

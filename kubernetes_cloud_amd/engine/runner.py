@@ -359,7 +359,7 @@ class StepRunner:
         on_gpu = self.device.type == "cuda"
         self.use_graphs = on_gpu if use_graphs is None else (use_graphs and on_gpu)
         self._graphs: dict = {}
-        self._pool = None
+        self._pool = self._side = None
         self._static: dict = {}
         self.step_launches: dict = {}
         self._outbufs: dict = {}
@@ -594,7 +594,11 @@ class StepRunner:
 
     def _capture(self, st, Bb, Kb, mc=False):
         saved = [t.clone() for t in self._step_state()]
-        s = torch.cuda.Stream()
+        # one stream for warm-up and capture: what the ops keep per stream (zeroed counters) exists before the capture,
+        # outside the graphs' shared pool, where another graph's replay would overwrite it
+        if self._side is None:
+            self._side = torch.cuda.Stream()
+        s = self._side
         s.wait_stream(torch.cuda.current_stream())
         with torch.cuda.stream(s):
             for _ in range(2):  # warm up (allocator, hipBLASLt heuristics)
@@ -608,7 +612,7 @@ class StepRunner:
         # thread-local capture: the RCCL process-group watchdog thread polls its work events while a
         # capture runs; under the default global mode that query fails ("operation not permitted when
         # stream is capturing") and the watchdog aborts the process
-        with torch.cuda.graph(g, pool=self._pool, capture_error_mode="thread_local"):
+        with torch.cuda.graph(g, pool=self._pool, stream=s, capture_error_mode="thread_local"):
             self._step_body(st, Bb, Kb, mc)
         self._graphs[(Bb, Kb, mc)] = g
         return g

@@ -180,6 +180,10 @@ def _workspace(device, floats: int, nblk: int):
     key = (str(device), torch.cuda.current_stream(device).cuda_stream)
     ws = _WS.get(key)
     if ws is None or ws[0].numel() < floats or ws[1].numel() < nblk:
+        if torch.cuda.is_current_stream_capturing():
+            # memory of the graph's pool: other graphs of the pool write it between replays, so it serves one launch and
+            # its counters are cleared by the graph itself (callers that warm up on the capturing stream avoid this)
+            return (torch.empty(floats, device=device, dtype=torch.float32), torch.zeros(nblk, device=device, dtype=torch.int32))
         f = max(floats, ws[0].numel() if ws else 0, 1 << 20)
         n = max(nblk, ws[1].numel() if ws else 0, 4096)
         ws = (torch.empty(f, device=device, dtype=torch.float32), torch.zeros(n, device=device, dtype=torch.int32))

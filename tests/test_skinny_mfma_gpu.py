@@ -222,3 +222,33 @@ def test_consumer_merged_row_stats(M, N, monkeypatch):
     ref = sm.mm_reference([(sm.ln_on_load_reference(outs[True][0], sm.row_stats_reference(outs[True][0], 1e-5),
                                                      gam, bet), wn, None)])
     _close(outs[True][1], ref, 1.5e-2)
+
+
+def test_split_counters_live_outside_a_graphs_pool():
+    """Two graphs of one memory pool, each with a split product and the other's intermediates over its scratch, replayed
+    in turn: every replay equals the eager product, on a stream the ops know and on one they meet in the capture."""
+    g = torch.Generator(device=DEV).manual_seed(1)
+    N, K, M = 640, 4096, 8
+    x, w = torch.randn(M, K, generator=g, device=DEV).bfloat16(), _w(N, K, torch.bfloat16, g)
+    want = sm.mm(x, w)
+    assert sm.plan([sm.job([sm.part(x, w)], N, want)], M, torch.bfloat16)[0] > 1
+    for warm in (True, False):
+        s = torch.cuda.Stream()
+        if warm:
+            with torch.cuda.stream(s):
+                sm.mm(x, w)
+        torch.cuda.synchronize()
+        known = dict(sm._WS)
+        pool, graphs, outs = torch.cuda.graph_pool_handle(), [], []
+        for i in range(3):
+            graphs.append(torch.cuda.CUDAGraph())
+            with torch.cuda.graph(graphs[-1], pool=pool, stream=s):
+                noise = [torch.full((n,), 7.0, device=DEV) for n in (64, 4096, 1 << 20)] if i != 1 else []
+                outs.append(sm.mm(x, w))
+                del noise
+        assert all(known.get(k) is v for k, v in sm._WS.items())  # nothing kept from within a capture
+        for i in (0, 1, 2, 1, 0, 2, 2, 1):
+            outs[i].zero_()
+            graphs[i].replay()
+            torch.cuda.synchronize()
+            assert torch.equal(outs[i], want), (warm, i)
