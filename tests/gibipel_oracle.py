@@ -37,13 +37,13 @@ def frequencies(rot):
     return out
 
 
-def rotate(x, pos, rot):
-    """One head's vector at a position: pairs (i, i + dims / 2) of its first dims turn."""
+def rotate(x, rot):
+    """[T, heads, D], row t at position t: pairs (i, i + dims / 2) of a head's first dims turn."""
     y, n = x.clone(), rot["dims"] // 2
+    t = torch.arange(x.shape[0], dtype=x.dtype)[:, None]
     for i, f in enumerate(frequencies(rot)):
-        c, s = math.cos(pos * f), math.sin(pos * f)
-        y[i] = x[i] * c - x[i + n] * s
-        y[i + n] = x[i + n] * c + x[i] * s
+        c, s, u, v = torch.cos(t * f), torch.sin(t * f), x[:, :, i], x[:, :, i + n]
+        y[:, :, i], y[:, :, i + n] = u * c - v * s, v * c + u * s
     return y
 
 
@@ -95,11 +95,7 @@ def attention_inputs(h, w, p, mx, eps):
     T, D = h.shape[0], mx["dim"]
     q, k, v = (h @ w[p + n].T + w[p + n + ".b"] for n in "qkv")
     q, k = rms(q, eps) * w[p + "q.norm"], rms(k, eps) * w[p + "k.norm"]
-    q, k = q.view(T, mx["heads"], D).clone(), k.view(T, mx["kv_heads"], D).clone()
-    for t in range(T):
-        for x in (q, k):
-            for a in range(x.shape[1]):
-                x[t, a] = rotate(x[t, a], t, mx["rot"])
+    q, k = rotate(q.view(T, mx["heads"], D), mx["rot"]), rotate(k.view(T, mx["kv_heads"], D), mx["rot"])
     return q, k, v.view(T, mx["kv_heads"], mx["vdim"])
 
 
@@ -220,7 +216,7 @@ def random_weights(cfg, seed=0):
     """Weights whose mechanisms all matter: query rows that pick keys out, gates on both sides of their caps,
     corrections that change the choice. bfloat16 values in float64."""
     g = torch.Generator().manual_seed(seed)
-    r = lambda *s: torch.randn(*s, generator=g)  # noqa: E731
+    r = lambda *s: torch.randn(s, generator=g)  # noqa: E731
     w = {}
     for n, s in shapes(cfg).items():
         last = n.rsplit(".", 1)[-1]
@@ -231,7 +227,7 @@ def random_weights(cfg, seed=0):
         elif last == "sink":
             t = 1 + r(*s)
         elif last == "correction":
-            t = 0.3 * r(*s)
+            t = 0.15 * r(*s)
         elif n.endswith("f.b"):
             t = 2 + 2 * r(*s)
         elif last == "b":
