@@ -45,7 +45,8 @@ the headline always prints):
 ``--megusun`` runs none of this: it prints one line with Megusun's prefill / decode throughput beside
 GPT-J of equal size and each kernel's distance from its roofline (bench/megusun_bench.py). ``--rezusun`` does
 the same for Rezusun beside Megusun and GPT-J (bench/rezusun_bench.py), ``--begopel`` for Begopel beside Rezusun and
-GPT-J (bench/begopel_bench.py).
+GPT-J (bench/begopel_bench.py), ``--gibipel`` for Gibipel beside Begopel and the routed Megusun
+(bench/gibipel_bench.py).
 
 ``KCA_BENCH_SHARED_GPU=1`` (rehearsal only, parallel/shared_gpu.py): N ranks
 share cuda:0 with gloo collectives staged through the host, so the N > 1 paths
@@ -105,6 +106,8 @@ def main():
                     help="the same for Rezusun beside Megusun and GPT-J (bench/rezusun_bench.py)")
     ap.add_argument("--begopel", choices=["models", "kernels", "all"], default=None,
                     help="the same for Begopel beside Rezusun and GPT-J (bench/begopel_bench.py)")
+    ap.add_argument("--gibipel", choices=["models", "kernels", "all"], default=None,
+                    help="the same for Gibipel beside Begopel and the routed Megusun (bench/gibipel_bench.py)")
     # rehearsal shrink flags (tests/test_bench_shared_gpu.py): NOT the BASELINE config
     ap.add_argument("--layers", type=int, default=0)
     ap.add_argument("--hidden", type=int, default=0)
@@ -123,7 +126,7 @@ def main():
               + json.dumps({"world_size": int(os.environ.get("WORLD_SIZE", "1"))}), flush=True)
         return
 
-    for design in ("megusun", "rezusun", "begopel"):
+    for design in ("megusun", "rezusun", "begopel", "gibipel"):
         what = getattr(args, design)
         if what:
             mb = _load_bench(design + "_bench")

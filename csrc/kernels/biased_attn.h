@@ -64,12 +64,6 @@ __device__ __forceinline__ int blocks_seen(const BiasedArgs& p, int pos) {
 __device__ __forceinline__ int block_row(const BiasedArgs& p, int end) {
   return (int)((unsigned)(end & ((1 << p.shift) - 1)) * p.pool_mul >> 20);
 }
-// element c of a rotated head (pairs half apart)
-__device__ __forceinline__ float rotated(const float* u, int c, int half, const float* cs, const float* sn) {
-  if (c < half) return u[c] * cs[c] - u[c + half] * sn[c];
-  if (c < 2 * half) return u[c] * cs[c - half] + u[c - half] * sn[c - half];
-  return u[c];
-}
 __host__ __device__ __forceinline__ int pool_lds(int rb, int dim, int rot) { return (rb + 1) * dim + rot; }  // floats
 
 template <typename E>
@@ -86,7 +80,7 @@ __device__ __forceinline__ float gate_of(float z) {
 constexpr int MAX_SPLITS = 256;
 
 template <typename E, int RB, int LP, bool VEC, bool POOL>
-__global__ void __launch_bounds__(256) biased_rows_kernel(BiasedArgs p) {
+__global__ void __launch_bounds__(256, sizeof(E) == 2 && LP <= 16 ? 4 : 1) biased_rows_kernel(BiasedArgs p) {
   constexpr int KT = LP >= 64 ? 4 : (LP >= 32 ? 8 : 16);  // keys per tile of a wave
   constexpr int KP = 64 / LP, NPASS = KT / KP;            // keys per pass, passes
   static_assert(KP <= KT, "a pass covers at most one tile");
@@ -120,10 +114,35 @@ __global__ void __launch_bounds__(256) biased_rows_kernel(BiasedArgs p) {
   auto mxf = [](float x, float y) { return fmaxf(x, y); };
   float q[RB][8];
   Raw8<E> kown;  // the row's own key, normed and rounded as the page holds it
+  // a tile's keys and values (POOL: the first tile's before the norms; more in flight would cost resident waves)
+  Raw8<E> kx[NPASS], vx[NPASS];
+  auto fetch = [&](int k0) {
+#pragma unroll
+    for (int n = 0; n < NPASS; ++n) {
+      const int key = min(k0 + n * KP + jj, hi - 1);
+      const bool mean = POOL && key < nbs;
+      const int at = !POOL ? key : mean ? key * p.pool + p.pool - 1 : key - nbs + first;
+      const long long pg = tbl[at >> p.shift];
+      const E *kr, *vr;
+      if (mean) {
+        const long long in = (long long)g * p.per + block_row(p, at);
+        kr = reinterpret_cast<const E*>(p.kb) + pg * p.kb_sp + in * D;
+        vr = reinterpret_cast<const E*>(p.vb) + pg * p.vb_sp + in * Vd;
+      } else {
+        const long long in = ((long long)g << p.shift) + (at & pmask);
+        kr = kc + pg * p.k_sp + in * D;
+        vr = vc + pg * p.v_sp + in * Vd;
+      }
+      if (!POOL && p.append && key == kv - 1) kx[n] = kown;
+      else ld8g<E, VEC>(kr + ll * 8, D - ll * 8, kx[n]);
+      ld8g<E, VEC>((p.append && key == kv - 1 ? vn : vr) + ll * 8, Vd - ll * 8, vx[n]);
+    }
+  };
+  if (POOL && lo + wv * KT < hi) fetch(lo + wv * KT);
   if constexpr (POOL) {
     if (p.append) {  // norms over the whole projections, this group's heads normed in LDS, then rotated
       __shared__ float red[2][4];
-      float *qs = merged + 4 * RB * Vd, *ks = qs + RB * D, *cs = ks + D, *sn = cs + p.rot / 2;
+      float *qs = merged + 4 * RB * Vd, *cs = qs + (RB + 1) * D, *sn = cs + p.rot / 2;  // heads: queries, then the key
       const E *gq = reinterpret_cast<const E*>(p.qn), *gk = reinterpret_cast<const E*>(p.kn);
       float sq = 0.f, sk = 0.f;
       const int nq = p.H * D, nk = p.G * D;
@@ -140,25 +159,57 @@ __global__ void __launch_bounds__(256) biased_rows_kernel(BiasedArgs p) {
 #pragma unroll
         for (int i = 0; i < 8; ++i) sk = fmaf(u.f(i), u.f(i), sk);
       }
-      for (int i = tid; i < p.rot / 2; i += 256) sincosf((float)pos * p.freq[i], sn + i, cs + i);
+      constexpr int MINE = ((RB + 1) * 8 * LP + 255) / 256;  // this thread's elements of the heads, and their partners
+      const int half = p.rot / 2;
+      float own[MINE], gain[MINE], other[MINE], gain2[MINE];
+#pragma unroll
+      for (int j = 0; j < MINE; ++j) {
+        const int i = min(tid + 256 * j, (RB + 1) * D - 1), r = i / D, c = i - r * D;
+        const int col = r < RB ? (h0 + min(r, nh - 1)) * D + c : g * D + c, turn = c < half ? half : c < 2 * half ? -half : 0;
+        const E *xs = xr + (r < RB ? p.o_q : p.o_k) + col, *gs = (r < RB ? gq : gk) + col;
+        own[j] = El<E>::ld(xs);
+        gain[j] = El<E>::ld(gs);
+        other[j] = El<E>::ld(xs + turn);
+        gain2[j] = El<E>::ld(gs + turn);
+      }
+      for (int i = tid; i < half; i += 256) sincosf((float)pos * p.freq[i], sn + i, cs + i);
       sq = lanes_reduce<64>(sq, add);
       sk = lanes_reduce<64>(sk, add);
       if (lane == 0) red[0][wv] = sq, red[1][wv] = sk;
       __syncthreads();
       const float rq = 1.f / sqrtf((red[0][0] + red[0][1] + red[0][2] + red[0][3]) / (float)nq + p.eps);
       const float rk = 1.f / sqrtf((red[1][0] + red[1][1] + red[1][2] + red[1][3]) / (float)nk + p.eps);
-      for (int i = tid; i < (RB + 1) * D; i += 256) {
-        const int r = i / D, c = i - r * D;
-        const int qc = (h0 + min(r, nh - 1)) * D + c, kcol = g * D + c;
-        qs[i] = r < RB ? El<E>::ld(xr + p.o_q + qc) * rq * El<E>::ld(gq + qc) : El<E>::ld(xr + p.o_k + kcol) * rk * El<E>::ld(gk + kcol);
+#pragma unroll
+      for (int j = 0; j < MINE; ++j) {
+        const int i = tid + 256 * j, r = i / D, c = i - r * D;
+        if (r > RB) break;
+        const float n = r < RB ? rq : rk;
+        float u = own[j] * n * gain[j];
+        if (c < 2 * half) {
+          const int f = c < half ? c : c - half;
+          u = u * cs[f] + (c < half ? -1.f : 1.f) * (other[j] * n * gain2[j]) * sn[f];
+        }
+        qs[i] = r < RB ? u * p.scale : u;
       }
       __syncthreads();
 #pragma unroll
-      for (int i = 0; i < 8; ++i) {
-        const int c = ll * 8 + i;
+      for (int r = 0; r <= RB; ++r) {
+        const float* u = qs + r * D + ll * 8;
+        float v[8];
+        if constexpr (VEC) {
+          const int o = ll * 8 < D ? 0 : -ll * 8;  // (past the head: in bounds, and zero)
+          load8f(u + o, v);
 #pragma unroll
-        for (int r = 0; r < RB; ++r) q[r][i] = c < D ? rotated(qs + r * D, c, p.rot / 2, cs, sn) * p.scale : 0.f;
-        El<E>::st(kown.v + i, c < D ? rotated(ks, c, p.rot / 2, cs, sn) : 0.f);
+          for (int i = 0; i < 8; ++i) v[i] = o ? 0.f : v[i];
+        } else {
+#pragma unroll
+          for (int i = 0; i < 8; ++i) v[i] = ll * 8 + i < D ? u[i] : 0.f;
+        }
+#pragma unroll
+        for (int i = 0; i < 8; ++i) {
+          if (r < RB) q[r < RB ? r : 0][i] = v[i];
+          else El<E>::st(kown.v + i, v[i]);
+        }
       }
     } else {
 #pragma unroll
@@ -206,27 +257,10 @@ __global__ void __launch_bounds__(256) biased_rows_kernel(BiasedArgs p) {
 #pragma unroll
   for (int j = 0; j < PPL; ++j) mx[j] = -INFINITY, l[j] = 0.f;
   for (int k0 = lo + wv * KT; k0 < hi; k0 += 4 * KT) {
-    Raw8<E> kx[NPASS], vx[NPASS];
+    if (!POOL || k0 > lo + wv * KT) fetch(k0);
 #pragma unroll
-    for (int n = 0; n < NPASS; ++n) {
-      const int key = min(k0 + n * KP + jj, hi - 1);
-      const bool own = p.append && key == kv - 1, mean = POOL && key < nbs;
-      const int at = !POOL ? key : mean ? key * p.pool + p.pool - 1 : key - nbs + first;
-      const long long pg = tbl[at >> p.shift];
-      const E *kr, *vr;
-      if (mean) {
-        const long long in = (long long)g * p.per + block_row(p, at);
-        kr = reinterpret_cast<const E*>(p.kb) + pg * p.kb_sp + in * D;
-        vr = reinterpret_cast<const E*>(p.vb) + pg * p.vb_sp + in * Vd;
-      } else {
-        const long long in = ((long long)g << p.shift) + (at & pmask);
-        kr = kc + pg * p.k_sp + in * D;
-        vr = vc + pg * p.v_sp + in * Vd;
-      }
-      if (own) kx[n] = kown;
-      else ld8g<E, VEC>(kr + ll * 8, D - ll * 8, kx[n]);
-      ld8g<E, VEC>((own ? vn : vr) + ll * 8, Vd - ll * 8, vx[n]);
-    }
+    for (int n = 0; n < NPASS; ++n)  // (the page does not hold the new key yet)
+      if (POOL && p.append && min(k0 + n * KP + jj, hi - 1) == kv - 1) kx[n] = kown;
     float bv[PPL];
 #pragma unroll
     for (int j = 0; j < PPL; ++j) {
@@ -455,7 +489,7 @@ __global__ void __launch_bounds__(256, DV > 128 ? 1 : 2) biased_tile_kernel(Bias
   const bf16_t* xr = reinterpret_cast<const bf16_t*>(p.x) + row * p.ld;
 
   // this thread's 16-B chunks of a tile: element offset from the tile's first row, LDS offset
-  int off[CPT], ldo[CPT], vrow[CPT], row_of[POOL ? CPT : 1];  // (POOL: the offset within the row, and the row)
+  int off[CPT], ldo[CPT], vrow[CPT], col[POOL ? CPT : 1];  // (col: within the row)
   bool on[CPT];
 #pragma unroll
   for (int i = 0; i < CPT; ++i) {
@@ -463,12 +497,12 @@ __global__ void __launch_bounds__(256, DV > 128 ? 1 : 2) biased_tile_kernel(Bias
     const bool key = c < CK;
     const int r = key ? c / (DK / 8) : cv / (DV / 8), ch = key ? c % (DK / 8) : cv % (DV / 8);
     on[i] = c < NC && ch * 8 < (key ? D : Vd);
-    off[i] = on[i] ? (POOL ? 0 : r * (key ? D : Vd)) + ch * 8 : 0;
-    if constexpr (POOL) row_of[i] = min(r, BN - 1);
+    off[i] = on[i] ? r * (key ? D : Vd) + ch * 8 : 0;
+    if constexpr (POOL) col[i] = on[i] ? ch * 8 : 0;
     ldo[i] = key ? img_off<DK>(r, ch) : TK + img_off<DV>(r, ch);
     vrow[i] = key ? -1 : r;
   }
-  struct Pages { int v[POOL ? CPT : 1]; };  // of a tile (POOL: of each chunk's row)
+  struct Pages { int pg, v[POOL ? CPT : 1]; };  // of a tile (of tokens; of block means: of each chunk's row)
   auto end_of = [&](int t, int i) {          // last position of the block in chunk i's row
     const int c = tid + 256 * i, r = c < CK ? c / (DK / 8) : min(c - CK, CV - 1) / (DV / 8);
     return min(t * BN + r, nbm - 1) * p.pool + p.pool - 1;
@@ -476,37 +510,29 @@ __global__ void __launch_bounds__(256, DV > 128 ? 1 : 2) biased_tile_kernel(Bias
   auto page = [&](int tn) {
     Pages r;
     const int t = min(tn, ntiles - 1);
-    if constexpr (POOL) {
+    if (POOL && t < nbt) {
 #pragma unroll
-      for (int i = 0; i < CPT; ++i) r.v[i] = tbl[(t < nbt ? end_of(t, i) : (t + tt0) * BN) >> p.shift];
+      for (int i = 0; i < CPT; ++i) r.v[POOL ? i : 0] = tbl[end_of(t, i) >> p.shift];
     } else {
-      r.v[0] = tbl[t * BN >> p.shift];
+      r.pg = tbl[(t + tt0) * BN >> p.shift];
     }
     return r;
   };
   auto load = [&](int tn, const Pages& pgs, u32x4 (&st)[CPT]) {  // tile t of these pages (tiles past the end: the last again)
     const int t = min(tn, ntiles - 1);
-    if constexpr (POOL) {
-      const bool mean = t < nbt;
-      const int k0 = (t + tt0) * BN, kr = k0 & ((1 << p.shift) - 1);
+    if (POOL && t < nbt) {
 #pragma unroll
       for (int i = 0; i < CPT; ++i) {
         const bool key = 256 * i + 255 < CK || (256 * i < CK && tid + 256 * i < CK);
-        const bf16_t* base;
-        if (mean) {
-          const long long in = (long long)g * p.per + block_row(p, end_of(t, i));
-          base = key ? reinterpret_cast<const bf16_t*>(p.kb) + pgs.v[i] * p.kb_sp + in * D
-                     : reinterpret_cast<const bf16_t*>(p.vb) + pgs.v[i] * p.vb_sp + in * Vd;
-        } else {
-          const long long in = ((long long)g << p.shift) + kr + row_of[i];
-          base = key ? kc + pgs.v[i] * p.k_sp + in * D : vc + pgs.v[i] * p.v_sp + in * Vd;
-        }
-        const u32x4 v = *reinterpret_cast<const u32x4*>(base + off[i]);
-        st[i] = on[i] && (mean ? t * BN + vrow[i] < nbm : k0 + vrow[i] < kv_hi) ? v : u32x4{0u, 0u, 0u, 0u};
+        const long long in = (long long)g * p.per + block_row(p, end_of(t, i));
+        const bf16_t* base = key ? reinterpret_cast<const bf16_t*>(p.kb) + pgs.v[POOL ? i : 0] * p.kb_sp + in * D
+                                 : reinterpret_cast<const bf16_t*>(p.vb) + pgs.v[POOL ? i : 0] * p.vb_sp + in * Vd;
+        const u32x4 v = *reinterpret_cast<const u32x4*>(base + col[POOL ? i : 0]);
+        st[i] = on[i] && t * BN + vrow[i] < nbm ? v : u32x4{0u, 0u, 0u, 0u};
       }
       return;
     }
-    const int pg = pgs.v[0], k0 = t * BN;
+    const int pg = pgs.pg, k0 = (t + tt0) * BN;
     const long long o0 = ((long long)g << p.shift) + (k0 & ((1 << p.shift) - 1));
     const bf16_t *kb = kc + pg * p.k_sp + o0 * D, *vb = vc + pg * p.v_sp + o0 * Vd;
 #pragma unroll

@@ -235,21 +235,25 @@ __global__ void __launch_bounds__(NW * 64) route_mfma_kernel(RouteArgs p, GroupA
 #pragma unroll
     for (int i = 0; i < 4; ++i) acc[i] = f32x4{0.f, 0.f, 0.f, 0.f};
     auto steps = [&](auto ntc) {
-      constexpr int NTC = decltype(ntc)::value;
-#pragma unroll 2
-      for (int k2 = wv * 2; k2 < nk; k2 += NW * 2)  // 64 columns at a time: whole cache lines of every row
+      constexpr int NTC = decltype(ntc)::value, AH = NTC > 2 ? 4 : 8;  // k steps whose loads fly together
+      for (int k0 = wv * 2; k0 < nk; k0 += NW * AH) {  // 64 columns at a time: whole cache lines of every row
+        u32x4 a[AH][NTC], b[AH];
 #pragma unroll
-        for (int u = 0; u < 2; ++u) {
-          const int c = (k2 + u) * 32 + g * 8;
-          const u32x4 zero = {0u, 0u, 0u, 0u};
-          const u32x4 b = c < d ? *reinterpret_cast<const u32x4*>(h + c) : zero;
+        for (int j = 0; j < AH; ++j) {  // (no load is conditional; columns past d multiply zeros)
+          const int c = (k0 + (j & 1) + (j >> 1) * NW * 2) * 32 + g * 8, cc = min(c, d - 8);
+          const uint32_t keep = c < d ? ~0u : 0u;
+          b[j] = *reinterpret_cast<const u32x4*>(h + cc) & u32x4{keep, keep, keep, keep};
 #pragma unroll
-          for (int i = 0; i < NTC; ++i) {
-            const u32x4 a = c < d ? *reinterpret_cast<const u32x4*>(w[i] + c) : zero;
-            acc[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8, a), __builtin_bit_cast(bf16x8, b),
-                                                             acc[i], 0, 0, 0);
-          }
+          for (int i = 0; i < NTC; ++i) a[j][i] = *reinterpret_cast<const u32x4*>(w[i] + cc);
         }
+        asm volatile("" ::: "memory");
+#pragma unroll
+        for (int j = 0; j < AH; ++j)
+#pragma unroll
+          for (int i = 0; i < NTC; ++i)
+            acc[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8, a[j][i]), __builtin_bit_cast(bf16x8, b[j]),
+                                                             acc[i], 0, 0, 0);
+      }
     };
     if (nt == 1) steps(std::integral_constant<int, 1>{});
     else if (nt == 2) steps(std::integral_constant<int, 2>{});
@@ -289,25 +293,34 @@ struct ExpertArgs {
   const int* tiles;
   const int* ntiles;
   int top, N, K, up, scale;  // up: gate-and-up (x gathered by token, silu product); scale: the weight applies here
+  // gemv: a shared expert beside them, `tokens` rows in order, without a weight (ws null: none)
+  const void* xs;       // [tokens][Ks]
+  const void* ws;       // [2Ns or Ns][Ks]
+  void* ys;             // [tokens][Ns]
+  int tokens, Ns, Ks;
 };
 
 // ------------------------------------------------------------------------------------------------ gemv
-// Workgroup: one tile (<= MT rows of one expert) x 4 waves, a wave streams two weight rows (gate and up
-// of one output, or two outputs); the activation rows of a K chunk are staged in LDS for the four.
+// Workgroup: one tile (<= MT rows of one expert, or of the shared one: the first tiles) x 4 waves, a wave streams two
+// weight rows (gate and up of one output, or two outputs); the activation rows of a K chunk are staged in LDS for the four.
 template <typename E, int MT, bool VEC>
 __global__ void __launch_bounds__(256) expert_gemv_kernel(ExpertArgs p) {
   constexpr int KC = 2048, EPL = 16 / (int)sizeof(E), NL = KC / (64 * EPL);  // elements per lane and load
   extern __shared__ __attribute__((aligned(16))) char raw[];
   E* xs = reinterpret_cast<E*>(raw);  // [MT][KC]
-  if ((int)blockIdx.y >= *p.ntiles) return;
+  const int nsh = p.ws ? (p.tokens + MT - 1) / MT : 0;
+  const bool sh = (int)blockIdx.y < nsh;
+  const int tile = (int)blockIdx.y - nsh, N = sh ? p.Ns : p.N, K = sh ? p.Ks : p.K;
+  if ((!sh && tile >= *p.ntiles) || (int)blockIdx.x * (p.up ? 4 : 8) >= N) return;
   const int tid = threadIdx.x, lane = tid & 63, wv = tid >> 6;
-  const int* tl = p.tiles + blockIdx.y * 5;
-  const int ex = tl[0], lo = tl[1], nr = tl[2], K = p.K;
+  const int* tl = p.tiles + (sh ? 0 : tile) * 5;
+  const int ex = sh ? 0 : tl[0], lo = sh ? blockIdx.y * MT : tl[1], nr = sh ? min(MT, p.tokens - lo) : tl[2];
   const int n0 = p.up ? blockIdx.x * 4 + wv : (blockIdx.x * 4 + wv) * 2;
-  const int rows = p.up ? 2 * p.N : p.N;
-  const int ra = min(n0, p.N - 1), rb = p.up ? p.N + ra : min(n0 + 1, p.N - 1);
-  const E* wa = reinterpret_cast<const E*>(p.w) + ((long long)ex * rows + ra) * K;
-  const E* wb = reinterpret_cast<const E*>(p.w) + ((long long)ex * rows + rb) * K;
+  const int rows = p.up ? 2 * N : N;
+  const int ra = min(n0, N - 1), rb = p.up ? N + ra : min(n0 + 1, N - 1);
+  const E* w = reinterpret_cast<const E*>(sh ? p.ws : p.w);
+  const E* wa = w + ((long long)ex * rows + ra) * K;
+  const E* wb = w + ((long long)ex * rows + rb) * K;
   float acc[2][MT];
 #pragma unroll
   for (int r = 0; r < MT; ++r) acc[0][r] = acc[1][r] = 0.f;
@@ -326,8 +339,8 @@ __global__ void __launch_bounds__(256) expert_gemv_kernel(ExpertArgs p) {
     }
     __syncthreads();
     for (int r = 0; r < nr; ++r) {
-      const long long src = p.up ? p.perm[lo + r] / p.top : lo + r;
-      const E* x = reinterpret_cast<const E*>(p.x) + src * K + k0;
+      const long long src = p.up && !sh ? p.perm[lo + r] / p.top : lo + r;
+      const E* x = reinterpret_cast<const E*>(sh ? p.xs : p.x) + src * K + k0;
       if constexpr (VEC) {
         for (int i = tid * EPL; i < kn; i += 256 * EPL)
           *reinterpret_cast<u32x4*>(xs + r * KC + i) = *reinterpret_cast<const u32x4*>(x + i);
@@ -376,17 +389,17 @@ __global__ void __launch_bounds__(256) expert_gemv_kernel(ExpertArgs p) {
     if (r >= nr) break;
     float a = wave_sum(acc[0][r]), b = wave_sum(acc[1][r]);
     if (lane) continue;
-    if (p.scale) {
+    if (p.scale && !sh) {
       const float s = p.wts[p.perm[lo + r]];
       a *= s;
       b *= s;
     }
-    E* y = reinterpret_cast<E*>(p.y) + (long long)(lo + r) * p.N;
+    E* y = reinterpret_cast<E*>(sh ? p.ys : p.y) + (long long)(lo + r) * N;
     if (p.up) {
-      if (n0 < p.N) ste<E>(y + n0, a * sigmoid(a) * b);
+      if (n0 < N) ste<E>(y + n0, a * sigmoid(a) * b);
     } else {
-      if (n0 < p.N) ste<E>(y + n0, a);
-      if (n0 + 1 < p.N) ste<E>(y + n0 + 1, b);
+      if (n0 < N) ste<E>(y + n0, a);
+      if (n0 + 1 < N) ste<E>(y + n0 + 1, b);
     }
   }
 }
@@ -536,7 +549,8 @@ __global__ void __launch_bounds__(512, 2) expert_gemm_kernel(ExpertArgs p) {
 
 template <typename E, bool VEC>
 int gemv_go(const ExpertArgs& a, int mt, int max_tiles, hipStream_t s) {
-  const dim3 g((a.N + (a.up ? 4 : 8) - 1) / (a.up ? 4 : 8), max_tiles);
+  const int n = a.ws && a.Ns > a.N ? a.Ns : a.N;
+  const dim3 g((n + (a.up ? 4 : 8) - 1) / (a.up ? 4 : 8), max_tiles + (a.ws ? (a.tokens + mt - 1) / mt : 0));
 #define GO(M)                                                                                                  \
   do {                                                                                                         \
     constexpr int lds = M * 2048 * (int)sizeof(E);                                                             \
@@ -587,8 +601,10 @@ KCA_API int kca_moe_route(int dtype, const void* h, const void* wr, const void* 
                           int T, int d, int E, int top, int softmax, const void* fix, int groups, int keep, hipStream_t s) {
   const RouteArgs a{h, wr, wsg, (int*)ids, (float*)wts, (float*)sg, T, d, E, top, softmax, groups, keep, (const float*)fix};
   if (!route_ok(a)) return 1;
-  if (dtype == 1 && d % 8 == 0 && al16(h) && al16(wr) && al16(wsg) && route_lds<8, false>(a) <= MAX_LDS)
-    return route_go<8, false>(a, GroupArgs{}, s);
+  if (dtype == 1 && d % 8 == 0 && al16(h) && al16(wr) && al16(wsg)) {
+    if (T <= 1024 && route_lds<16, false>(a) <= MAX_LDS) return route_go<16, false>(a, GroupArgs{}, s);
+    if (route_lds<8, false>(a) <= MAX_LDS) return route_go<8, false>(a, GroupArgs{}, s);
+  }
   const int lds = ((softmax ? 3 : 1) * E + 1) * 4;
   if (dtype == 1) hipLaunchKernelGGL(route_rows_kernel<bf16_t>, dim3(T), dim3(256), lds, s, a);
   else if (dtype == 0) hipLaunchKernelGGL(route_rows_kernel<float>, dim3(T), dim3(256), lds, s, a);
@@ -623,12 +639,14 @@ KCA_API int kca_moe_route_group(const void* h, const void* wr, const void* wsg, 
 }
 
 // One expert product of every tile. mt: the tiles' row limit (1, 2, 4, 8: gemv; 128: gemm, bf16 with
-// K % 8 == 0 and N % 4 == 0).
+// K % 8 == 0 and N % 4 == 0). ws: a shared expert's product over all tokens beside them (gemv; nullable).
 KCA_API int kca_moe_expert(int dtype, const void* x, const void* w, void* y, const void* perm, const void* wts,
                            const void* tiles, const void* ntiles, int max_tiles, int mt, int top, int N, int K, int up,
-                           int scale, hipStream_t s) {
-  if (max_tiles < 1 || max_tiles > 65535 || N < 1 || K < 1 || top < 1 || !x || !w || !y || !perm || !wts || !tiles || !ntiles) return 1;
-  const ExpertArgs a{x, w, y, (const int*)perm, (const float*)wts, (const int*)tiles, (const int*)ntiles, top, N, K, up, scale};
+                           int scale, const void* xs, const void* ws, void* ys, int tokens, int Ns, int Ks, hipStream_t s) {
+  if (max_tiles < 1 || max_tiles > 32767 || N < 1 || K < 1 || top < 1 || !x || !w || !y || !perm || !wts || !tiles || !ntiles) return 1;
+  if (ws && (!xs || !ys || tokens < 1 || tokens > 32767 || Ns < 1 || Ks < 1 || mt == 128)) return 1;
+  const ExpertArgs a{x, w, y, (const int*)perm, (const float*)wts, (const int*)tiles, (const int*)ntiles, top, N, K, up, scale,
+                     xs, ws, ys, tokens, Ns, Ks};
   if (mt == 128) {
     if (dtype != 1 || K % 8 || N % 4 || !al16(x) || !al16(w) || (uintptr_t)y % 8) return 10;
     const void* kern = up ? (const void*)expert_gemm_kernel<true> : (const void*)expert_gemm_kernel<false>;
@@ -637,7 +655,8 @@ KCA_API int kca_moe_expert(int dtype, const void* x, const void* w, void* y, con
     else hipLaunchKernelGGL(expert_gemm_kernel<false>, dim3((N + 255) / 256 * max_tiles), dim3(512), GEMM_LDS, s, a);
     return hipGetLastError() == hipSuccess ? 0 : 4;
   }
-  const bool vec = K % (dtype == 1 ? 8 : 4) == 0 && al16(x) && al16(w);
+  const int v = dtype == 1 ? 8 : 4;
+  const bool vec = K % v == 0 && al16(x) && al16(w) && (!ws || (Ks % v == 0 && al16(xs) && al16(ws)));
   if (dtype == 0) return vec ? gemv_go<float, true>(a, mt, max_tiles, s) : gemv_go<float, false>(a, mt, max_tiles, s);
   if (dtype == 1) return vec ? gemv_go<bf16_t, true>(a, mt, max_tiles, s) : gemv_go<bf16_t, false>(a, mt, max_tiles, s);
   return 3;

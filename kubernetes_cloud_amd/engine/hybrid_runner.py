@@ -263,10 +263,12 @@ class HybridRunner(StepRunner):
     def _routed(self, L, h, rule):
         """A post-norm layer's routed experts (and the shared one)."""
         mlp, T = L.spec.mlp, h.shape[0]
-        ids, wts, _, g = moe.route_group(h, L.router, mlp.top, None,
-                                         moe.tile_rows(T, mlp.top, mlp.outputs, h.shape[1], mlp.ff, h.dtype), rule)
-        y = moe.experts(h, ids, wts, L.gate_up, L.down, g, mlp.scale_in)
-        a = None
+        mt = moe.tile_rows(T, mlp.top, mlp.outputs, h.shape[1], mlp.ff, h.dtype)
+        ids, wts, _, g = moe.route_group(h, L.router, mlp.top, None, mt, rule)
+        if mlp.shared_ff and moe.shared_ok(T, mt):
+            y, a = moe.experts(h, ids, wts, L.gate_up, L.down, g, mlp.scale_in, (L.w_up, L.w_down))
+            return NormedSum(L.norm2, a, y, g.inv, wts)
+        y, a = moe.experts(h, ids, wts, L.gate_up, L.down, g, mlp.scale_in), None
         if mlp.shared_ff:
             act = torch.empty(T, mlp.shared_ff, device=h.device, dtype=h.dtype)
             a = self._linear(moe.act_rows(self._linear(h, L.w_up), act, gated=True), L.w_down)

@@ -359,7 +359,7 @@ class StepRunner:
         on_gpu = self.device.type == "cuda"
         self.use_graphs = on_gpu if use_graphs is None else (use_graphs and on_gpu)
         self._graphs: dict = {}
-        self._pool = self._side = None
+        self._pool = self._capture_stream = None
         self._static: dict = {}
         self.step_launches: dict = {}
         self._outbufs: dict = {}
@@ -596,9 +596,9 @@ class StepRunner:
         saved = [t.clone() for t in self._step_state()]
         # one stream for warm-up and capture: what the ops keep per stream (zeroed counters) exists before the capture,
         # outside the graphs' shared pool, where another graph's replay would overwrite it
-        if self._side is None:
-            self._side = torch.cuda.Stream()
-        s = self._side
+        if self._capture_stream is None:
+            self._capture_stream = torch.cuda.Stream()
+        s = self._capture_stream
         s.wait_stream(torch.cuda.current_stream())
         with torch.cuda.stream(s):
             for _ in range(2):  # warm up (allocator, hipBLASLt heuristics)

@@ -123,7 +123,7 @@ _SIGS.update({
     "kca_moe_route": [I, P, P, P, P, P, P, I, I, I, I, I, P, I, I, P],
     "kca_moe_group": [P, I, I, I, P, P, P, I, P, P],
     "kca_moe_route_group": [P, P, P, P, P, P, I, I, I, I, I, I, P, I, I, I, P, P, P, I, P, P],
-    "kca_moe_expert": [I, P, P, P, P, P, P, P, I, I, I, I, I, I, I, P],
+    "kca_moe_expert": [I, P, P, P, P, P, P, P, I, I, I, I, I, I, I, P, P, P, I, I, I, P],
     "kca_act_rows": [I, I, P, LL, P, P, P, LL, I, I, F, P],
     "kca_norm_residual": [I, P, P, P, P, LL, P, P, P, P, F, P, P, P, I, I, I, P],
 })

@@ -135,12 +135,17 @@ def append(sp: BiasedHeads, wt: BiasedWeights, x, k_pages, v_pages, table, pos, 
     _call("kca_biased_append", _args(sp, wt, x, k_pages, v_pages, table, pos, slots), code, x.shape[0])
 
 
-def rows_plan(sp: BiasedHeads, rows: int, max_kv: int) -> tuple[int, int, int, int]:
-    """(splits, keys per split, workspace floats, counters) of the rows kernel: enough for either head grouping."""
+def rows_plan(sp: BiasedHeads, rows: int, max_kv: int, target: int = 0, least: int = 64) -> tuple[int, int, int, int]:
+    """(splits, keys per split, workspace floats, counters) of the rows kernel: enough for either head grouping.
+    ``target``: workgroups to aim for with splits of one size, of ``least`` keys or more (0: ``decode_chunk``'s choice)."""
     hg = sp.heads // sp.kv_heads
     rb = 4 if hg > 1 else 1
     sub = -(-hg // rb)
-    chunk = max(decode_chunk(rows, sp.kv_heads * sub, max_kv), -(-max_kv // MAX_SPLITS))
+    if target:
+        n = min(MAX_SPLITS, max(1, target // (rows * sp.kv_heads * sub)), -(-max_kv // least))
+        chunk = -(-max_kv // (32 * n)) * 32
+    else:
+        chunk = max(decode_chunk(rows, sp.kv_heads * sub, max_kv), -(-max_kv // MAX_SPLITS))
     n = -(-max_kv // chunk)
     return n, chunk, (rows * sp.kv_heads * sub * rb * n * (sp.vdim + 2) if n > 1 else 0), rows * sp.heads
 

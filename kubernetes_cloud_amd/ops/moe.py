@@ -15,6 +15,7 @@ from . import _lib
 from .rms_shift import native_dt
 
 GEMM_ROWS = 128
+SHARED_ROWS = 16  # tokens up to which a shared expert's weights stream beside the routed ones'
 
 
 @dataclasses.dataclass(frozen=True)
@@ -133,33 +134,51 @@ def group(ids: torch.Tensor, E: int, mt: int) -> Groups:
     return g
 
 
+def shared_ok(T: int, mt: int) -> bool:
+    """Whether a shared expert streams beside the routed ones' (``experts``): few tokens, streaming products."""
+    return mt != GEMM_ROWS and T <= SHARED_ROWS
+
+
 def experts(h: torch.Tensor, ids: torch.Tensor, weights: torch.Tensor, gate_up: torch.Tensor, down: torch.Tensor,
-            g: Groups, scale_in: bool = True) -> torch.Tensor:
-    """Output rows [n, d] of the routed experts in ``g``'s sorted order."""
+            g: Groups, scale_in: bool = True, shared: tuple | None = None):
+    """Output rows [n, d] of the routed experts in ``g``'s sorted order. ``shared`` (gate and up [2F', d], down [d, F']): an
+    ungated expert for every token in the same launches (``shared_ok``) -> (rows, its output [T, d])."""
     E, F2, d = gate_up.shape
-    F, top, n = F2 // 2, ids.shape[1], ids.numel()
-    code = native_dt(h, gate_up, down)
+    F, top, n, T = F2 // 2, ids.shape[1], ids.numel(), h.shape[0]
+    code = native_dt(h, gate_up, down, *(shared or ()))
     if code is None:
         flat, wt = ids.reshape(-1).long(), weights.reshape(-1)
         y = torch.empty(n, d, dtype=h.dtype)
+
+        def ff(x, up, dn, s_in=1.0):
+            u = up.float() @ (x * s_in)
+            k = u.shape[0] // 2
+            return dn.float() @ (torch.nn.functional.silu(u[:k]) * u[k:])
+
         for pos, a in enumerate(g.perm.tolist()):
             if a < 0:
                 break
-            x, e = h[a // top].float(), int(flat[a])
-            s_in, s_out = (float(wt[a]), 1.0) if scale_in else (1.0, float(wt[a]))
-            u = gate_up[e].float() @ (x * s_in)
-            y[pos] = (down[e].float() @ (torch.nn.functional.silu(u[:F]) * u[F:]) * s_out).to(h.dtype)
-        return y
+            e, w = int(flat[a]), float(wt[a])
+            y[pos] = (ff(h[a // top].float(), gate_up[e], down[e], w if scale_in else 1.0) * (1.0 if scale_in else w)).to(h.dtype)
+        return y if shared is None else (y, torch.stack([ff(r.float(), *shared).to(h.dtype) for r in h]))
     assert h.is_contiguous() and gate_up.is_contiguous() and down.is_contiguous() and down.shape == (E, d, F)
     act = torch.empty(n, F, device=h.device, dtype=h.dtype)
     y = torch.empty(n, d, device=h.device, dtype=h.dtype)
     mx = g.tiles.shape[0]
     common = (g.perm.data_ptr(), weights.data_ptr(), g.tiles.data_ptr(), g.ntiles.data_ptr(), mx, g.mt, top)
+    up_s = down_s = (None, None, None, 0, 0, 0)
+    if shared is not None:
+        w_up, w_down = shared
+        Fs = w_down.shape[1]
+        assert shared_ok(T, g.mt) and w_up.is_contiguous() and w_down.is_contiguous() and w_up.shape == (2 * Fs, d)
+        act_s, y_s = torch.empty(T, Fs, device=h.device, dtype=h.dtype), torch.empty(T, d, device=h.device, dtype=h.dtype)
+        up_s = (h.data_ptr(), w_up.data_ptr(), act_s.data_ptr(), T, Fs, d)
+        down_s = (act_s.data_ptr(), w_down.data_ptr(), y_s.data_ptr(), T, d, Fs)
     _lib.call("kca_moe_expert", code, h.data_ptr(), gate_up.data_ptr(), act.data_ptr(), *common, F, d, 1,
-              int(scale_in), _lib.stream())
+              int(scale_in), *up_s, _lib.stream())
     _lib.call("kca_moe_expert", code, act.data_ptr(), down.data_ptr(), y.data_ptr(), *common, d, F, 0,
-              int(not scale_in), _lib.stream())
-    return y
+              int(not scale_in), *down_s, _lib.stream())
+    return y if shared is None else (y, y_s)
 
 
 ACT_ROWS = {"gelu": 0, "silu_gated": 1, "gelu_tanh_gated": 2, "tanh": 3, "relu2": 4, "softcap": 5}
@@ -192,4 +211,4 @@ def act_rows(x: torch.Tensor, out: torch.Tensor, gated: bool, row_scale: torch.T
     return out
 
 
-__all__ = ["Router", "SIGMOID", "route", "group", "route_group", "experts", "act_rows", "tile_rows", "Groups"]
+__all__ = ["Router", "SIGMOID", "route", "group", "route_group", "experts", "shared_ok", "act_rows", "tile_rows", "Groups"]

@@ -24,7 +24,7 @@ from . import biased_attention as ba
 from .decode import gather_kv
 from .rms_shift import native_dt
 
-rows_plan = ba.rows_plan
+SPLIT_TARGET, SPLIT_MIN = 1024, 96
 
 
 @dataclasses.dataclass(frozen=True)
@@ -88,6 +88,12 @@ def rotary_frequencies(dims: int, base: float, scaling: tuple | None = None) -> 
                 f = (1 - s) * f / factor + s * f
         out.append(f)
     return torch.tensor(out, dtype=torch.float64).float()
+
+
+def rows_plan(sp: PooledHeads, rows: int, max_kv: int) -> tuple[int, int, int, int]:
+    """``biased_attention.rows_plan`` over the keys that are seen: about four workgroups a CU, of 96 keys or more
+    (a window bounds the rows' keys, so they differ little and splits of one size fill the chip evenly)."""
+    return ba.rows_plan(sp, rows, max_kv, SPLIT_TARGET, SPLIT_MIN)
 
 
 def tiles_ok(sp: PooledHeads, dtype, page_size: int, ld: int, ldo: int) -> bool:
