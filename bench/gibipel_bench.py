@@ -72,6 +72,7 @@ def run_kernels(size="4096x8", T=4096, cached=2048, batches=(1, 8, 32), ring=4):
     from kubernetes_cloud_amd.ops import matrix_memory as mm
     from kubernetes_cloud_amd.ops import moe
     from kubernetes_cloud_amd.ops import pooled_attention as pa
+    from kubernetes_cloud_amd.ops import side_step as ss
     from kubernetes_cloud_amd.ops.norm_residual import NormedSum, postnorm
     d, _, _, ah, ag, mh, E, ident, groups, keep, top, ff, _ = SIZES[size]
     dev = torch.device("cuda", torch.cuda.current_device())
@@ -118,7 +119,7 @@ def run_kernels(size="4096x8", T=4096, cached=2048, batches=(1, 8, 32), ring=4):
     V = mh * D
     sp = mm.MemoryHeads(mh, D, D, (0, V, 2 * V, 3 * V, 4 * V, 4 * V + 16), 15.0, 1e-5)
     cols = 4 * V + 32
-    wt = mm.MemoryWeights(torch.zeros(mh, **bf), torch.ones(mh, **bf) * 3, torch.ones(V, **bf))
+    wt = mw = mm.MemoryWeights(torch.zeros(mh, **bf), torch.ones(mh, **bf) * 3, torch.ones(V, **bf))
     state = lambda n: mm.MemoryState(*(torch.zeros(n, w, device=dev) for w in (mh * D * D, mh * D, mh)))  # noqa: E731
     for n_seq in (1, 4):
         L = T // n_seq
@@ -163,7 +164,11 @@ def run_kernels(size="4096x8", T=4096, cached=2048, batches=(1, 8, 32), ring=4):
         ws, cnt = torch.empty(max(wsf, 1), device=dev), torch.zeros(blk, **i32)
         us = _time([lambda c=c: pa.attend_rows(sp, wt, x, c, pos, slot, o, cached, fused=True, ws=ws, cnt=cnt) for c in cs])
         rec(f"pooled_rows B={B} cached={cached} seen={seen} H={ah} G={ag}", us, B * seen * KV * 4, like="biased_rows")
-        del cs
+        ms = mm.MemoryHeads(mh, D, D, (0, V, 2 * V, 3 * V, 4 * V, 4 * V + 16), 15.0, 1e-5)
+        xm, om, sts = torch.randn(B, 4 * V + 32, **bf), torch.empty(B, V, **bf), [state(B) for _ in cs]
+        us = _time([lambda c=c, s=s: ss.step((sp, wt, x, c, o), (ms, mw, xm, s, om), pos, slot, cached, ws, cnt) for c, s in zip(cs, sts)])
+        rec(f"side_step B={B} (pooled_rows and memory_step)", us, B * (seen * KV * 4 + mh * D * (D + 1) * 8), like="biased_rows, delta_step head")
+        del cs, sts
     return out
 
 

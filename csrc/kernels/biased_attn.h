@@ -80,7 +80,7 @@ __device__ __forceinline__ float gate_of(float z) {
 constexpr int MAX_SPLITS = 256;
 
 template <typename E, int RB, int LP, bool VEC, bool POOL>
-__global__ void __launch_bounds__(256, sizeof(E) == 2 && LP <= 16 ? 4 : 1) biased_rows_kernel(BiasedArgs p) {
+__device__ __forceinline__ void rows_body(const BiasedArgs& p, int bx, int by, int sp, int ny) {  // workgroup (bx, by, sp), ny of by
   constexpr int KT = LP >= 64 ? 4 : (LP >= 32 ? 8 : 16);  // keys per tile of a wave
   constexpr int KP = 64 / LP, NPASS = KT / KP;            // keys per pass, passes
   static_assert(KP <= KT, "a pass covers at most one tile");
@@ -88,12 +88,12 @@ __global__ void __launch_bounds__(256, sizeof(E) == 2 && LP <= 16 ? 4 : 1) biase
   __shared__ __attribute__((aligned(16))) float sc[4][KT][RB], als[4][RB];
   __shared__ float wm[4][RB], wl[4][RB];
   __shared__ int s_last;
-  extern __shared__ __attribute__((aligned(16))) float merged[];  // [4][RB][vdim] then reused
+  extern __shared__ __attribute__((aligned(16))) float merged[];  // [4][RB][vdim] then reused; POOL: + the prepared heads
   const int tid = threadIdx.x, lane = tid & 63, wv = tid >> 6;
   const int D = p.dim, Vd = p.vdim, Hg = p.H / p.G;
   const int nsub = (Hg + RB - 1) / RB;
-  const int row = p.row_of ? p.row_of[blockIdx.x] : (int)blockIdx.x;
-  const int g = blockIdx.y / nsub, sub = blockIdx.y % nsub, sp = blockIdx.z;
+  const int row = p.row_of ? p.row_of[bx] : bx;
+  const int g = by / nsub, sub = by % nsub;
   const int h0 = g * Hg + sub * RB, nh = min(RB, Hg - sub * RB);
   const int pos = p.pos[row], slot = p.slot[row];
   const int nbs = POOL ? blocks_seen(p, pos) : 0;                 // keys [0, nbs): block means,
@@ -369,7 +369,7 @@ __global__ void __launch_bounds__(256, sizeof(E) == 2 && LP <= 16 ? 4 : 1) biase
     }
   }
   // waves -> this split's (m, l, acc)
-  const long long blk = ((long long)blockIdx.x * gridDim.y + blockIdx.y);
+  const long long blk = (long long)bx * ny + by;
   const int stride = RB * (Vd + 2);
   float* part = p.ws + (blk * p.nsplit + sp) * stride;
   for (int s = wv; s < RB; s += 4) {
@@ -449,6 +449,11 @@ __global__ void __launch_bounds__(256, sizeof(E) == 2 && LP <= 16 ? 4 : 1) biase
   const E* gr = xr + p.o_g + h0 * Vd;
   for (int i = tid; i < nh * Vd; i += 256)
     El<E>::st(orow + i, POOL ? merged[i] * p.mul : p.o_g >= 0 ? merged[i] * gate_of<E>(El<E>::ld(gr + i)) : merged[i]);
+}
+
+template <typename E, int RB, int LP, bool VEC, bool POOL>
+__global__ void __launch_bounds__(256, sizeof(E) == 2 && LP <= 16 ? 4 : 1) biased_rows_kernel(BiasedArgs p) {
+  rows_body<E, RB, LP, VEC, POOL>(p, blockIdx.x, blockIdx.y, blockIdx.z, gridDim.y);
 }
 
 // ---------------------------------------------------------------------------------------- tile kernel
@@ -742,10 +747,15 @@ __global__ void __launch_bounds__(256, DV > 128 ? 1 : 2) biased_tile_kernel(Bias
     }
 }
 
+template <bool POOL>
+size_t rows_lds(const BiasedArgs& p, int rb) {
+  return ((size_t)4 * rb * p.vdim + (POOL ? pool_lds(rb, p.dim, p.rot) : 0)) * 4;
+}
+
 template <typename E, int RB, int LP, bool VEC, bool POOL>
 int rows_go(const BiasedArgs& p, int rows, hipStream_t s) {
   const int Hg = p.H / p.G, nsub = (Hg + RB - 1) / RB;
-  const size_t lds = ((size_t)4 * RB * p.vdim + (POOL ? pool_lds(RB, p.dim, p.rot) : 0)) * 4;
+  const size_t lds = rows_lds<POOL>(p, RB);
   hipLaunchKernelGGL((biased_rows_kernel<E, RB, LP, VEC, POOL>), dim3(rows, p.G * nsub, p.nsplit), dim3(256), lds, s, p);
   return hipGetLastError() == hipSuccess ? 0 : 4;
 }
@@ -804,20 +814,34 @@ static bool vec_ok(const BiasedArgs& p) {
          p.v_sp % 8 == 0 && (uintptr_t)p.qn % 16 == 0 && (uintptr_t)p.kn % 16 == 0;
 }
 
-// One query token per row. nsplit * chunk must cover the keys of every row (at most max_kv).
-template <bool POOL>
-int rows_entry(const BiasedArgs& p, int dtype, int rows, long long ws_floats, long long n_cnt, int max_kv, hipStream_t s) {
+static bool pool_ok(const BiasedArgs& p) {
+  return args_ok(p) && p.window >= 1 && p.pool >= 1 && p.per >= ((1 << p.shift) + p.pool - 1) / p.pool && p.shift <= 10 && p.kb && p.vb &&
+         p.pool_mul == (unsigned)(((1 << 20) + p.pool - 1) / p.pool) && p.pool <= (1 << 20) && p.qn && p.kn && p.rot >= 0 &&
+         p.rot % 2 == 0 && p.rot <= p.dim && (p.rot == 0 || p.freq) && !p.bias && p.o_g < 0;
+}
+static bool pool_vec(const BiasedArgs& p) {
+  return vec_ok(p) && (uintptr_t)p.kb % 16 == 0 && (uintptr_t)p.vb % 16 == 0 && p.kb_sp % 8 == 0 && p.vb_sp % 8 == 0;
+}
+
+// 0: the rows kernel may run. nsplit * chunk must cover the keys of every row (at most max_kv).
+static int rows_check(const BiasedArgs& p, int rows, long long ws_floats, long long n_cnt, int max_kv) {
   if (!args_ok(p) || !p.pos || !p.slot || !p.out || rows < 1 || p.nsplit < 1 || p.chunk < 1 || p.nsplit > MAX_SPLITS)
     return 1;
   if ((long long)p.nsplit * p.chunk < max_kv) return 2;
-  const bool vec = vec_ok(p);
-  const int rb = rb_for(p.H / p.G, vec), nsub = (p.H / p.G + rb - 1) / rb;
+  const int rb = rb_for(p.H / p.G, vec_ok(p)), nsub = (p.H / p.G + rb - 1) / rb;
   if (p.nsplit > 1) {
     const long long blk = (long long)rows * p.G * nsub;
     if (!p.ws || !p.cnt || n_cnt < blk || ws_floats < blk * p.nsplit * rb * (p.vdim + 2)) return 5;
   }
-  if (dtype == 0) return rows_dispatch<float, POOL>(p, rows, vec, s);
-  if (dtype == 1) return rows_dispatch<bf16_t, POOL>(p, rows, vec, s);
+  return 0;
+}
+
+// One query token per row.
+template <bool POOL>
+int rows_entry(const BiasedArgs& p, int dtype, int rows, long long ws_floats, long long n_cnt, int max_kv, hipStream_t s) {
+  if (const int rc = rows_check(p, rows, ws_floats, n_cnt, max_kv)) return rc;
+  if (dtype == 0) return rows_dispatch<float, POOL>(p, rows, vec_ok(p), s);
+  if (dtype == 1) return rows_dispatch<bf16_t, POOL>(p, rows, vec_ok(p), s);
   return 3;
 }
 

@@ -104,15 +104,6 @@ __global__ void __launch_bounds__(256) mean_kernel(BiasedArgs p, int T) {
   }
 }
 
-bool pool_ok(const BiasedArgs& p) {
-  return args_ok(p) && p.window >= 1 && p.pool >= 1 && p.per >= ((1 << p.shift) + p.pool - 1) / p.pool && p.shift <= 10 && p.kb && p.vb &&
-         p.pool_mul == (unsigned)(((1 << 20) + p.pool - 1) / p.pool) && p.pool <= (1 << 20) && p.qn && p.kn && p.rot >= 0 &&
-         p.rot % 2 == 0 && p.rot <= p.dim && (p.rot == 0 || p.freq) && !p.bias && p.o_g < 0;
-}
-bool pool_vec(const BiasedArgs& p) {
-  return vec_ok(p) && (uintptr_t)p.kb % 16 == 0 && (uintptr_t)p.vb % 16 == 0 && p.kb_sp % 8 == 0 && p.vb_sp % 8 == 0;
-}
-
 template <typename E, int V>
 int prep_go(const BiasedArgs& p, int T, hipStream_t s) {
   const int lds = ((p.rot * 4 + 15) & ~15) + (p.H + p.G) * p.dim * (int)sizeof(E);

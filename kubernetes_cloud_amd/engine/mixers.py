@@ -21,6 +21,7 @@ from ..ops import latent_attention as la
 from ..ops import matrix_memory as mm
 from ..ops import moe
 from ..ops import pooled_attention as pa
+from ..ops import side_step as ss
 
 
 class Mixer:
@@ -231,15 +232,17 @@ class PooledAttentionMixer(Mixer):
         _, _, w, c = pa.rows_plan(self.sp, rows, self.sp.visible(max_kv))
         return {"ws": (w, torch.float32), "cnt": (c, torch.int32)}
 
-    def __call__(self, x, out, b):
+    def pages(self):
         c, i = self.cache, self.index
-        pages = pa.PooledCache(c.k[i], c.v[i], c.k[i + 1], c.v[i + 1], c.table)
-        a = (self.sp, self.wt, x, pages, b.pos, b.slots)
+        return pa.PooledCache(c.k[i], c.v[i], c.k[i + 1], c.v[i + 1], c.table)
+
+    def __call__(self, x, out, b):
+        a = (self.sp, self.wt, x, self.pages(), b.pos, b.slots)
         if b.single:
             pa.attend_rows(*a, out, b.max_kv, fused=True, ws=b.bufs.get("ws"), cnt=b.bufs.get("cnt"))
             return
         pa.prepare(*a)
-        if out.is_cuda and pa.tiles_ok(self.sp, out.dtype, c.page_size, x.stride(0), out.stride(0)):
+        if out.is_cuda and pa.tiles_ok(self.sp, out.dtype, self.cache.page_size, x.stride(0), out.stride(0)):
             if b.tiles is not None:
                 pa.attend_tiles(*a, out, b.tiles)
             if b.row_of is not None:
@@ -262,8 +265,11 @@ class MatrixMemoryMixer(Mixer):
         sp, r = self.sp, self.run
         return {f"mem{r}": (1, sp.heads * sp.dim * sp.vdim), f"memn{r}": (1, sp.heads * sp.dim), f"memm{r}": (1, sp.heads)}
 
+    def memory(self):
+        return mm.MemoryState(*(self.state[f"{k}{self.run}"][0] for k in ("mem", "memn", "memm")))
+
     def __call__(self, x, out, b):
-        st = mm.MemoryState(*(self.state[f"{k}{self.run}"][0] for k in ("mem", "memn", "memm")))
+        st = self.memory()
         if b.single:
             mm.memory_step(self.sp, self.wt, x, st, b.pos, b.slots, out)
         else:
@@ -297,6 +303,16 @@ class SumMixer(SideBySideMixer):
         mx = layer.spec.mixer
         for m, mul in zip(self.sides, (mx.left_mul, mx.right_mul)):
             m.weigh(mul)
+        self.pooled_memory = [type(m) for m in self.sides] == [PooledAttentionMixer, MatrixMemoryMixer]
+
+    def __call__(self, x, out, b):
+        if b.single and self.pooled_memory:  # a decode step of both in one launch
+            (l, r), (xl, xr), (ol, orr) = self.sides, (x[:, c] for c in self.cols), (out[:, o] for o in self.outs)
+            if ss.step_ok(l.sp, r.sp, xl):
+                ss.step((l.sp, l.wt, xl, l.pages(), ol), (r.sp, r.wt, xr, r.memory(), orr), b.pos, b.slots, b.max_kv,
+                        b.bufs.get("ws"), b.bufs.get("cnt"))
+                return
+        super().__call__(x, out, b)
 
 
 MIXERS = {DiffAttentionSpec: DiffAttentionMixer, GatedRecurrenceSpec: GatedRecurrenceMixer,

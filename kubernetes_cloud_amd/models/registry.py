@@ -68,7 +68,7 @@ def _gibipel() -> Family:
         from ..engine.hybrid_runner import HybridRunner
         return HybridRunner
     return Family("gibipel", gibipel.read_config, build_hybrid, gibipel.to_native, gibipel.from_native, runner,
-                  ("norm_residual", "pooled_attn", "matrix_memory", "moe", "act_rows", "gemv", "skinny_mfma"))
+                  ("norm_residual", "pooled_attn", "matrix_memory", "side_step", "moe", "act_rows", "gemv", "skinny_mfma"))
 
 
 def _causal_lm() -> Family:

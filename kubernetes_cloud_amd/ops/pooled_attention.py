@@ -137,6 +137,15 @@ def attend_rows(sp: PooledHeads, wt: PooledWeights, x, c: PooledCache, pos, slot
         if fused:
             _prepare_reference(sp, wt, x, c, pos, slots)
         return _reference(sp, wt, x, c, pos, slots, out, range(x.shape[0]) if row_of is None else row_of.tolist())
+    a, n, wsn, cn, kv, keep = rows_args(sp, wt, x, c, pos, slots, out, max_len, fused, row_of, ws, cnt)
+    ba._call("kca_pooled_rows", a, code, n, wsn, cn, kv)
+    del keep
+    return out
+
+
+def rows_args(sp, wt, x, c, pos, slots, out, max_len, fused, row_of, ws, cnt):
+    """The rows kernel's descriptor -> (descriptor, rows, workspace floats, counters, most keys, what must stay alive until
+    the launch)."""
     n = x.shape[0] if row_of is None else row_of.shape[0]
     kv = sp.visible(max_len)
     splits, chunk, wsf, blocks = rows_plan(sp, n, kv)
@@ -149,8 +158,7 @@ def attend_rows(sp: PooledHeads, wt: PooledWeights, x, c: PooledCache, pos, slot
     a.append, a.nsplit, a.chunk, a.row_of = int(fused), splits, chunk, _lib.ptr(row_of)
     a.ws, a.cnt = _lib.ptr(ws), _lib.ptr(cnt)
     assert row_of is None or row_of.dtype == torch.int32
-    ba._call("kca_pooled_rows", a, code, n, ws.numel() if ws is not None else 0, cnt.numel() if cnt is not None else 0, kv)
-    return out
+    return a, n, ws.numel() if ws is not None else 0, cnt.numel() if cnt is not None else 0, kv, (ws, cnt)
 
 
 def attend_tiles(sp: PooledHeads, wt: PooledWeights, x, c: PooledCache, pos, slots, out, tiles: torch.Tensor):

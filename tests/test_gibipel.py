@@ -24,6 +24,7 @@ from kubernetes_cloud_amd.ops import diff_attention as da
 from kubernetes_cloud_amd.ops import matrix_memory as mm
 from kubernetes_cloud_amd.ops import moe
 from kubernetes_cloud_amd.ops import pooled_attention as pa
+from kubernetes_cloud_amd.ops import side_step as ss
 from kubernetes_cloud_amd.ops.norm_residual import Embedded, NormedSum, postnorm
 
 
@@ -565,6 +566,40 @@ def test_extreme_gates(device, dtype, kind, how):
     for cuts in ([200], [64, 2, 70, 64], [120] + [1] * 20 + [60]):
         got = d.cut(cuts, device, dtype)
         assert torch.isfinite(got).all() and rel(got, want) < (3e-5 if dtype == F32 else 2.5e-2), (cuts, rel(got, want))
+
+
+@pytest.mark.gpu
+@pytest.mark.parametrize("heads,groups,dim,vdim,mdim,mvdim", [(8, 2, 64, 64, 48, 40), (5, 1, 128, 96, 128, 136), (6, 3, 40, 128, 104, 64),
+                                                              (12, 2, 24, 56, 64, 24), (4, 1, 128, 128, 72, 128)])
+def test_both_mixers_in_one_launch(heads, groups, dim, vdim, mdim, mvdim):
+    """The decode step of attention and memory together leaves what the two steps leave: outputs, pages, block means, state."""
+    T = 70
+    d = Pooled(left(heads, groups, dim, vdim, 30, 5, 16), T, seed=91)
+    e = Memory(right(3, mdim, mvdim), T, seed=92)
+    runs = []
+    for together in (False, True):
+        c, st, got = d.cache(4, "cuda", BF16, 32), e.state(3, "cuda"), []
+        d.step([(d.x[:20], 0, 1), (d.x[:40], 0, 0)], c, "cuda", BF16, 40)
+        e.run([(e.x[:20], 0, 1), (e.x[:40], 0, 0)], st, "cuda", BF16)
+        for t in range(28):
+            pos, slots = (torch.tensor(v, dtype=torch.int32, device="cuda") for v in ([20 + t, 40 + t], [1, 0]))
+            xs = torch.cat([torch.stack([m.x[20 + t], m.x[40 + t]]) for m in (d, e)], 1).to("cuda", BF16)
+            xa, xm = xs[:, :d.x.shape[1]], xs[:, d.x.shape[1]:]
+            oa, om = torch.empty(2, heads * vdim, device="cuda", dtype=BF16), torch.empty(2, 3 * mvdim, device="cuda", dtype=BF16)
+            wa, wm = d.weights("cuda", BF16), e.weights("cuda", BF16)
+            if together:
+                assert ss.step_ok(d.sp, e.sp, xa)
+                ss.step((d.sp, wa, xa, c, oa), (e.sp, wm, xm, st, om), pos, slots, 41 + t)
+            else:
+                pa.attend_rows(d.sp, wa, xa, c, pos, slots, oa, 41 + t, fused=True)
+                mm.memory_step(e.sp, wm, xm, st, pos, slots, om)
+            got += [oa, om]
+        runs.append(got + [c.k, c.v, c.kb, c.vb, st.s, st.n, st.m])
+    want = d.want(d.x), e.want(e.x)
+    for j in range(2):
+        assert rel(torch.stack([o[0] for o in runs[1][j:56:2]]), want[j][20:48]) < 2e-2
+    for a, b in zip(*runs):
+        assert rel(b, a.double().cpu()) < 5e-3
 
 
 # -------------------------------------------------------------------------------------------- models
