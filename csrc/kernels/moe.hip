@@ -18,6 +18,7 @@
 // activations are [n][F], their outputs [n][d]; the residual pass (rms_shift.hip) sums a token's outputs
 // through `inv`.
 #include "common.h"
+#include "lanes.h"
 
 #include <type_traits>
 
@@ -113,8 +114,57 @@ __device__ __forceinline__ void pick_softmax(const RouteArgs& p, float* z, float
   for (int k = lane; k < p.top; k += 64) p.wts[(long long)t * p.top + k] = w[k] / (total + 1e-20f);
 }
 
+__device__ __forceinline__ float lane_of(float v, int j) {
+  return __int_as_float(__builtin_amdgcn_readlane(__float_as_int(v), j));
+}
+
+// Both rules for up to 64 outputs, one a lane: choices by rank, all at once. (NaN counts as the least; ties go to the
+// lower index, so ranks are distinct.)
+__device__ __forceinline__ void pick_lanes(const RouteArgs& p, const float* z, float fix, int t, int lane, int* ids_lds) {
+  const bool on = lane < p.E;
+  float s = on ? z[lane] : -INFINITY, c;
+  if (p.softmax) {
+    auto add = [](float a, float b) { return a + b; };
+    auto big = [](float a, float b) { return fmaxf(a, b); };
+    const float mx = lanes_reduce<64>(s, big), e = on ? expf(s - mx) : 0.f;
+    s = e / lanes_reduce<64>(e, add);
+    c = on ? s + fix : -INFINITY;
+    if (c != c) c = -INFINITY;
+    if (p.keep < p.groups) {
+      const int size = p.E / p.groups, g = lane / size;
+      float best = -INFINITY;
+      int ahead = 0;  // groups before this lane's
+      for (int j = 0; j < size; ++j) best = fmaxf(best, __shfl(c, g * size + j, 64));
+      for (int j = 0; j < p.groups; ++j) {
+        const float o = lane_of(best, j * size);
+        ahead += o > best || (o == best && j < g);
+      }
+      if (ahead >= p.keep) c = -INFINITY;
+    }
+  } else {
+    c = s != s ? -INFINITY : s;
+  }
+  int rank = 0;
+  for (int j = 0; j < p.E; ++j) {
+    const float o = lane_of(c, j);
+    rank += o > c || (o == c && j < lane);
+  }
+  const bool take = on && rank < p.top;
+  float w = sigmoid(s);
+  if (p.softmax) w = s / (lanes_reduce<64>(take ? s : 0.f, [](float a, float b) { return a + b; }) + 1e-20f);
+  if (take) {
+    p.ids[(long long)t * p.top + rank] = lane;
+    if (ids_lds) ids_lds[t * p.top + rank] = lane;
+    p.wts[(long long)t * p.top + rank] = w;
+  }
+}
+
+// this lane's correction, requested early
+__device__ __forceinline__ float lane_fix(const RouteArgs& p, int lane) { return p.fix && p.E <= 64 && lane < p.E ? p.fix[lane] : 0.f; }
+
 // One wave: the top experts of one token from its logits z[E] (LDS; softmax: E floats each at c and w).
-__device__ __forceinline__ void pick(const RouteArgs& p, float* z, float* c, float* w, int t, int lane, int* ids_lds = nullptr) {
+__device__ __forceinline__ void pick(const RouteArgs& p, float* z, float* c, float* w, float fix, int t, int lane, int* ids_lds = nullptr) {
+  if (p.E <= 64) return pick_lanes(p, z, fix, t, lane, ids_lds);
   if (p.softmax) return pick_softmax(p, z, c, w, t, lane, ids_lds);
   for (int k = 0; k < p.top; ++k) {
     float best;
@@ -145,7 +195,7 @@ __global__ void __launch_bounds__(256) route_rows_kernel(RouteArgs p) {
     if (lane == 0) z[e] = s;
   }
   __syncthreads();
-  if (wv == 0) pick(p, z, z + n, z + n + p.E, t, lane);
+  if (wv == 0) pick(p, z, z + n, z + n + p.E, lane_fix(p, lane), t, lane);
   if (threadIdx.x == 64 && p.wsg) p.sg[t] = sigmoid(z[p.E]);
 }
 
@@ -223,6 +273,7 @@ __global__ void __launch_bounds__(NW * 64) route_mfma_kernel(RouteArgs p, GroupA
   const int t0 = blockIdx.x * 16, d = p.d;
   const bf16_t* h = reinterpret_cast<const bf16_t*>(p.h) + (long long)min(t0 + r16, p.T - 1) * d;
   const int nk = (d + 31) / 32;
+  const float fix = lane_fix(p, lane);
   for (int e0 = 0; e0 < n; e0 += 64) {
     const bf16_t* w[4];
 #pragma unroll
@@ -275,7 +326,7 @@ __global__ void __launch_bounds__(NW * 64) route_mfma_kernel(RouteArgs p, GroupA
   for (int r = wv; r < 16; r += NW) {
     if (t0 + r >= p.T) break;
     if (p.wsg && lane == 0) p.sg[t0 + r] = sigmoid(z[r * zs + p.E]);
-    pick(p, z + r * zs, z + zr + r * zs, z + 2 * zr + r * zs, t0 + r, lane, GROUP ? sids : nullptr);
+    pick(p, z + r * zs, z + zr + r * zs, z + 2 * zr + r * zs, fix, t0 + r, lane, GROUP ? sids : nullptr);
   }
   if constexpr (GROUP) {
     __syncthreads();
