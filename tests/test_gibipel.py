@@ -367,7 +367,7 @@ def test_norm_over_all_heads(device, dtype):
 
 @pytest.mark.gpu
 @pytest.mark.parametrize("dtype", [F32, BF16])
-@pytest.mark.parametrize("shape", [(8, 2, 64, 64, 300, 4), (9, 3, 96, 80, 700, 16), (3, 3, 24, 40, 5, 2), (5, 1, 11, 13, 900, 1), (2, 1, 128, 256, 256, 64)])
+@pytest.mark.parametrize("shape", [(8, 4, 64, 80, 300, 4), (9, 3, 96, 80, 700, 16), (3, 3, 24, 40, 5, 2), (5, 1, 11, 13, 900, 1), (2, 1, 128, 256, 256, 64)])
 def test_pooled_decode_over_key_splits(dtype, shape):
     """Rows of unequal length over a long cache cut in splits: prepared portions, then fused single tokens."""
     H, G, D, E, window, pool = shape
@@ -569,7 +569,7 @@ def test_extreme_gates(device, dtype, kind, how):
 
 
 @pytest.mark.gpu
-@pytest.mark.parametrize("heads,groups,dim,vdim,mdim,mvdim", [(8, 2, 64, 64, 48, 40), (5, 1, 128, 96, 128, 136), (6, 3, 40, 128, 104, 64),
+@pytest.mark.parametrize("heads,groups,dim,vdim,mdim,mvdim", [(8, 4, 56, 64, 40, 56), (5, 1, 128, 96, 128, 136), (6, 3, 40, 128, 104, 64),
                                                               (12, 2, 24, 56, 64, 24), (4, 1, 128, 128, 72, 128)])
 def test_both_mixers_in_one_launch(heads, groups, dim, vdim, mdim, mvdim):
     """The decode step of attention and memory together leaves what the two steps leave: outputs, pages, block means, state."""
