@@ -99,7 +99,6 @@ def _args(sp: BiasedHeads, wt: BiasedWeights, x, k_pages, v_pages, table, pos, s
     assert all(t is None or (t.is_contiguous() and t.numel() == D and t.dtype == x.dtype) for t in (wt.q_norm, wt.k_norm))
     assert wt.bias is None or (wt.bias.is_contiguous() and wt.bias.dtype == torch.float32 and wt.bias.shape[0] == H)
     assert wt.sink is None or (wt.sink.is_contiguous() and wt.sink.dtype == torch.float32 and wt.sink.numel() == H)
-    _abi()
     a, p = _Args(), _lib.ptr
     a.x, a.ld = x.data_ptr(), x.stride(0)
     a.o_q, a.o_k, a.o_v, a.o_g = sp.at
@@ -116,6 +115,8 @@ def _args(sp: BiasedHeads, wt: BiasedWeights, x, k_pages, v_pages, table, pos, s
 
 
 def _call(name, a, *args):
+    if name.startswith("kca_biased"):  # (the pooled entry points check theirs)
+        _abi()
     fn = getattr(_lib.require(), name)
     kinds = [ctypes.c_longlong if i in (2, 3) and name.endswith("_rows") else ctypes.c_int for i in range(len(args))]
     fn.argtypes, fn.restype = [ctypes.c_void_p, *kinds, ctypes.c_void_p], ctypes.c_int
