@@ -1,6 +1,6 @@
 """Mixture of gated experts (``csrc/kernels/moe.hip``): top-k router (sigmoid scores, or softmax scores with a correction
-of the choice, expert groups and identity experts), grouping by expert, expert products with the router weight on the expert's input (or output), and the strided feed-forward
-activations (``csrc/kernels/act_rows.hip``).
+of the choice, expert groups and identity experts), grouping by expert, expert products with the router weight on the
+expert's input (or output), and the strided feed-forward activations (``csrc/kernels/act_rows.hip``).
 
 Expert weights are stacked: gate-and-up [E, 2F, d] (gate rows first), down [E, d, F].
 """

@@ -14,6 +14,7 @@ block lives and is shared, copied and given back with the page of its last token
 """
 from __future__ import annotations
 
+import ctypes
 import dataclasses
 import math
 
@@ -109,7 +110,7 @@ def _args(sp: PooledHeads, wt: PooledWeights, x, c: PooledCache, pos, slots, out
     assert all(t.is_contiguous() and t.numel() == n * D and t.dtype == x.dtype
                for t, n in ((wt.q_norm, sp.heads), (wt.k_norm, G)))
     assert wt.freq.is_contiguous() and wt.freq.dtype == torch.float32 and wt.freq.numel() == sp.rot // 2
-    if _lib.require().kca_pooled_attn_abi() != ba.ctypes.sizeof(ba._Args):
+    if _lib.require().kca_pooled_attn_abi() != ctypes.sizeof(ba._Args):
         raise RuntimeError("kca_pooled_attn descriptor: C and ctypes sizes differ")
     core = ba.BiasedHeads(sp.heads, G, D, E, sp.scale, sp.eps, (*sp.at, -1))
     a = ba._args(core, ba.BiasedWeights(sink=wt.sink), x, c.k, c.v, c.table, pos, slots, out)
